@@ -10,6 +10,44 @@ from __future__ import annotations
 from dataclasses import dataclass
 
 
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Latent attention: keys and values are linear images of one cached
+    latent per token (plus one rotated key part all heads share)."""
+    heads: int
+    dim: int                        # unrotated query/key size per head
+    rot_dim: int                    # rotated query/key size per head
+    vdim: int                       # value size per head
+    kv_rank: int                    # latent size
+    scale: float                    # factor on the scores
+    rope_base: float = 10000.0
+    rope_dims: int | None = None    # rotated part of rot_dim (None: all)
+    window: int | None = None       # keys a query sees, itself included
+    kv_from: int | None = None      # layer whose latents this layer reads
+
+    @property
+    def rotation(self) -> tuple[float, int]:
+        return (self.rope_base, self.rope_dims or self.rot_dim)
+
+
+@dataclass(frozen=True)
+class GatedMLPSpec:
+    """Clamped gated unit: g = min(gate, limit), u = clamp(up, +-limit),
+    y = g * sigmoid(alpha * g) * (u + shift)."""
+    ff: int
+    limit: float
+    alpha: float = 1.702
+    shift: float = 1.0
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    """One layer of a model whose layers differ: both sublayers read the
+    same normed input and are summed into a 32-bit residual."""
+    mixer: LatentAttentionSpec
+    mlp: GatedMLPSpec | None
+
+
 @dataclass
 class ModelConfig:
     name: str
@@ -37,14 +75,50 @@ class ModelConfig:
     attn_bias: bool = False   # bias on q/k/v AND o_proj (OPT)
     qkv_bias: bool = False    # bias on q/k/v only (qwen2)
     embed_scale: float = 1.0  # gemma multiplies embeddings by sqrt(hidden)
+    # models described layer by layer (None: every layer is the one the
+    # fields above describe)
+    layers: tuple[LayerSpec, ...] | None = None
 
     def __post_init__(self):
+        if self.layers is not None:
+            self.layers = tuple(self.layers)
+            self._check_layers()
         if self.head_dim is None:
             self.head_dim = self.hidden_size // self.num_heads
+
+    def _check_layers(self):
+        for i, lay in enumerate(self.layers):
+            m = lay.mixer
+            if min(m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank) < 1 or \
+                    m.rotation[1] % 2 or m.rotation[1] > m.rot_dim:
+                raise ValueError(f"layer {i}: bad mixer sizes {m}")
+            if m.window is not None and m.window < 1:
+                raise ValueError(f"layer {i}: window {m.window}")
+            if m.kv_from is None:
+                continue
+            if not 0 <= m.kv_from < i:
+                raise ValueError(f"layer {i}: kv_from {m.kv_from}")
+            src = self.layers[m.kv_from].mixer
+            if src.kv_from is not None or \
+                    (src.kv_rank, src.rot_dim, src.rotation) != \
+                    (m.kv_rank, m.rot_dim, m.rotation):
+                raise ValueError(f"layer {i} cannot read the latents of "
+                                 f"layer {m.kv_from}: {src} vs {m}")
 
     @property
     def params_b(self) -> float:
         """Rough parameter count in billions."""
+        if self.layers is not None:
+            n = 2 * self.vocab_size * self.hidden_size
+            for lay in self.layers:
+                m, h = lay.mixer, self.hidden_size
+                n += h * m.heads * (m.dim + m.rot_dim + 2 * m.vdim) + \
+                    m.kv_rank * m.heads * (m.dim + m.vdim)
+                if m.kv_from is None:
+                    n += h * (m.kv_rank + m.rot_dim)
+                if lay.mlp is not None:
+                    n += 3 * h * lay.mlp.ff
+            return n / 1e9
         h, l, v = self.hidden_size, self.num_layers, self.vocab_size
         kvh = self.num_kv_heads * self.head_dim
         attn = h * (self.num_heads * self.head_dim) + 2 * h * kvh + \
@@ -52,6 +126,26 @@ class ModelConfig:
         mlp = (3 if self.act == "silu_glu" else 2) * h * self.intermediate_size
         emb = v * h * (1 if self.tie_embeddings else 2)
         return (l * (attn + mlp) + emb) / 1e9
+
+
+def layered_config(name: str, layers, width: int, vocab: int,
+                   norm_eps: float = 1e-5,
+                   max_seq_len: int = 131072) -> ModelConfig:
+    """A ModelConfig of a layer-by-layer model. The engine-wide fields
+    follow from the layers: cached tokens may be dropped once they are
+    outside every layer's window."""
+    layers = tuple(layers)
+    windows = [lay.mixer.window for lay in layers]
+    m = layers[0].mixer
+    return ModelConfig(
+        name, vocab_size=vocab, hidden_size=width, num_layers=len(layers),
+        num_heads=max(lay.mixer.heads for lay in layers), num_kv_heads=1,
+        intermediate_size=max((lay.mlp.ff for lay in layers if lay.mlp),
+                              default=0),
+        max_seq_len=max_seq_len, head_dim=m.dim + m.rot_dim,
+        norm_eps=norm_eps, parallel_residual=True, single_norm=True,
+        sliding_window=None if None in windows else max(windows),
+        layers=layers)
 
 
 _REGISTRY: dict[str, ModelConfig] = {}
@@ -187,3 +281,35 @@ register(ModelConfig("tiny-opt", vocab_size=256, hidden_size=64,
                      intermediate_size=128, max_seq_len=128,
                      norm="layernorm", act="relu", pos="learned",
                      tie_embeddings=True, mlp_bias=True, attn_bias=True))
+
+
+# --- Pimazen family (latent attention in parallel with a clamped gated MLP) --
+def _pimazen(name: str, n_layers: int, width: int, vocab: int, ff, mixer,
+             share_every: int = 0, limit: float = 7.0, **kw) -> ModelConfig:
+    """Equal layers; with share_every = n, n - 1 of n layers read the
+    latents of the first one of their group."""
+    layers = []
+    for i in range(n_layers):
+        first = i - i % share_every if share_every else i
+        src = None if first == i else first
+        layers.append(LayerSpec(
+            LatentAttentionSpec(kv_from=src, **mixer),
+            GatedMLPSpec(ff, limit) if ff else None))
+    return register(layered_config(name, layers, width, vocab, **kw))
+
+
+_pimazen("tiny-pimazen", 3, 64, 256, 96,
+         dict(heads=3, dim=24, rot_dim=8, vdim=16, kv_rank=40, window=24,
+              scale=32 ** -0.5), share_every=2, max_seq_len=256)
+_pimazen("smoke-pimazen", 4, 256, 512, 384,
+         dict(heads=4, dim=64, rot_dim=32, vdim=64, kv_rank=128, window=96,
+              scale=96 ** -0.5), share_every=2, max_seq_len=1024)
+# sized like the layers of llama2-7b / mistral-7b and a narrower model
+_pimazen("pimazen-7b", 32, 4096, 32000, 11008,
+         dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512,
+              window=4096, scale=192 ** -0.5, rope_base=1000000.0),
+         share_every=2, max_seq_len=32768)
+_pimazen("pimazen-1b", 16, 2048, 32000, 5632,
+         dict(heads=16, dim=64, rot_dim=32, vdim=64, kv_rank=256,
+              window=2048, scale=96 ** -0.5), share_every=2,
+         max_seq_len=32768)

@@ -1,0 +1,159 @@
+"""Layers of models described layer by layer: latent attention beside a
+clamped gated MLP, both fed by one norm, summed into a 32-bit residual.
+
+Serving runs a layer as two products around the attention (ops/latent.py):
+one wide projection of the normed input (queries, latent, gates, both MLP
+inputs) and one output projection of [gated heads | MLP activation], so the
+parallel sum never leaves the accumulators. `fuse()` builds those weights
+from the loaded parameters.
+
+Tensor parallelism: heads and MLP columns are sharded, the latent
+projection (and so the cache) is replicated; the shared output projection
+makes it one all-reduce per layer.
+"""
+from __future__ import annotations
+
+import torch
+from torch import nn
+
+from .. import ops
+from ..ops import latent as L
+from ..parallel import ColumnParallelLinear, RowParallelLinear, reduce_from_tp
+from .config import GatedMLPSpec, LatentAttentionSpec, LayerSpec, ModelConfig
+
+
+class LatentAttention(nn.Module):
+    """Parameters of one latent-attention mixer."""
+
+    def __init__(self, cfg: ModelConfig, spec: LatentAttentionSpec, dtype,
+                 tp: int):
+        super().__init__()
+        if spec.heads % tp:
+            raise ValueError(f"{spec.heads} heads do not divide tp={tp}")
+        D, H = cfg.hidden_size, spec.heads
+
+        def col(n, k):
+            return ColumnParallelLinear(k, n, tp_size=tp, dtype=dtype)
+
+        self.q_proj = col(H * (spec.dim + spec.rot_dim), D)
+        if spec.kv_from is None:
+            self.dkv_proj = ops.Linear(D, spec.kv_rank + spec.rot_dim,
+                                       bias=False, dtype=dtype)
+            self.kv_norm = ops.RMSNorm(spec.kv_rank, eps=cfg.norm_eps,
+                                       dtype=dtype)
+        self.uk_proj = col(H * spec.dim, spec.kv_rank)
+        self.uv_proj = col(H * spec.vdim, spec.kv_rank)
+        self.g_proj = col(H * spec.vdim, D)
+        self.o_proj = RowParallelLinear(H * spec.vdim, D, tp_size=tp,
+                                        dtype=dtype)
+
+
+class GatedMLP(nn.Module):
+    """Parameters of one clamped gated MLP."""
+
+    def __init__(self, cfg: ModelConfig, spec: GatedMLPSpec, dtype, tp: int):
+        super().__init__()
+        D = cfg.hidden_size
+        self.gate_proj = ColumnParallelLinear(D, spec.ff, tp_size=tp,
+                                              dtype=dtype)
+        self.up_proj = ColumnParallelLinear(D, spec.ff, tp_size=tp,
+                                            dtype=dtype)
+        self.down_proj = RowParallelLinear(spec.ff, D, tp_size=tp,
+                                           dtype=dtype)
+
+
+class ParallelBlock(nn.Module):
+    def __init__(self, cfg: ModelConfig, spec: LayerSpec, dtype, tp: int):
+        super().__init__()
+        self.spec, self.tp, self.dtype = spec, tp, dtype
+        m = spec.mixer
+        self.norm1 = ops.RMSNorm(cfg.hidden_size, eps=cfg.norm_eps,
+                                 dtype=dtype)
+        self.attn = LatentAttention(cfg, m, dtype, tp)
+        self.mlp = (GatedMLP(cfg, spec.mlp, dtype, tp) if spec.mlp else None)
+        self.lay = L.LatentLayout(
+            heads=m.heads // tp, dim=m.dim, rot=m.rot_dim, vdim=m.vdim,
+            rank=m.kv_rank, ff=spec.mlp.ff // tp if spec.mlp else 0,
+            own_latent=m.kv_from is None)
+        self.expandable = (L.latent_flash_supported(self.lay, dtype) and
+                           dtype == torch.bfloat16)
+        self.wide_w = None
+
+    @torch.no_grad()
+    def fuse(self) -> list[torch.Tensor]:
+        """Serving weights from the loaded parameters; returns those the
+        decode GEMM may keep a copy of. Parameters whose rows appear
+        unpadded in the wide weight become views of it."""
+        a, m, lay = self.attn, self.mlp, self.lay
+        own = lay.own_latent
+        self.wide_w = L.pack_wide(
+            lay, a.q_proj.weight, a.dkv_proj.weight if own else None,
+            a.g_proj.weight, m and m.gate_proj.weight,
+            m and m.up_proj.weight)
+        self.out_w = L.pack_out(lay, a.o_proj.weight, m and m.down_proj.weight)
+        uk = a.uk_proj.weight.view(lay.heads, lay.dim, lay.rank)
+        uv = a.uv_proj.weight.view(lay.heads, lay.vdim, lay.rank)
+        pad = nn.functional.pad
+        r = lay.rc - lay.rank
+        self.absorb_w = L.pack_heads(
+            pad(uk, (0, r, 0, lay.dimc - lay.dim)))
+        self.expand_w = L.pack_heads(
+            pad(uv, (0, r, 0, lay.vc - lay.vdim)).transpose(1, 2))
+        self.context_w = L.pack_expand(lay, a.uk_proj.weight,
+                                       a.uv_proj.weight)
+
+        def adopt(lin, row, padded):
+            n = lin.weight.shape[0]
+            if n == padded:
+                lin.weight = nn.Parameter(self.wide_w[row:row + n],
+                                          requires_grad=False)
+
+        if lay.qc == lay.dim + lay.rot:
+            adopt(a.q_proj, 0, lay.off_kv)
+        if own and lay.ec == lay.rank + lay.rot:
+            adopt(a.dkv_proj, lay.off_kv, lay.ec)
+        adopt(a.g_proj, lay.off_g, lay.off_gate - lay.off_g)
+        if m is not None:
+            adopt(m.gate_proj, lay.off_gate, lay.fc)
+            adopt(m.up_proj, lay.off_up, lay.fc)
+        return [self.wide_w, self.out_w]
+
+    def step(self, x, delta, batch, cache, rope, contexts):
+        """x [T, D] fp32 residual before this layer without `delta`, the
+        last layer's pending output; adds delta to x in place and returns
+        this layer's own. `contexts` keeps gathered latents for the layers
+        that read the same ones."""
+        lay, spec = self.lay, self.spec.mixer
+        T = x.shape[0]
+        h = ops.rmsnorm_res32(x, delta, self.norm1.weight, self.norm1.eps,
+                              self.dtype,
+                              operand=ops.decode_ready(self.wide_w, T))
+        y = ops.fast_linear(h, self.wide_w)
+        z = torch.empty(T, lay.n_z, dtype=y.dtype, device=y.device)
+        zs = None
+        if ops.decode_ready(self.out_w, T):
+            zs = ops.decode_operand(T, lay.n_z, z)
+        norm = self.attn.kv_norm if lay.own_latent else None
+        L.latent_prep(y, lay, *rope, batch.positions, batch.slots, cache,
+                      norm and norm.weight, norm.eps if norm else 0.0,
+                      self.spec.mlp, z, zs)
+        if batch.t_short:
+            q_lat = L.latent_absorb(y, lay, self.absorb_w, batch.t_short)
+            o_lat = L.latent_attend(q_lat, y, lay, cache, batch, spec.scale,
+                                    spec.window)
+            L.latent_expand(o_lat, lay, self.expand_w, y, z, zs)
+        if batch.long_plans:
+            slots, meta = batch.long_plans[spec.window]
+            key = (cache.data_ptr(), spec.window)
+            if key not in contexts:
+                contexts[key] = cache.view(-1, lay.ec).index_select(0, slots)
+            ctx = contexts[key]
+            kv = nn.functional.linear(ctx[:, :lay.rc], self.context_w)
+            L.latent_flash(y, lay, kv, ctx, meta, batch.max_q_long,
+                           spec.scale, spec.window, z)
+        if zs is not None:
+            z._rb_swz = zs
+            if self.tp == 1:
+                return ops.decode_linear_raw(z, self.out_w)[0]
+        out = ops.linear_f32(z, self.out_w)
+        return reduce_from_tp(out) if self.tp > 1 else out

@@ -11,6 +11,7 @@ TP-shards each tensor for the local rank.
 from __future__ import annotations
 
 import json
+import warnings
 from pathlib import Path
 
 import torch
@@ -20,6 +21,8 @@ from .transformer import Transformer
 
 
 def detect_family(cfg: ModelConfig) -> str:
+    if cfg.layers is not None:
+        return "pimazen"
     if cfg.pos == "learned":
         return "gpt2" if cfg.act == "gelu_tanh" else "opt"
     if cfg.parallel_residual:
@@ -88,6 +91,24 @@ def _map_falcon(name: str):
     return n
 
 
+_PIMAZEN = {"mix.q": "attn.q_proj", "mix.dkv": "attn.dkv_proj",
+            "mix.dkv.norm": "attn.kv_norm", "mix.uk": "attn.uk_proj",
+            "mix.uv": "attn.uv_proj", "mix.g": "attn.g_proj",
+            "mix.o": "attn.o_proj", "mlp.gate": "mlp.gate_proj",
+            "mlp.up": "mlp.up_proj", "mlp.down": "mlp.down_proj",
+            "norm1": "norm1"}
+_PIMAZEN_TOP = {"embed": "embed", "final.norm": "norm_f", "head": "lm_head"}
+
+
+def _map_pimazen(name: str):
+    if name in _PIMAZEN_TOP:
+        return _PIMAZEN_TOP[name] + ".weight"
+    layer, _, rest = name.partition(".")
+    if layer[:1] == "l" and layer[1:].isdigit() and rest in _PIMAZEN:
+        return f"blocks.{layer[1:]}.{_PIMAZEN[rest]}.weight"
+    return name
+
+
 def _split_falcon_qkv(w: torch.Tensor, cfg: ModelConfig):
     """Falcon fuses QKV as [n_kv_groups, (g_q + 2), head_dim, hidden] with
     the group's q heads followed by its k and v head."""
@@ -104,7 +125,8 @@ def convert_hf_state_dict(hf_state: dict, cfg: ModelConfig) -> dict:
     family = detect_family(cfg)
     out: dict[str, torch.Tensor] = {}
     mapper = {"llama": _map_llama, "opt": _map_opt,
-              "falcon": _map_falcon, "gpt2": _map_gpt2}[family]
+              "falcon": _map_falcon, "gpt2": _map_gpt2,
+              "pimazen": _map_pimazen}[family]
     for name, w in hf_state.items():
         if name.endswith(".rotary_emb.inv_freq"):
             continue
@@ -196,10 +218,96 @@ def load_safetensors_dir(path: str | Path) -> dict:
     return state
 
 
+def config_from_pimazen(d: dict, name: str = "pimazen") -> ModelConfig:
+    """ModelConfig from a Pimazen config.json. A layer type or kind this
+    framework does not have is an error; an unknown key is reported."""
+    from .config import (GatedMLPSpec, LatentAttentionSpec, LayerSpec,
+                         layered_config)
+
+    def only(obj, known, where):
+        extra = set(obj) - set(known)
+        if extra:
+            warnings.warn(f"{where}: keys without effect: {sorted(extra)}")
+        return obj
+
+    only(d, ("architecture", "layers", "norm", "vocab", "width",
+             "max_seq_len"), "config")
+    layers = []
+    for i, lay in enumerate(d["layers"]):
+        where = f"layer {i}"
+        only(lay, ("type", "mixer", "mlp"), where)
+        if lay["type"] != "latent_attention":
+            raise ValueError(f"{where}: type {lay['type']!r}")
+        m = only(lay["mixer"], ("heads", "dim", "rot_dim", "vdim", "kv_rank",
+                                "scale", "rot", "mask", "kv_from"), where)
+        rot = only(m["rot"], ("base", "dims"), where)
+        mask = only(m.get("mask") or {}, ("size",), where)
+        mixer = LatentAttentionSpec(
+            heads=m["heads"], dim=m["dim"], rot_dim=m["rot_dim"],
+            vdim=m["vdim"], kv_rank=m["kv_rank"], scale=float(m["scale"]),
+            rope_base=float(rot["base"]), rope_dims=rot["dims"],
+            window=mask.get("size"), kv_from=m.get("kv_from"))
+        mlp = lay.get("mlp")
+        if mlp is not None:
+            only(mlp, ("kind", "ff", "limit"), where)
+            if mlp["kind"] != "dense":
+                raise ValueError(f"{where}: mlp kind {mlp['kind']!r}")
+            mlp = GatedMLPSpec(mlp["ff"], float(mlp["limit"]))
+        layers.append(LayerSpec(mixer, mlp))
+    kw = {"max_seq_len": d["max_seq_len"]} if "max_seq_len" in d else {}
+    return layered_config(name, layers, d["width"], d["vocab"],
+                          norm_eps=float(only(d["norm"], ("eps",),
+                                              "norm")["eps"]), **kw)
+
+
+def config_to_pimazen(cfg: ModelConfig) -> dict:
+    """The config.json of a Pimazen model (inverse of config_from_pimazen)."""
+    layers = []
+    for lay in cfg.layers:
+        m = lay.mixer
+        mixer = {"heads": m.heads, "dim": m.dim, "rot_dim": m.rot_dim,
+                 "vdim": m.vdim, "kv_rank": m.kv_rank, "scale": m.scale,
+                 "rot": {"base": m.rope_base, "dims": m.rotation[1]}}
+        if m.window is not None:
+            mixer["mask"] = {"size": m.window}
+        if m.kv_from is not None:
+            mixer["kv_from"] = m.kv_from
+        mlp = None if lay.mlp is None else {
+            "kind": "dense", "ff": lay.mlp.ff, "limit": lay.mlp.limit}
+        layers.append({"type": "latent_attention", "mixer": mixer,
+                       "mlp": mlp})
+    return {"architecture": "Pimazen", "layers": layers,
+            "norm": {"eps": cfg.norm_eps}, "vocab": cfg.vocab_size,
+            "width": cfg.hidden_size, "max_seq_len": cfg.max_seq_len}
+
+
+def config_from_dir(path: str | Path, default: str | None = None
+                    ) -> ModelConfig:
+    """The configuration of a checkpoint directory: a registered name or
+    explicit fields this framework wrote, a Pimazen config, or an HF one;
+    `default` names the registry entry of a directory that says nothing."""
+    from .config import get_config, list_configs, register
+    marker = Path(path) / "config.json"
+    meta = json.loads(marker.read_text()) if marker.exists() else {}
+    if meta.get("runbooks_amd_config") in list_configs():
+        return get_config(meta["runbooks_amd_config"])
+    if "runbooks_amd_fields" in meta:
+        return register(ModelConfig(**meta["runbooks_amd_fields"]))
+    if {"architecture", "model_type", "architectures"} & set(meta):
+        return config_from_hf_json(marker)
+    if default is None:
+        raise ValueError(f"no model configuration in {marker}")
+    return get_config(default)
+
+
 def config_from_hf_json(path: str | Path) -> ModelConfig:
     """Derive a ModelConfig from an HF config.json (for models not in the
     registry)."""
     d = json.loads(Path(path).read_text())
+    if "architecture" in d:
+        if d["architecture"] != "Pimazen":
+            raise ValueError(f"unsupported architecture {d['architecture']}")
+        return config_from_pimazen(d)
     mt = d.get("model_type", "llama")
     if mt == "gemma":
         heads = d["num_attention_heads"]

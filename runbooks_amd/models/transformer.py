@@ -7,13 +7,16 @@ One implementation, three family knobs (ModelConfig):
   * pos: RoPE (fused kernel) or learned embeddings (OPT)
   * parallel_residual: falcon's attn+mlp-in-parallel block
   * GQA/MQA via num_kv_heads (llama2-70b 8, falcon-40b 8, falcon-7b 1)
+  * layers: models described layer by layer (models/latent.py)
 
-Three forward modes:
+Forward modes:
   * ``forward(tokens)``             — training, full causal attention
   * ``prefill(...)``                — fills the paged KV cache, returns
                                       last-position logits
   * ``decode(...)``                 — one token per sequence against the
                                       paged cache (gfx950 decode kernel)
+  * ``forward_ragged(...)``         — portions of several sequences in one
+                                      batch (layer-by-layer models)
 
 TP: attention QKV is column-parallel (head-sharded), the output
 projection row-parallel (one xGMI all-reduce); MLP up column / down row
@@ -24,6 +27,7 @@ cache — 288 GB HBM per GPU makes that the right trade on MI355X.
 from __future__ import annotations
 
 import math
+import os
 
 import torch
 from torch import nn
@@ -36,6 +40,8 @@ from ..parallel import (
     gather_from_tp,
 )
 from .config import ModelConfig
+from .latent import ParallelBlock
+from .ragged import RaggedBatch
 
 
 def _norm_module(cfg: ModelConfig, dtype):
@@ -276,8 +282,15 @@ class Transformer(nn.Module):
         self.embed = nn.Embedding(cfg.vocab_size, cfg.hidden_size, dtype=dtype)
         if cfg.pos == "learned":
             self.embed_pos = nn.Embedding(cfg.max_seq_len, cfg.hidden_size, dtype=dtype)
-        self.blocks = nn.ModuleList(Block(cfg, dtype, self.tp)
-                                    for _ in range(cfg.num_layers))
+        # layer-by-layer models take ragged batches (portions of prompts
+        # beside decoded tokens) through forward_ragged
+        self.ragged = cfg.layers is not None
+        if self.ragged:
+            self.blocks = nn.ModuleList(ParallelBlock(cfg, lay, dtype, self.tp)
+                                        for lay in cfg.layers)
+        else:
+            self.blocks = nn.ModuleList(Block(cfg, dtype, self.tp)
+                                        for _ in range(cfg.num_layers))
         self.norm_f = _norm_module(cfg, dtype)
         # vocab-parallel head at TP>1 (untied vocab divisible by tp):
         # each rank's head GEMM shrinks tp-fold; full logits reassemble
@@ -295,7 +308,19 @@ class Transformer(nn.Module):
                                       bias=False, dtype=dtype)
         if cfg.tie_embeddings:
             self.lm_head.weight = self.embed.weight
-        if cfg.pos == "rope":
+        if self.ragged:
+            self.windows = sorted({lay.mixer.window for lay in cfg.layers},
+                                  key=lambda w: (w is None, w))
+            # one table per distinct rotation
+            rotations = [lay.mixer.rotation for lay in cfg.layers]
+            distinct = sorted(set(rotations))
+            self._rope_of = [distinct.index(r) for r in rotations]
+            for i, (base, dims) in enumerate(distinct):
+                cos, sin = ops.rope_tables(dims, cfg.max_seq_len, base)
+                self.register_buffer(f"rope_cos_{i}", cos, persistent=False)
+                self.register_buffer(f"rope_sin_{i}", sin, persistent=False)
+            self._decode_cu = {}
+        elif cfg.pos == "rope":
             cos, sin = ops.rope_tables(cfg.head_dim, cfg.max_seq_len, cfg.rope_theta)
             self.register_buffer("rope_cos", cos, persistent=False)
             self.register_buffer("rope_sin", sin, persistent=False)
@@ -328,6 +353,8 @@ class Transformer(nn.Module):
     # -- training --------------------------------------------------------------
     def forward(self, tokens: torch.Tensor) -> torch.Tensor:
         """tokens [B, S] -> logits [B, S, V] (training / eval, no cache)."""
+        if self.ragged:
+            raise NotImplementedError(f"{self.cfg.name}: serving only")
         B, S = tokens.shape
         positions = torch.arange(S, device=tokens.device, dtype=torch.int32)
         positions = positions.repeat(B)
@@ -360,6 +387,8 @@ class Transformer(nn.Module):
     def prefill(self, tokens, positions, caches, slot_mapping):
         """tokens [B, S]; caches: list of (k_cache, v_cache) per layer.
         Returns last-position logits [B, V]."""
+        if self.ragged:
+            raise NotImplementedError("prefill through forward_ragged")
         B, S = tokens.shape
         x = self._embed(tokens, positions)
         for blk, (kc, vc) in zip(self.blocks, caches):
@@ -377,13 +406,21 @@ class Transformer(nn.Module):
         ``nsplit`` fixes the paged-decode work split (required under
         hipGraph capture, serve/graph.py)."""
         B = tokens.shape[0]
+        if self.ragged:
+            if B not in self._decode_cu:
+                self._decode_cu[B] = torch.arange(
+                    B + 1, dtype=torch.int32, device=tokens.device)
+            return self.forward_ragged(RaggedBatch(
+                tokens=tokens, positions=positions, slots=slot_mapping,
+                cu_q=self._decode_cu[B], seq_lens=seq_lens,
+                block_tables=block_tables, rows=None, n_short=B, t_short=B,
+                max_q=1, max_keys=None), caches)
         x = self._embed(tokens.view(B, 1), positions)
-        import os as _os
         if (ops.use_hip(x) and x.dtype == torch.bfloat16 and B <= 32 and
                 self.cfg.norm == "rmsnorm" and
                 not self.cfg.parallel_residual and not self.cfg.single_norm
                 and self.cfg.hidden_size % 16 == 0 and
-                _os.environ.get("RB_FUSED_RESID", "1") == "1"):
+                os.environ.get("RB_FUSED_RESID", "1") == "1"):
             # fused residual chain: zero standalone adds in the hot loop
             delta = None
             for blk, (kc, vc) in zip(self.blocks, caches):
@@ -411,16 +448,77 @@ class Transformer(nn.Module):
         logits = self.lm_head(x)
         return gather_from_tp(logits) if self._lm_vocab_parallel else logits
 
+    @torch.no_grad()
+    def forward_ragged(self, batch: RaggedBatch, caches):
+        """One step of a layer-by-layer model: every token of the batch,
+        logits [rows, V] fp32 at the wanted ones. The residual stays fp32;
+        each layer's output is added by the norm that follows it."""
+        x = self.embed(batch.tokens).float()
+        delta, contexts = None, {}
+        for blk, cache, r in zip(self.blocks, caches, self._rope_of):
+            rope = (getattr(self, f"rope_cos_{r}"),
+                    getattr(self, f"rope_sin_{r}"))
+            delta = blk.step(x, delta, batch, cache, rope, contexts)
+        if batch.rows is not None:
+            x = x.index_select(0, batch.rows)
+            delta = delta.index_select(delta.dim() - 2, batch.rows)
+        w, n = self.lm_head.weight, x.shape[0]
+        ready = ops.decode_ready(w, n)
+        y = ops.rmsnorm_res32(x, delta, self.norm_f.weight, self.norm_f.eps,
+                              self.dtype, operand=ready)
+        logits = (ops.fast_linear(y, w).float() if ready
+                  else ops.linear_f32(y, w))
+        return gather_from_tp(logits) if self._lm_vocab_parallel else logits
+
     # -- cache helpers ----------------------------------------------------------
     def local_kv_heads(self) -> int:
         return self.blocks[0].attn.hkv
 
+    def kv_bytes_per_block(self, fp8: bool = False) -> int:
+        """Cache bytes of one block over all layers."""
+        if self.ragged:
+            return sum(b.lay.ec for b in self.blocks if b.lay.own_latent) * \
+                ops.BLOCK_SIZE * self.embed.weight.element_size()
+        elem = self.cfg.head_dim + 16 if fp8 else self.cfg.head_dim * 2
+        return 2 * self.cfg.num_layers * self.local_kv_heads() * \
+            ops.BLOCK_SIZE * elem
+
+    def decode_nsplit(self, batch: int, caches) -> int | None:
+        """Work split of the paged-decode kernel for a captured batch (None
+        where the model's own kernels choose it)."""
+        if self.ragged:
+            return None
+        from ..ops.attention import _is_vt
+        from ..serve.graph import fixed_nsplit
+        return fixed_nsplit(batch, self.local_kv_heads(),
+                            mfma=_is_vt(*caches[0][:2]))
+
+    def check_serving(self, device, fp8: bool) -> None:
+        """Raise when the serving kernels do not cover this model."""
+        if self.ragged:
+            if fp8:
+                raise NotImplementedError(
+                    f"{self.cfg.name}: no fp8 cache for latent attention")
+        elif torch.device(device).type == "cuda" and \
+                self.cfg.head_dim not in (64, 128, 256):
+            raise NotImplementedError(
+                f"paged decode supports head_dim 64/128/256 on gfx950; "
+                f"{self.cfg.name} has {self.cfg.head_dim}")
+
     def alloc_caches(self, num_blocks: int, device, fp8: bool = False):
+        if self.ragged:
+            # a layer that reads another's latents shares its cache
+            caches = []
+            for blk in self.blocks:
+                src = blk.spec.mixer.kv_from
+                caches.append(caches[src] if src is not None else
+                              ops.alloc_latent_cache(num_blocks, blk.lay,
+                                                     device, self.dtype))
+            return caches
         # Transposed-V blocks feed the MFMA decode kernel's direct V^T
         # fragment reads (GQA/MQA models, bf16, Dh<=128). The cache
         # shape is the routing signal all the way down (kv_append,
         # paged_decode). RB_DECODE_MFMA=0 reverts to the scalar path.
-        import os
         attn = self.blocks[0].attn
         vt = ((fp8 or self.dtype == torch.bfloat16)
               and attn.hq // attn.hkv >= 4 and self.cfg.head_dim <= 128
@@ -433,15 +531,9 @@ class Transformer(nn.Module):
                 for _ in range(self.cfg.num_layers)]
 
 
-def fuse_for_inference(model: "Transformer",
-                       load_in_8bit: bool = False) -> "Transformer":
-    """Fuse each block's QKV and gate/up weights into single tensors for
-    serving: one wide GEMM per group instead of 2-3 skinny ones (the
-    batch-<=32 decode GEMMs are weight-bandwidth bound, and hipBLASLt is
-    markedly more efficient at the fused N — profiles/). The original
-    parameters become views into the fused tensor, so no extra HBM and
-    the separate-projection training path keeps working.
-    """
+def _fuse_projections(model: "Transformer") -> list[torch.Tensor]:
+    """Fused qkv and gate/up weights; returns every layer's serving
+    weights."""
     for blk in model.blocks:
         attn = blk.attn
         if (attn.q_proj.bias is None and
@@ -460,12 +552,11 @@ def fuse_for_inference(model: "Transformer",
             attn.v_proj.weight = nn.Parameter(fused[qo + kvo:],
                                               requires_grad=False)
         mlp = blk.mlp
-        import os as _os
         # geglu_packed GPU-validated (GPUTEST r2: vs fp32 tanh-gelu ref);
         # default-on, RB_FUSED_GEGLU=0 reverts to eager
         glu_fusable = model.cfg.act == "silu_glu" or (
             model.cfg.act == "gelu_glu" and
-            _os.environ.get("RB_FUSED_GEGLU", "1") == "1")
+            os.environ.get("RB_FUSED_GEGLU", "1") == "1")
         if glu_fusable and mlp.gate_proj.bias is None:
             fused = torch.cat([mlp.gate_proj.weight.data,
                                mlp.up_proj.weight.data],
@@ -476,9 +567,29 @@ def fuse_for_inference(model: "Transformer",
                                                 requires_grad=False)
             mlp.up_proj.weight = nn.Parameter(fused[half:],
                                               requires_grad=False)
+    return [w for blk in model.blocks
+            for w in (getattr(blk.attn, "_qkv_w", None),
+                      getattr(blk.mlp, "_gateup_w", None),
+                      blk.attn.o_proj.weight, blk.mlp.down_proj.weight)
+            if w is not None]
 
+
+def fuse_for_inference(model: "Transformer",
+                       load_in_8bit: bool = False) -> "Transformer":
+    """Fuse each block's QKV and gate/up weights into single tensors for
+    serving: one wide GEMM per group instead of 2-3 skinny ones (the
+    batch-<=32 decode GEMMs are weight-bandwidth bound, and hipBLASLt is
+    markedly more efficient at the fused N — profiles/). The original
+    parameters become views into the fused tensor, so no extra HBM and
+    the separate-projection training path keeps working.
+    """
+    if model.ragged:
+        weights = [w for blk in model.blocks for w in blk.fuse()]
+    else:
+        weights = _fuse_projections(model)
     if not load_in_8bit and torch.cuda.is_available() and ops.has_hip() and \
-            _os.environ.get("RB_DECODE_GEMM", "1") == "1":
+            os.environ.get("RB_DECODE_GEMM", "1") == "1" and \
+            model.dtype == torch.bfloat16:
         # Register fragment-lane-major weight copies for the v2 decode
         # GEMM (csrc/decode_gemm.hip): doubles decode-weight memory, which
         # 288 GB HBM3E affords for every BASELINE config at TP=1 except
@@ -486,15 +597,8 @@ def fuse_for_inference(model: "Transformer",
         # guard: keep at least ~35% of the GPU free for KV cache.
         from ..ops.linear import register_decode_weight
         ext = ops.ext()
-        cands = []
-        for blk in model.blocks:
-            for w in (getattr(blk.attn, "_qkv_w", None),
-                      getattr(blk.mlp, "_gateup_w", None),
-                      blk.attn.o_proj.weight,
-                      blk.mlp.down_proj.weight):
-                if w is not None and ext.decode_gemm_supported(
-                        32, w.shape[0], w.shape[1]):
-                    cands.append(w)
+        cands = [w for w in weights
+                 if ext.decode_gemm_supported(32, w.shape[0], w.shape[1])]
         if model.lm_head.weight.shape[0] % 32 == 0 and \
                 ext.decode_gemm_supported(32, model.lm_head.weight.shape[0],
                                           model.lm_head.weight.shape[1]):
@@ -512,14 +616,9 @@ def fuse_for_inference(model: "Transformer",
         # prefill/big-M GEMMs: 288 GB HBM3E makes both-copies the right
         # trade on MI355X.
         from ..ops.linear import quantize_fp8
-        for blk in model.blocks:
-            for w in (getattr(blk.attn, "_qkv_w", None),
-                      getattr(blk.mlp, "_gateup_w", None),
-                      blk.attn.o_proj.weight,
-                      blk.mlp.down_proj.weight):
-                if w is not None and w.shape[0] % 64 == 0 and \
-                        w.shape[1] % 256 == 0:
-                    quantize_fp8(w)
+        for w in weights:
+            if w.shape[0] % 64 == 0 and w.shape[1] % 256 == 0:
+                quantize_fp8(w)
         if model.lm_head.weight.shape[0] % 64 == 0 and \
                 model.lm_head.weight.shape[1] % 256 == 0:
             quantize_fp8(model.lm_head.weight)

@@ -10,7 +10,9 @@ from .adamw import FusedAdamW  # noqa: F401
 from .attention import (causal_attention, flash_prefill, paged_decode,  # noqa: F401
                         paged_decode_ref, paged_decode_with_operand)
 from .kvcache import BLOCK_SIZE, alloc_kv_cache, kv_append, kv_append_ref  # noqa: F401
-from .linear import Linear, decode_linear_raw, fast_linear  # noqa: F401
-from .norm import RMSNorm, rmsnorm, rmsnorm_ref  # noqa: F401
+from .latent import alloc_latent_cache  # noqa: F401
+from .linear import (Linear, decode_linear_raw, decode_operand,  # noqa: F401
+                     decode_ready, fast_linear, linear_f32)
+from .norm import RMSNorm, rmsnorm, rmsnorm_ref, rmsnorm_res32  # noqa: F401
 from .rope import rope, rope_ref, rope_tables  # noqa: F401
 from .sampling import sample_tokens  # noqa: F401

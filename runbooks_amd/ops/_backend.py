@@ -13,20 +13,45 @@ import importlib
 
 import torch
 
-_EXT = None
-_EXT_ERR: Exception | None = None
+# The kernels are built as three modules (setup.py): ops shared by every
+# served model, latent attention, and the rest.
+_MODULES = ("_hip_core", "_hip_latent", "_hip")
+_BUILD_HINT = ("Run `PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext "
+               "--inplace` at the repo root.")
+
+
+class _Extension:
+    """All built kernel modules as one namespace. A function whose module
+    is not built raises on use, naming the cause."""
+
+    def __init__(self):
+        self.mods, self.errors = {}, {}
+        for name in _MODULES:
+            try:
+                self.mods[name] = importlib.import_module(
+                    f"runbooks_amd.ops.{name}")
+            except Exception as e:  # noqa: BLE001
+                self.errors[name] = e
+
+    def __getattr__(self, fn):
+        for mod in self.__dict__["mods"].values():
+            f = getattr(mod, fn, None)
+            if f is not None:
+                self.__dict__[fn] = f
+                return f
+        raise RuntimeError(
+            f"runbooks_amd: kernel {fn!r} is in no built gfx950 extension "
+            f"module. {_BUILD_HINT} Import errors: {self.errors!r}")
+
+
+_EXT: _Extension | None = None
 
 
 def _load():
-    global _EXT, _EXT_ERR
-    if _EXT is not None or _EXT_ERR is not None:
-        return _EXT
-    try:
-        _EXT = importlib.import_module("runbooks_amd.ops._hip")
-    except Exception as e:  # noqa: BLE001
-        _EXT_ERR = e
-        _EXT = None
-    return _EXT
+    global _EXT
+    if _EXT is None:
+        _EXT = _Extension()
+    return _EXT if _EXT.mods else None
 
 
 def has_hip() -> bool:
@@ -35,14 +60,12 @@ def has_hip() -> bool:
 
 
 def ext():
-    """Return the extension module; raise loudly if we're on a GPU without it."""
+    """Return the extension namespace; raise loudly if nothing is built."""
     m = _load()
     if m is None:
         raise RuntimeError(
-            "runbooks_amd: GPU tensor seen but the gfx950 HIP extension is not "
-            "built. Run `PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext "
-            f"--inplace` at the repo root. Import error: {_EXT_ERR!r}"
-        )
+            "runbooks_amd: GPU tensor seen but the gfx950 HIP extension is "
+            f"not built. {_BUILD_HINT} Import errors: {_EXT.errors!r}")
     return m
 
 

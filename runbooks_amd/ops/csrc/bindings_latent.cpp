@@ -1,0 +1,41 @@
+// Python bindings of the latent-attention kernels.
+
+#include <torch/extension.h>
+
+void latent_prep(at::Tensor y, at::Tensor cos, at::Tensor sin,
+                 at::Tensor positions, at::Tensor slots,
+                 c10::optional<at::Tensor> cache, c10::optional<at::Tensor> w,
+                 at::Tensor z, c10::optional<at::Tensor> swz, int64_t heads,
+                 int64_t dimc, int64_t rotc, int64_t rank, int64_t rc,
+                 int64_t off_kv, int64_t off_gate, int64_t off_up, int64_t fc,
+                 int64_t off_act, double eps, double limit, double alpha,
+                 double shift);
+void head_gemm(at::Tensor x, int64_t x_off, int64_t xh, at::Tensor w,
+               int64_t K, int64_t N, at::Tensor out, int64_t o_off, int64_t oh,
+               c10::optional<at::Tensor> gate, int64_t g_off,
+               c10::optional<at::Tensor> swz, int64_t T, int64_t H);
+int64_t latent_attend_rows(int64_t rows, int64_t rc, int64_t rotc, bool bf16);
+at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
+                         int64_t q_head, at::Tensor cache,
+                         at::Tensor block_tables, at::Tensor cu_q,
+                         at::Tensor seq_lens, int64_t n_seqs, int64_t max_q,
+                         int64_t nsplit, double scale, int64_t window,
+                         int64_t rc);
+void latent_flash(at::Tensor y, at::Tensor kv, at::Tensor ctx, at::Tensor meta,
+                  at::Tensor z, int64_t heads, int64_t dimc, int64_t rotc,
+                  int64_t vc, int64_t rc, int64_t off_g, int64_t max_q,
+                  double scale, int64_t window);
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.doc() = "runbooks_amd gfx950 HIP kernels: latent attention";
+  m.def("latent_prep", &latent_prep,
+        "rotations, latent norm, cache write and gated activation");
+  m.def("head_gemm", &head_gemm,
+        "per-head product with an optional sigmoid gate");
+  m.def("latent_attend_rows", &latent_attend_rows,
+        "query rows one workgroup of latent_attend covers");
+  m.def("latent_attend", &latent_attend,
+        "attention over the paged latent cache");
+  m.def("latent_flash", &latent_flash,
+        "flash attention of long portions on expanded keys and values");
+}

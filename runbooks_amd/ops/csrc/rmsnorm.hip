@@ -367,6 +367,130 @@ std::vector<at::Tensor> rmsnorm_res_slab_fwd_dec(at::Tensor x,
   return {sum, y, swz};
 }
 
+// Norm of a 32-bit residual: x += delta in place, y = rmsnorm(x) * w in w's
+// dtype. `nd` delta terms of type DT (0: none; > 1: the uncombined split-K
+// slab of decode_gemm_raw) lie n_rows * D apart. swz as above (bf16 only).
+namespace {
+template <typename T, typename DT, int V>
+__global__ void rmsnorm_res32_kernel(float *__restrict__ x,
+                                     const DT *__restrict__ delta, int nd,
+                                     const T *__restrict__ w,
+                                     T *__restrict__ y,
+                                     uint16_t *__restrict__ swz,
+                                     int64_t n_rows, int D, float eps) {
+  __shared__ float red[BLOCK / RB_WAVE];
+  const int nvec = D / V;
+  for (int64_t row = blockIdx.x; row < n_rows; row += gridDim.x) {
+    float *xr = x + row * D;
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < nvec; i += BLOCK) {
+      float f[V];
+      if constexpr (V == 8) {
+        rb::VIO<float>::load(xr + i * 8, f);
+        rb::VIO<float>::load(xr + i * 8 + 4, f + 4);
+      } else {
+        f[0] = xr[i];
+      }
+      for (int s = 0; s < nd; ++s) {
+        const DT *dp = delta + ((int64_t)s * n_rows + row) * D + i * V;
+        float d[V];
+        if constexpr (V == 8) {
+          rb::VIO<DT>::load(dp, d);
+          if constexpr (rb::VIO<DT>::W == 4) rb::VIO<DT>::load(dp + 4, d + 4);
+        } else {
+          d[0] = rb::bf16_to_f32_or_id(*dp);
+        }
+#pragma unroll
+        for (int k = 0; k < V; ++k) f[k] += d[k];
+      }
+      if (nd > 0) {
+        if constexpr (V == 8) {
+          rb::VIO<float>::store(xr + i * 8, f);
+          rb::VIO<float>::store(xr + i * 8 + 4, f + 4);
+        } else {
+          xr[i] = f[0];
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < V; ++k) ss += f[k] * f[k];
+    }
+    ss = rb::block_reduce_sum(ss, red);
+    const float ir = 1.0f / sqrtf(ss / (float)D + eps);
+    for (int i = threadIdx.x; i < nvec; i += BLOCK) {
+      if constexpr (V == 8) {
+        float f[8], g[8];               // this thread's own values of pass 1
+        rb::VIO<float>::load(xr + i * 8, f);
+        rb::VIO<float>::load(xr + i * 8 + 4, f + 4);
+        rb::VIO<T>::load(w + i * 8, g);
+        if constexpr (rb::VIO<T>::W == 4) rb::VIO<T>::load(w + i * 8 + 4, g + 4);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) f[k] = f[k] * ir * g[k];
+        rb::VIO<T>::store(y + row * D + i * 8, f);
+        if constexpr (rb::VIO<T>::W == 4)
+          rb::VIO<T>::store(y + row * D + i * 8 + 4, f + 4);
+        if constexpr (sizeof(T) == 2) {
+          if (swz != nullptr)
+            rb::VIO<T>::store(swz + (i >> 1) * 512 + (i & 1) * 256 + row * 8,
+                              f);
+        }
+      } else {
+        rb::store_scalar(y + row * D + i,
+                         xr[i] * ir * rb::bf16_to_f32_or_id(w[i]));
+      }
+    }
+    __syncthreads();
+  }
+}
+}  // namespace
+
+std::vector<at::Tensor> rmsnorm_res32(at::Tensor x,
+                                      c10::optional<at::Tensor> delta,
+                                      at::Tensor w, double eps, bool want_swz) {
+  TORCH_CHECK(x.is_cuda() && x.is_contiguous() && w.is_contiguous() &&
+              x.dim() == 2 && x.scalar_type() == at::kFloat &&
+              w.numel() == x.size(1), "rmsnorm_res32: x [T, D] f32, w [D]");
+  const int64_t n_rows = x.size(0);
+  const int D = (int)x.size(1);
+  const bool bf16 = w.scalar_type() == at::kBFloat16;
+  TORCH_CHECK(bf16 || w.scalar_type() == at::kFloat, "rmsnorm_res32: w dtype");
+  TORCH_CHECK(!want_swz || (bf16 && n_rows <= 32 && D % 16 == 0),
+              "rmsnorm_res32: operand shape");
+  auto y = at::empty(x.sizes(), w.options());
+  auto swz = at::empty({want_swz ? (int64_t)(D / 16) * 512 : 0}, w.options());
+  int nd = 0;
+  bool d16 = false;
+  void *dp = nullptr;
+  if (delta.has_value()) {
+    const at::Tensor &d = *delta;
+    TORCH_CHECK(d.is_cuda() && d.is_contiguous() && d.size(-1) == D &&
+                d.size(-2) == n_rows && (d.dim() == 2 || d.dim() == 3),
+                "rmsnorm_res32: delta shape");
+    d16 = d.scalar_type() == at::kBFloat16;
+    TORCH_CHECK(d16 || d.scalar_type() == at::kFloat,
+                "rmsnorm_res32: delta dtype");
+    nd = d.dim() == 3 ? (int)d.size(0) : 1;
+    dp = d.data_ptr();
+  }
+  if (n_rows == 0) return {y, swz};
+  auto stream = at::hip::getCurrentHIPStream();
+  const dim3 grid(std::min<int64_t>(n_rows, 4096));
+#define RB_RES32(T, DT, V)                                                   \
+  hipLaunchKernelGGL((rmsnorm_res32_kernel<T, DT, V>), grid, dim3(BLOCK), 0, \
+                     stream, x.data_ptr<float>(), (const DT *)dp, nd,        \
+                     (const T *)w.data_ptr(), (T *)y.data_ptr(),             \
+                     want_swz ? (uint16_t *)swz.data_ptr() : nullptr,        \
+                     n_rows, D, (float)eps)
+#define RB_RES32_V(V)                                  \
+  if (bf16 && d16) RB_RES32(uint16_t, uint16_t, V);    \
+  else if (bf16) RB_RES32(uint16_t, float, V);         \
+  else if (d16) RB_RES32(float, uint16_t, V);          \
+  else RB_RES32(float, float, V)
+  if (D % 8 == 0) { RB_RES32_V(8); } else { RB_RES32_V(1); }
+#undef RB_RES32_V
+#undef RB_RES32
+  return {y, swz};
+}
+
 std::vector<at::Tensor> rmsnorm_bwd(at::Tensor x, at::Tensor w, at::Tensor dy,
                                     at::Tensor inv_rms) {
   TORCH_CHECK(x.is_cuda() && dy.is_contiguous() && x.is_contiguous(), "rmsnorm_bwd: bad args");

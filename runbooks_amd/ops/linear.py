@@ -133,6 +133,27 @@ def decode_linear_raw(x, weight):
     return out, out.dtype == torch.float32
 
 
+def decode_ready(weight: torch.Tensor, m: int) -> bool:
+    """True when a product of m rows with `weight` runs on the decode GEMM
+    (so that its producer should emit the swizzled operand)."""
+    return (m <= 32 and _USE_DECODE_GEMM and weight.is_cuda and
+            _registry_get(_FP8_REGISTRY, weight) is None and
+            _registry_get(_DECODE_W_REGISTRY, weight) is not None)
+
+
+def decode_operand(m: int, k: int, like: torch.Tensor) -> torch.Tensor:
+    """Buffer for a decode-GEMM operand of m <= 32 rows and k columns,
+    [k/16][2][32][8] (filled by the kernels that produce the rows)."""
+    return torch.empty((k // 16) * 512, dtype=like.dtype, device=like.device)
+
+
+def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """x @ weight^T with the fp32 accumulator as the result."""
+    if x.is_cuda and x.dtype == torch.bfloat16:
+        return torch.mm(x, weight.t(), out_dtype=torch.float32)
+    return F.linear(x, weight).float()
+
+
 class Linear(torch.nn.Linear):
     """nn.Linear with the decode-GEMM fast path."""
 

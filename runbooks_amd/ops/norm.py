@@ -44,6 +44,25 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float = 1e-5) -> torch.T
     return rmsnorm_ref(x, weight, eps)
 
 
+def rmsnorm_res32(x: torch.Tensor, delta: torch.Tensor | None,
+                  weight: torch.Tensor, eps: float, dtype: torch.dtype,
+                  operand: bool = False) -> torch.Tensor:
+    """Norm of a 32-bit residual: x [T, D] fp32 += delta in place, returns
+    rmsnorm(x) * weight in `dtype`. delta: fp32 or `dtype` [T, D], an
+    uncombined fp32 split-K slab [split, T, D], or None. operand=True also
+    attaches the decode GEMM's pre-swizzled operand (T <= 32)."""
+    if not _backend.use_hip(x):
+        if delta is not None:
+            x += delta.float() if delta.dim() == 2 else delta.sum(0)
+        return rmsnorm_ref(x, weight, eps).to(dtype)
+    y, swz = _backend.ext().rmsnorm_res32(
+        x, None if delta is None else delta.contiguous(), weight, eps,
+        operand)
+    if operand:
+        y._rb_swz = swz
+    return y
+
+
 class RMSNorm(torch.nn.Module):
     def __init__(self, dim: int, eps: float = 1e-5, dtype=None):
         super().__init__()

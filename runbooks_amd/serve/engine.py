@@ -11,6 +11,13 @@ when capacity allows, then all running sequences decode as one batch —
 decode batches hit the gfx950 paged-decode kernel
 (ops/csrc/attention_decode.hip).
 
+Models that take ragged batches (model.ragged, the layer-by-layer ones)
+run one batch per step instead: the next portion of every prompt being
+read, up to `prefill_chunk` tokens, beside one token of every decoding
+sequence (`_step_ragged` -> `run_portions`). A step of single tokens only
+is the captured decode graph there too. Their windows are exact in prompts
+and decoding alike.
+
 Sliding-window attention (mistral, cfg.sliding_window): enforced here as
 pure KV bookkeeping — RoPE is applied at absolute positions when keys
 are written, so attention over any suffix of the cache is exact, and the
@@ -31,6 +38,7 @@ import torch
 
 from .. import ops
 from ..models import Transformer, build_model
+from ..models.ragged import Portion, StepPlan
 from ..parallel import comm
 from ..utils.trace import get_tracer
 
@@ -86,6 +94,8 @@ class Request:
     # tokens whose KV blocks were freed by the sliding window (always a
     # multiple of BLOCK_SIZE; blocks[] maps retained positions only)
     dropped: int = 0
+    # tokens whose KV is in the cache (ragged models)
+    computed: int = 0
     finished: bool = False
     created: float = field(default_factory=time.time)
 
@@ -106,7 +116,7 @@ class Engine:
             model = build_model(model, dtype=dtype, seed=seed,
                                 device=self.device)
         self.model = model.to(self.device).eval()
-        if torch.cuda.is_available():
+        if torch.cuda.is_available() or model.ragged:
             # TP>1 included: each rank fuses ITS OWN qkv / gate-up weight
             # shards and registers decode-GEMM layouts for them — the
             # collective order (o/down all-reduce per layer) is untouched,
@@ -119,11 +129,6 @@ class Engine:
                   "(fp8 decode path is single-GPU; 288 GB/GPU rarely "
                   "needs 8-bit at TP>1)", flush=True)
         self.cfg = model.cfg
-        if torch.cuda.is_available() and model.cfg.head_dim not in (64, 128,
-                                                                    256):
-            raise NotImplementedError(
-                f"paged decode supports head_dim 64/128/256 on gfx950; "
-                f"{model.cfg.name} has {model.cfg.head_dim}")
         self.bs = ops.BLOCK_SIZE
         self.max_batch = max_batch
         # Admission budget per step: the default 1 matches the classic
@@ -138,6 +143,9 @@ class Engine:
         import os as _os0
         self.kv_fp8 = (kv_fp8 if kv_fp8 is not None
                        else _os0.environ.get("RB_KV_FP8", "0") == "1")
+        model.check_serving(self.device, self.kv_fp8)
+        # ragged models: most prompt tokens of one step
+        self.prefill_chunk = 2048
         if kv_blocks is None:
             kv_blocks = self._auto_kv_blocks(mem_fraction)
         if comm.is_dist() and comm.world_size() > 1 and model.tp > 1:
@@ -177,7 +185,8 @@ class Engine:
         # so the worker-follow protocol (serve/tp_worker.py) sees every
         # collective.
         self.tp = comm.world_size()
-        self.use_graphs = torch.cuda.is_available() and self.tp == 1
+        self.use_graphs = (torch.device(self.device).type == "cuda" and
+                           self.tp == 1)
         # Prefix caching (opt-in, RB_PREFIX_CACHE=1 or prefix_cache=True):
         # full 16-token prompt-prefix chunks are shared across requests by
         # refcount — a hit skips the KV writes for those chunks (the
@@ -197,10 +206,7 @@ class Engine:
                       "prefix_hit_blocks": 0, "window_dropped_blocks": 0}
 
     def _auto_kv_blocks(self, mem_fraction: float) -> int:
-        elem = (self.cfg.head_dim + 16) if self.kv_fp8 \
-            else self.cfg.head_dim * 2
-        bytes_per_block = (2 * self.cfg.num_layers * self.model.local_kv_heads()
-                           * self.bs * elem)
+        bytes_per_block = self.model.kv_bytes_per_block(self.kv_fp8)
         if torch.cuda.is_available():
             free, _total = torch.cuda.mem_get_info(self.device)
             budget = int(free * mem_fraction) - (2 << 30)  # activations headroom
@@ -373,14 +379,9 @@ class Engine:
         starts = [max(0, v + 1 - W) if W else 0 for v in vpos]
 
         if self.use_graphs and B <= self.max_batch:
-            if self._graphed is None:
-                from .graph import GraphedDecoder
-                self._graphed = GraphedDecoder(
-                    self.model, self.caches, self.max_batch,
-                    self.max_blocks_per_seq, self.dummy_block, dev)
-            logits = self._graphed.decode(last, pos, slots,
-                                          [r.blocks for r in reqs],
-                                          [v + 1 for v in vpos], starts)
+            logits = self._graph_decode(last, pos, slots,
+                                        [r.blocks for r in reqs],
+                                        [v + 1 for v in vpos], starts)
         else:
             maxb = max(len(r.blocks) for r in reqs)
             bt = torch.zeros(B, maxb, dtype=torch.int32)
@@ -401,6 +402,234 @@ class Engine:
             logits = self.model.decode(tokens, positions, self.caches, slot_t,
                                        bt, seq_lens, seq_starts=start_t)
         return self._sample_batch(logits, reqs)
+
+    def _graph_decode(self, *args):
+        if self._graphed is None:
+            from .graph import GraphedDecoder
+            self._graphed = GraphedDecoder(
+                self.model, self.caches, self.max_batch,
+                self.max_blocks_per_seq, self.dummy_block, self.device)
+        return self._graphed.decode(*args)
+
+    # -- ragged steps (layer-by-layer models) -----------------------------------
+    def _release_front(self, r: Request, next_pos: int) -> None:
+        """Give back the blocks no query at `next_pos` or later can see."""
+        w = self.cfg.sliding_window
+        while w and r.blocks and r.dropped + self.bs <= next_pos - w + 1:
+            self.allocator.release([r.blocks.pop(0)])
+            r.dropped += self.bs
+            self.stats["window_dropped_blocks"] += 1
+
+    def blocks_missing(self, r: Request, n: int) -> int:
+        """Blocks request r still needs to hold its next n tokens."""
+        need = r.computed + n - r.dropped
+        return max(0, -(-need // self.bs) - len(r.blocks))
+
+    def run_portions(self, entries):
+        """Run the next tokens of several requests as one batch.
+
+        entries: (request, tokens, want) with `want` the places among the
+        tokens whose logits are returned, [n_wanted, V] in entry order
+        (None when nothing is wanted). Cache blocks are taken here; the
+        caller sees to it that they suffice."""
+        portions = []
+        for r, tokens, want in entries:
+            if r.computed + len(tokens) > self.cfg.max_seq_len:
+                raise ValueError(
+                    f"request {r.request_id}: {r.computed + len(tokens)} "
+                    f"tokens, max_seq_len {self.cfg.max_seq_len}")
+            self._release_front(r, r.computed)
+            r.blocks.extend(self.allocator.alloc(
+                self.blocks_missing(r, len(tokens))))
+            portions.append(Portion(list(tokens), r.computed, r.dropped,
+                                    r.blocks, list(want)))
+        plan = StepPlan(portions)
+        wanted = sum(len(p.want) for p in portions)
+        if self.use_graphs and wanted == len(portions) and \
+                len(portions) <= self.max_batch and \
+                all(len(p.tokens) == 1 for p in portions):
+            vpos = [p.start - p.dropped for p in portions]
+            logits = self._graph_decode(
+                [p.tokens[0] for p in portions], [p.start for p in portions],
+                [p.blocks[v // self.bs] * self.bs + v % self.bs
+                 for p, v in zip(portions, vpos)],
+                [p.blocks for p in portions], [v + 1 for v in vpos])
+        else:
+            if self.tp > 1:
+                from .tp_worker import broadcast_ragged
+                broadcast_ragged(plan, self.device)
+            logits = self.forward_plan(plan)
+        for r, tokens, _ in entries:
+            r.computed += len(tokens)
+        return logits if wanted else None
+
+    def forward_plan(self, plan: StepPlan):
+        m = self.model
+        batch = plan.build(self.bs, m.windows, self.device,
+                           expand=all(b.expandable for b in m.blocks))
+        return m.forward_ragged(batch, self.caches)
+
+    def open_request(self, prompt_ids=()) -> Request:
+        """A request the caller feeds itself, through run_portions."""
+        req = Request(self._next_id, list(prompt_ids))
+        self._next_id += 1
+        return req
+
+    def close_request(self, r: Request) -> None:
+        """Give back what a request holds in the cache."""
+        self.allocator.release(r.blocks)
+        r.blocks = []
+        r.finished = True
+
+    def _admit_ragged(self) -> Request | None:
+        """Move the next waiting request to the running ones; whole blocks
+        of its prompt that the prefix cache holds need no computing (the
+        last prompt token always runs, for its logits)."""
+        if not self.waiting or len(self.running) >= self.max_batch:
+            return None
+        req = self.waiting.pop(0)
+        hits = 0
+        if self.prefix_cache_enabled:
+            for k in range(1, (len(req.prompt_ids) - 1) // self.bs + 1):
+                key = tuple(req.prompt_ids[:k * self.bs])
+                b = self._pc.get(key)
+                if b is None:
+                    break
+                self.allocator.share(b)
+                self._pc.move_to_end(key)
+                req.blocks.append(b)
+                hits += 1
+        if hits:
+            self.stats["prefix_hits"] += 1
+            self.stats["prefix_hit_blocks"] += hits
+            req.computed = hits * self.bs
+        self.running.append(req)
+        return req
+
+    def _publish_prefix(self, r: Request, before: int) -> None:
+        """Offer the prompt blocks a portion completed to later requests."""
+        last = min(r.computed, len(r.prompt_ids)) // self.bs
+        for k in range(before // self.bs + 1, last + 1):
+            key = tuple(r.prompt_ids[:k * self.bs])
+            i = k - 1 - r.dropped // self.bs
+            if key not in self._pc and i >= 0:
+                self._pc[key] = r.blocks[i]
+                self.allocator.share(r.blocks[i])
+
+    def _take_blocks(self, r: Request, n: int, preempt: bool) -> bool:
+        """Blocks for r's next n tokens, from the free ones, then idle
+        prefix blocks, then (for a decoding request) by preempting the
+        newest other request."""
+        self._release_front(r, r.computed)
+        while True:
+            need = self.blocks_missing(r, n)
+            short = need - len(self.allocator.free)
+            if short <= 0:
+                r.blocks.extend(self.allocator.alloc(need))
+                return True
+            if self.prefix_cache_enabled:
+                self._evict_prefix(short)
+                if need <= len(self.allocator.free):
+                    continue
+            if not (preempt and self._preempt_newest(exclude=r)):
+                return False
+
+    def _step_ragged(self) -> list[Request]:
+        self.stats["steps"] += 1
+        finished: list[Request] = []
+        self._sweep_finished(finished)
+        # decoding requests first: prompts must not starve them
+        planned: list[tuple[Request, int]] = []
+        preempted = self.stats["preemptions"]
+        for r in list(self.running):
+            if r in self.running and r.computed == r.seq_len - 1:
+                if self._take_blocks(r, 1, preempt=True):
+                    planned.append((r, 1))
+                else:
+                    self._preempt(r)
+        planned = [(r, n) for r, n in planned if r in self.running]
+        # then prompts, within the step's token budget: they take free and
+        # idle blocks only, as many tokens as those hold
+        budget = self.prefill_chunk
+        queue = [r for r in self.running if r.computed < r.seq_len - 1]
+        while budget > 0:
+            fresh = not queue
+            if fresh and self.stats["preemptions"] > preempted:
+                break
+            r = queue.pop(0) if queue else self._admit_ragged()
+            if r is None:
+                break
+            n = min(budget, r.seq_len - r.computed)
+            if not self._take_blocks(r, n, preempt=False):
+                n -= self.bs * (self.blocks_missing(r, n) -
+                                len(self.allocator.free))
+                if n <= 0 or not self._take_blocks(r, n, preempt=False):
+                    if fresh:
+                        self._unadmit(r)
+                    break
+            planned.append((r, n))
+            budget -= n
+        if not planned:
+            if self.running or self.waiting:
+                self._resolve_stall()
+            return finished
+        tr = get_tracer()
+        entries = []
+        for r, n in planned:
+            ids = r.prompt_ids + r.output_ids
+            done = r.computed + n == len(ids)
+            entries.append((r, ids[r.computed:r.computed + n],
+                            [n - 1] if done else []))
+        n_dec = sum(1 for _, t, w in entries if w and len(t) == 1)
+        before = [r.computed for r, _ in planned]
+        try:
+            if tr:
+                name = "decode" if n_dec == len(entries) else "prefill"
+                with tr.span(name, batch=len(entries),
+                             tokens=sum(n for _, n in planned)):
+                    logits = self.run_portions(entries)
+            else:
+                logits = self.run_portions(entries)
+        except Exception:
+            # a failing batch must not leak its cache blocks
+            for r, _ in planned:
+                if r in self.running:
+                    self.running.remove(r)
+                self.close_request(r)
+            raise
+        ready = []
+        for (r, toks, want), b in zip(entries, before):
+            if b < len(r.prompt_ids):
+                if self.prefix_cache_enabled:
+                    self._publish_prefix(r, b)
+                self.stats["prefills"] += bool(want)
+            else:
+                self.stats["decode_tokens"] += 1
+            if want:
+                ready.append(r)
+        if ready:
+            for r, t in zip(ready, self._sample_batch(logits, ready)):
+                r.output_ids.append(t)
+        self._sweep_finished(finished)
+        return finished
+
+    def _unadmit(self, r: Request) -> None:
+        self.running.remove(r)
+        self.allocator.release(r.blocks)
+        r.blocks, r.computed, r.dropped = [], 0, 0
+        self.waiting.insert(0, r)
+
+    def _resolve_stall(self) -> None:
+        """Nothing could be planned: preempt the newest of several running
+        requests; a lone request that does not fit never will."""
+        if len(self.running) > 1:
+            self._preempt(self.running[-1])
+            return
+        r = self.running.pop() if self.running else self.waiting.pop(0)
+        self.close_request(r)
+        raise RuntimeError(
+            f"request of {r.seq_len} tokens cannot fit the KV cache "
+            f"({self.allocator.num_blocks} blocks)")
 
     def _sample_batch(self, logits, reqs: list[Request]) -> list[int]:
         seed = self.seed + 1_000_003 * reqs[0].seq_len
@@ -446,7 +675,7 @@ class Engine:
         tokens become part of the prompt for the re-prefill."""
         self.allocator.release(r.blocks)
         r.blocks = []
-        r.dropped = 0
+        r.dropped = r.computed = 0
         r.prompt_ids = r.prompt_ids + r.output_ids
         r.max_new_tokens -= len(r.output_ids)
         r.output_ids = []
@@ -480,6 +709,8 @@ class Engine:
     # -- scheduler step ----------------------------------------------------------
     def step(self) -> list[Request]:
         """One engine iteration. Returns requests finished this step."""
+        if self.model.ragged:
+            return self._step_ragged()
         self.stats["steps"] += 1
         finished = []
         # sweep first: requests already satisfied (cancel() capped their
@@ -568,7 +799,8 @@ class Engine:
     def _sweep_finished(self, finished: list[Request]) -> None:
         for r in list(self.running):
             if (len(r.output_ids) >= r.max_new_tokens
-                    or (r.stop_ids and r.output_ids[-1] in r.stop_ids)
+                    or (r.stop_ids and r.output_ids and
+                        r.output_ids[-1] in r.stop_ids)
                     or r.seq_len >= self.cfg.max_seq_len):
                 r.finished = True
                 self.allocator.release(r.blocks)

@@ -71,10 +71,7 @@ class GraphedDecoder:
 
     # -- capture -----------------------------------------------------------
     def _capture(self, b: int):
-        hkv = self.model.local_kv_heads()
-        from ..ops.attention import _is_vt
-        nsplit = fixed_nsplit(b, hkv,
-                              mfma=_is_vt(*self.caches[0][:2]))
+        nsplit = self.model.decode_nsplit(b, self.caches)
         args = (self.tokens[:b], self.positions[:b], self.caches,
                 self.slots[:b], self.block_tables[:b], self.seq_lens[:b])
         kw = dict(nsplit=nsplit, seq_starts=self.seq_starts[:b])

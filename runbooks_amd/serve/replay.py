@@ -1,0 +1,91 @@
+"""Trace replay: given token ids through the serving engine, step by step.
+
+    bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR
+                  --max-tokens N [--device cuda:0] < steps.jsonl
+
+Each input line is one engine step,
+
+    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17], "want": [1]}],
+     "end": ["b"]}
+
+the next tokens of each named request and the places among them whose
+logits to write; `end` closes requests after the step. A step's entries run
+as one batch (Engine.run_portions). Logits go to OUT/<step>.f32 as
+little-endian fp32 [wanted, vocab]; `done <step>` follows every step. The
+cache pool holds --max-tokens tokens.
+"""
+from __future__ import annotations
+
+import argparse
+import json
+import sys
+from pathlib import Path
+
+
+def _arguments(argv):
+    p = argparse.ArgumentParser(prog="trace_run", description=__doc__,
+                                formatter_class=argparse.
+                                RawDescriptionHelpFormatter)
+    p.add_argument("--model", required=True)
+    p.add_argument("--dtype", choices=["bfloat16", "float32"],
+                   default="bfloat16")
+    p.add_argument("--out", required=True)
+    p.add_argument("--max-tokens", type=int, required=True)
+    p.add_argument("--max-requests", type=int, default=4,
+                   help="live requests at any time")
+    p.add_argument("--device", default="cuda:0")
+    return p.parse_args(argv)
+
+
+def build_engine(model_dir, dtype, device, max_tokens: int,
+                 max_requests: int = 4):
+    from .. import ops
+    from ..models import build_model
+    from ..models.load import config_from_dir, load_pretrained
+    from .engine import Engine
+    model = build_model(config_from_dir(model_dir), dtype=dtype, tp=1,
+                        device=device)
+    if not model.ragged:
+        raise SystemExit(f"{model.cfg.name}: the engine runs this family's "
+                         f"prompts whole; replay needs portions")
+    load_pretrained(model, model_dir)
+    # one more block for the padding rows of captured batches
+    blocks = -(-max_tokens // ops.BLOCK_SIZE) + 1
+    return Engine(model, device=device, dtype=dtype, kv_blocks=blocks,
+                  max_batch=max_requests, prefix_cache=False, kv_fp8=False)
+
+
+def replay(engine, lines, out_dir, say=print) -> None:
+    live = {}
+    for line in lines:
+        if not line.strip():
+            continue
+        step = json.loads(line)
+        entries = []
+        for e in step["entries"]:
+            if e["id"] not in live:
+                live[e["id"]] = engine.open_request()
+            if e["tokens"]:
+                entries.append((live[e["id"]], e["tokens"], e["want"]))
+        logits = engine.run_portions(entries) if entries else None
+        if logits is not None:
+            logits.float().cpu().numpy().astype("<f4").tofile(
+                Path(out_dir) / f"{step['step']}.f32")
+        for name in step.get("end", ()):
+            engine.close_request(live.pop(name))
+        say(f"done {step['step']}", flush=True)
+
+
+def main(argv=None) -> int:
+    a = _arguments(argv)
+    if a.device.startswith("cuda"):
+        from ..ops.build import ensure_built
+        ensure_built(("core", "latent"))
+    import torch
+    # true 32-bit products
+    torch.backends.cuda.matmul.allow_tf32 = False
+    torch.set_float32_matmul_precision("highest")
+    engine = build_engine(a.model, getattr(torch, a.dtype), a.device,
+                          a.max_tokens, a.max_requests)
+    replay(engine, sys.stdin, a.out)
+    return 0

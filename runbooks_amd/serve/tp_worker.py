@@ -9,7 +9,8 @@ their own weight shards and KV caches and discard the logits (the
 vocab-parallel lm_head all-gather assembles full logits on every rank,
 so the collective schedule stays symmetric).
 
-Ops: 1 = prefill, 2 = decode, 0 = shutdown.
+Ops: 1 = prefill, 2 = decode, 3 = ragged step (the flattened plan, from
+which every rank builds the same batch), 0 = shutdown.
 """
 from __future__ import annotations
 
@@ -19,6 +20,7 @@ import torch.distributed as dist
 OP_SHUTDOWN = 0
 OP_PREFILL = 1
 OP_DECODE = 2
+OP_RAGGED = 3
 
 
 def _bcast(t: torch.Tensor) -> torch.Tensor:
@@ -52,6 +54,14 @@ def broadcast_decode(tokens, positions, slots, block_tables, seq_lens,
     _bcast(seq_starts)
 
 
+def broadcast_ragged(plan, device):
+    """Called by rank 0's engine before model.forward_ragged."""
+    flat = plan.flatten().to(device)
+    _bcast(torch.tensor([OP_RAGGED, flat.numel(), 0, 0], dtype=torch.int64,
+                        device=device))
+    _bcast(flat)
+
+
 def broadcast_shutdown(device):
     hdr = torch.tensor([OP_SHUTDOWN, 0, 0, 0], dtype=torch.int64,
                        device=device)
@@ -73,6 +83,10 @@ def worker_loop(engine) -> None:
             positions = _bcast(torch.zeros(s, dtype=torch.int32, device=dev))
             slots = _bcast(torch.zeros(s, dtype=torch.int32, device=dev))
             model.prefill(tokens, positions, caches, slots)
+        elif op == OP_RAGGED:
+            from ..models.ragged import StepPlan
+            flat = _bcast(torch.zeros(b, dtype=torch.int64, device=dev))
+            engine.forward_plan(StepPlan.unflatten(flat.cpu()))
         elif op == OP_DECODE:
             tokens = _bcast(torch.zeros(b, dtype=torch.long, device=dev))
             positions = _bcast(torch.zeros(b, dtype=torch.int32, device=dev))

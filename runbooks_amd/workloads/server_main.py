@@ -14,7 +14,6 @@ examples/llama2-7b/server.yaml, container-contract.md:50-56) — loads
 """
 from __future__ import annotations
 
-import json
 import os
 import sys
 from pathlib import Path
@@ -39,8 +38,8 @@ def main():
         return 0
     import torch
 
-    from ..models import build_model, get_config, list_configs
-    from ..models.load import config_from_hf_json, load_pretrained
+    from ..models import build_model
+    from ..models.load import config_from_dir, load_pretrained
     from ..parallel import comm
     from ..serve import Engine
     from ..serve.http import serve_forever
@@ -58,22 +57,9 @@ def main():
         if ckpts:
             model_dir = ckpts[-1]
             print(f"server: serving latest checkpoint {model_dir}")
-    arch = os.environ.get("PARAM_MODEL") or "llama2-7b"
-    marker = model_dir / "config.json"
-    cfg = None
-    if marker.exists():
-        meta = json.loads(marker.read_text())
-        name = meta.get("runbooks_amd_config")
-        if name and name in list_configs():
-            cfg = get_config(name)
-        elif "runbooks_amd_fields" in meta:
-            from ..models import ModelConfig
-            from ..models.config import register
-            cfg = register(ModelConfig(**meta["runbooks_amd_fields"]))
-        elif "model_type" in meta or "architectures" in meta:
-            cfg = config_from_hf_json(marker)
-    if cfg is None:
-        cfg = get_config(arch)
+    cfg = config_from_dir(model_dir,
+                          default=os.environ.get("PARAM_MODEL")
+                          or "llama2-7b")
 
     dtype = torch.bfloat16 if torch.cuda.is_available() else torch.float32
     model = build_model(cfg, dtype=dtype)

@@ -17,7 +17,41 @@ from torch.utils import cpp_extension  # noqa: E402
 ROOT = Path(__file__).parent
 CSRC = ROOT / "runbooks_amd" / "ops" / "csrc"
 
-sources = sorted(str(p) for p in CSRC.glob("*.hip")) + [str(CSRC / "bindings.cpp")]
+# One extension module per group, so that a caller can build just what a
+# model needs (RB_EXT_GROUPS=core,latent): `core` holds the ops every
+# served model runs, `latent` the latent-attention kernels, `main` the rest.
+CORE = ("rmsnorm", "decode_gemm", "sampling")
+
+
+def _group_of(stem: str) -> str:
+    if stem in CORE:
+        return "core"
+    return "latent" if stem.startswith("latent_") else "main"
+
+
+MODULES = {"core": ("_hip_core", "bindings_core.cpp"),
+           "latent": ("_hip_latent", "bindings_latent.cpp"),
+           "main": ("_hip", "bindings.cpp")}
+
+# *_hip.hip are build-time copies torch's extension builder leaves behind
+kernels = [p for p in sorted(CSRC.glob("*.hip"))
+           if not p.stem.endswith("_hip")]
+groups = os.environ.get("RB_EXT_GROUPS", ",".join(MODULES)).split(",")
+
+# packed fp32 instructions stay off in device code
+HIP_FLAGS = ["-O3", "-std=c++17", "--offload-arch=gfx950",
+             "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+
+def _extension(group: str):
+    module, bindings = MODULES[group]
+    return cpp_extension.CUDAExtension(
+        name=f"runbooks_amd.ops.{module}",
+        sources=[str(p) for p in kernels if _group_of(p.stem) == group]
+        + [str(CSRC / bindings)],
+        extra_compile_args={"cxx": ["-O3", "-std=c++17"],
+                            "nvcc": HIP_FLAGS})
+
 
 setup(
     name="runbooks_amd",
@@ -41,15 +75,6 @@ setup(
         "kubectl-notebook = runbooks_amd.cli.main:kubectl_notebook",
         "kubectl-applybuild = runbooks_amd.cli.main:kubectl_applybuild",
     ]},
-    ext_modules=[
-        cpp_extension.CUDAExtension(
-            name="runbooks_amd.ops._hip",
-            sources=sources,
-            extra_compile_args={
-                "cxx": ["-O3", "-std=c++17"],
-                "nvcc": ["-O3", "-std=c++17", "--offload-arch=gfx950"],
-            },
-        )
-    ],
+    ext_modules=[_extension(g) for g in groups],
     cmdclass={"build_ext": cpp_extension.BuildExtension.with_options(use_ninja=True)},
 )
