@@ -6,8 +6,9 @@ sequential JSON lines: the llama2-7b LoRA fine-tune step (DP over
 RCCL/xGMI, "finetune samples/sec") first, then "Server tokens/sec"
 (paged-KV batch-32 decode on the same model), bf16, synthetic token
 data, random-init weights. The reference publishes no numbers; this
-bench ESTABLISHES the baseline. --mode train / serve
-select a single metric.
+bench ESTABLISHES the baseline. --mode train / serve select a single
+metric; --mode latent measures prefill and decode of the latent-attention
+models beside llama models of equal layer sizes.
 
 Launch (driver):
   python bench.py --gpus 1 --steps K --warmup W
@@ -189,12 +190,87 @@ def bench_serve(args) -> dict:
     }
 
 
+# latent-attention model, and the model of equal width, heads and mlp
+LATENT_PAIRS = (("pimazen-7b", "llama2-7b"), ("pimazen-1b", "llama-1b"))
+
+
+def bench_latent(args) -> list[dict]:
+    """Prefill (whole prompts, one at a time) and decode (a full batch at a
+    given context) through the engine's own step, each latent-attention
+    model beside its pair; one result per model and workload."""
+    import gc
+
+    from runbooks_amd.serve import Engine
+
+    on_gpu = torch.cuda.is_available()
+    pairs = LATENT_PAIRS if on_gpu else (("tiny-pimazen", "tiny-llama"),)
+    prompts, contexts = ((512, 2048), (128, 2048)) if on_gpu else ((32,), (16,))
+    batch = args.serve_batch if on_gpu else 2
+    dtype = torch.bfloat16 if on_gpu else torch.float32
+    g = torch.Generator().manual_seed(17)
+    results = []
+
+    def measure(name, what, seq, tokens, dt, steps):
+        results.append({
+            "metric": f"{what}_tokens_per_sec", "value": tokens / dt,
+            "unit": "tokens/sec", "n_gpus": 1, "steps": steps,
+            "warmup": args.warmup, "ms_per_step": dt / steps * 1e3,
+            "higher_is_better": True, "scaling": "weak",
+            "vs_baseline": None, "dtype": str(dtype).split(".")[-1],
+            "data": "synthetic",
+            "config": {"model": name, "seq_len": seq,
+                       "global_batch": 1 if what == "prefill" else batch,
+                       "parallelism": "tp1"}})
+
+    for name in (m for pair in pairs for m in pair):
+        need = batch * (max(contexts) + 256) + 4096
+        eng = Engine(name, dtype=dtype, kv_blocks=need // 16,
+                     max_batch=batch, seed=17, prefix_cache=False)
+        vocab = eng.cfg.vocab_size
+
+        def prompt(n):
+            return torch.randint(0, vocab, (n,), generator=g).tolist()
+
+        for n in prompts:
+            for i in range(args.warmup + args.steps):
+                if i == args.warmup:
+                    _sync()
+                    t0 = time.perf_counter()
+                eng.submit(prompt(n), max_new_tokens=1)
+                while eng.has_work():
+                    eng.step()
+            _sync()
+            measure(name, "prefill", n, n * args.steps,
+                    time.perf_counter() - t0, args.steps)
+        for n in contexts:
+            reqs = [eng.submit(prompt(n), max_new_tokens=1 << 30)
+                    for _ in range(batch)]
+            while not all(len(r.output_ids) > 1 for r in reqs):
+                eng.step()
+            for i in range(args.warmup + args.steps):
+                if i == args.warmup:
+                    _sync()
+                    t0 = time.perf_counter()
+                eng.step()
+            _sync()
+            measure(name, "decode", n, batch * args.steps,
+                    time.perf_counter() - t0, args.steps)
+            for r in reqs:
+                eng.cancel(r.request_id)
+            eng.step()
+        del eng
+        gc.collect()
+        if on_gpu:
+            torch.cuda.empty_cache()
+    return results
+
+
 def main():
     p = argparse.ArgumentParser()
     p.add_argument("--gpus", type=int, default=1)
     p.add_argument("--steps", type=int, default=20)
     p.add_argument("--warmup", type=int, default=5)
-    p.add_argument("--mode", choices=["both", "train", "serve"],
+    p.add_argument("--mode", choices=["both", "train", "serve", "latent"],
                    default="both")
     p.add_argument("--model", default=None)
     p.add_argument("--seq-len", type=int, default=512)
@@ -236,6 +312,8 @@ def main():
             if torch.cuda.is_available():
                 torch.cuda.empty_cache()
         results.append(bench_serve(args))
+    if args.mode == "latent":
+        results += bench_latent(args)
     if comm.rank() == 0:
         for r in results:
             if r:

@@ -177,6 +177,10 @@ register(ModelConfig("llama2-70b", vocab_size=32000, hidden_size=8192,
                      num_layers=80, num_heads=64, num_kv_heads=8,
                      intermediate_size=28672))
 
+register(ModelConfig("llama-1b", vocab_size=32000, hidden_size=2048,
+                     num_layers=16, num_heads=32, num_kv_heads=32,
+                     intermediate_size=5632))
+
 register(ModelConfig("llama3-8b", vocab_size=128256, hidden_size=4096,
                      num_layers=32, num_heads=32, num_kv_heads=8,
                      intermediate_size=14336, max_seq_len=8192,
@@ -304,12 +308,12 @@ _pimazen("tiny-pimazen", 3, 64, 256, 96,
 _pimazen("smoke-pimazen", 4, 256, 512, 384,
          dict(heads=4, dim=64, rot_dim=32, vdim=64, kv_rank=128, window=96,
               scale=96 ** -0.5), share_every=2, max_seq_len=1024)
-# sized like the layers of llama2-7b / mistral-7b and a narrower model
+# layers of the width, heads and mlp of llama2-7b and llama-1b
 _pimazen("pimazen-7b", 32, 4096, 32000, 11008,
          dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512,
               window=4096, scale=192 ** -0.5, rope_base=1000000.0),
          share_every=2, max_seq_len=32768)
 _pimazen("pimazen-1b", 16, 2048, 32000, 5632,
-         dict(heads=16, dim=64, rot_dim=32, vdim=64, kv_rank=256,
+         dict(heads=32, dim=64, rot_dim=32, vdim=64, kv_rank=256,
               window=2048, scale=96 ** -0.5), share_every=2,
          max_seq_len=32768)

@@ -12,12 +12,15 @@
 // A query at retained position i sees keys j with 0 <= i - j < window
 // (window 0: all earlier keys).
 //
-// MFMA kernel (bf16): 4 waves, 64-key tiles staged once into LDS (next tile
-// prefetched to registers). QK: each wave scores 16 keys for all rows, one
-// fp32 exchange through LDS for the row-wise online softmax, PV: each wave
-// owns a quarter of the latent columns and reads the same LDS rows
-// transposed (ds_read_b64_tr_b16). `nsplit` workgroups share a sequence's
-// keys; latent_combine merges their partial sums.
+// MFMA kernel (bf16): 8 waves, 64-key tiles staged once into double-buffered
+// LDS (the tile after next is in registers). QK: each wave scores 16 keys for
+// one part of the rows, whose q it keeps in registers (with 16 rows, for one
+// half of the columns); one fp32 exchange through LDS for the row-wise online
+// softmax; PV: each wave owns an eighth of the latent columns and reads the
+// same LDS rows transposed (ds_read_b64_tr_b16). Two barriers per tile: one
+// interval holds softmax(t) and the staging of tile t+1, the other PV(t) and
+// QK(t+1). `nsplit` workgroups share a sequence's keys; latent_combine merges
+// their partial sums.
 //
 // The scalar kernel covers fp32 and sizes beyond the MFMA tiles: one
 // workgroup per row, a wave per key, lanes across the cache row.
@@ -29,11 +32,13 @@
 
 namespace {
 
-constexpr int BLOCK = 256;
+constexpr int BLOCK = 512;             // MFMA kernel
+constexpr int ROWS_BLOCK = 256;        // scalar kernel
 constexpr int TK = 64;                 // keys per tile
 constexpr int ROTP = 64;               // padded rotated part
 constexpr int PAGE = 16;               // tokens per cache block
 constexpr int SSTRIDE = 68;            // floats per score row
+constexpr int PSTRIDE = 72;            // 16-bit weights per row
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
 typedef __attribute__((ext_vector_type(4))) float f32x4v;
@@ -65,31 +70,52 @@ RB_DEV bf16x8v read_column8(const char *p, int stride4) {
   return r.v;
 }
 
+// maximum over aligned groups of N lanes (N = 8, 16, 32)
+template <int N> RB_DEV float group_max(float v) {
+  auto dpp = [](float x, auto ctrl) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(
+        0, __float_as_int(x), decltype(ctrl)::value, 0xf, 0xf, true));
+  };
+  v = fmaxf(v, dpp(v, std::integral_constant<int, 0xB1>{}));   // lane ^ 1
+  v = fmaxf(v, dpp(v, std::integral_constant<int, 0x4E>{}));   // lane ^ 2
+  v = fmaxf(v, dpp(v, std::integral_constant<int, 0x141>{}));  // 7 - lane
+  if constexpr (N >= 16)
+    v = fmaxf(v, dpp(v, std::integral_constant<int, 0x140>{}));  // 15 - lane
+  if constexpr (N >= 32) v = fmaxf(v, __shfl_xor(v, 16, 64));
+  return v;
+}
+
 template <int RP, int MT>
 __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   constexpr int M = MT * 16;
   constexpr int COLS = RP + ROTP;
   constexpr int STRIDE = (COLS + 8) * 2;       // LDS row bytes
-  constexpr int STEPS = COLS / 32;
+  constexpr int KH = MT == 1 ? 2 : 1;          // column halves in QK
+  constexpr int QT = MT == 4 ? 2 : 1;          // row tiles per wave in QK
+  constexpr int NS = COLS / 32 / KH;           // QK steps per wave
   constexpr int CPP = COLS / 64;               // 16 B chunks per lane and key
-  constexpr int CT = RP / 64;                  // column tiles per wave
+  constexpr int CG = RP / 16 < 8 ? RP / 16 : 8;  // waves that own columns
+  constexpr int CT = RP / 16 / CG;             // their column tiles
   constexpr int TPR = BLOCK / M;               // softmax threads per row
   constexpr int KPT = TK / TPR;                // their keys
 
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  char *kv_s = smem;                           // [TK][STRIDE]
-  char *q_s = kv_s + TK * STRIDE;              // [M][STRIDE]
-  float *s_s = reinterpret_cast<float *>(q_s + M * STRIDE);  // [M][SSTRIDE]
-  float *alpha_s = s_s + M * SSTRIDE;          // [M]
+  char *kv_s = smem;                           // [2][TK][STRIDE]
+  float *s_s = reinterpret_cast<float *>(kv_s + 2 * TK * STRIDE);
+                                               // [KH][M][SSTRIDE]
+  uint16_t *p_s = reinterpret_cast<uint16_t *>(s_s + KH * M * SSTRIDE);
+                                               // [M][PSTRIDE]
+  float *alpha_s = reinterpret_cast<float *>(p_s + M * PSTRIDE);  // [M]
   float *l_s = alpha_s + M;                    // [M]
 
   const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
   const int l16 = lane & 15, grp = lane >> 4;
+  const int kg = wid & 3, part = wid >> 2;     // QK role: keys, rows/columns
   const int split = blockIdx.x, seq = blockIdx.z;
   const int q0 = a.cu_q[seq], nq = a.cu_q[seq + 1] - q0;
+  const int n_keys = a.seq_lens[seq];
   const int rows = nq * a.heads, row0 = blockIdx.y * M;
   if (row0 >= rows) return;
-  const int n_keys = a.seq_lens[seq];
   const int v0 = n_keys - nq;                  // retained position of query 0
   const int tok_lo = row0 / a.heads;
   const int tok_hi = (min(row0 + M, rows) - 1) / a.heads;
@@ -97,7 +123,8 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   const int key_lo = a.window > 0 ? max(0, v0 + tok_lo - a.window + 1) : 0;
   const int base = key_lo & ~(PAGE - 1);
   const int tiles = (key_hi - base + TK - 1) / TK;
-  const int per = (tiles + a.nsplit - 1) / a.nsplit;
+  // short contexts use fewer splits: at least two tiles each
+  const int per = max(2, (tiles + a.nsplit - 1) / a.nsplit);
   const int t0 = split * per, t1 = min(tiles, t0 + per);
   const int64_t grow0 = (int64_t)q0 * a.heads + row0;   // first global row
 
@@ -115,71 +142,65 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   const int *table = a.tables + (int64_t)seq * a.table_width;
   const u32x4v zero4 = (u32x4v)(0u);
 
-  // ---- q rows (zero-padded) and the padding columns of the key tile -----
-  for (int c = tid; c < M * (COLS / 8); c += BLOCK) {
-    const int m = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
-    u32x4v v = zero4;
-    if (row0 + m < rows) {
-      const int64_t g = grow0 + m;
-      if (col < RP) {
-        if (col < a.rc)
-          v = *reinterpret_cast<const u32x4v *>(
-              (const uint16_t *)a.q_lat + g * a.rc + col);
-      } else if (col - RP < a.rotc) {
-        v = *reinterpret_cast<const u32x4v *>(
-            (const uint16_t *)a.q_rot + (g / a.heads) * a.q_row +
-            (g % a.heads) * a.q_head + col - RP);
-      }
-    }
-    *reinterpret_cast<u32x4v *>(q_s + m * STRIDE + col * 2) = v;
-  }
-  for (int c = tid; c < TK * (COLS / 8); c += BLOCK) {
-    const int key = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
-    if (col < RP ? col >= a.rc : col - RP >= a.rotc)
-      *reinterpret_cast<u32x4v *>(kv_s + key * STRIDE + col * 2) = zero4;
-  }
-
-  // ---- tile loader: 8 lanes per key, 32 keys per pass, 2 passes ---------
+  // ---- tile loader: 8 lanes per key ---------------------------------------
+  // Branch-free: keys beyond the last one repeat it (their scores are masked),
+  // lanes beyond the row's last chunk repeat that chunk.
   const int lkey = tid >> 3, lchunk = tid & 7;
-  const int chunks = a.ec / 8;
-  u32x4v reg[2][CPP];
-  int page[2];
-  auto fetch_pages = [&](int t) {
-#pragma unroll
-    for (int p = 0; p < 2; ++p) {
-      const int key = base + t * TK + p * 32 + lkey;
-      page[p] = key < key_hi ? table[key / PAGE] : 0;
-    }
+  const int last_chunk = a.ec / 8 - 1, split_chunk = a.rc / 8;
+  u32x4v reg[CPP];
+  int page = 0;
+  auto fetch_page = [&](int t) {
+    page = table[min(base + t * TK + lkey, key_hi - 1) / PAGE];
   };
   auto fetch = [&](int t) {
+    const int key = min(base + t * TK + lkey, key_hi - 1);
+    const uint16_t *src = cache + ((int64_t)page * PAGE + key % PAGE) * a.ec;
 #pragma unroll
-    for (int p = 0; p < 2; ++p) {
-      const int key = base + t * TK + p * 32 + lkey;
-      const bool ok = key < key_hi;
-      const uint16_t *src =
-          cache + ((int64_t)page[p] * PAGE + key % PAGE) * a.ec;
+    for (int i = 0; i < CPP; ++i)
+      reg[i] = *reinterpret_cast<const u32x4v *>(
+          src + min(lchunk + i * 8, last_chunk) * 8);
+  };
+  auto stage = [&](char *dst) {
 #pragma unroll
-      for (int i = 0; i < CPP; ++i) {
-        const int c = lchunk + i * 8;
-        reg[p][i] = (ok && c < chunks)
-                        ? *reinterpret_cast<const u32x4v *>(src + c * 8)
-                        : zero4;
-      }
+    for (int i = 0; i < CPP; ++i) {
+      const int c = min(lchunk + i * 8, last_chunk);
+      const int col = c * 8 + (c < split_chunk ? 0 : RP - a.rc);
+      *reinterpret_cast<u32x4v *>(dst + lkey * STRIDE + col * 2) = reg[i];
     }
   };
-  auto stage = [&]() {
+  fetch_page(t0);
+
+  // ---- this wave's q fragments (zero beyond the real columns) -------------
+  bf16x8v qf[QT][NS];
 #pragma unroll
-    for (int p = 0; p < 2; ++p)
+  for (int qt = 0; qt < QT; ++qt) {
+    const int m = (KH == 2 ? 0 : part * QT + qt) * 16 + l16;
+    const bool ok = (KH == 2 || part * QT + qt < MT) && row0 + m < rows;
+    const int row = ok ? row0 + m : 0;
+    const int tok = q0 + row / a.heads, head = row % a.heads;
+    const uint16_t *ql = (const uint16_t *)a.q_lat +
+                         ((int64_t)tok * a.heads + head) * a.rc;
+    const uint16_t *qr = (const uint16_t *)a.q_rot + tok * a.q_row +
+                         head * a.q_head - RP;
 #pragma unroll
-      for (int i = 0; i < CPP; ++i) {
-        const int c = lchunk + i * 8;
-        if (c < chunks) {
-          const int col = c * 8 < a.rc ? c * 8 : RP + c * 8 - a.rc;
-          *reinterpret_cast<u32x4v *>(kv_s + (p * 32 + lkey) * STRIDE +
-                                      col * 2) = reg[p][i];
-        }
-      }
-  };
+    for (int s = 0; s < NS; ++s) {
+      const int col = ((KH == 2 ? part * NS : 0) + s) * 32 + grp * 8;
+      const bool in = col < RP ? col < a.rc : col - RP < a.rotc;
+      union { u32x4v u; bf16x8v v; } c;
+      const u32x4v v = *reinterpret_cast<const u32x4v *>(
+          in ? (col < RP ? ql : qr) + col : ql);
+      c.u = (ok && in) ? v : zero4;
+      qf[qt][s] = c.v;
+    }
+  }
+
+  // padding columns of both key tiles
+  if (a.rc < RP || a.rotc < ROTP)
+    for (int c = tid; c < 2 * TK * (COLS / 8); c += BLOCK) {
+      const int key = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
+      if (col < RP ? col >= a.rc : col - RP >= a.rotc)
+        *reinterpret_cast<u32x4v *>(kv_s + key * STRIDE + col * 2) = zero4;
+    }
 
   // ---- softmax role of this thread --------------------------------------
   const int srow = tid / TPR, spart = tid % TPR;
@@ -194,44 +215,96 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
 #pragma unroll
     for (int m = 0; m < MT; ++m) acc[c][m] = (f32x4v)(0.0f);
 
-  fetch_pages(t0);
-  fetch(t0);
-  if (t0 + 1 < t1) fetch_pages(t0 + 1);
-
-  for (int t = t0; t < t1; ++t) {
-    __syncthreads();                           // last tile fully read
-    stage();
-    __syncthreads();
-    if (t + 1 < t1) {
-      fetch(t + 1);
-      if (t + 2 < t1) fetch_pages(t + 2);
-    }
-
-    // ---- scores: wave's 16 keys x all rows ------------------------------
-    f32x4v sc[MT];
+  // ---- scores of a staged tile: 16 keys x this wave's rows ---------------
+  auto scores = [&](const char *tile) {
+    // key fragments come in groups, one group of LDS reads ahead of the
+    // products; two accumulators per row tile shorten the dependent chain
+    constexpr int G = NS == 18 && MT > 1 ? 3 : NS % 6 == 0 ? 6 :
+                      NS % 5 == 0 ? 5 : NS % 4 == 0 ? 4 :
+                      NS % 3 == 0 ? 3 : NS;
+    static_assert(NS % G == 0, "QK groups");
+    f32x4v sc[QT][2];
 #pragma unroll
-    for (int m = 0; m < MT; ++m) sc[m] = (f32x4v)(0.0f);
+    for (int q = 0; q < QT; ++q) sc[q][0] = sc[q][1] = (f32x4v)(0.0f);
+    const char *krow = tile + (kg * 16 + l16) * STRIDE + grp * 16 +
+                       (KH == 2 ? part * NS * 64 : 0);
+    bf16x8v kf[2][G];
 #pragma unroll
-    for (int s = 0; s < STEPS; ++s) {
-      const int off = (s * 32 + grp * 8) * 2;
-      const bf16x8v kf = *reinterpret_cast<const bf16x8v *>(
-          kv_s + (wid * 16 + l16) * STRIDE + off);
+    for (int s = 0; s < G; ++s)
+      kf[0][s] = *reinterpret_cast<const bf16x8v *>(krow + s * 64);
 #pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        const bf16x8v qf = *reinterpret_cast<const bf16x8v *>(
-            q_s + (m * 16 + l16) * STRIDE + off);
-        sc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf, kf, sc[m], 0, 0, 0);
+    for (int g = 0; g < NS / G; ++g) {
+      if (g + 1 < NS / G) {
+#pragma unroll
+        for (int s = 0; s < G; ++s)
+          kf[(g + 1) & 1][s] = *reinterpret_cast<const bf16x8v *>(
+              krow + ((g + 1) * G + s) * 64);
       }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int s = 0; s < G; ++s)
+#pragma unroll
+        for (int q = 0; q < QT; ++q)
+          sc[q][s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              qf[q][g * G + s], kf[g & 1][s], sc[q][s & 1], 0, 0, 0);
+      __builtin_amdgcn_sched_barrier(0);
     }
 #pragma unroll
-    for (int m = 0; m < MT; ++m)
+    for (int q = 0; q < QT; ++q) {
+      const int m0 = KH == 2 ? part * M : (part * QT + q) * 16;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        s_s[(m * 16 + grp * 4 + r) * SSTRIDE + wid * 16 + l16] =
-            sc[m][r] * a.scale;
-    __syncthreads();
+        s_s[(m0 + grp * 4 + r) * SSTRIDE + kg * 16 + l16] =
+            (sc[q][0][r] + sc[q][1][r]) * a.scale;
+    }
+  };
 
-    // ---- online softmax; P replaces the scores of its row ---------------
+  // ---- O^T += C^T P^T on the wave's latent columns ------------------------
+  auto accumulate = [&](const char *tile) {
+    if (wid >= CG) return;
+    bf16x8v pf[2][MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks)
+        pf[ks][m] = *reinterpret_cast<const bf16x8v *>(
+            p_s + (m * 16 + l16) * PSTRIDE + ks * 32 + grp * 8);
+      const float al = alpha_s[m * 16 + l16];
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[c][m][r] *= al;
+    }
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      const char *vrow = tile + (ks * 32 + grp * 8 + (l16 >> 2)) * STRIDE +
+                         (wid * (CT * 16) + (l16 & 3) * 4) * 2;
+      bf16x8v vf[CT];
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+        vf[c] = read_column8(vrow + c * 32, 4 * STRIDE);
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+          acc[c][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              vf[c], pf[ks][m], acc[c][m], 0, 0, 0);
+    }
+  };
+
+  fetch(t0);
+  if (t0 + 1 < t1) fetch_page(t0 + 1);
+  stage(kv_s);
+  if (t0 + 1 < t1) fetch(t0 + 1);
+  if (t0 + 2 < t1) fetch_page(t0 + 2);
+  __syncthreads();
+  scores(kv_s);
+
+  for (int t = t0; t < t1; ++t) {
+    char *tile = kv_s + ((t - t0) & 1) * TK * STRIDE;
+    char *next = kv_s + ((t - t0 + 1) & 1) * TK * STRIDE;
+    __syncthreads();                   // scores(t) written, PV(t-1) done
+    // ---- online softmax ---------------------------------------------------
     {
       float p[KPT];
       float mx = -INFINITY;
@@ -239,67 +312,43 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
       const int k0 = base + t * TK + spart * KPT;
 #pragma unroll
       for (int j = 0; j < KPT; ++j) {
+        p[j] = sr[j];
+        if constexpr (KH == 2) p[j] += sr[M * SSTRIDE + j];
+      }
+#pragma unroll
+      for (int j = 0; j < KPT; ++j) {
         const bool vis = k0 + j <= qpos && k0 + j >= kmin;
-        p[j] = vis ? sr[j] : -INFINITY;
+        p[j] = vis ? p[j] : -INFINITY;
         mx = fmaxf(mx, p[j]);
       }
+      const float m_new = fmaxf(m_run, group_max<TPR>(mx));
+      // rows that have seen no key yet keep a finite reference
+      const float ref = m_new == -INFINITY ? 0.0f : m_new;
+      const float alpha = __expf(m_run - ref);   // 0 before the first key
+      float sum = 0.0f;
 #pragma unroll
-      for (int o = TPR / 2; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
-      const float m_new = fmaxf(m_run, mx);
-      float alpha = 1.0f;
-      if (m_new != -INFINITY) {
-        alpha = __expf(m_run - m_new);         // 0 on the first visible tile
-        float sum = 0.0f;
-#pragma unroll
-        for (int j = 0; j < KPT; ++j) {
-          p[j] = __expf(p[j] - m_new);
-          sum += p[j];
-        }
-        l_run = l_run * alpha + sum;
-        m_run = m_new;
-      } else {
-#pragma unroll
-        for (int j = 0; j < KPT; ++j) p[j] = 0.0f;
+      for (int j = 0; j < KPT; ++j) {
+        p[j] = __expf(p[j] - ref);
+        sum += p[j];
       }
-      // a row's threads are lanes of one wave: all have read their scores
-      uint32_t *pr = reinterpret_cast<uint32_t *>(s_s + srow * SSTRIDE) +
-                     spart * (KPT / 2);
+      l_run = l_run * alpha + sum;
+      m_run = m_new;
+      uint32_t *pr =
+          reinterpret_cast<uint32_t *>(p_s + srow * PSTRIDE + spart * KPT);
 #pragma unroll
       for (int j = 0; j < KPT; j += 2)
         pr[j / 2] = rb::f32_to_bf16(p[j]) |
                     ((uint32_t)rb::f32_to_bf16(p[j + 1]) << 16);
       if (spart == 0) alpha_s[srow] = alpha;
     }
-    __syncthreads();
-
-    // ---- O^T += C^T P^T on the wave's latent columns --------------------
-    bf16x8v pf[2][MT];
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-      const float al = alpha_s[m * 16 + l16];
-#pragma unroll
-      for (int c = 0; c < CT; ++c)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) acc[c][m][r] *= al;
-#pragma unroll
-      for (int ks = 0; ks < 2; ++ks)
-        pf[ks][m] = *reinterpret_cast<const bf16x8v *>(
-            reinterpret_cast<const char *>(s_s + (m * 16 + l16) * SSTRIDE) +
-            (ks * 32 + grp * 8) * 2);
+    if (t + 1 < t1) {
+      stage(next);
+      if (t + 2 < t1) fetch(t + 2);
+      if (t + 3 < t1) fetch_page(t + 3);
     }
-#pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      const char *vrow = kv_s + (ks * 32 + grp * 8 + (l16 >> 2)) * STRIDE +
-                         (wid * (RP / 4) + (l16 & 3) * 4) * 2;
-#pragma unroll
-      for (int c = 0; c < CT; ++c) {
-        const bf16x8v vf = read_column8(vrow + c * 32, 4 * STRIDE);
-#pragma unroll
-        for (int m = 0; m < MT; ++m)
-          acc[c][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[ks][m],
-                                                              acc[c][m], 0, 0, 0);
-      }
-    }
+    __syncthreads();                   // P(t) and tile t+1 are there
+    accumulate(tile);
+    if (t + 1 < t1) scores(next);
   }
 
   // ---- row sums, then O^T: lane holds 4 consecutive columns of one row ---
@@ -315,6 +364,7 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
     }
   }
   __syncthreads();
+  if (wid >= CG) return;
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
     const int row = m * 16 + l16;
@@ -323,7 +373,7 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
     const float inv = l > 0.0f ? 1.0f / l : 0.0f;
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
-      const int col = wid * (RP / 4) + c * 16 + grp * 4;
+      const int col = wid * (CT * 16) + c * 16 + grp * 4;
       if (col >= a.rc) continue;
       if (a.nsplit > 1) {
         *reinterpret_cast<f32x4v *>(
@@ -342,30 +392,35 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   }
 }
 
-// one block per row: merge the splits
+// One block per row merges the splits (at most 64). Each wave reads all
+// splits' statistics at once; splits without keys get weight 0 and the
+// address of one that has some, so every load is unconditional.
 __global__ __launch_bounds__(128) void latent_combine_kernel(
     const float *__restrict__ part_o, const float *__restrict__ part_ml,
     uint16_t *__restrict__ out, int nsplit, int total_rows, int rc) {
   const int64_t row = blockIdx.x;
-  float mx = -INFINITY;
-  for (int s = 0; s < nsplit; ++s)
-    mx = fmaxf(mx, part_ml[((int64_t)s * total_rows + row) * 2]);
-  float l = 0.0f;
-  for (int s = 0; s < nsplit; ++s) {
-    const float *ml = part_ml + ((int64_t)s * total_rows + row) * 2;
-    if (ml[1] > 0.0f) l += ml[1] * __expf(ml[0] - mx);
+  const int lane = threadIdx.x & 63;
+  float m = -INFINITY, l = 0.0f;
+  if (lane < nsplit) {
+    const float2 ml = *reinterpret_cast<const float2 *>(
+        part_ml + ((int64_t)lane * total_rows + row) * 2);
+    m = ml.x;
+    l = ml.y;
   }
-  const float inv = l > 0.0f ? 1.0f / l : 0.0f;
+  const bool has = l > 0.0f;
+  const float mx = rb::wave_reduce_max(m);
+  float w = has ? __expf(m - mx) : 0.0f;
+  w /= rb::wave_reduce_sum(l * w);
+  const int src = has ? lane : __builtin_ctzll(__ballot(has));
   for (int c = threadIdx.x * 4; c < rc; c += blockDim.x * 4) {
     f32x4v o = (f32x4v)(0.0f);
+#pragma unroll 8
     for (int s = 0; s < nsplit; ++s) {
-      const float *ml = part_ml + ((int64_t)s * total_rows + row) * 2;
-      if (!(ml[1] > 0.0f)) continue;
-      const float w = __expf(ml[0] - mx) * inv;
+      const float ws = __shfl(w, s, 64);
       const f32x4v p = *reinterpret_cast<const f32x4v *>(
-          part_o + ((int64_t)s * total_rows + row) * rc + c);
+          part_o + ((int64_t)__shfl(src, s, 64) * total_rows + row) * rc + c);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] += w * p[e];
+      for (int e = 0; e < 4; ++e) o[e] += ws * p[e];
     }
     uint2 w2;
     w2.x = rb::f32_to_bf16(o[0]) | ((uint32_t)rb::f32_to_bf16(o[1]) << 16);
@@ -378,7 +433,7 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
 // scalar kernel: block = one (token, head) row, wave = every fourth key
 // ---------------------------------------------------------------------------
 template <typename T, int NE>
-__global__ __launch_bounds__(BLOCK) void latent_attend_rows_kernel(
+__global__ __launch_bounds__(ROWS_BLOCK) void latent_attend_rows_kernel(
     AttendArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   float *o_s = reinterpret_cast<float *>(smem);        // [4][ec]
@@ -438,7 +493,7 @@ __global__ __launch_bounds__(BLOCK) void latent_attend_rows_kernel(
     w[k] = ml_s[k][1] > 0.0f ? expf(ml_s[k][0] - mx) : 0.0f;
     lt += w[k] * ml_s[k][1];
   }
-  for (int e = threadIdx.x; e < a.rc; e += BLOCK) {
+  for (int e = threadIdx.x; e < a.rc; e += ROWS_BLOCK) {
     float v = 0.0f;
 #pragma unroll
     for (int k = 0; k < 4; ++k) v += w[k] * o_s[k * a.ec + e];
@@ -453,8 +508,10 @@ int padded_rank(int64_t rc) {
 
 template <int RP, int MT>
 void launch_attend(const AttendArgs &a, dim3 grid, hipStream_t stream) {
-  constexpr size_t shmem = (size_t)(TK + MT * 16) * ((RP + ROTP + 8) * 2) +
-                           (size_t)MT * 16 * (SSTRIDE + 2) * sizeof(float);
+  constexpr int planes = MT == 1 ? 2 : 1;
+  constexpr size_t shmem =
+      (size_t)2 * TK * ((RP + ROTP + 8) * 2) +
+      (size_t)MT * 16 * ((planes * SSTRIDE + 2) * sizeof(float) + PSTRIDE * 2);
   static_assert(shmem <= 160 * 1024, "LDS");
   static bool once = [] {
     return hipFuncSetAttribute(
@@ -538,7 +595,7 @@ at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
     auto go = [&](auto tag, auto n) {
       using E = decltype(tag);
       hipLaunchKernelGGL((latent_attend_rows_kernel<E, decltype(n)::value>),
-                         grid, dim3(BLOCK), shmem, stream, a);
+                         grid, dim3(ROWS_BLOCK), shmem, stream, a);
     };
     auto pick = [&](auto tag) {
       if (ne == 2) go(tag, std::integral_constant<int, 2>{});
@@ -551,7 +608,7 @@ at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
     return out;
   }
 
-  a.nsplit = (int)std::max<int64_t>(1, nsplit);
+  a.nsplit = (int)std::min<int64_t>(64, std::max<int64_t>(1, nsplit));
   at::Tensor po, pml;
   if (a.nsplit > 1) {
     const auto f32 = q_lat.options().dtype(at::kFloat);

@@ -105,42 +105,28 @@ __global__ __launch_bounds__(BLOCK, 2) void latent_flash_kernel(FlashArgs a) {
   const int last = rel + min(nq, q0 + wid * 32 + 32) - 1;
   const int tile0 = wg_lo / KB, tile1 = (wg_hi + KB - 1) / KB;
 
-  // zero the padding columns once
-  for (int c = tid; c < KB * (DQ / 8); c += BLOCK) {
-    const int key = c / (DQ / 8), d = (c % (DQ / 8)) * 8;
-    if (d >= a.dimc + a.rotc)
-      *reinterpret_cast<u32x4v *>(k_s + key * KSTRIDE + d * 2) = zero4;
-  }
-  for (int c = tid; c < KB * (DV / 8); c += BLOCK) {
-    const int key = c / (DV / 8), d = (c % (DV / 8)) * 8;
-    if (d >= a.vc)
-      *reinterpret_cast<u32x4v *>(v_s + key * VSTRIDE + d * 2) = zero4;
-  }
-
   const int lkey = tid >> 3, lchunk = tid & 7;
   const int kvrow = a.heads * (a.dimc + a.vc);
   u32x4v kr[2][KC], vr[2][VC];
+  // Branch-free: keys beyond the last one repeat it (masked), columns beyond
+  // the real ones hold finite values (q is zero there, or they are not kept).
   auto fetch = [&](int t) {
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
-      const int key = t * KB + p * 32 + lkey;
-      const bool ok = key < wg_hi;
-      const int64_t krow = k_row0 + (ok ? key : 0);
+      const int64_t krow = k_row0 + min(t * KB + p * 32 + lkey, wg_hi - 1);
       const uint16_t *kvp = a.kv + krow * kvrow + h * (a.dimc + a.vc);
       const uint16_t *cp = a.ctx + krow * a.ec + a.rc - a.dimc;
 #pragma unroll
       for (int i = 0; i < KC; ++i) {
         const int d = (lchunk + i * 8) * 8;
-        const uint16_t *src = d < a.dimc ? kvp + d : cp + d;
-        kr[p][i] = (ok && d < a.dimc + a.rotc)
-                       ? *reinterpret_cast<const u32x4v *>(src) : zero4;
+        kr[p][i] = *reinterpret_cast<const u32x4v *>(
+            d < a.dimc ? kvp + d : d < a.dimc + a.rotc ? cp + d : kvp);
       }
 #pragma unroll
       for (int i = 0; i < VC; ++i) {
         const int d = (lchunk + i * 8) * 8;
-        vr[p][i] = (ok && d < a.vc)
-                       ? *reinterpret_cast<const u32x4v *>(kvp + a.dimc + d)
-                       : zero4;
+        vr[p][i] = *reinterpret_cast<const u32x4v *>(
+            kvp + a.dimc + (d < a.vc ? d : 0));
       }
     }
   };

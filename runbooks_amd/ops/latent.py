@@ -322,14 +322,14 @@ def latent_expand(o_lat, lay, w_expand, y, z, swz=None):
 
 def attend_split(n_seqs: int, row_tiles: int, max_keys: int | None,
                  window: int | None, max_q: int) -> int:
-    """Cache splits per (sequence, row tile): enough workgroups for the
-    chip, each with at least two 64-key tiles."""
+    """Cache splits per (sequence, row tile): one workgroup per CU, each
+    with at least two 64-key tiles."""
     keys = max_keys
     if window is not None:
         w = window + max_q - 1
         keys = w if keys is None else min(keys, w)
     base = max(1, n_seqs * row_tiles)
-    fill = max(1, -(-512 // base))
+    fill = max(1, -(-256 // base))
     if keys is not None:
         fill = min(fill, -(-keys // 128))
     return max(1, min(32, fill))
