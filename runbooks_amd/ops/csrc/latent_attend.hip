@@ -408,17 +408,25 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
     l = ml.y;
   }
   const bool has = l > 0.0f;
+  const int first = __ffsll((unsigned long long)__ballot(has)) - 1;
   const float mx = rb::wave_reduce_max(m);
   float w = has ? __expf(m - mx) : 0.0f;
   w /= rb::wave_reduce_sum(l * w);
-  const int src = has ? lane : __builtin_ctzll(__ballot(has));
+  // through LDS: not every lane takes part in the loop below
+  __shared__ float w_s[64];
+  __shared__ int src_s[64];
+  if (threadIdx.x < 64) {
+    w_s[lane] = w;
+    src_s[lane] = has ? lane : max(first, 0);
+  }
+  __syncthreads();
   for (int c = threadIdx.x * 4; c < rc; c += blockDim.x * 4) {
     f32x4v o = (f32x4v)(0.0f);
 #pragma unroll 8
     for (int s = 0; s < nsplit; ++s) {
-      const float ws = __shfl(w, s, 64);
+      const float ws = w_s[s];
       const f32x4v p = *reinterpret_cast<const f32x4v *>(
-          part_o + ((int64_t)__shfl(src, s, 64) * total_rows + row) * rc + c);
+          part_o + ((int64_t)src_s[s] * total_rows + row) * rc + c);
 #pragma unroll
       for (int e = 0; e < 4; ++e) o[e] += ws * p[e];
     }

@@ -1,0 +1,659 @@
+"""Latent attention and the Pimazen family on the CPU path: every op and
+whole engine runs against the plain oracle (tests/latent_oracle.py)."""
+import io
+import json
+import os
+
+import numpy as np
+import pytest
+import torch
+
+import latent_oracle as oracle
+from latent_helpers import (MODELS, load, make, make_engine, rel_err, run_cut,
+                            tokens_of, write_checkpoint)
+from runbooks_amd import ops
+from runbooks_amd.models import get_config
+from runbooks_amd.models.config import (GatedMLPSpec, LatentAttentionSpec,
+                                        LayerSpec, layered_config)
+from runbooks_amd.models.load import (config_from_dir, config_from_pimazen,
+                                      config_to_pimazen, load_pretrained)
+from runbooks_amd.models.ragged import Portion, StepPlan
+from runbooks_amd.ops import latent as L
+
+TOL = 2e-5
+
+
+# --- single mechanisms -------------------------------------------------------
+
+def test_norm_of_a_32_bit_residual():
+    g = torch.Generator().manual_seed(0)
+    x = torch.randn(5, 24, generator=g)
+    d = torch.randn(5, 24, generator=g)
+    w = torch.rand(24, generator=g)
+    for delta, add in ((None, 0), (d, d), (torch.stack([d, d]), 2 * d)):
+        y = x.clone()
+        got = ops.rmsnorm_res32(y, delta, w, 3e-3, torch.float32)
+        assert torch.allclose(y, x + add)
+        ref = oracle.rms_norm((x + add).double(), w.double(), 3e-3)
+        assert torch.allclose(got.double(), ref, atol=1e-5)
+
+
+@pytest.mark.parametrize("dims", [2, 6, 8])
+def test_interleaved_rotation(dims):
+    x = torch.randn(7, 3, 8)
+    pos = torch.tensor([0, 1, 5, 900, 17, 2, 63])
+    cos, sin = ops.rope_tables(dims, 1000, 777.0)
+    got = L.rope_interleaved_ref(x, cos, sin, pos)
+    ref = oracle.rotate_interleaved(x.double(), pos, 777.0, dims)
+    assert torch.allclose(got.double(), ref, atol=1e-5)
+    assert torch.equal(got[0], x[0])             # position 0 does not turn
+    assert torch.equal(got[..., dims:], x[..., dims:])
+
+
+def test_clamped_gated_unit():
+    g = torch.tensor([[-9.0, -0.5, 0.3, 1.1, 8.0]])
+    u = torch.tensor([[5.0, -7.0, 0.2, -0.4, 0.9]])
+    eye = torch.eye(5, dtype=torch.float64)
+    for limit, alpha, shift in ((1.0, 1.702, 1.0), (0.4, 1.0, 0.0)):
+        got = L.clamped_glu_ref(g, u, limit, alpha, shift)
+        both = torch.cat([g, u], 1).double()
+        sel = torch.eye(10, dtype=torch.float64)
+        ref = oracle.clamped_glu(both, sel[:5], sel[5:], eye, limit, alpha,
+                                 shift)
+        assert torch.allclose(got.double(), ref, atol=1e-6)
+    # the gate is bounded above only
+    low = L.clamped_glu_ref(torch.tensor([-3.0]), torch.tensor([0.0]), 1.0,
+                            1.702, 1.0)
+    assert float(low) == pytest.approx(-3 / (1 + np.exp(3 * 1.702)), rel=1e-5)
+
+
+def _layout(own=True):
+    return L.LatentLayout(heads=3, dim=20, rot=12, vdim=18, rank=36, ff=50,
+                          own_latent=own)
+
+
+def test_wide_projection_layout_and_prep():
+    """The padded wide product and its epilogue give the oracle's queries,
+    cached rows and MLP activation; a layer without latents of its own
+    leaves the cache alone."""
+    lay, D, T = _layout(), 40, 9
+    g = torch.Generator().manual_seed(1)
+    r = lambda *s: torch.randn(*s, generator=g)  # noqa: E731
+    q, dkv = r(3 * 32, D), r(48, D)
+    gw, gate, up = r(3 * 18, D), r(50, D), r(50, D)
+    h, w = r(T, D) * 0.2, torch.rand(36, generator=g)
+    pos = torch.arange(T, dtype=torch.int32) + 4
+    slots = torch.tensor([40, 3, 17, 16, 15, 31, 32, 5, 63],
+                         dtype=torch.int32)
+    cos, sin = ops.rope_tables(12, 64, 100.0)
+    mlp = GatedMLPSpec(50, 0.7)
+    y = h @ L.pack_wide(lay, q, dkv, gw, gate, up).T
+    cache = L.alloc_latent_cache(4, lay, "cpu", torch.float32)
+    z = torch.full((T, lay.n_z), 7.0)
+    L.latent_prep(y, lay, cos, sin, pos, slots, cache, w, 1e-3, mlp, z)
+
+    hd = h.double()
+    qr = (hd @ q.double().T).view(T, 3, 32)
+    got = y[:, :lay.off_kv].view(T, 3, lay.qc)
+    assert torch.allclose(got[..., :20].double(), qr[..., :20], atol=1e-4)
+    assert torch.allclose(
+        got[..., lay.dimc:lay.dimc + 12].double(),
+        oracle.rotate_interleaved(qr[..., 20:], pos, 100.0, 12), atol=1e-4)
+    c, kr = oracle.latent_and_key(hd, dkv.double(), w.double(), 1e-3, 36,
+                                  {"base": 100.0, "dims": 12}, pos)
+    rows = cache.view(-1, lay.ec)[slots.long()].double()
+    assert torch.allclose(rows[:, :36], c, atol=1e-4)
+    assert torch.allclose(rows[:, lay.rc:lay.rc + 12], kr, atol=1e-4)
+    untouched = sorted(set(range(64)) - set(slots.tolist()))
+    assert not cache.view(-1, lay.ec)[untouched].any()
+    act = oracle.clamped_glu(hd, gate.double(), up.double(),
+                             torch.eye(50, dtype=torch.float64), 0.7)
+    assert torch.allclose(z[:, lay.off_act:lay.off_act + 50].double(), act,
+                          atol=1e-4)
+    assert not z[:, lay.off_act + 50:].any()
+
+    other = _layout(own=False)
+    y2 = h @ L.pack_wide(other, q, None, gw, gate, up).T
+    before = cache.clone()
+    L.latent_prep(y2, other, cos, sin, pos, slots, cache, None, 0.0, mlp, z)
+    assert torch.equal(cache, before)
+    assert torch.allclose(y2[:, :other.off_kv], y[:, :lay.off_kv])
+
+
+def _attention_case(window, portions, seed=0, peak=None, lay=None):
+    """Both attention forms on one batch, and the oracle's answer.
+
+    peak (seq, query, key, other): the query scores `key` far above all
+    others, and `other` second."""
+    lay = lay or L.LatentLayout(heads=2, dim=12, rot=8, vdim=10, rank=20,
+                                ff=0, own_latent=True)
+    g = torch.Generator().manual_seed(seed)
+    H, R = lay.heads, lay.rank
+    T = sum(len(p.tokens) for p in portions)
+    y = torch.zeros(T, lay.n_y)
+    q = torch.randn(T, H, lay.dim + lay.rot, generator=g)
+    gate = torch.randn(T, H * lay.vdim, generator=g)
+    cache = L.alloc_latent_cache(64, lay, "cpu", torch.float32)
+    flat = cache.view(-1, lay.ec)
+    flat[:, :R] = torch.randn(len(flat), R, generator=g)
+    flat[:, lay.rc:lay.rc + lay.rot] = torch.randn(len(flat), lay.rot,
+                                                   generator=g)
+    uk = torch.randn(H, lay.dim, R, generator=g) / R ** 0.5
+    uv = torch.randn(H, lay.vdim, R, generator=g) / R ** 0.5
+
+    def slot(p, i):
+        return p.blocks[i // 16] * 16 + i % 16
+
+    row = 0
+    rows_of = []
+    for p in portions:
+        rows_of.append(row)
+        row += len(p.tokens)
+    if peak is not None:
+        s, qi, key, other = peak
+        p = portions[s]
+        t = rows_of[s] + qi - (p.start - p.dropped)
+        for k, gain in ((key, 9.0), (other, 6.0)):
+            flat[slot(p, k), lay.rc:lay.rc + lay.rot] = 0
+            flat[slot(p, k), lay.rc + (0 if k == key else 1)] = gain
+        q[t, :, lay.dim:] = 0
+        q[t, :, lay.dim] = 9.0
+        q[t, :, lay.dim + 1] = 9.0
+    y[:, :lay.off_kv].view(T, H, lay.qc)[..., :lay.dim] = q[..., :lay.dim]
+    y[:, :lay.off_kv].view(T, H, lay.qc)[
+        ..., lay.dimc:lay.dimc + lay.rot] = q[..., lay.dim:]
+    y[:, lay.off_g:lay.off_gate].view(T, H, lay.vc)[..., :lay.vdim] = \
+        gate.view(T, H, lay.vdim)
+
+    ref = []
+    for p, r0 in zip(portions, rows_of):
+        n = p.start - p.dropped + len(p.tokens)
+        kv = flat[[slot(p, i) for i in range(n)]].double()
+        c, kr = kv[:, :R], kv[:, lay.rc:lay.rc + lay.rot]
+        k = torch.cat([torch.einsum("kr,hdr->khd", c, uk.double()),
+                       kr[:, None].expand(n, H, lay.rot)], -1)
+        v = torch.einsum("kr,hvr->khv", c, uv.double())
+        nq = len(p.tokens)
+        qq = torch.zeros(n, H, k.shape[-1], dtype=torch.float64)
+        qq[n - nq:] = q[r0:r0 + nq].double()
+        o = oracle.softmax_attention(qq, k, v, 0.21,
+                                     oracle.window_mask(n, window))[n - nq:]
+        ref.append(o.reshape(nq, -1) *
+                   torch.sigmoid(gate[r0:r0 + nq].double()))
+
+    pad = torch.nn.functional.pad
+    out = {}
+    for name, expand in (("latent", False), ("expanded", True)):
+        import runbooks_amd.models.ragged as ragged
+        keep, ragged.ABSORB_MAX = ragged.ABSORB_MAX, 0
+        try:
+            b = StepPlan(portions).build(16, [window], "cpu", expand=expand)
+        finally:
+            ragged.ABSORB_MAX = keep
+        z = torch.zeros(T, lay.n_z)
+        if expand:
+            slots, meta = b.long_plans[window]
+            ctx = flat.index_select(0, slots)
+            kv = ctx[:, :lay.rc] @ L.pack_expand(
+                lay, uk.reshape(-1, R), uv.reshape(-1, R)).T
+            L.latent_flash(y, lay, kv, ctx, meta, b.max_q_long, 0.21, window,
+                           z)
+        else:
+            wa = pad(uk, (0, lay.rc - R, 0, lay.dimc - lay.dim))
+            we = pad(uv, (0, lay.rc - R, 0, lay.vc - lay.vdim))
+            ql = L.latent_absorb(y, lay, wa, T)
+            ol = L.latent_attend(ql, y, lay, cache, b, 0.21, window)
+            L.latent_expand(ol, lay, we.transpose(1, 2), y, z)
+        out[name] = z[:, :lay.off_act].view(T, H, lay.vc)[
+            ..., :lay.vdim].reshape(T, -1)
+    return out, torch.cat(ref), rows_of
+
+
+def _portions(*spec, seed=3):
+    g = torch.Generator().manual_seed(seed)
+    free = torch.randperm(64, generator=g).tolist()
+    out = []
+    for n, start, dropped in spec:
+        nb = -(-(start + n - dropped) // 16)
+        out.append(Portion([0] * n, start, dropped,
+                           [free.pop() for _ in range(nb)], []))
+    return out
+
+
+@pytest.mark.parametrize("window", [None, 1, 7, 16, 33])
+def test_both_attention_forms(window):
+    drop = 0 if window is None else 16
+    ps = _portions((1, 0, 0), (5, 0, 0), (1, 47, 0), (2, 15, 0),
+                   (40, 60, drop), (17, 16, 0))
+    out, ref, _ = _attention_case(window, ps)
+    for name, got in out.items():
+        assert (got.double() - ref).abs().max() < TOL, name
+
+
+@pytest.mark.parametrize("window,inside", [(20, True), (20, False),
+                                           (None, True)])
+@pytest.mark.parametrize("query", [31, 32, 47, 70])
+def test_standout_key_at_the_window_edge(window, inside, query):
+    """The oldest visible key, given a score far above the rest, takes the
+    whole output; the next older one has no effect at all."""
+    ps = _portions((40, 40, 0), (60, 20, 0))
+    s = 1
+    key = 0 if window is None else query - window + (1 if inside else 0)
+    out, ref, rows = _attention_case(window, ps, peak=(s, query, key,
+                                                       query - 3))
+    t = rows[s] + query - 20
+    flat_out, _, _ = _attention_case(window, ps, peak=(s, query, query,
+                                                       query - 3))
+    for name, got in out.items():
+        assert (got.double() - ref).abs().max() < TOL
+    # the standout key decides the answer only when it is visible
+    alone = _attention_case(1, ps, peak=(s, query, query, query - 3))[1]
+    differs = (out["latent"][t] - flat_out["latent"][t]).abs().max()
+    assert differs > 1e-2
+    assert alone.shape == ref.shape
+
+
+# --- whole models -------------------------------------------------------------
+
+@pytest.mark.parametrize("name", list(MODELS))
+@pytest.mark.parametrize("cuts", [[1000], [1], [2], [3, 40, 2, 1, 17],
+                                  [33, 1], [16], [64, 5]])
+def test_any_cut_of_the_prompt(name, cuts):
+    cfg, W = make(name)
+    toks = tokens_of(cfg, 90 if name == "wide" else 150)
+    ref = oracle.forward(cfg, W, toks)
+    eng = make_engine(cfg, W)
+    assert rel_err(run_cut(eng, toks, cuts), ref) < TOL
+    assert len(eng.allocator.free) == eng.allocator.num_blocks
+
+
+def test_residual_after_every_layer():
+    cfg, W = make("mixed")
+    toks = tokens_of(cfg, 70)
+    want = []
+    oracle.forward(cfg, W, toks, layers_out=want)
+    eng = make_engine(cfg, W)
+    got, blocks = [], eng.model.blocks
+    for i, blk in enumerate(blocks):
+        step = blk.step
+
+        def spy(x, delta, *a, _step=step, _first=i == 0):
+            if not _first:
+                got.append(x + delta)
+            out = _step(x, delta, *a)
+            return out
+        blk.step = spy
+    run_cut(eng, toks, [1000])
+    assert len(got) == len(blocks) - 1
+    for g, w in zip(got, want):
+        assert (g.double() - w).abs().max() < 1e-4
+
+
+@pytest.mark.parametrize("layer,delta", [(0, 1), (0, -1), (1, 1), (2, -1),
+                                         (3, 1), (3, -1)])
+def test_a_window_off_by_one_shows(layer, delta):
+    """The comparison above is sharp: the oracle with one window moved by a
+    token differs far beyond its tolerance."""
+    cfg, W = make("mixed")
+    toks = tokens_of(cfg, 150)
+    ref = oracle.forward(cfg, W, toks)
+    wrong = json.loads(json.dumps(cfg))
+    wrong["layers"][layer]["mixer"]["mask"]["size"] += delta
+    assert rel_err(oracle.forward(wrong, W, toks), ref) > 50 * TOL
+
+
+@pytest.mark.parametrize("change", [
+    lambda c: c["layers"][1]["mixer"].update(scale=0.31),
+    lambda c: c["layers"][0]["mlp"].update(limit=1.31),
+    lambda c: c["norm"].update(eps=2e-3),
+    lambda c: [c["layers"][i]["mixer"]["rot"].update(base=510.0)
+               for i in (0, 1)],
+])
+def test_every_constant_is_read(change):
+    cfg, W = make("mixed")
+    toks = tokens_of(cfg, 60)
+    ref = oracle.forward(cfg, W, toks)
+    change(cfg)
+    moved = oracle.forward(cfg, W, toks)
+    assert rel_err(moved, ref) > 20 * TOL
+    assert rel_err(run_cut(make_engine(cfg, W), toks, [25]), moved) < TOL
+
+
+def test_first_tokens_and_single_token_prompt():
+    cfg, W = make("mixed")
+    for n in (1, 2, 3):
+        toks = tokens_of(cfg, n, seed=n)
+        ref = oracle.forward(cfg, W, toks)
+        for cuts in ([n], [1]):
+            assert rel_err(run_cut(make_engine(cfg, W), toks, cuts), ref) < TOL
+
+
+@pytest.mark.parametrize("name", ["mixed", "full"])
+def test_unequal_requests_in_one_batch(name):
+    """Portions beside single tokens, requests that pause, end and make way:
+    every logit as if the request were alone, on a pool that only just
+    holds the live ones."""
+    cfg, W = make(name)
+    lens = [130, 3, 61, 1, 97, 40]
+    seqs = [tokens_of(cfg, n, seed=i) for i, n in enumerate(lens)]
+    refs = [oracle.forward(cfg, W, s) for s in seqs]
+    eng = make_engine(cfg, W, kv_blocks=23)
+    g = torch.Generator().manual_seed(5)
+    waiting, live = list(range(len(seqs))), {}
+    used, reused = set(), False
+    while waiting or live:
+        while waiting and len(live) < 3:
+            i = waiting.pop(0)
+            live[i] = [eng.open_request(), 0]
+        entries, ids = [], []
+        for i, (r, at) in live.items():
+            if len(live) > 1 and int(torch.randint(0, 4, (1,),
+                                                   generator=g)) == 0:
+                continue
+            n = [1, 1, 2, 7, 34, 50][int(torch.randint(0, 6, (1,),
+                                                       generator=g))]
+            n = min(n, len(seqs[i]) - at)
+            entries.append((r, seqs[i][at:at + n], range(n)))
+            ids.append((i, at, n))
+        if not entries:
+            continue
+        logits = eng.run_portions(entries)
+        row = 0
+        for (i, at, n), (r, _, _) in zip(ids, entries):
+            assert rel_err(logits[row:row + n], refs[i][at:at + n]) < 2 * TOL
+            row += n
+            live[i][1] = at + n
+            reused |= bool(used & set(r.blocks))
+            if at + n == len(seqs[i]):
+                used |= set(r.blocks)
+                eng.close_request(r)
+                del live[i]
+    assert reused
+    assert len(eng.allocator.free) == eng.allocator.num_blocks
+
+
+def test_stale_pages_do_not_leak():
+    """A page's former content must not reach its next owner."""
+    cfg, W = make("full")
+    eng = make_engine(cfg, W, kv_blocks=12)
+    toks = tokens_of(cfg, 100, seed=8)
+    ref = oracle.forward(cfg, W, toks)
+    for c in eng.caches:
+        c.fill_(50.0)
+    assert rel_err(run_cut(eng, toks, [7, 1, 40]), ref) < TOL
+    assert rel_err(run_cut(eng, toks, [50]), ref) < TOL
+
+
+def test_cache_is_shared_and_bounded_by_the_window():
+    cfg, W = make("mixed")
+    eng = make_engine(cfg, W)
+    assert eng.caches[1] is eng.caches[0] and eng.caches[3] is eng.caches[2]
+    assert eng.caches[2] is not eng.caches[0]
+    r = eng.open_request()
+    run_cut(eng, tokens_of(cfg, 400), [50, 1, 1], req=r)
+    held = len(r.blocks) * 16
+    assert r.dropped > 250 and held <= 64 + 50 + 32
+    full = make_engine(*make("full"))
+    r = full.open_request()
+    run_cut(full, tokens_of(cfg, 200)[:200] and tokens_of(make("full")[0],
+                                                         200), [64], req=r)
+    assert r.dropped == 0
+
+
+def test_pool_and_length_limits_are_errors():
+    cfg, W = make("full")
+    eng = make_engine(cfg, W, kv_blocks=4)
+    with pytest.raises(RuntimeError, match="exhausted"):
+        run_cut(eng, tokens_of(cfg, 80), [80])
+    eng.cfg.max_seq_len = 20
+    with pytest.raises(ValueError, match="max_seq_len"):
+        run_cut(eng, tokens_of(cfg, 30), [30])
+
+
+# --- scheduler ------------------------------------------------------------------
+
+def _assert_greedy(cfg, W, req, prompt, n):
+    ids = req.prompt_ids + req.output_ids
+    assert ids[:len(prompt)] == prompt and len(ids) == len(prompt) + n
+    ref = oracle.forward(cfg, W, ids).argmax(-1).tolist()
+    assert ref[len(prompt) - 1:-1] == ids[len(prompt):]
+
+
+def test_greedy_generation_long():
+    cfg, W = make("mixed")
+    eng = make_engine(cfg, W)
+    prompt = tokens_of(cfg, 30)
+    out = eng.generate(prompt, max_new_tokens=200)
+    ref = oracle.forward(cfg, W, prompt + out).argmax(-1).tolist()
+    assert ref[29:-1] == out
+
+
+@pytest.mark.parametrize("chunk,blocks,prefix", [
+    (2048, 128, True), (20, 128, False), (33, 40, True), (16, 24, False), (200, 13, False)])
+def test_scheduler_batches(chunk, blocks, prefix):
+    """Admission, prompt portions beside decoding, preemption on a small
+    pool and the prefix cache: the greedy continuation never changes."""
+    cfg, W = make("full")
+    eng = make_engine(cfg, W, kv_blocks=blocks, prefix_cache=prefix,
+                      max_batch=4)
+    eng.prefill_chunk = chunk
+    base = tokens_of(cfg, 100, seed=4)
+    prompts = [base[:n] for n in (1, 60, 100, 33, 100, 17)] + \
+        [tokens_of(cfg, 70, seed=9)]
+    reqs = [eng.submit(p, max_new_tokens=30) for p in prompts]
+    steps = 0
+    while eng.has_work():
+        eng.step()
+        steps += 1
+        assert steps < 2000
+    for r, p in zip(reqs, prompts):
+        _assert_greedy(cfg, W, r, p, 30)
+    if prefix:
+        assert eng.stats["prefix_hit_blocks"] > 0
+    if blocks == 13:
+        assert eng.stats["preemptions"] > 0
+    eng.flush_prefix_cache()
+    assert len(eng.allocator.free) == eng.allocator.num_blocks
+
+
+def test_scheduler_cancel_stop_and_sampling():
+    cfg, W = make("mixed")
+    eng = make_engine(cfg, W)
+    a = eng.submit(tokens_of(cfg, 20), max_new_tokens=50)
+    first = make_engine(cfg, W).generate(tokens_of(cfg, 40), 9)
+    b = eng.submit(tokens_of(cfg, 40), max_new_tokens=50,
+                   stop_token_ids=(first[4],))
+    c = eng.submit(tokens_of(cfg, 15), max_new_tokens=6, temperature=0.8,
+                   seed=3, logprobs=2)
+    for _ in range(4):
+        eng.step()
+    eng.cancel(a.request_id)
+    while eng.has_work():
+        eng.step()
+    assert a.finished and len(a.output_ids) < 10
+    assert b.output_ids == first[:first.index(first[4]) + 1]
+    assert len(c.output_ids) == 6 and len(c.logprob_data) == 6
+    again = make_engine(cfg, W)
+    d = again.submit(tokens_of(cfg, 15), max_new_tokens=6, temperature=0.8,
+                     seed=3)
+    while again.has_work():
+        again.step()
+    assert d.output_ids == c.output_ids
+
+
+def test_prompt_that_never_fits_is_refused():
+    cfg, W = make("full")
+    eng = make_engine(cfg, W, kv_blocks=5)
+    eng.submit(tokens_of(cfg, 90), max_new_tokens=2)
+    with pytest.raises(RuntimeError, match="cannot fit"):
+        for _ in range(20):
+            eng.step()
+    assert len(eng.allocator.free) == eng.allocator.num_blocks
+    assert not eng.has_work()
+
+
+def test_failed_step_releases_blocks():
+    cfg, W = make("mixed")
+    eng = make_engine(cfg, W)
+    eng.submit(tokens_of(cfg, 20))
+
+    def boom(*_):
+        raise RuntimeError("injected")
+    eng.forward_plan, keep = boom, eng.forward_plan
+    with pytest.raises(RuntimeError, match="injected"):
+        eng.step()
+    assert len(eng.allocator.free) == eng.allocator.num_blocks
+    eng.forward_plan = keep
+    assert len(eng.generate(tokens_of(cfg, 5), 3)) == 3
+
+
+# --- configuration, weights, command line -------------------------------------
+
+def test_checkpoint_directory_round_trip(tmp_path):
+    cfg, W = make("mixed")
+    d = write_checkpoint(tmp_path / "m", cfg, W)
+    mc = config_from_dir(d)
+    assert config_from_pimazen(config_to_pimazen(mc)).layers == mc.layers
+    assert mc.sliding_window == 64 and mc.norm_eps == 2e-5
+    assert config_from_pimazen(make("full")[0]).sliding_window is None
+    from runbooks_amd.models import build_model
+    m = build_model(mc, dtype=torch.float32)
+    load_pretrained(m, d)
+    ref = load(cfg, W, torch.float32)
+    for (k, a), (_, b) in zip(m.state_dict().items(),
+                              ref.state_dict().items()):
+        assert torch.equal(a, b), k
+    del W["l2.mix.uk"]
+    with pytest.raises(KeyError):
+        load_pretrained(build_model(mc, dtype=torch.float32),
+                        write_checkpoint(tmp_path / "bad", cfg, W))
+
+
+def test_configuration_errors():
+    cfg, _ = make("mixed")
+
+    def broken(f):
+        c = json.loads(json.dumps(cfg))
+        f(c)
+        return c
+    for f in (lambda c: c["layers"][0].update(type="other"),
+              lambda c: c["layers"][0]["mlp"].update(kind="sparse"),
+              lambda c: c["layers"][0]["mixer"].update(kv_from=2),
+              lambda c: c["layers"][3]["mixer"].update(kv_from=1),
+              lambda c: c["layers"][3]["mixer"].update(kv_rank=32),
+              lambda c: c["layers"][1]["mixer"]["rot"].update(base=501.0),
+              lambda c: c["layers"][0]["mixer"]["mask"].update(size=0)):
+        with pytest.raises(ValueError):
+            config_from_pimazen(broken(f))
+    with pytest.warns(UserWarning, match="without effect"):
+        config_from_pimazen(broken(lambda c: c.update(extra=1)))
+
+
+def test_registry_and_packing_keep_parameters():
+    mc = get_config("tiny-pimazen")
+    from runbooks_amd.models import build_model
+    m = build_model(mc, dtype=torch.float32)
+    before = {k: v.clone() for k, v in m.state_dict().items()}
+    for blk in m.blocks:
+        blk.fuse()
+    for k, v in m.state_dict().items():
+        assert torch.equal(v, before[k]), k
+    assert mc.params_b > 0
+    # a partially rotated key part
+    spec = LatentAttentionSpec(heads=2, dim=8, rot_dim=8, vdim=8, kv_rank=16,
+                               scale=0.25, rope_base=50.0, rope_dims=4,
+                               window=6)
+    pc = layered_config("p", [LayerSpec(spec, None)], 16, 20, max_seq_len=64)
+    from runbooks_amd.serve import Engine
+    eng = Engine(build_model(pc, dtype=torch.float32), device="cpu",
+                 kv_blocks=16)
+    cfg = config_to_pimazen(pc)
+    names = {"q_proj": "q", "dkv_proj": "dkv", "kv_norm": "dkv.norm",
+             "uk_proj": "uk", "uv_proj": "uv", "g_proj": "g", "o_proj": "o"}
+    W = {}
+    for k, v in eng.model.state_dict().items():
+        p = k.split(".")
+        if p[0] == "blocks":
+            W["l0.norm1" if p[2] == "norm1" else
+              f"l0.mix.{names[p[3]]}"] = v
+        else:
+            W[{"embed": "embed", "norm_f": "final.norm",
+               "lm_head": "head"}[p[0]]] = v
+    toks = tokens_of(cfg, 40)
+    assert rel_err(run_cut(eng, toks, [9]), oracle.forward(cfg, W, toks)) < TOL
+
+
+def test_synthetic_model_loads_and_serves(tmp_path):
+    from runbooks_amd.models import build_model
+    from runbooks_amd.serve import Engine
+    from runbooks_amd.workloads.model_loader import materialize_synthetic
+    materialize_synthetic("tiny-pimazen", tmp_path)
+    mc = config_from_dir(tmp_path)
+    m = load_pretrained(build_model(mc, dtype=torch.float32, seed=5),
+                        tmp_path)
+    out = Engine(m, device="cpu", kv_blocks=32).generate([1, 2, 3], 5)
+    assert len(out) == 5
+
+
+def test_http_server_serves_the_family():
+    from fastapi.testclient import TestClient
+    from runbooks_amd.serve import ByteTokenizer, Engine
+    from runbooks_amd.serve.http import build_app
+    eng = Engine("tiny-pimazen", device="cpu", dtype=torch.float32,
+                 kv_blocks=64)
+    with TestClient(build_app(eng, ByteTokenizer(),
+                              model_name="tiny-pimazen")) as client:
+        r = client.post("/v1/completions", json={
+            "prompt": "hello", "max_tokens": 4, "temperature": 0.0})
+        assert r.status_code == 200
+        assert r.json()["usage"]["completion_tokens"] == 4
+
+
+def test_fp8_cache_is_refused():
+    with pytest.raises(NotImplementedError, match="fp8"):
+        make_engine(*make("mixed"), kv_fp8=True)
+
+
+def test_replay_command(tmp_path, capsys, monkeypatch):
+    from runbooks_amd.serve.replay import main
+    cfg, W = make("mixed")
+    d = write_checkpoint(tmp_path / "m", cfg, W)
+    a, b = tokens_of(cfg, 60, 1), tokens_of(cfg, 9, 2)
+    steps = [
+        {"step": 0, "entries": [{"id": "a", "tokens": a[:40],
+                                 "want": [0, 39]}], "end": []},
+        {"step": 1, "entries": [{"id": "b", "tokens": b[:8], "want": []}],
+         "end": []},
+        {"step": 2, "entries": [{"id": "b", "tokens": b[8:], "want": [0]},
+                                {"id": "a", "tokens": a[40:], "want": [19]}],
+         "end": ["a", "b"]},
+        {"step": 3, "entries": [{"id": "a", "tokens": b, "want": [8]}],
+         "end": ["a"]}]
+    monkeypatch.setattr("sys.stdin", io.StringIO(
+        "".join(json.dumps(s) + "\n" for s in steps)))
+    out = tmp_path / "out"
+    out.mkdir()
+    assert main(["--model", str(d), "--dtype", "float32", "--out", str(out),
+                 "--max-tokens", "128", "--device", "cpu"]) == 0
+    assert [ln for ln in capsys.readouterr().out.splitlines()
+            if ln.startswith("done")] == [f"done {i}" for i in range(4)]
+    ra, rb = oracle.forward(cfg, W, a), oracle.forward(cfg, W, b)
+    want = {0: ra[[0, 39]], 2: torch.stack([rb[8], ra[59]]), 3: rb[8:]}
+    assert sorted(os.listdir(out)) == ["0.f32", "2.f32", "3.f32"]
+    for k, ref in want.items():
+        got = torch.from_numpy(np.fromfile(out / f"{k}.f32", dtype="<f4"))
+        assert rel_err(got.view(ref.shape), ref) < TOL
+
+
+def test_plan_flattens():
+    ps = _portions((3, 20, 16), (1, 0, 0))
+    ps[0].want = [0, 2]
+    back = StepPlan.unflatten(StepPlan(ps).flatten())
+    assert back.portions == ps
+
+
+def test_kv_blocks_follow_the_latent_cache():
+    m = load(*make("mixed"), torch.float32)
+    # two of the four layers own latents
+    per_token = (40 + 16) + (24 + 8)
+    assert m.kv_bytes_per_block() == per_token * 16 * 4
