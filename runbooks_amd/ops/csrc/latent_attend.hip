@@ -60,15 +60,20 @@ struct AttendArgs {
 };
 
 // 8 values down a column of row-major 16-bit LDS rows: lane i of each 16-lane
-// group gets column i of the 4 rows its group addresses, twice (rows +0..3
-// and +4..7). `p` is this lane's 8-byte piece of the first 4 rows.
-RB_DEV bf16x8v read_column8(const char *p, int stride4) {
+// group gets column i of the 4 rows its group addresses, twice: `lo` and `hi`
+// are this lane's 8-byte pieces of rows 0..3 and 4..7.
+RB_DEV bf16x8v read_column8(const char *lo, const char *hi) {
   typedef __attribute__((address_space(3))) s16x4v *lds4;
   union { s16x4v h[2]; bf16x8v v; } r;
-  r.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)p);
-  r.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)(p + stride4));
+  r.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)lo);
+  r.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)hi);
   return r.v;
 }
+
+// The key tile's rows are unpadded; 16-byte chunk c of key k lies at chunk
+// c ^ (k & 7), which spreads both the row-wise reads (16 keys, one chunk) and
+// the column-wise ones (8 keys, two chunks) over the banks.
+RB_DEV int tile_chunk(int key, int chunk) { return (chunk ^ (key & 7)) * 16; }
 
 // maximum over aligned groups of N lanes (N = 8, 16, 32)
 template <int N> RB_DEV float group_max(float v) {
@@ -89,7 +94,7 @@ template <int RP, int MT>
 __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   constexpr int M = MT * 16;
   constexpr int COLS = RP + ROTP;
-  constexpr int STRIDE = (COLS + 8) * 2;       // LDS row bytes
+  constexpr int STRIDE = COLS * 2;             // LDS row bytes
   constexpr int KH = MT == 1 ? 2 : 1;          // column halves in QK
   constexpr int QT = MT == 4 ? 2 : 1;          // row tiles per wave in QK
   constexpr int NS = COLS / 32 / KH;           // QK steps per wave
@@ -147,28 +152,33 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   // lanes beyond the row's last chunk repeat that chunk.
   const int lkey = tid >> 3, lchunk = tid & 7;
   const int last_chunk = a.ec / 8 - 1, split_chunk = a.rc / 8;
-  u32x4v reg[CPP];
-  int page = 0;
-  auto fetch_page = [&](int t) {
-    page = table[min(base + t * TK + lkey, key_hi - 1) / PAGE];
+  u32x4v reg[CPP], reg0[CPP];
+  auto page_of = [&](int t) {
+    return table[min(base + t * TK + lkey, key_hi - 1) / PAGE];
   };
-  auto fetch = [&](int t) {
+  auto fetch = [&](u32x4v *dst, int t, int page) {
     const int key = min(base + t * TK + lkey, key_hi - 1);
     const uint16_t *src = cache + ((int64_t)page * PAGE + key % PAGE) * a.ec;
 #pragma unroll
     for (int i = 0; i < CPP; ++i)
-      reg[i] = *reinterpret_cast<const u32x4v *>(
+      dst[i] = *reinterpret_cast<const u32x4v *>(
           src + min(lchunk + i * 8, last_chunk) * 8);
   };
-  auto stage = [&](char *dst) {
+  auto stage = [&](char *dst, const u32x4v *src) {
 #pragma unroll
     for (int i = 0; i < CPP; ++i) {
       const int c = min(lchunk + i * 8, last_chunk);
-      const int col = c * 8 + (c < split_chunk ? 0 : RP - a.rc);
-      *reinterpret_cast<u32x4v *>(dst + lkey * STRIDE + col * 2) = reg[i];
+      *reinterpret_cast<u32x4v *>(
+          dst + lkey * STRIDE +
+          tile_chunk(lkey, c < split_chunk ? c : c - split_chunk + RP / 8)) =
+          src[i];
     }
   };
-  fetch_page(t0);
+  // the first two tiles are on their way before anything else
+  int page = page_of(t0), page1 = page_of(t0 + 1);
+  fetch(reg0, t0, page);
+  if (t0 + 1 < t1) fetch(reg, t0 + 1, page1);
+  if (t0 + 2 < t1) page = page_of(t0 + 2);
 
   // ---- this wave's q fragments (zero beyond the real columns) -------------
   bf16x8v qf[QT][NS];
@@ -199,7 +209,8 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
     for (int c = tid; c < 2 * TK * (COLS / 8); c += BLOCK) {
       const int key = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
       if (col < RP ? col >= a.rc : col - RP >= a.rotc)
-        *reinterpret_cast<u32x4v *>(kv_s + key * STRIDE + col * 2) = zero4;
+        *reinterpret_cast<u32x4v *>(kv_s + key * STRIDE +
+                                    tile_chunk(key, col / 8)) = zero4;
     }
 
   // ---- softmax role of this thread --------------------------------------
@@ -226,19 +237,21 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
     f32x4v sc[QT][2];
 #pragma unroll
     for (int q = 0; q < QT; ++q) sc[q][0] = sc[q][1] = (f32x4v)(0.0f);
-    const char *krow = tile + (kg * 16 + l16) * STRIDE + grp * 16 +
-                       (KH == 2 ? part * NS * 64 : 0);
+    const char *krow = tile + (kg * 16 + l16) * STRIDE;
+    const int s_first = KH == 2 ? part * NS : 0;
+    auto fragment = [&](int s) {
+      return *reinterpret_cast<const bf16x8v *>(
+          krow + tile_chunk(l16, (s_first + s) * 4 + grp));
+    };
     bf16x8v kf[2][G];
 #pragma unroll
-    for (int s = 0; s < G; ++s)
-      kf[0][s] = *reinterpret_cast<const bf16x8v *>(krow + s * 64);
+    for (int s = 0; s < G; ++s) kf[0][s] = fragment(s);
 #pragma unroll
     for (int g = 0; g < NS / G; ++g) {
       if (g + 1 < NS / G) {
 #pragma unroll
         for (int s = 0; s < G; ++s)
-          kf[(g + 1) & 1][s] = *reinterpret_cast<const bf16x8v *>(
-              krow + ((g + 1) * G + s) * 64);
+          kf[(g + 1) & 1][s] = fragment((g + 1) * G + s);
       }
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
@@ -278,11 +291,14 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
       const char *vrow = tile + (ks * 32 + grp * 8 + (l16 >> 2)) * STRIDE +
-                         (wid * (CT * 16) + (l16 & 3) * 4) * 2;
+                         (l16 & 1) * 8;
+      const int vchunk = wid * (CT * 2) + ((l16 >> 1) & 1);
       bf16x8v vf[CT];
 #pragma unroll
       for (int c = 0; c < CT; ++c)
-        vf[c] = read_column8(vrow + c * 32, 4 * STRIDE);
+        vf[c] = read_column8(
+            vrow + tile_chunk(l16 >> 2, vchunk + c * 2),
+            vrow + 4 * STRIDE + tile_chunk((l16 >> 2) + 4, vchunk + c * 2));
 #pragma unroll
       for (int c = 0; c < CT; ++c)
 #pragma unroll
@@ -292,11 +308,7 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
     }
   };
 
-  fetch(t0);
-  if (t0 + 1 < t1) fetch_page(t0 + 1);
-  stage(kv_s);
-  if (t0 + 1 < t1) fetch(t0 + 1);
-  if (t0 + 2 < t1) fetch_page(t0 + 2);
+  stage(kv_s, reg0);
   __syncthreads();
   scores(kv_s);
 
@@ -342,9 +354,9 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
       if (spart == 0) alpha_s[srow] = alpha;
     }
     if (t + 1 < t1) {
-      stage(next);
-      if (t + 2 < t1) fetch(t + 2);
-      if (t + 3 < t1) fetch_page(t + 3);
+      stage(next, reg);
+      if (t + 2 < t1) fetch(reg, t + 2, page);
+      if (t + 3 < t1) page = page_of(t + 3);
     }
     __syncthreads();                   // P(t) and tile t+1 are there
     accumulate(tile);
@@ -518,7 +530,7 @@ template <int RP, int MT>
 void launch_attend(const AttendArgs &a, dim3 grid, hipStream_t stream) {
   constexpr int planes = MT == 1 ? 2 : 1;
   constexpr size_t shmem =
-      (size_t)2 * TK * ((RP + ROTP + 8) * 2) +
+      (size_t)2 * TK * ((RP + ROTP) * 2) +
       (size_t)MT * 16 * ((planes * SSTRIDE + 2) * sizeof(float) + PSTRIDE * 2);
   static_assert(shmem <= 160 * 1024, "LDS");
   static bool once = [] {
