@@ -221,3 +221,30 @@ template <> struct VIO<float> {
 };
 
 }  // namespace rb
+
+// ---------------------------------------------------------------------------
+// Transposed 16-bit LDS reads (gfx950 ds_read_b64_tr_b16).
+// ---------------------------------------------------------------------------
+namespace rb {
+
+// 8 values down a column of row-major 16-bit LDS rows: lane i of each 16-lane
+// group gets column i of the 4 rows its group addresses, twice. `lo` and `hi`
+// are this lane's 8-byte pieces (row i / 4, columns 4 (i % 4)..) of rows 0..3
+// and 4..7.
+RB_DEV __attribute__((ext_vector_type(8))) __bf16 lds_column8(const char *lo,
+                                                               const char *hi) {
+  typedef __attribute__((ext_vector_type(4))) short s16x4;
+  typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
+  typedef __attribute__((address_space(3))) s16x4 *lds4;
+  union { s16x4 h[2]; bf16x8v v; } r;
+  r.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)lo);
+  r.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)hi);
+  return r.v;
+}
+
+// two floats -> packed bf16 words (round to nearest even)
+RB_DEV uint32_t pack_bf16x2(float lo, float hi) {
+  return f32_to_bf16(lo) | ((uint32_t)f32_to_bf16(hi) << 16);
+}
+
+}  // namespace rb

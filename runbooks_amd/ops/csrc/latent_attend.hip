@@ -42,7 +42,6 @@ constexpr int PSTRIDE = 72;            // 16-bit weights per row
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
 typedef __attribute__((ext_vector_type(4))) float f32x4v;
-typedef __attribute__((ext_vector_type(4))) short s16x4v;
 typedef __attribute__((ext_vector_type(4))) unsigned int u32x4v;
 
 struct AttendArgs {
@@ -58,17 +57,6 @@ struct AttendArgs {
   float *part_o;                       // [nsplit, T*H, rc]
   float *part_ml;                      // [nsplit, T*H, 2]
 };
-
-// 8 values down a column of row-major 16-bit LDS rows: lane i of each 16-lane
-// group gets column i of the 4 rows its group addresses, twice: `lo` and `hi`
-// are this lane's 8-byte pieces of rows 0..3 and 4..7.
-RB_DEV bf16x8v read_column8(const char *lo, const char *hi) {
-  typedef __attribute__((address_space(3))) s16x4v *lds4;
-  union { s16x4v h[2]; bf16x8v v; } r;
-  r.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)lo);
-  r.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)hi);
-  return r.v;
-}
 
 // The key tile's rows are unpadded; 16-byte chunk c of key k lies at chunk
 // c ^ (k & 7), which spreads both the row-wise reads (16 keys, one chunk) and
@@ -174,44 +162,43 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
           src[i];
     }
   };
-  // the first two tiles are on their way before anything else
-  int page = page_of(t0), page1 = page_of(t0 + 1);
-  fetch(reg0, t0, page);
-  if (t0 + 1 < t1) fetch(reg, t0 + 1, page1);
-  if (t0 + 2 < t1) page = page_of(t0 + 2);
+  // the first two tiles and q are on their way before anything else
+  const int page0 = page_of(t0), page1 = page_of(t0 + 1);
+  int page = page_of(t0 + 2);
+  fetch(reg0, t0, page0);
 
-  // ---- this wave's q fragments (zero beyond the real columns) -------------
-  bf16x8v qf[QT][NS];
+  // q rows come once per workgroup, through the second key buffer
+  constexpr int QCHUNKS = M * (COLS / 8), QN = (QCHUNKS + BLOCK - 1) / BLOCK;
+  u32x4v qreg[QN];
 #pragma unroll
-  for (int qt = 0; qt < QT; ++qt) {
-    const int m = (KH == 2 ? 0 : part * QT + qt) * 16 + l16;
-    const bool ok = (KH == 2 || part * QT + qt < MT) && row0 + m < rows;
+  for (int i = 0; i < QN; ++i) {
+    const int c = min(tid + i * BLOCK, QCHUNKS - 1);
+    const int m = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
+    const bool ok = row0 + m < rows &&
+                    (col < RP ? col < a.rc : col - RP < a.rotc);
     const int row = ok ? row0 + m : 0;
     const int tok = q0 + row / a.heads, head = row % a.heads;
-    const uint16_t *ql = (const uint16_t *)a.q_lat +
-                         ((int64_t)tok * a.heads + head) * a.rc;
-    const uint16_t *qr = (const uint16_t *)a.q_rot + tok * a.q_row +
-                         head * a.q_head - RP;
-#pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      const int col = ((KH == 2 ? part * NS : 0) + s) * 32 + grp * 8;
-      const bool in = col < RP ? col < a.rc : col - RP < a.rotc;
-      union { u32x4v u; bf16x8v v; } c;
-      const u32x4v v = *reinterpret_cast<const u32x4v *>(
-          in ? (col < RP ? ql : qr) + col : ql);
-      c.u = (ok && in) ? v : zero4;
-      qf[qt][s] = c.v;
-    }
+    const uint16_t *src =
+        ok && col >= RP
+            ? (const uint16_t *)a.q_rot + tok * a.q_row + head * a.q_head +
+                  col - RP
+            : (const uint16_t *)a.q_lat +
+                  ((int64_t)tok * a.heads + head) * a.rc + (ok ? col : 0);
+    const u32x4v v = *reinterpret_cast<const u32x4v *>(src);
+    qreg[i] = ok ? v : zero4;
   }
+  if (t0 + 1 < t1) fetch(reg, t0 + 1, page1);
 
-  // padding columns of both key tiles
-  if (a.rc < RP || a.rotc < ROTP)
-    for (int c = tid; c < 2 * TK * (COLS / 8); c += BLOCK) {
+  // padding columns of the key tiles
+  auto clear_padding = [&](char *tile) {
+    if (a.rc == RP && a.rotc == ROTP) return;
+    for (int c = tid; c < TK * (COLS / 8); c += BLOCK) {
       const int key = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
       if (col < RP ? col >= a.rc : col - RP >= a.rotc)
-        *reinterpret_cast<u32x4v *>(kv_s + key * STRIDE +
+        *reinterpret_cast<u32x4v *>(tile + key * STRIDE +
                                     tile_chunk(key, col / 8)) = zero4;
     }
+  };
 
   // ---- softmax role of this thread --------------------------------------
   const int srow = tid / TPR, spart = tid % TPR;
@@ -225,6 +212,8 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   for (int c = 0; c < CT; ++c)
 #pragma unroll
     for (int m = 0; m < MT; ++m) acc[c][m] = (f32x4v)(0.0f);
+
+  bf16x8v qf[QT][NS];                  // this wave's q fragments
 
   // ---- scores of a staged tile: 16 keys x this wave's rows ---------------
   auto scores = [&](const char *tile) {
@@ -296,7 +285,7 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
       bf16x8v vf[CT];
 #pragma unroll
       for (int c = 0; c < CT; ++c)
-        vf[c] = read_column8(
+        vf[c] = rb::lds_column8(
             vrow + tile_chunk(l16 >> 2, vchunk + c * 2),
             vrow + 4 * STRIDE + tile_chunk((l16 >> 2) + 4, vchunk + c * 2));
 #pragma unroll
@@ -308,9 +297,31 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
     }
   };
 
+  clear_padding(kv_s);
   stage(kv_s, reg0);
+  char *q_s = kv_s + TK * STRIDE;
+#pragma unroll
+  for (int i = 0; i < QN; ++i) {
+    const int c = min(tid + i * BLOCK, QCHUNKS - 1);
+    const int m = c / (COLS / 8);
+    *reinterpret_cast<u32x4v *>(
+        q_s + m * STRIDE + tile_chunk(m, c % (COLS / 8))) = qreg[i];
+  }
   __syncthreads();
+#pragma unroll
+  for (int q = 0; q < QT; ++q) {
+    const int m = (KH == 2 ? 0 : (part * QT + q) * 16) + l16;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      qf[q][s] = *reinterpret_cast<const bf16x8v *>(
+          q_s + m * STRIDE +
+          tile_chunk(m, ((KH == 2 ? part * NS : 0) + s) * 4 + grp));
+  }
   scores(kv_s);
+  if (t0 + 1 < t1 && (a.rc < RP || a.rotc < ROTP)) {
+    __syncthreads();                   // q has been read by all waves
+    clear_padding(q_s);
+  }
 
   for (int t = t0; t < t1; ++t) {
     char *tile = kv_s + ((t - t0) & 1) * TK * STRIDE;
@@ -349,8 +360,7 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
           reinterpret_cast<uint32_t *>(p_s + srow * PSTRIDE + spart * KPT);
 #pragma unroll
       for (int j = 0; j < KPT; j += 2)
-        pr[j / 2] = rb::f32_to_bf16(p[j]) |
-                    ((uint32_t)rb::f32_to_bf16(p[j + 1]) << 16);
+        pr[j / 2] = rb::pack_bf16x2(p[j], p[j + 1]);
       if (spart == 0) alpha_s[srow] = alpha;
     }
     if (t + 1 < t1) {
@@ -393,10 +403,8 @@ __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
             col) = acc[c][m];
       } else {
         uint2 o;
-        o.x = rb::f32_to_bf16(acc[c][m][0] * inv) |
-              ((uint32_t)rb::f32_to_bf16(acc[c][m][1] * inv) << 16);
-        o.y = rb::f32_to_bf16(acc[c][m][2] * inv) |
-              ((uint32_t)rb::f32_to_bf16(acc[c][m][3] * inv) << 16);
+        o.x = rb::pack_bf16x2(acc[c][m][0] * inv, acc[c][m][1] * inv);
+        o.y = rb::pack_bf16x2(acc[c][m][2] * inv, acc[c][m][3] * inv);
         *reinterpret_cast<uint2 *>((uint16_t *)a.out + (grow0 + row) * a.rc +
                                    col) = o;
       }
@@ -443,8 +451,8 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
       for (int e = 0; e < 4; ++e) o[e] += ws * p[e];
     }
     uint2 w2;
-    w2.x = rb::f32_to_bf16(o[0]) | ((uint32_t)rb::f32_to_bf16(o[1]) << 16);
-    w2.y = rb::f32_to_bf16(o[2]) | ((uint32_t)rb::f32_to_bf16(o[3]) << 16);
+    w2.x = rb::pack_bf16x2(o[0], o[1]);
+    w2.y = rb::pack_bf16x2(o[2], o[3]);
     *reinterpret_cast<uint2 *>(out + row * rc + c) = w2;
   }
 }

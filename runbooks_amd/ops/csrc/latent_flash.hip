@@ -28,7 +28,6 @@ constexpr int KB = 64;                 // keys per tile
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
 typedef __attribute__((ext_vector_type(16))) float f32x16v;
-typedef __attribute__((ext_vector_type(4))) short s16x4v;
 typedef __attribute__((ext_vector_type(4))) unsigned int u32x4v;
 
 struct FlashArgs {
@@ -41,14 +40,6 @@ struct FlashArgs {
   int heads, dimc, rotc, vc, rc, ec, off_g, window;
   float scale_log2e;
 };
-
-RB_DEV bf16x8v read_column8(const char *p, int stride4) {
-  typedef __attribute__((address_space(3))) s16x4v *lds4;
-  union { s16x4v h[2]; bf16x8v v; } r;
-  r.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)p);
-  r.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds4)(p + stride4));
-  return r.v;
-}
 
 RB_DEV unsigned pack2(float lo, float hi) {
   union { __bf16 b[2]; unsigned u; } c;
@@ -222,7 +213,7 @@ __global__ __launch_bounds__(BLOCK, 2) void latent_flash_kernel(FlashArgs a) {
             (16 * (g & 1) + (i & 3) * 4) * 2;
 #pragma unroll
         for (int d = 0; d < DT; ++d) {
-          const bf16x8v vf = read_column8(vp + d * 64, 4 * VSTRIDE);
+          const bf16x8v vf = rb::lds_column8(vp + d * 64, vp + d * 64 + 4 * VSTRIDE);
           acc[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pf.v, acc[d],
                                                            0, 0, 0);
         }
@@ -252,8 +243,8 @@ __global__ __launch_bounds__(BLOCK, 2) void latent_flash_kernel(FlashArgs a) {
         o[e] = acc[d][rq * 4 + e] * inv / (1.0f + __expf(-g));
       }
       uint2 w;
-      w.x = rb::f32_to_bf16(o[0]) | ((uint32_t)rb::f32_to_bf16(o[1]) << 16);
-      w.y = rb::f32_to_bf16(o[2]) | ((uint32_t)rb::f32_to_bf16(o[3]) << 16);
+      w.x = rb::pack_bf16x2(o[0], o[1]);
+      w.y = rb::pack_bf16x2(o[2], o[3]);
       *reinterpret_cast<uint2 *>(zp + c) = w;
     }
 }

@@ -194,8 +194,8 @@ __global__ __launch_bounds__(BLOCK) void head_gemm_kernel(
             rb::bf16_to_f32((uint16_t)(gu[r >> 1] >> (16 * (r & 1)))));
     }
     uint2 o;
-    o.x = rb::f32_to_bf16(v[0]) | ((uint32_t)rb::f32_to_bf16(v[1]) << 16);
-    o.y = rb::f32_to_bf16(v[2]) | ((uint32_t)rb::f32_to_bf16(v[3]) << 16);
+    o.x = rb::pack_bf16x2(v[0], v[1]);
+    o.y = rb::pack_bf16x2(v[2], v[3]);
     *reinterpret_cast<uint2 *>(out + a.o_off + m * a.os + (int64_t)h * a.oh +
                                n) = o;
     if (swz != nullptr) {

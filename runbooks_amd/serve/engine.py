@@ -640,7 +640,7 @@ class Engine:
         if len(params) == 1 and plain:
             t, p = params.pop()
             toks = ops.sample_tokens(logits, t, top_p=p, seed=seed)
-            out = [int(x) for x in toks]
+            out = toks.tolist()          # one copy for the whole batch
         else:
             # heterogeneous sampling params / custom seeds: row-by-row
             out = []
