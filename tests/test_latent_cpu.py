@@ -234,8 +234,8 @@ def test_both_attention_forms(window):
                                            (None, True)])
 @pytest.mark.parametrize("query", [31, 32, 47, 70])
 def test_standout_key_at_the_window_edge(window, inside, query):
-    """The oldest visible key, given a score far above the rest, takes the
-    whole output; the next older one has no effect at all."""
+    """A key whose score stands out, just inside or just outside the window
+    (or at the very start without one): both forms follow the oracle."""
     ps = _portions((40, 40, 0), (60, 20, 0))
     s = 1
     key = 0 if window is None else query - window + (1 if inside else 0)
@@ -246,11 +246,9 @@ def test_standout_key_at_the_window_edge(window, inside, query):
                                                        query - 3))
     for name, got in out.items():
         assert (got.double() - ref).abs().max() < TOL
-    # the standout key decides the answer only when it is visible
-    alone = _attention_case(1, ps, peak=(s, query, query, query - 3))[1]
+    # where the standout key lies decides the answer
     differs = (out["latent"][t] - flat_out["latent"][t]).abs().max()
     assert differs > 1e-2
-    assert alone.shape == ref.shape
 
 
 # --- whole models -------------------------------------------------------------
@@ -393,10 +391,10 @@ def test_cache_is_shared_and_bounded_by_the_window():
     run_cut(eng, tokens_of(cfg, 400), [50, 1, 1], req=r)
     held = len(r.blocks) * 16
     assert r.dropped > 250 and held <= 64 + 50 + 32
-    full = make_engine(*make("full"))
+    cfg, W = make("full")
+    full = make_engine(cfg, W)
     r = full.open_request()
-    run_cut(full, tokens_of(cfg, 200)[:200] and tokens_of(make("full")[0],
-                                                         200), [64], req=r)
+    run_cut(full, tokens_of(cfg, 200), [64], req=r)
     assert r.dropped == 0
 
 
