@@ -82,6 +82,87 @@ class LightningSpec:
 
 
 @dataclass(frozen=True)
+class GatedDeltaSpec:
+    """Gated delta rule with one decay per head and key channel: q, k, v pass
+    a short causal convolution and silu, q and k become unit vectors;
+    S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; RMS norm per
+    head, sigmoid gate. Decay logits and gate come through a bottleneck."""
+    heads: int
+    kv_heads: int                   # q/k heads
+    dim: int
+    vdim: int
+    conv: int                       # taps of the convolution
+    decay_rank: int
+    gate_rank: int
+
+    rotation = None
+
+
+@dataclass(frozen=True)
+class AttentionSpec:
+    """Grouped-query attention with RMS norms of queries and keys, rotation
+    of the first rope_dims dimensions in neighbouring pairs, and a learned
+    sink in the softmax. A query sees the keys of its own chunk, counted
+    from the sequence's start."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float                    # factor on the scores
+    rope_dims: int
+    rope_base: float = 10000.0
+    chunk: int | None = None        # tokens per chunk (None: one chunk)
+
+    @property
+    def rotation(self):
+        return (self.rope_base, self.rope_dims)
+
+
+@dataclass(frozen=True)
+class MinGRUSpec:
+    """Gated recurrence S <- (1 - z) S + z c whose gates read only the
+    current token; the result is S silu(gate)."""
+    width: int
+
+
+@dataclass(frozen=True)
+class TwinSpec:
+    """Two mixers side by side on the same input; their results are added
+    with a factor each."""
+    left: AttentionSpec
+    right: MinGRUSpec
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+    @property
+    def rotation(self):
+        return self.left.rotation
+
+    @property
+    def chunk(self):
+        return self.left.chunk
+
+
+@dataclass(frozen=True)
+class SquaredReluSpec:
+    """Feed-forward down(relu(up)^2)."""
+    ff: int
+
+
+@dataclass(frozen=True)
+class MoESpec:
+    """`top` of `experts` squared-ReLU units per token, by softmax scores
+    plus a correction, out of the `keep` best of `groups` groups; weighted
+    by the scores. A shared unit of size shared_ff (0: none) is added."""
+    ff: int                         # of one expert
+    experts: int
+    top: int
+    groups: int = 1
+    keep: int = 1
+    shared_ff: int = 0
+
+
+@dataclass(frozen=True)
 class GLUSpec:
     """Gated unit act(gate) * up."""
     ff: int
@@ -93,13 +174,31 @@ class LayerSpec:
     """One layer of a model whose layers differ, on a 32-bit residual. With
     a latent mixer both sublayers read the same normed input and are summed;
     with the others they follow each other, each behind a norm of its own."""
-    mixer: LatentAttentionSpec | SharedKVAttentionSpec | LightningSpec
-    mlp: GatedMLPSpec | GLUSpec | None
+    mixer: (LatentAttentionSpec | SharedKVAttentionSpec | LightningSpec |
+            GatedDeltaSpec | TwinSpec)
+    mlp: GatedMLPSpec | GLUSpec | SquaredReluSpec | MoESpec | None
+    weights_of: int | None = None   # layer whose parameters this one uses
 
     @property
     def attends(self) -> bool:
-        """The mixer reads cached keys (else it carries a state)."""
-        return not isinstance(self.mixer, LightningSpec)
+        """The mixer reads cached keys."""
+        return not isinstance(self.mixer, (LightningSpec, GatedDeltaSpec))
+
+    @property
+    def reach(self) -> int | None:
+        """Most keys a query sees, itself included (None: all)."""
+        return getattr(self.mixer, "window", None) or \
+            getattr(self.mixer, "chunk", None)
+
+    def first_key(self, pos: int) -> int:
+        """First position that a query at `pos` or later can see."""
+        if not self.attends:
+            return pos
+        chunk = getattr(self.mixer, "chunk", None)
+        if chunk is not None:
+            return pos - pos % chunk
+        window = getattr(self.mixer, "window", None)
+        return 0 if window is None else max(0, pos - window + 1)
 
 
 @dataclass(frozen=True)
@@ -123,7 +222,7 @@ class ModelConfig:
     intermediate_size: int
     max_seq_len: int = 4096
     head_dim: int | None = None
-    norm: str = "rmsnorm"            # rmsnorm | layernorm
+    norm: str = "rmsnorm"            # rmsnorm | layernorm | dyt
     norm_eps: float = 1e-5
     act: str = "silu_glu"            # silu_glu | gelu | relu
     pos: str = "rope"                # rope | learned
@@ -143,6 +242,10 @@ class ModelConfig:
     # fields above describe)
     layers: tuple[LayerSpec, ...] | None = None
     loop: LoopSpec | None = None
+    # residual streams with learned mixing (None: one plain residual), and
+    # the factor on a sublayer's result that goes with them
+    streams: int | None = None
+    residual_mult: float = 1.0
 
     def __post_init__(self):
         if self.layers is not None:
@@ -156,18 +259,37 @@ class ModelConfig:
         """(layer, starts a loop pass) in the order of execution."""
         n, loop = len(self.layers), self.loop
         if loop is None:
-            return [(i, False) for i in range(n)]
+            return [(self.owner(i), False) for i in range(n)]
         body = range(loop.start, loop.stop)
         return ([(i, False) for i in range(loop.start)] +
                 [(i, i == loop.start) for _ in range(loop.times)
                  for i in body] +
                 [(i, False) for i in range(loop.stop, n)])
 
+    def owner(self, i: int) -> int:
+        """The layer whose parameters layer i uses."""
+        while self.layers[i].weights_of is not None:
+            i = self.layers[i].weights_of
+        return i
+
+    @property
+    def owners(self) -> list[int]:
+        """Layers with parameters of their own."""
+        return [i for i, lay in enumerate(self.layers)
+                if lay.weights_of is None]
+
+    def first_key(self, pos: int) -> int:
+        """First position that a query at `pos` or later can see in any
+        layer."""
+        return min(lay.first_key(pos) for lay in self.layers)
+
     @property
     def kernel_groups(self) -> tuple[str, ...]:
         """Kernel modules (ops/build.py) that serving this model needs."""
         if self.layers is None:
             return ("core", "main")
+        if self.streams is not None:
+            return ("core", "hybrid", "streams")
         latent = any(isinstance(lay.mixer, LatentAttentionSpec)
                      for lay in self.layers)
         return ("core", "latent" if latent else "hybrid")
@@ -175,17 +297,27 @@ class ModelConfig:
     def _check_layers(self):
         checks = {LatentAttentionSpec: self._check_latent,
                   SharedKVAttentionSpec: self._check_shared_kv,
-                  LightningSpec: self._check_lightning}
+                  LightningSpec: self._check_lightning,
+                  GatedDeltaSpec: self._check_delta,
+                  TwinSpec: self._check_twin}
         for i, lay in enumerate(self.layers):
             if getattr(lay.mixer, "window", None) is not None and \
                     lay.mixer.window < 1:
                 raise ValueError(f"layer {i}: window {lay.mixer.window}")
             checks[type(lay.mixer)](i, lay.mixer)
-            latent = isinstance(lay.mixer, LatentAttentionSpec)
+            kinds = ((SquaredReluSpec, MoESpec) if self.streams is not None
+                     else GatedMLPSpec
+                     if isinstance(lay.mixer, LatentAttentionSpec)
+                     else GLUSpec)
             if lay.mlp is not None and (
-                    lay.mlp.ff < 1 or
-                    latent != isinstance(lay.mlp, GatedMLPSpec)):
+                    lay.mlp.ff < 1 or not isinstance(lay.mlp, kinds)):
                 raise ValueError(f"layer {i}: mlp {lay.mlp}")
+            if isinstance(lay.mixer, (GatedDeltaSpec, TwinSpec)) != \
+                    (self.streams is not None):
+                raise ValueError(f"layer {i}: residual of {lay.mixer}")
+            if isinstance(lay.mlp, MoESpec):
+                self._check_moe(i, lay.mlp)
+            self._check_owner(i, lay)
             if getattr(lay.mlp, "act", "gelu_tanh") != "gelu_tanh":
                 raise ValueError(f"layer {i}: activation {lay.mlp.act}")
         if self.loop is not None:
@@ -196,6 +328,41 @@ class ModelConfig:
             if any(getattr(lay.mixer, "kv_from", None) is not None
                    for lay in self.layers):
                 raise ValueError("no loop over layers that share latents")
+
+        if self.streams is not None and (self.streams < 1 or self.loop or
+                                         self.norm != "dyt"):
+            raise ValueError(f"bad streams {self.streams}")
+
+    def _check_owner(self, i, lay):
+        """Layer i's weights_of leads to a layer like it that has some."""
+        seen, j = {i}, lay.weights_of
+        while j is not None:
+            if j in seen or not 0 <= j < len(self.layers) or self.loop or \
+                    (self.layers[j].mixer, self.layers[j].mlp) != \
+                    (lay.mixer, lay.mlp):
+                raise ValueError(f"layer {i} cannot use the weights of "
+                                 f"layer {lay.weights_of}")
+            seen.add(j)
+            j = self.layers[j].weights_of
+
+    def _check_delta(self, i, m):
+        if min(m.heads, m.kv_heads, m.dim, m.vdim, m.conv, m.decay_rank,
+               m.gate_rank) < 1 or m.heads % m.kv_heads:
+            raise ValueError(f"layer {i}: bad mixer sizes {m}")
+
+    def _check_twin(self, i, m):
+        a = m.left
+        if min(a.heads, a.kv_heads, a.dim, a.vdim, m.right.width) < 1 or \
+                a.heads % a.kv_heads or a.rope_dims % 2 or \
+                not 0 <= a.rope_dims <= a.dim or \
+                (a.chunk is not None and a.chunk < 1):
+            raise ValueError(f"layer {i}: bad mixer sizes {m}")
+
+    def _check_moe(self, i, m):
+        if m.experts < 1 or m.groups < 1 or m.experts % m.groups or \
+                not 1 <= m.keep <= m.groups or m.shared_ff < 0 or \
+                not 1 <= m.top <= m.experts // m.groups * m.keep:
+            raise ValueError(f"layer {i}: bad mixture {m}")
 
     def _check_latent(self, i, m):
         if min(m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank) < 1 or \
@@ -227,19 +394,33 @@ class ModelConfig:
         """Rough parameter count in billions."""
         if self.layers is not None:
             n = 2 * self.vocab_size * self.hidden_size
-            for lay in self.layers:
+            for lay in (self.layers[i] for i in self.owners):
                 m, h = lay.mixer, self.hidden_size
                 if isinstance(m, SharedKVAttentionSpec):
                     n += h * m.dim * (2 * m.heads + m.kv_heads)
                 elif isinstance(m, LightningSpec):
                     n += h * m.heads * (2 * m.dim + 3 * m.vdim)
+                elif isinstance(m, GatedDeltaSpec):
+                    n += h * (2 * m.kv_heads * m.dim + m.decay_rank +
+                              m.gate_rank + 2 * m.heads * m.vdim)
+                    n += m.heads * (m.decay_rank * m.dim +
+                                    m.gate_rank * m.vdim)
+                elif isinstance(m, TwinSpec):
+                    a = m.left
+                    n += h * (a.heads + a.kv_heads) * (a.dim + a.vdim) + \
+                        4 * h * m.right.width
                 else:
                     n += h * m.heads * (m.dim + m.rot_dim + 2 * m.vdim) + \
                         m.kv_rank * m.heads * (m.dim + m.vdim)
                     if m.kv_from is None:
                         n += h * (m.kv_rank + m.rot_dim)
-                if lay.mlp is not None:
+                if isinstance(lay.mlp, (MoESpec, SquaredReluSpec)):
+                    n += 2 * h * (lay.mlp.ff * getattr(lay.mlp, "experts", 1)
+                                  + getattr(lay.mlp, "shared_ff", 0))
+                elif lay.mlp is not None:
                     n += 3 * h * lay.mlp.ff
+                if self.streams is not None:
+                    n += h * h * (1 + (lay.mlp is not None))
             if self.loop is not None:
                 n += 2 * self.hidden_size ** 2
             return n / 1e9
@@ -255,7 +436,7 @@ class ModelConfig:
 def layered_config(name: str, layers, width: int, vocab: int,
                    norm_eps: float = 1e-5, max_seq_len: int = 131072,
                    norm: str = "rmsnorm",
-                   loop: LoopSpec | None = None) -> ModelConfig:
+                   loop: LoopSpec | None = None, **kw) -> ModelConfig:
     """A ModelConfig of a layer-by-layer model. The engine-wide fields
     follow from the layers: cached tokens may be dropped once they are
     outside every attention layer's window."""
@@ -264,20 +445,22 @@ def layered_config(name: str, layers, width: int, vocab: int,
     latent = isinstance(mixers[0], LatentAttentionSpec)
     if any(isinstance(m, LatentAttentionSpec) != latent for m in mixers):
         raise ValueError("latent layers do not mix with others")
-    windows = [lay.mixer.window for lay in layers if lay.attends]
+    # sizes of the attention (a twin mixer's left side)
+    heads = [getattr(m, "left", m) for m in mixers]
+    windows = [lay.reach for lay in layers if lay.attends]
     return ModelConfig(
         name, vocab_size=vocab, hidden_size=width, num_layers=len(layers),
-        num_heads=max(m.heads for m in mixers),
+        num_heads=max(m.heads for m in heads),
         num_kv_heads=1 if latent else max(getattr(m, "kv_heads", 1)
-                                          for m in mixers),
+                                          for m in heads),
         intermediate_size=max((lay.mlp.ff for lay in layers if lay.mlp),
                               default=0),
         max_seq_len=max_seq_len,
-        head_dim=mixers[0].dim + getattr(mixers[0], "rot_dim", 0),
+        head_dim=heads[0].dim + getattr(heads[0], "rot_dim", 0),
         norm=norm, norm_eps=norm_eps, parallel_residual=latent,
         single_norm=latent,
         sliding_window=None if None in windows else max(windows, default=1),
-        layers=layers, loop=loop)
+        layers=layers, loop=loop, **kw)
 
 
 _REGISTRY: dict[str, ModelConfig] = {}
@@ -489,3 +672,58 @@ _keralorn("keralorn-1b", "AL" * 8, 2048, 32000, 5632,
                rope_base=500000.0,
                rope_scaling=RopeScaling(8.0, 1.0, 4.0, 8192), window=2048),
           dict(heads=32, dim=64, vdim=64), max_seq_len=32768)
+
+
+# --- Gokapel family (gated delta rule, chunked attention beside a minGRU,
+# squared-ReLU units and mixtures of them; residual streams, dynamic tanh) ----
+def _gokapel(name: str, pattern: str, width: int, vocab: int, ff: int,
+             mixture: dict, delta: dict, attention: dict, gru: int, **kw):
+    """`pattern`: one letter a layer, D delta or P attention beside a minGRU
+    (lower case: the feed-forward is a mixture), or a digit: the weights of
+    that layer."""
+    made = {"d": GatedDeltaSpec(**delta),
+            "p": TwinSpec(AttentionSpec(**attention), MinGRUSpec(gru),
+                          0.6, 0.5)}
+    layers: list[LayerSpec] = []
+    for c in pattern:
+        if c.isdigit():
+            src = layers[int(c)]
+            layers.append(LayerSpec(src.mixer, src.mlp, int(c)))
+        else:
+            layers.append(LayerSpec(
+                made[c.lower()],
+                SquaredReluSpec(ff) if c.isupper() else MoESpec(**mixture)))
+    kw = {"streams": 4, "residual_mult": 0.7, "embed_scale": width ** 0.5,
+          "norm_eps": 1e-6, **kw}
+    return register(layered_config(name, layers, width, vocab, norm="dyt",
+                                   tie_embeddings=True, **kw))
+
+
+_gokapel("tiny-gokapel", "DpPd0", 64, 256, 96,
+         dict(ff=24, experts=8, top=2, groups=4, keep=2, shared_ff=40),
+         dict(heads=4, kv_heads=2, dim=16, vdim=24, conv=4, decay_rank=8,
+              gate_rank=12),
+         dict(heads=4, kv_heads=2, dim=24, vdim=16, scale=24 ** -0.5,
+              rope_dims=16, chunk=24), 40, max_seq_len=256)
+_gokapel("smoke-gokapel", "DpdP1", 256, 512, 512,
+         dict(ff=128, experts=8, top=2, groups=2, keep=1, shared_ff=128),
+         dict(heads=4, kv_heads=4, dim=64, vdim=64, conv=4, decay_rank=32,
+              gate_rank=32),
+         dict(heads=4, kv_heads=2, dim=64, vdim=64, scale=64 ** -0.5,
+              rope_dims=32, chunk=96), 256, max_seq_len=1024)
+# layers of the width and heads of llama2-7b and llama-1b; a dense layer has
+# llama's feed-forward parameters, and so has what a token uses of a mixture
+_gokapel("gokapel-7b", "DpPd" * 4, 4096, 32000, 16384,
+         dict(ff=2048, experts=32, top=6, groups=4, keep=2, shared_ff=4096),
+         dict(heads=32, kv_heads=32, dim=128, vdim=128, conv=4,
+              decay_rank=128, gate_rank=128),
+         dict(heads=32, kv_heads=32, dim=128, vdim=128, scale=128 ** -0.5,
+              rope_dims=64, rope_base=500000.0, chunk=4096), 4096,
+         max_seq_len=32768)
+_gokapel("gokapel-1b", "DpPd" * 4, 2048, 32000, 8192,
+         dict(ff=1024, experts=32, top=6, groups=4, keep=2, shared_ff=2048),
+         dict(heads=16, kv_heads=16, dim=128, vdim=128, conv=4,
+              decay_rank=128, gate_rank=128),
+         dict(heads=32, kv_heads=32, dim=64, vdim=64, scale=64 ** -0.5,
+              rope_dims=32, rope_base=500000.0, chunk=2048), 2048,
+         max_seq_len=32768)

@@ -21,6 +21,8 @@ from .transformer import Transformer
 
 def detect_family(cfg: ModelConfig) -> str:
     if cfg.layers is not None:
+        if cfg.streams is not None:
+            return "gokapel"
         latent = isinstance(cfg.layers[0].mixer, LatentAttentionSpec)
         return "pimazen" if latent else "keralorn"
     if cfg.pos == "learned":
@@ -129,6 +131,58 @@ def _map_keralorn(name: str):
     return name
 
 
+_GOKAPEL = {
+    **{f"mix.{n}": f"mixer.{n}_proj.weight" for n in
+       ("q", "k", "v", "b", "a1", "a2", "g1", "g2", "o")},
+    **{f"mix.{n}.conv": f"mixer.{n}_conv" for n in ("q", "k", "v")},
+    "mix.A_log": "mixer.a_log", "mix.dt_bias": "mixer.dt_bias",
+    "mix.norm": "mixer.norm.weight",
+    **{f"mix.left.{n}": f"mixer.left.{n}_proj.weight"
+       for n in ("q", "k", "v", "o")},
+    "mix.left.q.norm": "mixer.left.q_norm.weight",
+    "mix.left.k.norm": "mixer.left.k_norm.weight",
+    "mix.left.sink": "mixer.left.sink",
+    **{f"mix.right.{n}": f"mixer.right.{n}_proj.weight"
+       for n in ("z", "x", "g", "o")},
+    "mix.right.z.b": "mixer.right.z_proj.bias",
+    "mix.right.x.b": "mixer.right.x_proj.bias",
+    "mlp.up": "mlp.up_proj.weight", "mlp.down": "mlp.down_proj.weight",
+    "mlp.router": "mlp.router.weight", "mlp.correction": "mlp.correction",
+    "mlp.shared.up": "mlp.shared.up_proj.weight",
+    "mlp.shared.down": "mlp.shared.down_proj.weight",
+    **{f"{a}{n}": f"join{n}.{b}" for n in "12" for a, b in
+       (("ls", "scale"), ("rg", "gate.weight"))},
+    **{f"{a}{n}.{c}": f"join{n}.{b}" for n in "12" for a, c, b in
+       (("rg", "b", "gate.bias"), ("hc", "in", "inp"), ("hc", "out", "out"),
+        ("hc", "mix", "mix"))}}
+
+
+def _map_gokapel(name: str, cfg: ModelConfig):
+    """Experts keep their numbers; blocks count the layers that have
+    parameters."""
+    if name == "embed":
+        return "embed.weight"
+    base, kind = next(((name[:-len(end)], k) for end, k in
+                       ((".b", "bias"), (".alpha", "alpha"))
+                       if name.endswith(end)), (name, "weight"))
+    if base == "final.norm":
+        return f"norm_f.{kind}"
+    layer, _, rest = name.partition(".")
+    if layer[:1] != "l" or not layer[1:].isdigit() or \
+            int(layer[1:]) not in cfg.owners:
+        return name
+    block = f"blocks.{cfg.owners.index(int(layer[1:]))}."
+    if rest in _GOKAPEL:
+        return block + _GOKAPEL[rest]
+    if base.partition(".")[2] in ("norm1", "norm2"):
+        return f"{block}{base.partition('.')[2]}.{kind}"
+    part = rest.split(".")
+    if len(part) == 3 and part[0] == "mlp" and part[1][:1] == "e" and \
+            part[1][1:].isdigit() and part[2] in ("up", "down"):
+        return f"{block}mlp.experts.{part[1][1:]}.{part[2]}_proj.weight"
+    return name
+
+
 def _split_falcon_qkv(w: torch.Tensor, cfg: ModelConfig):
     """Falcon fuses QKV as [n_kv_groups, (g_q + 2), head_dim, hidden] with
     the group's q heads followed by its k and v head."""
@@ -147,7 +201,8 @@ def convert_hf_state_dict(hf_state: dict, cfg: ModelConfig) -> dict:
     mapper = {"llama": _map_llama, "opt": _map_opt,
               "falcon": _map_falcon, "gpt2": _map_gpt2,
               "pimazen": _map_pimazen,
-              "keralorn": _map_keralorn}[family]
+              "keralorn": _map_keralorn,
+              "gokapel": lambda n: _map_gokapel(n, cfg)}[family]
     for name, w in hf_state.items():
         if name.endswith(".rotary_emb.inv_freq"):
             continue
@@ -335,6 +390,133 @@ def config_to_keralorn(cfg: ModelConfig) -> dict:
     return out
 
 
+def tensor_shapes(path: str | Path) -> dict:
+    """Shapes of a checkpoint directory's tensors, from the headers."""
+    from safetensors import safe_open
+    shapes = {}
+    for f in sorted(Path(path).glob("*.safetensors")):
+        with safe_open(str(f), framework="pt") as st:
+            for name in st.keys():
+                shapes[name] = tuple(st.get_slice(name).get_shape())
+    return shapes
+
+
+def config_from_gokapel(d: dict, shapes: dict, name: str = "gokapel"
+                        ) -> ModelConfig:
+    """ModelConfig from a Gokapel config.json and the shapes of its tensors
+    (the inner sizes of the delta mixer's decay and gate projections stand
+    only there). A type or kind this framework does not have is an error; an
+    unknown key is reported."""
+    from .config import (AttentionSpec, GatedDeltaSpec, LayerSpec, MinGRUSpec,
+                         MoESpec, SquaredReluSpec, TwinSpec, layered_config)
+
+    def rows(i, tensor):
+        seen = set()
+        while d["layers"][i].get("weights_of") is not None and i not in seen:
+            seen.add(i)
+            i = d["layers"][i]["weights_of"]
+        full = f"l{i}.mix.{tensor}"
+        if full not in shapes:
+            raise ValueError(f"no tensor {full} to take a size from")
+        return shapes[full][0]
+
+    def delta(m, where, i):
+        _only(m, ("heads", "kv_heads", "dim", "vdim", "conv"), where)
+        return GatedDeltaSpec(m["heads"], m["kv_heads"], m["dim"], m["vdim"],
+                              m["conv"], rows(i, "a1"), rows(i, "g1"))
+
+    def parallel(m, where, i):
+        _only(m, ("left", "right", "left_scale", "right_scale"), where)
+        a = _only(m["left"], ("heads", "kv_heads", "dim", "vdim", "scale",
+                              "rot", "mask"), where + " left")
+        rot = _only(a["rot"], ("base", "dims"), where)
+        mask = _only(a.get("mask") or {}, ("size",), where)
+        right = _only(m["right"], ("width",), where + " right")
+        return TwinSpec(
+            AttentionSpec(a["heads"], a["kv_heads"], a["dim"], a["vdim"],
+                          float(a["scale"]), rot["dims"],
+                          float(rot["base"]), mask.get("size")),
+            MinGRUSpec(right["width"]), float(m["left_scale"]),
+            float(m["right_scale"]))
+
+    def feed_forward(m, where):
+        if m["kind"] == "dense":
+            return SquaredReluSpec(_only(m, ("kind", "ff"), where)["ff"])
+        if m["kind"] != "moe":
+            raise ValueError(f"{where}: mlp kind {m['kind']!r}")
+        _only(m, ("kind", "expert", "router", "shared"), where)
+        r = _only(m["router"], ("experts", "top", "groups"), where)
+        groups = _only(r.get("groups") or {"count": 1, "keep": 1},
+                       ("count", "keep"), where)
+        shared = _only(m.get("shared") or {}, ("ff",), where)
+        return MoESpec(_only(m["expert"], ("ff",), where)["ff"],
+                       r["experts"], r["top"], groups["count"],
+                       groups["keep"], shared.get("ff", 0))
+
+    mixers = {"channel_delta": delta, "parallel": parallel}
+    _only(d, ("architecture", "embedding", "layers", "norm", "residual_mult",
+              "streams", "vocab", "width", "max_seq_len"), "config")
+    layers = []
+    for i, lay in enumerate(d["layers"]):
+        where = f"layer {i}"
+        _only(lay, ("type", "mixer", "mlp", "weights_of"), where)
+        if lay["type"] not in mixers:
+            raise ValueError(f"{where}: type {lay['type']!r}")
+        mlp = lay.get("mlp")
+        layers.append(LayerSpec(
+            mixers[lay["type"]](lay["mixer"], where, i),
+            None if mlp is None else feed_forward(mlp, where),
+            lay.get("weights_of")))
+    kw = {"max_seq_len": d["max_seq_len"]} if "max_seq_len" in d else {}
+    return layered_config(
+        name, layers, d["width"], d["vocab"],
+        norm_eps=float(_only(d["norm"], ("eps",), "norm")["eps"]),
+        norm="dyt", tie_embeddings=True, streams=d["streams"],
+        residual_mult=float(d["residual_mult"]),
+        embed_scale=float(_only(d["embedding"], ("scale",),
+                                "embedding")["scale"]), **kw)
+
+
+def config_to_gokapel(cfg: ModelConfig) -> dict:
+    """The config.json of a Gokapel model (inverse of config_from_gokapel)."""
+    layers = []
+    for lay in cfg.layers:
+        m, f = lay.mixer, lay.mlp
+        if lay.attends:
+            a = m.left
+            left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim,
+                    "vdim": a.vdim, "scale": a.scale,
+                    "rot": {"base": a.rope_base, "dims": a.rope_dims}}
+            if a.chunk is not None:
+                left["mask"] = {"size": a.chunk}
+            mixer = {"left": left, "left_scale": m.left_scale,
+                     "right": {"width": m.right.width},
+                     "right_scale": m.right_scale}
+        else:
+            mixer = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim,
+                     "vdim": m.vdim, "conv": m.conv}
+        mlp = None
+        if f is not None and not hasattr(f, "experts"):
+            mlp = {"kind": "dense", "ff": f.ff}
+        elif f is not None:
+            mlp = {"kind": "moe", "expert": {"ff": f.ff},
+                   "router": {"experts": f.experts, "top": f.top,
+                              "groups": {"count": f.groups, "keep": f.keep}}}
+            if f.shared_ff:
+                mlp["shared"] = {"ff": f.shared_ff}
+        entry = {"type": "parallel" if lay.attends else "channel_delta",
+                 "mixer": mixer, "mlp": mlp}
+        if lay.weights_of is not None:
+            entry["weights_of"] = lay.weights_of
+        layers.append(entry)
+    return {"architecture": "Gokapel",
+            "embedding": {"scale": cfg.embed_scale}, "layers": layers,
+            "norm": {"eps": cfg.norm_eps},
+            "residual_mult": cfg.residual_mult, "streams": cfg.streams,
+            "vocab": cfg.vocab_size, "width": cfg.hidden_size,
+            "max_seq_len": cfg.max_seq_len}
+
+
 def config_from_pimazen(d: dict, name: str = "pimazen") -> ModelConfig:
     """ModelConfig from a Pimazen config.json. A layer type or kind this
     framework does not have is an error; an unknown key is reported."""
@@ -396,8 +578,9 @@ def config_to_pimazen(cfg: ModelConfig) -> dict:
 def config_from_dir(path: str | Path, default: str | None = None
                     ) -> ModelConfig:
     """The configuration of a checkpoint directory: a registered name or
-    explicit fields this framework wrote, a Pimazen or Keralorn config, or an
-    HF one; `default` names the registry entry of a directory that says nothing."""
+    explicit fields this framework wrote, a Pimazen, Keralorn or Gokapel
+    config, or an HF one; `default` names the registry entry of a directory
+    that says nothing."""
     from .config import get_config, list_configs, register
     marker = Path(path) / "config.json"
     meta = json.loads(marker.read_text()) if marker.exists() else {}
@@ -418,7 +601,9 @@ def config_from_hf_json(path: str | Path) -> ModelConfig:
     d = json.loads(Path(path).read_text())
     if "architecture" in d:
         readers = {"Pimazen": config_from_pimazen,
-                   "Keralorn": config_from_keralorn}
+                   "Keralorn": config_from_keralorn,
+                   "Gokapel": lambda d: config_from_gokapel(
+                       d, tensor_shapes(Path(path).parent))}
         if d["architecture"] not in readers:
             raise ValueError(f"unsupported architecture {d['architecture']}")
         return readers[d["architecture"]](d)

@@ -8,7 +8,7 @@ One implementation, three family knobs (ModelConfig):
   * parallel_residual: falcon's attn+mlp-in-parallel block
   * GQA/MQA via num_kv_heads (llama2-70b 8, falcon-40b 8, falcon-7b 1)
   * layers: models described layer by layer (models/latent.py,
-    models/hybrid.py)
+    models/hybrid.py, models/streams.py)
 
 Forward modes:
   * ``forward(tokens)``             — training, full causal attention
@@ -44,11 +44,14 @@ from .config import LatentAttentionSpec, ModelConfig
 from .hybrid import SequentialBlock
 from .latent import ParallelBlock
 from .ragged import RaggedBatch
+from .streams import StreamBlock
 
 
 def _norm_module(cfg: ModelConfig, dtype):
     if cfg.norm == "rmsnorm":
         return ops.RMSNorm(cfg.hidden_size, eps=cfg.norm_eps, dtype=dtype)
+    if cfg.norm == "dyt":
+        return ops.DynamicTanh(cfg.hidden_size, dtype=dtype)
     return nn.LayerNorm(cfg.hidden_size, eps=cfg.norm_eps, dtype=dtype)
 
 
@@ -288,12 +291,16 @@ class Transformer(nn.Module):
         # beside decoded tokens) through forward_ragged
         self.ragged = cfg.layers is not None
         if self.ragged:
+            latent = isinstance(cfg.layers[0].mixer, LatentAttentionSpec)
+            kind = (StreamBlock if cfg.streams is not None else
+                    ParallelBlock if latent else SequentialBlock)
             self.blocks = nn.ModuleList(
-                (ParallelBlock if isinstance(lay.mixer, LatentAttentionSpec)
-                 else SequentialBlock)(cfg, lay, dtype, self.tp)
-                for lay in cfg.layers)
-            # a looped layer runs, and has a cache, once per pass
+                kind(cfg, cfg.layers[i], dtype, self.tp) for i in cfg.owners)
+            # (layer, starts a loop pass), in the order of execution: a
+            # looped layer, or one whose weights another layer uses, runs,
+            # and has a cache, every time
             self.runs = cfg.layer_runs
+            self._block_of = {i: n for n, i in enumerate(cfg.owners)}
             if cfg.loop is not None:
                 self.loop_in = ops.Linear(2 * cfg.hidden_size,
                                           cfg.hidden_size, bias=False,
@@ -344,6 +351,10 @@ class Transformer(nn.Module):
         self.reset_parameters()
         if device is not None:
             self.to(device)
+
+    def block(self, layer: int):
+        """The block of a layer with parameters of its own."""
+        return self.blocks[self._block_of[layer]]
 
     def reset_parameters(self):
         for m in self.modules():
@@ -472,13 +483,18 @@ class Transformer(nn.Module):
         each layer's output is added by the norm that follows it."""
         x0 = self.embed(batch.tokens)
         x, delta, contexts = x0.to(torch.float32, copy=True), None, {}
+        if self.cfg.streams is not None:
+            x = (x * self.cfg.embed_scale)[:, None].repeat(
+                1, self.cfg.streams, 1)
         for (i, enters), cache in zip(self.runs, caches):
             if enters:
                 x, delta = self._enter_pass(x, delta, x0)
             r = self._rope_of[i]
             rope = None if r is None else (getattr(self, f"rope_cos_{r}"),
                                            getattr(self, f"rope_sin_{r}"))
-            delta = self.blocks[i].step(x, delta, batch, cache, rope, contexts)
+            delta = self.block(i).step(x, delta, batch, cache, rope, contexts)
+        if self.cfg.streams is not None:
+            return self._head_of_streams(x, delta, batch.rows)
         if batch.rows is not None:
             x = x.index_select(0, batch.rows)
             delta = delta.index_select(delta.dim() - 2, batch.rows)
@@ -488,6 +504,24 @@ class Transformer(nn.Module):
         logits = (ops.fast_linear(y, w).float() if ready
                   else ops.linear_f32(y, w))
         return gather_from_tp(logits) if self._lm_vocab_parallel else logits
+
+    def _head_of_streams(self, x, pending, rows):
+        """Logits of the streams' sum."""
+        if rows is not None:
+            x, pending = x.index_select(0, rows), pending.rows(rows)
+        w, D = self.lm_head.weight, self.cfg.hidden_size
+        ready = D % 32 == 0 and ops.decode_ready(w, x.shape[0])
+        y = ops.streams_norm(x, pending, self._all_streams, self._norm_f_v,
+                             self.dtype, operand=ready)
+        logits = (ops.fast_linear(y, w).float() if ready else
+                  ops.linear_f32(y[:, :D], w))
+        return gather_from_tp(logits) if self._lm_vocab_parallel else logits
+
+    def fuse_streams(self) -> None:
+        """What _head_of_streams reads, from the loaded parameters."""
+        self._norm_f_v = self.norm_f.packed()
+        self._all_streams = torch.ones(self.cfg.streams,
+                                       device=self._norm_f_v.device)
 
     def _enter_pass(self, x, delta, x0):
         """The residual a loop pass starts from: one product of the residual
@@ -507,7 +541,7 @@ class Transformer(nn.Module):
     def kv_bytes_per_block(self, fp8: bool = False) -> int:
         """Cache bytes of one block over all layers."""
         if self.ragged:
-            return max(1, sum(self.blocks[i].block_elements()
+            return max(1, sum(self.block(i).block_elements()
                               for i, _ in self.runs) *
                        self.embed.weight.element_size())
         elem = self.cfg.head_dim + 16 if fp8 else self.cfg.head_dim * 2
@@ -519,7 +553,7 @@ class Transformer(nn.Module):
         none)."""
         if not self.ragged:
             return 0
-        return sum(self.blocks[i].state_bytes() for i, _ in self.runs)
+        return sum(self.block(i).state_bytes() for i, _ in self.runs)
 
     def decode_nsplit(self, batch: int, caches) -> int | None:
         """Work split of the paged-decode kernel for a captured batch (None
@@ -538,11 +572,11 @@ class Transformer(nn.Module):
                 raise NotImplementedError(
                     f"{self.cfg.name}: no fp8 cache for layer-by-layer "
                     f"models")
-            for i, blk in enumerate(self.blocks):
+            for i, blk in zip(self.cfg.owners, self.blocks):
                 if torch.device(device).type == "cuda" and not blk.covered():
                     raise NotImplementedError(
                         f"{self.cfg.name}: no kernel for the sizes of layer "
-                        f"{i}: {blk.spec.mixer}")
+                        f"{i}: {blk.spec}")
         elif torch.device(device).type == "cuda" and \
                 self.cfg.head_dim not in (64, 128, 256):
             raise NotImplementedError(
@@ -558,8 +592,8 @@ class Transformer(nn.Module):
             for i, _ in self.runs:
                 src = getattr(self.cfg.layers[i].mixer, "kv_from", None)
                 caches.append(caches[src] if src is not None else
-                              self.blocks[i].alloc_cache(num_blocks, num_slots,
-                                                         device))
+                              self.block(i).alloc_cache(num_blocks, num_slots,
+                                                        device))
             return caches
         # Transposed-V blocks feed the MFMA decode kernel's direct V^T
         # fragment reads (GQA/MQA models, bf16, Dh<=128). The cache
@@ -632,6 +666,8 @@ def fuse_for_inference(model: "Transformer",
         weights = [w for blk in model.blocks for w in blk.fuse()]
         if model.cfg.loop is not None:
             weights.append(model.loop_in.weight)
+        if model.cfg.streams is not None:
+            model.fuse_streams()
     else:
         weights = _fuse_projections(model)
     if not load_in_8bit and torch.cuda.is_available() and ops.has_hip() and \

@@ -19,3 +19,5 @@ from .norm import (RMSNorm, join_res32, layernorm_res32, norm_res32,  # noqa: F4
 from .rope import rope, rope_frequencies, rope_ref, rope_tables  # noqa: F401
 from .sampling import sample_tokens  # noqa: F401
 from .shared_kv import alloc_shared_kv_cache  # noqa: F401
+from .streams import (DynamicTanh, Pending, pack_join, squared_relu,  # noqa: F401
+                      streams_norm)

@@ -10,13 +10,17 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
                       at::Tensor cu_q, at::Tensor seq_lens, int64_t n_seqs,
                       int64_t t_seqs, int64_t max_q, int64_t nsplit,
                       double scale, int64_t window, int64_t heads,
-                      int64_t rotc, at::Tensor z,
-                      c10::optional<at::Tensor> swz);
+                      int64_t hc, int64_t voff, at::Tensor z,
+                      c10::optional<at::Tensor> swz, int64_t chunk,
+                      c10::optional<at::Tensor> positions,
+                      c10::optional<at::Tensor> sink, double out_scale);
 void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
                      at::Tensor cu_q, at::Tensor seq_lens, int64_t first_seq,
                      int64_t n_seqs, int64_t max_q, double scale,
-                     int64_t window, int64_t heads, int64_t rotc,
-                     at::Tensor z);
+                     int64_t window, int64_t heads, int64_t hc, int64_t voff,
+                     at::Tensor z, int64_t chunk,
+                     c10::optional<at::Tensor> positions,
+                     c10::optional<at::Tensor> sink, double out_scale);
 int64_t lightning_chunk_size();
 void lightning_step(at::Tensor y, at::Tensor state, at::Tensor positions,
                     at::Tensor cu_q, at::Tensor slots, at::Tensor powers,

@@ -1,17 +1,18 @@
-// Attention in which a token's unrotated key doubles as its value: what the
-// kernels share.
+// Attention over paged rows that hold a token's key and value at once: what
+// the kernels share.
 //
-// One head of q, of k and of the result has `hc` columns: the rotated
-// dimensions (`rotc`, padded to 8) first, the others after them. A cached
-// row holds a token's key and value at once,
+// A row has `ec` columns. The key is its first `hc`, the value `vc` from
+// column `voff` on. Where a token's unrotated key doubles as its value, the
+// two overlap,
 //
 //   [ rotated | not rotated | rotated dimensions before rotation ]   (ec)
 //     \------- key (hc) -----/
-//               \------------------ value (hc) -----------------/
+//               \------------------ value (vc = hc) ------------/
 //
 // so the value's columns come in another order than the key's; the output
-// projection's weight has its columns in the value's order. The cache is
-// [blocks, kv heads, PAGE, ec]: a page of one head is contiguous.
+// projection's weight has its columns in the value's order. Otherwise the
+// value follows the key. The cache is [blocks, kv heads, PAGE, ec]: a page of
+// one head is contiguous.
 #pragma once
 
 #include "common.h"
@@ -31,14 +32,32 @@ struct Args {
   int64_t ny;
   const void *cache;
   const int *tables, *cu_q, *seq_lens;
-  int table_width, heads, kv, group, hc, rotc, ec, window, nsplit, total_rows;
+  int table_width, heads, kv, group, hc, vc, voff, ec, nsplit, total_rows;
+  int window;                          // keys a query sees (0: all)
+  int chunk;                           // or: keys of its own chunk (0: all)
+  const int *positions;                // [T], absolute; with chunks
+  const float *sink;                   // [heads], a further score, or null
   float scale;                         // MFMA kernels: times log2(e)
+  float out_scale;                     // factor on the result
   void *z;                             // [T, nz]; heads first
   int64_t nz;
   uint16_t *swz;                       // decode operand of z, or null
-  float *part_o;                       // [nsplit, T*H, hc]
+  float *part_o;                       // [nsplit, T*H, vc]
   float *part_ml;                      // [nsplit, T*H, 2]
 };
+
+// First key that a query at retained position `pos` sees, possibly below 0;
+// `dropped`: the absolute position of retained position 0.
+RB_DEV int first_key(const Args &a, int pos, int dropped) {
+  if (a.chunk > 0) {
+    const int p = pos + dropped;
+    return p - p % a.chunk - dropped;
+  }
+  return a.window > 0 ? pos - a.window + 1 : 0;
+}
+RB_DEV int dropped_of(const Args &a, int q0, int v0) {
+  return a.chunk > 0 ? a.positions[q0] - v0 : 0;
+}
 
 // LDS bytes between two cached rows: an odd number of 16-byte chunks
 RB_DEV __host__ constexpr int row_stride(int ec) {
@@ -88,7 +107,8 @@ RB_DEV void store4(const Args &a, int64_t t, int col, const float *v) {
                                (col & 7)) = w;
 }
 
-// Calls f with the padded head size and the chunks a lane copies per page.
+// Calls f with the padded head size (key's or value's, the larger) and the
+// chunks a lane copies per page.
 template <typename F> void pick_sizes(int hc, int ec, F f) {
   const int ni = (ec + 31) / 32;
   auto go = [&](auto hcp) {

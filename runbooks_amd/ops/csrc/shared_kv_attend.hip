@@ -1,5 +1,5 @@
-// Attention on shared keys and values over the paged cache: decoding and
-// short portions (gfx950). Layouts: shared_kv.h.
+// Attention over the paged rows of shared_kv.h: decoding and short portions
+// (gfx950).
 //
 // MFMA kernel (bf16): 16 query rows of one kv head per workgroup. Each of the
 // 4 waves walks tiles of 32 keys (two pages) of its own, through its own LDS,
@@ -60,7 +60,8 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
   const int tok_lo = row0 / a.group;
   const int tok_hi = (min(row0 + M, rows) - 1) / a.group;
   const int key_hi = v0 + tok_hi + 1;
-  const int key_lo = a.window > 0 ? max(0, v0 + tok_lo - a.window + 1) : 0;
+  const int dropped = dropped_of(a, q0, v0);
+  const int key_lo = max(0, first_key(a, v0 + tok_lo, dropped));
   const int page_lo = key_lo / PAGE, page_hi = (key_hi - 1) / PAGE;
   const int tiles = (page_hi - page_lo + 2) / 2;
   // short contexts use fewer splits: at least a tile per wave
@@ -109,7 +110,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
   const int row = row0 + l16;
   const bool row_ok = row < rows;
   const int qpos = row_ok ? v0 + row / a.group : -1;
-  const int kmin = a.window > 0 ? qpos - a.window + 1 : 0;
+  const int kmin = first_key(a, max(qpos, 0), dropped);
   bf16x8v qf[KS];
   {
     const int64_t gr = global_row(row_ok ? l16 : 0);
@@ -129,6 +130,11 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
 #pragma unroll
   for (int d = 0; d < DT; ++d) acc[d] = (f32x4v)(0.0f);
   float m_run = -INFINITY, l_run = 0.0f;
+  if (a.sink != nullptr && split == 0 && wid == 0 && row_ok) {
+    // counts once: l_run is summed over the lane groups
+    m_run = a.sink[g * a.group + row % a.group] * 1.4426950408889634f;
+    l_run = grp == 0 ? 1.0f : 0.0f;
+  }
 
   for (; t < t1; t += WAVES) {
     wave_fence();                              // the last tile has been read
@@ -176,7 +182,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
     l_run = l_run * alpha + sum;
     m_run = m_new;
     const char *vp = tile + (grp * 4 + (l16 >> 2)) * stride +
-                     (a.rotc + (l16 & 3) * 4) * 2;
+                     (a.voff + (l16 & 3) * 4) * 2;
 #pragma unroll
     for (int d = 0; d < DT; ++d) {
       const bf16x8v vf =
@@ -224,7 +230,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
     }
   }
   __syncthreads();
-  const int quads = a.hc / 4;
+  const int quads = a.vc / 4;
   for (int i = tid; i < M * quads; i += BLOCK) {
     const int m = i / quads, c = (i - m * quads) * 4;
     if (row0 + m >= rows) break;
@@ -235,11 +241,11 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
     const int64_t gr = global_row(m);
     if (a.nsplit > 1) {
       *reinterpret_cast<f32x4v *>(
-          a.part_o + ((int64_t)split * a.total_rows + gr) * a.hc + c) = o;
+          a.part_o + ((int64_t)split * a.total_rows + gr) * a.vc + c) = o;
     } else {
-      const float inv = 1.0f / out_s[m][1];
+      const float inv = a.out_scale / out_s[m][1];
       const float v[4] = {o[0] * inv, o[1] * inv, o[2] * inv, o[3] * inv};
-      store4(a, gr / a.heads, (int)(gr % a.heads) * a.hc + c, v);
+      store4(a, gr / a.heads, (int)(gr % a.heads) * a.vc + c, v);
     }
   }
 }
@@ -258,21 +264,21 @@ __global__ __launch_bounds__(64) void shared_kv_combine_kernel(Args a) {
   }
   const float mx = rb::wave_reduce_max(m);
   float w = l > 0.0f ? __builtin_amdgcn_exp2f(m - mx) : 0.0f;
-  w /= rb::wave_reduce_sum(l * w);
+  w *= a.out_scale / rb::wave_reduce_sum(l * w);
   __shared__ float w_s[64];
   w_s[lane] = w;
   __syncthreads();
-  for (int c = lane * 4; c < a.hc; c += 256) {
+  for (int c = lane * 4; c < a.vc; c += 256) {
     float o[4] = {0.0f, 0.0f, 0.0f, 0.0f};
     for (int s = 0; s < a.nsplit; ++s) {
       const float ws = w_s[s];
       if (ws == 0.0f) continue;                // its part was not written
       const f32x4v p = *reinterpret_cast<const f32x4v *>(
-          a.part_o + ((int64_t)s * a.total_rows + row) * a.hc + c);
+          a.part_o + ((int64_t)s * a.total_rows + row) * a.vc + c);
 #pragma unroll
       for (int e = 0; e < 4; ++e) o[e] += ws * p[e];
     }
-    store4(a, row / a.heads, (int)(row % a.heads) * a.hc + c, o);
+    store4(a, row / a.heads, (int)(row % a.heads) * a.vc + c, o);
   }
 }
 
@@ -282,7 +288,7 @@ __global__ __launch_bounds__(64) void shared_kv_combine_kernel(Args a) {
 template <typename T, int NE>
 __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  float *o_s = reinterpret_cast<float *>(smem);        // [4][hc]
+  float *o_s = reinterpret_cast<float *>(smem);        // [4][vc]
   __shared__ float ml_s[4][2];
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int seq = blockIdx.y;
@@ -291,7 +297,8 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
   const int tok = blockIdx.x / a.heads, head = blockIdx.x % a.heads;
   const int g = head / a.group;
   const int qpos = a.seq_lens[seq] - nq + tok;
-  const int lo = a.window > 0 ? max(0, qpos - a.window + 1) : 0;
+  const int v0 = a.seq_lens[seq] - nq;
+  const int lo = max(0, first_key(a, qpos, dropped_of(a, q0, v0)));
   const T *qp = (const T *)a.y + (q0 + tok) * a.ny + head * a.hc;
   const int *table = a.tables + (int64_t)seq * a.table_width;
 
@@ -303,6 +310,10 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
     o[i] = 0.0f;
   }
   float m = -INFINITY, l = 0.0f;
+  if (a.sink != nullptr && wid == 0) {
+    m = a.sink[head];
+    l = 1.0f;
+  }
   for (int key = lo + wid; key <= qpos; key += 4) {
     const T *c = (const T *)a.cache +
                  (((int64_t)table[key / PAGE] * a.kv + g) * PAGE + key % PAGE) *
@@ -321,8 +332,8 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
 #pragma unroll
     for (int i = 0; i < NE; ++i) {
       const int e = lane + i * 64;
-      if (e < a.hc)
-        o[i] = o[i] * al + p * rb::bf16_to_f32_or_id(c[a.rotc + e]);
+      if (e < a.vc)
+        o[i] = o[i] * al + p * rb::bf16_to_f32_or_id(c[a.voff + e]);
     }
   }
   if (lane == 0) {
@@ -331,7 +342,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
   }
 #pragma unroll
   for (int i = 0; i < NE; ++i)
-    if (lane + i * 64 < a.hc) o_s[wid * a.hc + lane + i * 64] = o[i];
+    if (lane + i * 64 < a.vc) o_s[wid * a.vc + lane + i * 64] = o[i];
   __syncthreads();
   float mx = -INFINITY, lt = 0.0f, w[4];
 #pragma unroll
@@ -341,12 +352,12 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
     w[k] = ml_s[k][1] > 0.0f ? expf(ml_s[k][0] - mx) : 0.0f;
     lt += w[k] * ml_s[k][1];
   }
-  for (int e = threadIdx.x; e < a.hc; e += BLOCK) {
+  for (int e = threadIdx.x; e < a.vc; e += BLOCK) {
     float v = 0.0f;
 #pragma unroll
-    for (int k = 0; k < 4; ++k) v += w[k] * o_s[k * a.hc + e];
-    v /= lt;
-    const int col = head * a.hc + e;
+    for (int k = 0; k < 4; ++k) v += w[k] * o_s[k * a.vc + e];
+    v *= a.out_scale / lt;
+    const int col = head * a.vc + e;
     rb::store_scalar((T *)a.z + (q0 + tok) * a.nz + col, v);
     if constexpr (sizeof(T) == 2) {
       if (a.swz != nullptr)
@@ -378,15 +389,34 @@ void launch_attend(const Args &a, dim3 grid, hipStream_t stream) {
 
 }  // namespace
 
+// The mask and the sink as both entry points take them.
+void check_mask(const at::Tensor &y, int64_t window, int64_t chunk,
+                const c10::optional<at::Tensor> &positions,
+                const c10::optional<at::Tensor> &sink, int64_t heads) {
+  TORCH_CHECK(window >= 0 && chunk >= 0 && (window == 0 || chunk == 0),
+              "shared_kv: window ", window, ", chunk ", chunk);
+  if (chunk > 0)
+    TORCH_CHECK(positions.has_value() && positions->is_cuda() &&
+                positions->scalar_type() == at::kInt &&
+                positions->is_contiguous() &&
+                positions->numel() == y.size(0), "shared_kv: positions");
+  if (sink.has_value())
+    TORCH_CHECK(sink->is_cuda() && sink->scalar_type() == at::kFloat &&
+                sink->is_contiguous() && sink->numel() == heads,
+                "shared_kv: sink [heads] f32");
+}
+
 // Attention of the first n_seqs sequences, whose t_seqs tokens are the first
 // ones of y; the heads' results go to z's first columns, and to the decode
 // operand `swz` when given.
 void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
                       at::Tensor cu_q, at::Tensor seq_lens, int64_t n_seqs,
                       int64_t t_seqs, int64_t max_q, int64_t nsplit,
-                      double scale,
-                      int64_t window, int64_t heads, int64_t rotc, at::Tensor z,
-                      c10::optional<at::Tensor> swz) {
+                      double scale, int64_t window, int64_t heads,
+                      int64_t hc, int64_t voff, at::Tensor z,
+                      c10::optional<at::Tensor> swz, int64_t chunk,
+                      c10::optional<at::Tensor> positions,
+                      c10::optional<at::Tensor> sink, double out_scale) {
   const auto dt = y.scalar_type();
   const bool bf16 = dt == at::kBFloat16;
   TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous() &&
@@ -397,11 +427,13 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
               cache.is_contiguous() && cache.scalar_type() == dt,
               "shared_kv_attend: cache [blocks, kv heads, 16, ec]");
   const int64_t T = y.size(0), G = cache.size(1), ec = cache.size(3);
-  const int64_t hc = ec - rotc;
-  TORCH_CHECK(heads % G == 0 && rotc >= 0 && hc >= 8 && hc % 8 == 0 &&
-              rotc % 8 == 0 && rotc <= hc && y.size(1) % 8 == 0 &&
+  const int64_t vc = ec - voff, wide = std::max(hc, vc);
+  TORCH_CHECK(heads % G == 0 && voff >= 0 && hc >= 8 && hc % 8 == 0 &&
+              voff % 8 == 0 && voff <= hc && hc <= ec && vc >= 8 &&
+              ec % 8 == 0 && y.size(1) % 8 == 0 &&
               z.size(1) % 8 == 0 && heads * hc <= y.size(1) &&
-              heads * hc <= z.size(1), "shared_kv_attend: layout");
+              heads * vc <= z.size(1), "shared_kv_attend: layout");
+  check_mask(y, window, chunk, positions, sink, heads);
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.is_contiguous() &&
               block_tables.scalar_type() == at::kInt &&
               cu_q.scalar_type() == at::kInt && cu_q.is_contiguous() &&
@@ -427,9 +459,14 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   a.kv = (int)G;
   a.group = (int)(heads / G);
   a.hc = (int)hc;
-  a.rotc = (int)rotc;
+  a.vc = (int)vc;
+  a.voff = (int)voff;
   a.ec = (int)ec;
   a.window = (int)window;
+  a.chunk = (int)chunk;
+  a.positions = chunk > 0 ? positions->data_ptr<int>() : nullptr;
+  a.sink = sink ? sink->data_ptr<float>() : nullptr;
+  a.out_scale = (float)out_scale;
   a.total_rows = (int)(t_seqs * heads);
   a.z = z.data_ptr();
   a.nz = z.size(1);
@@ -437,20 +474,20 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   a.nsplit = 1;
   auto stream = at::hip::getCurrentHIPStream();
 
-  if (!bf16 || hc > 256) {
-    TORCH_CHECK(hc <= 1024, "shared_kv_attend: heads of ", hc);
+  if (!bf16 || wide > 256) {
+    TORCH_CHECK(wide <= 1024, "shared_kv_attend: heads of ", wide);
     a.scale = (float)scale;
     const dim3 grid(max_q * heads, n_seqs);
-    const size_t shmem = 4 * hc * sizeof(float);
+    const size_t shmem = 4 * vc * sizeof(float);
     auto pick = [&](auto tag) {
       using E = decltype(tag);
       auto go = [&](auto n) {
         hipLaunchKernelGGL((shared_kv_rows_kernel<E, decltype(n)::value>),
                            grid, dim3(BLOCK), shmem, stream, a);
       };
-      if (hc <= 64) go(std::integral_constant<int, 1>{});
-      else if (hc <= 128) go(std::integral_constant<int, 2>{});
-      else if (hc <= 256) go(std::integral_constant<int, 4>{});
+      if (wide <= 64) go(std::integral_constant<int, 1>{});
+      else if (wide <= 128) go(std::integral_constant<int, 2>{});
+      else if (wide <= 256) go(std::integral_constant<int, 4>{});
       else go(std::integral_constant<int, 16>{});
     };
     if (bf16) pick(uint16_t{});
@@ -463,7 +500,7 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   at::Tensor po, pml;
   if (a.nsplit > 1) {
     const auto f32 = y.options().dtype(at::kFloat);
-    po = at::empty({a.nsplit, t_seqs * heads, hc}, f32);
+    po = at::empty({a.nsplit, t_seqs * heads, vc}, f32);
     pml = at::empty({a.nsplit, t_seqs * heads, 2}, f32);
     a.part_o = po.data_ptr<float>();
     a.part_ml = pml.data_ptr<float>();
@@ -471,7 +508,7 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   const int64_t tiles = (max_q * a.group + M - 1) / M;
   TORCH_CHECK(tiles * G <= 65535, "shared_kv_attend: portion of ", max_q);
   const dim3 grid(a.nsplit, tiles * G, n_seqs);
-  pick_sizes((int)hc, (int)ec, [&](auto h, auto n) {
+  pick_sizes((int)wide, (int)ec, [&](auto h, auto n) {
     launch_attend<decltype(h)::value, decltype(n)::value>(a, grid, stream);
   });
   if (a.nsplit > 1)

@@ -1,5 +1,4 @@
-// Attention on shared keys and values over the paged cache: long portions
-// (gfx950, bf16). Layouts: shared_kv.h.
+// Attention over the paged rows of shared_kv.h: long portions (gfx950, bf16).
 //
 // 128 query rows of one kv head per workgroup, 32 per wave; tiles of 64 keys
 // (four pages, one per wave to load) in LDS, the next one on its way in
@@ -54,17 +53,21 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
   const int tok = (q_ok ? qi : 0) / a.group;
   const int head = g * a.group + (q_ok ? qi : 0) % a.group;
   const int qpos = rel + tok;
-  const int win = a.window > 0 ? a.window : (1 << 30);
+  const int dropped = dropped_of(a, q_tok0, rel);
   const u32x4v zero4 = (u32x4v)(0u);
   const int stride = row_stride(a.ec);
 
   // key range of the workgroup, and of this wave's queries
   const int wg_hi = rel + (min(rows, q0 + QB) - 1) / a.group + 1;
-  const int wg_lo = max(0, rel + q0 / a.group - win + 1);
+  const int wg_lo = max(0, first_key(a, rel + q0 / a.group, dropped));
   const int wrow = q0 + wid * 32;
   const int first = rel + wrow / a.group;
   const int last =
       wrow < rows ? rel + (min(rows, wrow + 32) - 1) / a.group : -1;
+  // the first keys of the wave's first and last query, and of this lane's
+  const int lo_first = first_key(a, first, dropped);
+  const int lo_last = first_key(a, max(last, 0), dropped);
+  const int kmin = first_key(a, qpos, dropped);
   const int tile0 = wg_lo / KB, tile1 = (wg_hi + KB - 1) / KB;
   const int page_hi = (wg_hi - 1) / PAGE;
 
@@ -104,6 +107,10 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
 #pragma unroll
   for (int d = 0; d < DT; ++d) acc[d] = (f32x16v)(0.0f);
   float m_run = -INFINITY, l_run = 0.0f;
+  if (a.sink != nullptr) {
+    m_run = a.sink[head] * 1.4426950408889634f;
+    l_run = hi == 0 ? 1.0f : 0.0f;             // the halves are added up
+  }
 
   for (int t = tile0; t < tile1; ++t) {
     __syncthreads();
@@ -117,7 +124,7 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
 #pragma unroll
     for (int it = 0; it < 2; ++it) {
       const int k0 = t * KB + it * 32;
-      if (k0 > last || k0 + 31 < first - win + 1) continue;   // wave-uniform
+      if (k0 > last || k0 + 31 < lo_first) continue;          // wave-uniform
       f32x16v s = (f32x16v)(0.0f);
       const char *kp = smem + (it * 32 + col) * stride + hi * 16;
 #pragma unroll
@@ -128,12 +135,12 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
       float p[16];
 #pragma unroll
       for (int r = 0; r < 16; ++r) p[r] = s[r] * a.scale;
-      if (k0 + 31 > first || k0 < last - win + 1) {
+      if (k0 + 31 > first || k0 < lo_last) {
         // some key of this sub-tile is hidden from some query
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
-          const int d = qpos - (k0 + (r & 3) + 8 * (r >> 2) + 4 * hi);
-          if (d < 0 || d >= win) p[r] = -INFINITY;
+          const int key = k0 + (r & 3) + 8 * (r >> 2) + 4 * hi;
+          if (key > qpos || key < kmin) p[r] = -INFINITY;
         }
       }
       float mx = p[0];
@@ -169,7 +176,7 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
         const int i = lane & 15;
         const char *vp =
             smem + (it * 32 + ks * 16 + 4 * hi + (i >> 2)) * stride +
-            (a.rotc + 16 * ((lane >> 4) & 1) + (i & 3) * 4) * 2;
+            (a.voff + 16 * ((lane >> 4) & 1) + (i & 3) * 4) * 2;
 #pragma unroll
         for (int d = 0; d < DT; ++d) {
           const bf16x8v vf =
@@ -183,14 +190,14 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
 
   if (!q_ok) return;
   const float l = l_run + __shfl_xor(l_run, 32, 64);
-  const float inv = 1.0f / l;
-  uint16_t *zp = (uint16_t *)a.z + (q_tok0 + tok) * a.nz + head * a.hc;
+  const float inv = a.out_scale / l;
+  uint16_t *zp = (uint16_t *)a.z + (q_tok0 + tok) * a.nz + head * a.vc;
 #pragma unroll
   for (int d = 0; d < DT; ++d)
 #pragma unroll
     for (int rq = 0; rq < 4; ++rq) {
       const int c = d * 32 + 8 * rq + 4 * hi;
-      if (c >= a.hc) continue;
+      if (c >= a.vc) continue;
       uint2 w;
       w.x = rb::pack_bf16x2(acc[d][rq * 4] * inv, acc[d][rq * 4 + 1] * inv);
       w.y = rb::pack_bf16x2(acc[d][rq * 4 + 2] * inv,
@@ -218,12 +225,18 @@ void launch_flash(const Args &a, int first_seq, dim3 grid,
 
 }  // namespace
 
+void check_mask(const at::Tensor &y, int64_t window, int64_t chunk,
+                const c10::optional<at::Tensor> &positions,
+                const c10::optional<at::Tensor> &sink, int64_t heads);
+
 // Attention of the sequences first_seq .. first_seq + n_seqs - 1.
 void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
                      at::Tensor cu_q, at::Tensor seq_lens, int64_t first_seq,
                      int64_t n_seqs, int64_t max_q, double scale,
-                     int64_t window, int64_t heads, int64_t rotc,
-                     at::Tensor z) {
+                     int64_t window, int64_t heads, int64_t hc, int64_t voff,
+                     at::Tensor z, int64_t chunk,
+                     c10::optional<at::Tensor> positions,
+                     c10::optional<at::Tensor> sink, double out_scale) {
   TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous() &&
               y.scalar_type() == at::kBFloat16 && z.dim() == 2 &&
               z.is_contiguous() && z.size(0) == y.size(0) &&
@@ -231,12 +244,14 @@ void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   TORCH_CHECK(cache.dim() == 4 && cache.size(2) == PAGE &&
               cache.is_contiguous() && cache.scalar_type() == at::kBFloat16,
               "shared_kv_flash: cache [blocks, kv heads, 16, ec]");
-  const int64_t G = cache.size(1), ec = cache.size(3), hc = ec - rotc;
-  TORCH_CHECK(heads % G == 0 && rotc >= 0 && hc >= 8 && hc <= 256 &&
-              hc % 8 == 0 && rotc % 8 == 0 && rotc <= hc &&
+  const int64_t G = cache.size(1), ec = cache.size(3), vc = ec - voff;
+  TORCH_CHECK(heads % G == 0 && voff >= 0 && hc >= 8 && hc <= 256 &&
+              hc % 8 == 0 && voff % 8 == 0 && voff <= hc && hc <= ec &&
+              vc >= 8 && vc <= 256 && ec % 8 == 0 &&
               y.size(1) % 8 == 0 && z.size(1) % 8 == 0 &&
-              heads * hc <= y.size(1) && heads * hc <= z.size(1),
+              heads * hc <= y.size(1) && heads * vc <= z.size(1),
               "shared_kv_flash: layout");
+  check_mask(y, window, chunk, positions, sink, heads);
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.is_contiguous() &&
               block_tables.scalar_type() == at::kInt &&
               cu_q.scalar_type() == at::kInt && cu_q.is_contiguous() &&
@@ -259,9 +274,14 @@ void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   a.kv = (int)G;
   a.group = (int)(heads / G);
   a.hc = (int)hc;
-  a.rotc = (int)rotc;
+  a.vc = (int)vc;
+  a.voff = (int)voff;
   a.ec = (int)ec;
   a.window = (int)window;
+  a.chunk = (int)chunk;
+  a.positions = chunk > 0 ? positions->data_ptr<int>() : nullptr;
+  a.sink = sink ? sink->data_ptr<float>() : nullptr;
+  a.out_scale = (float)out_scale;
   a.scale = (float)(scale * 1.4426950408889634);
   a.z = z.data_ptr();
   a.nz = z.size(1);
@@ -269,7 +289,7 @@ void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   TORCH_CHECK(blocks <= 65535, "shared_kv_flash: portion of ", max_q);
   const dim3 grid(G, blocks, n_seqs);
   auto stream = at::hip::getCurrentHIPStream();
-  pick_sizes((int)hc, (int)ec, [&](auto h, auto n) {
+  pick_sizes((int)std::max(hc, vc), (int)ec, [&](auto h, auto n) {
     launch_flash<decltype(h)::value, decltype(n)::value>(a, (int)first_seq,
                                                          grid, stream);
   });

@@ -30,7 +30,7 @@ import torch
 
 from . import _backend
 from .kvcache import BLOCK_SIZE
-from .latent import _masked_softmax_ref, pad_to
+from .latent import pad_to
 
 
 MAX_HEAD = 1024                # padded head size the kernels run
@@ -60,6 +60,10 @@ class SharedKVLayout:
     @property
     def ec(self):              # one cached row
         return self.rotc + self.hc
+
+    @property
+    def voff(self):            # first column of the value in a row
+        return self.rotc
 
     @property
     def off_k(self):
@@ -139,7 +143,20 @@ def _prep_ref(y, lay, cos, sin, positions, slots, cache):
     q.copy_(rotate_halves_ref(q, cos, sin, positions))
 
 
-def _attend_ref(y, lay, cache, batch, seqs, scale, window, z):
+def visible_ref(qpos, kpos, window, chunk=None, dropped=0):
+    """[queries, keys]: the keys a query sees, of its window or its chunk
+    (absolute position = retained position + dropped)."""
+    seen = kpos[None] <= qpos[:, None]
+    if window is not None:
+        seen = seen & (kpos[None] > qpos[:, None] - window)
+    if chunk is not None:
+        seen = seen & ((kpos + dropped)[None] // chunk ==
+                       (qpos + dropped)[:, None] // chunk)
+    return seen
+
+
+def _attend_ref(y, lay, cache, batch, seqs, scale, window, z, chunk=None,
+                sink=None, out_scale=1.0):
     for b in seqs:
         t0, t1 = int(batch.cu_q[b]), int(batch.cu_q[b + 1])
         n = int(batch.seq_lens[b])
@@ -149,9 +166,18 @@ def _attend_ref(y, lay, cache, batch, seqs, scale, window, z):
         q = y[t0:t1, :lay.off_k].float().view(
             t1 - t0, lay.kv_heads, lay.group, lay.hc)
         s = torch.einsum("qgrd,kgd->grqk", q, rows[..., :lay.hc]) * scale
-        p = _masked_softmax_ref(s, pos[n - (t1 - t0):], pos, window)
-        o = torch.einsum("grqk,kgd->qgrd", p, rows[..., lay.rotc:])
-        z[t0:t1, :lay.off_k] = o.reshape(t1 - t0, -1).to(z.dtype)
+        dropped = int(batch.positions[t0]) - (n - (t1 - t0))
+        hidden = ~visible_ref(pos[n - (t1 - t0):], pos, window, chunk,
+                              dropped)
+        s = s.masked_fill(hidden, float("-inf"))
+        if sink is not None:      # one more entry of the denominator
+            extra = sink.view(lay.kv_heads, lay.group, 1, 1).expand(
+                *s.shape[:-1], 1)
+            s = torch.cat([s, extra], dim=-1)
+        p = torch.softmax(s, dim=-1)[..., :n]
+        o = torch.einsum("grqk,kgd->qgrd", p, rows[..., lay.voff:])
+        o = (o * out_scale).reshape(t1 - t0, -1)
+        z[t0:t1, :o.shape[1]] = o.to(z.dtype)
 
 
 # ---------------------------------------------------------------------------
@@ -180,33 +206,38 @@ def attend_split(n_seqs: int, workgroups: int, max_keys: int | None,
     return max(1, min(32, fill))
 
 
-def shared_kv_attend(y, lay, cache, batch, scale, window, z, swz=None):
+def shared_kv_attend(y, lay, cache, batch, scale, window, z, swz=None,
+                     chunk=None, sink=None, out_scale=1.0):
     """z's first t_short rows: attention of the batch's short portions. A
-    query at retained position i sees keys j with 0 <= i - j < window."""
+    query at retained position i sees keys j with 0 <= i - j < window, or
+    those up to its own of its chunk. `sink` [heads] fp32: one more entry of
+    the softmax's denominator. The result is multiplied by out_scale."""
     if not _backend.use_hip(y):
         return _attend_ref(y, lay, cache, batch, range(batch.n_short), scale,
-                           window, z)
+                           window, z, chunk, sink, out_scale)
     tiles = -(-batch.max_q * lay.group // 16) * lay.kv_heads
-    nsplit = attend_split(batch.n_short, tiles, batch.max_keys, window,
-                          batch.max_q)
+    nsplit = attend_split(batch.n_short, tiles, batch.max_keys,
+                          window or chunk, batch.max_q)
     _backend.ext().shared_kv_attend(
         y, cache, batch.block_tables, batch.cu_q, batch.seq_lens,
         batch.n_short, batch.t_short, batch.max_q, nsplit, scale, window or 0,
-        lay.heads, lay.rotc, z, swz)
+        lay.heads, lay.hc, lay.voff, z, swz, chunk or 0, batch.positions,
+        sink, out_scale)
 
 
 def shared_kv_flash_supported(lay: SharedKVLayout, dtype) -> bool:
-    return dtype == torch.bfloat16 and lay.hc <= 256
+    return dtype == torch.bfloat16 and max(lay.hc, lay.ec - lay.voff) <= 256
 
 
-def shared_kv_flash(y, lay, cache, batch, scale, window, z):
+def shared_kv_flash(y, lay, cache, batch, scale, window, z, chunk=None,
+                    sink=None, out_scale=1.0):
     """z's other rows: the same attention for the long portions."""
     n = batch.n_seqs - batch.n_short
     if not _backend.use_hip(y):
         return _attend_ref(y, lay, cache, batch,
                            range(batch.n_short, batch.n_seqs), scale, window,
-                           z)
+                           z, chunk, sink, out_scale)
     _backend.ext().shared_kv_flash(
         y, cache, batch.block_tables, batch.cu_q, batch.seq_lens,
         batch.n_short, n, batch.max_q_long, scale, window or 0, lay.heads,
-        lay.rotc, z)
+        lay.hc, lay.voff, z, chunk or 0, batch.positions, sink, out_scale)

@@ -427,8 +427,8 @@ class Engine:
     # -- ragged steps (layer-by-layer models) -----------------------------------
     def _release_front(self, r: Request, next_pos: int) -> None:
         """Give back the blocks no query at `next_pos` or later can see."""
-        w = self.cfg.sliding_window
-        while w and r.blocks and r.dropped + self.bs <= next_pos - w + 1:
+        first = self.cfg.first_key(next_pos)
+        while r.blocks and r.dropped + self.bs <= first:
             self.allocator.release([r.blocks.pop(0)])
             r.dropped += self.bs
             self.stats["window_dropped_blocks"] += 1
