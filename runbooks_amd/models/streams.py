@@ -111,7 +111,8 @@ class GatedDelta(nn.Module):
         if batch.n_seqs > batch.n_short:
             DR.delta_chunk(*args)
         z, swz = _new_z(self, y, self.out_w, filled=True)
-        DR.delta_out(o, lay, self.norm_w, y2, z, self.eps, swz)
+        DR.delta_out(o, lay, self.norm_w, y2, z, self.eps, swz, y, cache,
+                     batch)
         return z
 
     def alloc_cache(self, num_blocks, num_slots, device):
@@ -126,7 +127,7 @@ class GatedDelta(nn.Module):
             (lay.taps - 1) * lay.off_b * self.o_proj.weight.element_size()
 
     def covered(self) -> bool:
-        return self.lay.dc <= DR.MAX_DIM
+        return self.lay.dc <= DR.MAX_DIM and self.lay.vc <= DR.MAX_VALUE
 
 
 class ChunkedAttention(nn.Module):

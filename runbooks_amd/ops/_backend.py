@@ -13,10 +13,10 @@ import importlib
 
 import torch
 
-# The kernels are built as four modules (setup.py): ops shared by every
+# The kernels are built as five modules (setup.py): ops shared by every
 # served model, latent attention, attention on shared keys and values with
-# lightning attention, and the rest.
-_MODULES = ("_hip_core", "_hip_latent", "_hip_hybrid", "_hip")
+# lightning attention, layers around residual streams, and the rest.
+_MODULES = ("_hip_core", "_hip_latent", "_hip_hybrid", "_hip_streams", "_hip")
 _BUILD_HINT = ("Run `PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext "
                "--inplace` at the repo root.")
 

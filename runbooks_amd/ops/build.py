@@ -10,7 +10,8 @@ from pathlib import Path
 _OPS = Path(__file__).parent
 _ROOT = _OPS.parent.parent
 _MODULE = {"core": "_hip_core", "latent": "_hip_latent",
-           "hybrid": "_hip_hybrid", "main": "_hip"}
+           "hybrid": "_hip_hybrid", "streams": "_hip_streams",
+           "main": "_hip"}
 
 
 def _missing(groups) -> list[str]:

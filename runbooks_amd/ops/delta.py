@@ -12,8 +12,9 @@ with y2 a product of y's bottleneck columns. log g = -exp(a_log)
 softplus(logit + bias).
 
   * ``delta_step``   token after token: decoded tokens, short portions
-  * ``delta_chunk``  long portions in chunks of 16 tokens
-  * ``delta_out``    norm per head, weight, sigmoid gate -> z
+  * ``delta_chunk``  long portions in chunks of tokens
+  * ``delta_out``    norm per head, weight, sigmoid gate -> z; the
+                     convolution's last inputs -> the slots
 
 Sizes per head are padded to a multiple of 8 with zero rows of the packed
 weights. A sequence's slot holds S [heads, dim, vdim] and the convolution's
@@ -31,7 +32,8 @@ from . import _backend
 from .latent import _pad_rows, pad_to
 
 UNIT_EPS = 1e-6                # under the root of a unit vector's length
-MAX_DIM = 256                  # padded key size the kernels run
+MAX_DIM = 256                  # padded sizes per head the kernels run
+MAX_VALUE = 1024
 
 
 @dataclass(frozen=True)
@@ -178,8 +180,7 @@ def delta_step(y, y2, lay, conv_w, decay, state, batch, o):
                           range(batch.n_short))
     _backend.ext().delta_step(
         y, y2, conv_w, decay, *state, batch.positions, batch.cu_q,
-        batch.state_slots, o, batch.n_short, batch.t_short, batch.max_q,
-        lay.kv_heads, lay.dim)
+        batch.state_slots, o, batch.n_short, lay.kv_heads, lay.dim)
 
 
 def delta_chunk_supported(lay: DeltaLayout, dtype) -> bool:
@@ -198,9 +199,9 @@ def delta_chunk(y, y2, lay, conv_w, decay, state, batch, o):
         lay.kv_heads, lay.dim)
 
 
-def delta_out(o, lay, w, y2, z, eps, swz=None):
+def delta_out(o, lay, w, y2, z, eps, swz, y, state, batch):
     """z = rmsnorm per head(o) * w * sigmoid(gate), padding zero. w [vc]
-    fp32."""
+    fp32. After it the slots hold the convolution's last inputs."""
     if not _backend.use_hip(o):
         T = o.shape[0]
         r = o.view(T, lay.heads, lay.vc)
@@ -209,4 +210,6 @@ def delta_out(o, lay, w, y2, z, eps, swz=None):
         z[:, :lay.n_o] = ((r * w).view(T, -1) * g).to(z.dtype)
         z[:, lay.n_o:] = 0
         return
-    _backend.ext().delta_out(o, w, y2, lay.off_g, z, swz, lay.vdim, eps)
+    _backend.ext().delta_out(o, w, y2, lay.off_g, z, swz, lay.vdim, eps, y,
+                             state[1], batch.positions, batch.cu_q,
+                             batch.state_slots, batch.n_seqs)

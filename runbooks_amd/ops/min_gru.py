@@ -52,4 +52,4 @@ def min_gru(y, off: int, bias, state, batch, z, z_off: int, scale: float,
     if n_long:
         ext.min_gru_scan(y, off, bias, state, batch.positions, batch.cu_q,
                          batch.state_slots, batch.n_short, n_long, z, z_off,
-                         scale)
+                         scale, batch.max_q_long)

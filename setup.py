@@ -20,14 +20,17 @@ CSRC = ROOT / "runbooks_amd" / "ops" / "csrc"
 # One extension module per group, so that a caller can build just what a
 # model needs (RB_EXT_GROUPS=core,latent): `core` holds the ops every
 # served model runs, `latent` the latent-attention kernels, `hybrid` the
-# attention on shared keys and values and the lightning attention, `main`
-# the rest.
+# attention on shared keys and values and the lightning attention, `streams`
+# the layers around several residual streams, `main` the rest.
 CORE = ("rmsnorm", "layernorm", "glu", "decode_gemm", "sampling")
+STREAMS = ("streams", "qkv_prep", "delta", "min_gru", "moe")
 
 
 def _group_of(stem: str) -> str:
     if stem in CORE:
         return "core"
+    if stem in STREAMS:
+        return "streams"
     if stem.startswith(("shared_kv", "lightning")):
         return "hybrid"
     return "latent" if stem.startswith("latent_") else "main"
@@ -36,6 +39,7 @@ def _group_of(stem: str) -> str:
 MODULES = {"core": ("_hip_core", "bindings_core.cpp"),
            "latent": ("_hip_latent", "bindings_latent.cpp"),
            "hybrid": ("_hip_hybrid", "bindings_hybrid.cpp"),
+           "streams": ("_hip_streams", "bindings_streams.cpp"),
            "main": ("_hip", "bindings.cpp")}
 
 # *_hip.hip are build-time copies torch's extension builder leaves behind
