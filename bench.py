@@ -9,7 +9,9 @@ data, random-init weights. The reference publishes no numbers; this
 bench ESTABLISHES the baseline. --mode train / serve select a single
 metric; --mode latent (latent attention) and --mode hybrid (attention on
 shared keys and values, lightning attention) measure prefill and decode of
-those models beside llama models of equal layer sizes.
+those models beside llama models of equal layer sizes, --mode streams (gated
+delta rule, minGRU, mixtures on residual streams) beside hybrid models of as
+many layers.
 
 Launch (driver):
   python bench.py --gpus 1 --steps K --warmup W
@@ -196,7 +198,22 @@ def bench_serve(args) -> dict:
 PAIRS = {"latent": (("pimazen-7b", "llama2-7b"), ("pimazen-1b", "llama-1b"),
                     ("tiny-pimazen", "tiny-llama")),
          "hybrid": (("keralorn-7b", "llama2-7b"), ("keralorn-1b", "llama-1b"),
-                    ("tiny-keralorn", "tiny-llama"))}
+                    ("tiny-keralorn", "tiny-llama")),
+         "streams": (("gokapel-7b", "keralorn-7b"),
+                     ("gokapel-1b", "keralorn-1b"),
+                     ("tiny-gokapel", "tiny-keralorn"))}
+
+
+def _cut(name: str, layers: int):
+    """A registered model's first layers."""
+    import dataclasses
+
+    from runbooks_amd.models.config import get_config
+    cfg = get_config(name)
+    if cfg.layers is None or cfg.loop or cfg.num_layers <= layers:
+        return cfg
+    return dataclasses.replace(cfg, name=f"{name}-{layers}l",
+                               layers=cfg.layers[:layers], num_layers=layers)
 
 
 def bench_pairs(args) -> list[dict]:
@@ -205,6 +222,7 @@ def bench_pairs(args) -> list[dict]:
     pair; one result per model and workload."""
     import gc
 
+    from runbooks_amd.models.config import get_config
     from runbooks_amd.serve import Engine
 
     on_gpu = torch.cuda.is_available()
@@ -227,9 +245,15 @@ def bench_pairs(args) -> list[dict]:
                        "global_batch": 1 if what == "prefill" else batch,
                        "parallelism": "tp1"}})
 
-    for name in (m for pair in pairs for m in pair):
+    cfgs = []
+    for pair in pairs:
+        cfgs += [get_config(m) for m in pair]
+        if args.mode == "streams":     # as many layers as the first
+            cfgs[-1] = _cut(pair[1], cfgs[-2].num_layers)
+    for cfg in cfgs:
+        name = cfg.name
         need = batch * (max(contexts) + 256) + 4096
-        eng = Engine(name, dtype=dtype, kv_blocks=need // 16,
+        eng = Engine(cfg, dtype=dtype, kv_blocks=need // 16,
                      max_batch=batch, seed=17, prefix_cache=False)
         vocab = eng.cfg.vocab_size
 
@@ -276,7 +300,7 @@ def main():
     p.add_argument("--steps", type=int, default=20)
     p.add_argument("--warmup", type=int, default=5)
     p.add_argument("--mode", choices=["both", "train", "serve", "latent",
-                                      "hybrid"],
+                                      "hybrid", "streams"],
                    default="both")
     p.add_argument("--model", default=None)
     p.add_argument("--seq-len", type=int, default=512)

@@ -51,7 +51,7 @@ struct Args {
   const void *y, *y2;
   int64_t ny, ny2;
   int heads, kv, dim, dc, vc, taps, off_k, off_v, off_b;
-  const float *conv;                   // [off_b, taps]
+  const float *conv;                   // [taps, off_b]
   const float *decay;                  // [heads, dc + 1]
   float *state;                        // [slots, heads, dc, vc]
   void *tails;                         // [slots, taps - 1, off_b]
@@ -82,27 +82,38 @@ RB_DEV void conv(const Args &a, int q0, int t, bool fresh, int slot, int ch,
                  float *out) {
 #pragma unroll
   for (int k = 0; k < N; ++k) out[k] = 0.0f;
-  for (int j = 0; j < a.taps; ++j) {
-    const int s = t - (a.taps - 1) + j;
-    const T *p;
-    if (s >= 0) {
-      p = (const T *)a.y + (int64_t)(q0 + s) * a.ny + ch;
-    } else {
-      if (fresh) continue;
-      p = (const T *)a.tails +
-          ((int64_t)slot * (a.taps - 1) + a.taps - 1 + s) * a.off_b + ch;
-    }
-    float f[N];
+  auto load = [](const auto *p, float *f) {
+    using E = std::remove_cv_t<std::remove_reference_t<decltype(*p)>>;
     if constexpr (N == 8) {
-      rb::VIO<T>::load(p, f);
-      if constexpr (rb::VIO<T>::W == 4) rb::VIO<T>::load(p + 4, f + 4);
+      rb::VIO<E>::load(p, f);
+      if constexpr (rb::VIO<E>::W == 4) rb::VIO<E>::load(p + 4, f + 4);
     } else {
 #pragma unroll
       for (int k = 0; k < N; ++k) f[k] = rb::bf16_to_f32_or_id(p[k]);
     }
+  };
+  const T *now = (const T *)a.y + (int64_t)(q0 + t) * a.ny + ch;
+  for (int j0 = 0; j0 < a.taps; j0 += 4) {
+    float f[4][N], w[4][N];
+    // a tap that does not count reads the current token
 #pragma unroll
-    for (int k = 0; k < N; ++k)
-      out[k] += f[k] * a.conv[(int64_t)(ch + k) * a.taps + j];
+    for (int i = 0; i < 4; ++i) {
+      const int j = j0 + i, back = a.taps - 1 - j, s = t - back;
+      const T *p = now - (int64_t)back * a.ny;
+      if (s < 0)
+        p = (const T *)a.tails +
+            ((int64_t)slot * (a.taps - 1) + a.taps - 1 + s) * a.off_b + ch;
+      if (j >= a.taps || (s < 0 && fresh)) p = now;
+      load(p, f[i]);
+      load(a.conv + (int64_t)min(j, a.taps - 1) * a.off_b + ch, w[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int j = j0 + i;
+      const bool ok = j < a.taps && (t - (a.taps - 1) + j >= 0 || !fresh);
+#pragma unroll
+      for (int k = 0; k < N; ++k) out[k] += ok ? f[i][k] * w[i][k] : 0.0f;
+    }
   }
 #pragma unroll
   for (int k = 0; k < N; ++k) out[k] *= sigmoid<T>(out[k]);
@@ -236,14 +247,20 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
 // ---------------------------------------------------------------------------
 // chunks: operands
 // ---------------------------------------------------------------------------
+RB_DEV unsigned pack2(float lo, float hi) {
+  union { __bf16 b[2]; unsigned u; } c;
+  c.b[0] = (__bf16)lo;
+  c.b[1] = (__bf16)hi;
+  return c.u;
+}
 RB_DEV void split8(const float *f, u32x4v &big, u32x4v &small) {
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const float x = f[2 * i], y = f[2 * i + 1];
-    big[i] = rb::pack_bf16x2(x, y);
-    small[i] = rb::pack_bf16x2(
-        x - rb::bf16_to_f32((uint16_t)big[i]),
-        y - rb::bf16_to_f32((uint16_t)(big[i] >> 16)));
+    const unsigned b = pack2(x, y);
+    big[i] = b;
+    small[i] = pack2(x - __uint_as_float(b << 16),
+                     y - __uint_as_float(b & 0xffff0000u));
   }
 }
 
@@ -274,7 +291,8 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
   constexpr int RS = DCP + 4, AS = C + 4;      // floats per LDS row
   extern __shared__ __attribute__((aligned(16))) float lds[];
   float *q_s = lds, *k_s = q_s + C * RS, *g_s = k_s + C * RS;
-  float *a_s = g_s + C * RS, *p_s = a_s + C * AS, *b_s = p_s + C * AS;
+  float *a_s = g_s + C * RS;                   // A transposed
+  float *p_s = a_s + C * AS, *b_s = p_s + C * AS;
   float *v_s = b_s + C;
   const int VS = vb + 4;
 
@@ -427,11 +445,11 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     if ((off_diag || diag) && part == 0) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int t = ti * 4 + r;
-        const float b = b_s[t];
-        *reinterpret_cast<f32x4v *>(a_s + t * AS + tj * 4) =
-            (f32x4v){A[r][0] * b, A[r][1] * b, A[r][2] * b, A[r][3] * b};
-        *reinterpret_cast<f32x4v *>(p_s + t * AS + tj * 4) =
+        const float *b = b_s + ti * 4;
+        *reinterpret_cast<f32x4v *>(a_s + (tj * 4 + r) * AS + ti * 4) =
+            (f32x4v){A[0][r] * b[0], A[1][r] * b[1], A[2][r] * b[2],
+                     A[3][r] * b[3]};
+        *reinterpret_cast<f32x4v *>(p_s + (ti * 4 + r) * AS + tj * 4) =
             (f32x4v){P[r][0], P[r][1], P[r][2], P[r][3]};
       }
     }
@@ -479,16 +497,24 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
   __syncthreads();                             // q_s is free
   // ---- (I + A)^-1 of both right sides, a column per thread ----------------
   float x[C];
-  auto solve = [&]() {
+  auto solve = [&]() __attribute__((always_inline)) {
 #pragma unroll
-    for (int t = 1; t < C; ++t) {
-      float s = x[t];
+    for (int j = 0; j < C - 1; ++j) {
+      // A is read when it is needed: it does not fit the registers
+      if (j % 4 == 0) asm volatile("" ::: "memory");
 #pragma unroll
-      for (int j = 0; j < t; ++j) s -= a_s[t * AS + j] * x[j];
-      x[t] = s;
+      for (int i = 0; i < C / 4; ++i) {
+        if (i * 4 + 3 <= j) continue;
+        const f32x4v f = *reinterpret_cast<const f32x4v *>(a_s + j * AS +
+                                                           i * 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (i * 4 + e > j) x[i * 4 + e] -= f[e] * x[j];
+      }
     }
   };
-  auto solve_v = [&](int c, int c0) {          // staged column c
+  auto solve_v = [&](int c, int c0) __attribute__((always_inline)) {
+    // staged column c
 #pragma unroll
     for (int t = 0; t < C; ++t) x[t] = b_s[t] * v_s[t * VS + c];
     solve();
@@ -693,27 +719,30 @@ struct OutArgs {
   const void *y2, *y;
   void *z, *swz, *tails;
   const int *positions, *cu_q, *slots;
-  int taps, channels;
+  int taps, channels, tail_blocks;
 };
 
 // L lanes per head with NV times 8 columns each
 template <typename T, int L, int NV>
 __global__ __launch_bounds__(BLOCK) void delta_out_kernel(OutArgs a) {
   if (blockIdx.x >= a.tokens) {
-    const int seq = blockIdx.x - (int)a.tokens;
+    const int i = blockIdx.x - (int)a.tokens, seq = i / a.tail_blocks;
     const int q0 = a.cu_q[seq], n = a.cu_q[seq + 1] - q0;
     if (n <= 0) return;
     const bool fresh = a.positions[q0] == 0;
     const int keep = a.taps - 1;
     T *tail = (T *)a.tails + (int64_t)a.slots[seq] * keep * a.channels;
-    for (int c = threadIdx.x; c < a.channels; c += BLOCK)
-      for (int j = 0; j < keep; ++j) {
-        const int s = n - keep + j;            // token of the portion
-        T v = T(0);
-        if (s >= 0) v = ((const T *)a.y)[(int64_t)(q0 + s) * a.ny + c];
-        else if (!fresh) v = tail[(int64_t)(keep + s) * a.channels + c];
-        tail[(int64_t)j * a.channels + c] = v;
-      }
+    const int c = (i % a.tail_blocks * BLOCK + threadIdx.x) * 8;
+    if (c >= a.channels) return;
+    for (int j = 0; j < keep; ++j) {
+      const int s = n - keep + j;              // token of the portion
+      float v[8] = {};
+      if (s >= 0)
+        load8((const T *)a.y + (int64_t)(q0 + s) * a.ny + c, v);
+      else if (!fresh)
+        load8(tail + (int64_t)(keep + s) * a.channels + c, v);
+      store8(tail + (int64_t)j * a.channels + c, v);
+    }
     return;
   }
   constexpr int GROUPS = BLOCK / L;
@@ -782,7 +811,7 @@ Args check(const at::Tensor &y, const at::Tensor &y2, const at::Tensor &conv,
               tails.scalar_type() == dt && tails.size(0) == state.size(0) &&
               tails.size(2) == off_b && conv.dim() == 2 &&
               conv.is_contiguous() && conv.scalar_type() == at::kFloat &&
-              conv.size(0) == off_b && conv.size(1) == tails.size(1) + 1 &&
+              conv.size(1) == off_b && conv.size(0) == tails.size(1) + 1 &&
               decay.is_contiguous() && decay.scalar_type() == at::kFloat &&
               decay.numel() == H * (dc + 1) && y.size(1) % 8 == 0 &&
               off_b + H <= y.size(1) && y2.size(1) % 8 == 0 &&
@@ -807,7 +836,7 @@ Args check(const at::Tensor &y, const at::Tensor &y2, const at::Tensor &conv,
   a.dim = (int)dim;
   a.dc = (int)dc;
   a.vc = (int)vc;
-  a.taps = (int)conv.size(1);
+  a.taps = (int)conv.size(0);
   a.off_k = (int)(kv * dc);
   a.off_v = (int)(2 * kv * dc);
   a.off_b = (int)off_b;
@@ -927,7 +956,8 @@ void delta_out(at::Tensor o, at::Tensor w, at::Tensor y2, int64_t off_g,
               vc % 8 == 0 && vc >= 8 && vc <= 1024 && n % vc == 0 &&
               nz % 8 == 0 && nz >= n && off_g % 8 == 0 && off_g >= 0 &&
               y2.size(1) % 8 == 0 && off_g + n <= y2.size(1) && vdim >= 1 &&
-              vdim <= vc && tails.size(2) <= y.size(1), "delta_out: layout");
+              vdim <= vc && tails.size(2) <= y.size(1) && tails.size(2) % 8 == 0 &&
+              y.size(1) % 8 == 0, "delta_out: layout");
   TORCH_CHECK(positions.scalar_type() == at::kInt &&
               positions.is_contiguous() && positions.numel() == T &&
               cu_q.scalar_type() == at::kInt && cu_q.is_contiguous() &&
@@ -963,12 +993,13 @@ void delta_out(at::Tensor o, at::Tensor w, at::Tensor y2, int64_t off_g,
   a.slots = slots.data_ptr<int>();
   a.taps = (int)tails.size(1) + 1;
   a.channels = (int)tails.size(2);
+  a.tail_blocks = (a.channels + BLOCK * 8 - 1) / (BLOCK * 8);
   auto stream = at::hip::getCurrentHIPStream();
   auto launch = [&](auto tag, auto l, auto v) {
     using E = decltype(tag);
     hipLaunchKernelGGL(
         (delta_out_kernel<E, decltype(l)::value, decltype(v)::value>),
-        dim3(T + n_seqs), dim3(BLOCK), 0, stream, a);
+        dim3(T + n_seqs * a.tail_blocks), dim3(BLOCK), 0, stream, a);
   };
   constexpr std::integral_constant<int, 1> one{};
   auto pick = [&](auto tag) {

@@ -4,7 +4,7 @@
 //    the `keep` best groups; a wave per token.
 //  * moe_plan: (token, choice) pairs sorted by expert, in tiles of at most
 //    `tile` pairs of one expert; the list of tiles has a fixed length, its
-//    unused entries are empty.
+//    unused entries are empty, and the last one counts the used ones.
 //  * moe_gemm: one product per tile with its expert's weight. First product:
 //    relu^2, rows by pair number. Second: times the pair's weight, fp32, one
 //    part [T, N] per choice.
@@ -178,7 +178,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(
     e[2] = min(tile, mine - k * tile);
   }
   for (int k = used + i; k < n_tiles; k += 1024) {
-    tiles[k * 3] = 0;
+    tiles[k * 3] = k == n_tiles - 1 ? used : 0;
     tiles[k * 3 + 1] = 0;
     tiles[k * 3 + 2] = 0;
   }
@@ -315,11 +315,13 @@ constexpr int BUF = 2 * 128 * ROW;
 
 template <bool DOWN>
 __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
-                                                            int total) {
+                                                            int n_tiles) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   // neighbouring workgroups of one XCD share an expert
+  const int total = a.tiles[(n_tiles - 1) * 3] * nb;
   const int q8 = total / 8, r8 = total % 8;
   const int xcd = blockIdx.x % 8, pos = blockIdx.x / 8;
+  if (pos >= q8 + (xcd < r8)) return;
   const int wg = xcd * q8 + min(xcd, r8) + pos;
   const int *tile = a.tiles + wg / nb * 3;
   const int expert = tile[0], first = tile[1], count = tile[2];
@@ -342,22 +344,24 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
             ((int64_t)expert * a.N + min(n0 + row, a.N - 1)) * a.K + kc * 8;
     dst[i] = row * ROW + kc * 16;
   }
-  u32x4v xr[4], wr[4];
-  auto fetch = [&](int k0) {
+  struct Step { u32x4v x[4], w[4]; };          // a thread's part of a step
+  auto fetch = [&](Step &r, int k0) {
     const bool ok = k0 + kc * 8 < a.K;
+    const int k = ok ? k0 : 0;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      xr[i] = ok ? *reinterpret_cast<const u32x4v *>(xp[i] + k0)
-                 : (u32x4v)(0u);
-      wr[i] = ok ? *reinterpret_cast<const u32x4v *>(wp[i] + k0)
-                 : (u32x4v)(0u);
+      r.x[i] = *reinterpret_cast<const u32x4v *>(xp[i] + k);
+      r.w[i] = *reinterpret_cast<const u32x4v *>(wp[i] + k);
     }
   };
-  auto stage = [&](char *buf) {
+  auto stage = [&](const Step &r, int k0, char *buf) {
+    const bool ok = k0 + kc * 8 < a.K;
+    const u32x4v zero = (u32x4v)(0u);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      *reinterpret_cast<u32x4v *>(buf + dst[i]) = xr[i];
-      *reinterpret_cast<u32x4v *>(buf + 128 * ROW + dst[i]) = wr[i];
+      *reinterpret_cast<u32x4v *>(buf + dst[i]) = ok ? r.x[i] : zero;
+      *reinterpret_cast<u32x4v *>(buf + 128 * ROW + dst[i]) =
+          ok ? r.w[i] : zero;
     }
   };
   f32x4v acc[4][4];
@@ -365,15 +369,12 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = (f32x4v)(0.0f);
-  fetch(0);
-  stage(smem);
-  __syncthreads();
-  int cur = 0;
-  for (int k0 = 0; k0 < a.K; k0 += BK) {
-    const bool more = k0 + BK < a.K;
-    if (more) fetch(k0 + BK);
-    const char *xs = smem + cur * BUF, *ws = xs + 128 * ROW;
-#pragma unroll
+  // two steps ahead in registers, one in LDS
+  auto step = [&](int k0, char *buf, char *other, Step &free,
+                  const Step &next) __attribute__((always_inline)) {
+    fetch(free, k0 + 2 * BK);
+    const char *xs = buf, *ws = buf + 128 * ROW;
+#pragma unroll 1
     for (int ks = 0; ks < 2; ++ks) {
       bf16x8v xf[4], wf[4];
 #pragma unroll
@@ -391,9 +392,18 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
           acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
               wf[i], xf[j], acc[i][j], 0, 0, 0);
     }
-    if (more) stage(smem + (cur ^ 1) * BUF);
+    stage(next, k0 + BK, other);
     __syncthreads();
-    cur ^= 1;
+  };
+  Step r0, r1;
+  fetch(r0, 0);
+  fetch(r1, BK);
+  stage(r0, 0, smem);
+  __syncthreads();
+  for (int k0 = 0; k0 < a.K; k0 += 2 * BK) {
+    step(k0, smem, smem + BUF, r0, r1);
+    if (k0 + BK >= a.K) break;
+    step(k0 + BK, smem + BUF, smem, r1, r0);
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
@@ -417,9 +427,10 @@ template <bool DOWN> void launch_tile(const Args &a, int n_tiles,
                2 * BUF) == hipSuccess;
   }();
   TORCH_CHECK(once, "moe_gemm: LDS size");
-  const int nb = (a.N + 127) / 128, total = nb * n_tiles;
+  const int nb = (a.N + 127) / 128;
+  const int total = (nb * n_tiles + 7) / 8 * 8;
   hipLaunchKernelGGL((moe_tile_kernel<DOWN>), dim3(total), dim3(BLOCK),
-                     2 * BUF, stream, a, nb, total);
+                     2 * BUF, stream, a, nb, n_tiles);
 }
 
 }  // namespace
@@ -464,7 +475,7 @@ std::vector<at::Tensor> moe_plan(at::Tensor chosen, int64_t experts,
               experts <= MAX_EXPERTS && tile >= 1, "moe_plan: chosen i32");
   const int64_t n = chosen.numel();
   TORCH_CHECK(n < (1 << 30), "moe_plan: pairs");
-  const int64_t n_tiles = (n + tile - 1) / tile + std::min(n, experts);
+  const int64_t n_tiles = (n + tile - 1) / tile + std::min(n, experts) + 1;
   auto pairs = at::empty({n}, chosen.options());
   auto tiles = at::empty({n_tiles, 3}, chosen.options());
   if (n == 0) return {pairs, tiles};
@@ -512,7 +523,7 @@ at::Tensor moe_gemm(at::Tensor x, at::Tensor w, at::Tensor pairs,
     else launch_tile<false>(a, (int)n_tiles, stream);
     return out;
   }
-  const dim3 grid((N + 31) / 32, n_tiles);
+  const dim3 grid((N + 31) / 32, n_tiles - 1);
   auto launch = [&](auto tag, auto d) {
     hipLaunchKernelGGL((moe_rows_kernel<decltype(tag), decltype(d)::value>),
                        grid, dim3(BLOCK), 0, stream, a);

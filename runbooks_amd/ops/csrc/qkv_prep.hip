@@ -54,20 +54,30 @@ __global__ __launch_bounds__(BLOCK) void qkv_prep_kernel(
       ss[n][k] = p < a.half ? sr[p] : 0.0f;
     }
   const int n_heads = a.heads + a.kv;
+  float ahead[NV][8];
+  auto fetch = [&](int h) {
+#pragma unroll
+    for (int n = 0; n < NV; ++n) {
+      const int c = (n * L + lane) * 8;
+      // padding is zero; beyond it any address of the row
+      load8(yr + (int64_t)min(h, n_heads - 1) * a.hc + (c < a.hc ? c : 0),
+            ahead[n]);
+    }
+  };
+  fetch(threadIdx.x / L);
   for (int h0 = 0; h0 < n_heads; h0 += GROUPS) {
     const int h = h0 + threadIdx.x / L;
     const bool ok = h < n_heads, is_k = h >= a.heads;
     T *src = yr + (int64_t)h * a.hc;
     float v[NV][8], sum = 0.0f;
 #pragma unroll
-    for (int n = 0; n < NV; ++n) {
-      const int c = (n * L + lane) * 8;
-      if (ok && c < a.hc) {
-        load8(src + c, v[n]);                  // padding is zero
+    for (int n = 0; n < NV; ++n)
 #pragma unroll
-        for (int k = 0; k < 8; ++k) sum += v[n][k] * v[n][k];
+      for (int k = 0; k < 8; ++k) {
+        v[n][k] = (n * L + lane) * 8 < a.hc ? ahead[n][k] : 0.0f;
+        sum += v[n][k] * v[n][k];
       }
-    }
+    if (h0 + GROUPS < n_heads) fetch(h + GROUPS);
 #pragma unroll
     for (int o = L / 2; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
     const float inv = 1.0f / sqrtf(sum / a.dim + a.eps);

@@ -117,11 +117,12 @@ def pack_second(lay: DeltaLayout, a2, g2):
 
 
 def pack_conv(lay: DeltaLayout, q, k, v):
-    """[channels, taps] fp32 in y's order."""
+    """[taps, channels] fp32, channels in y's order."""
     return torch.cat([
         _pad_rows(q, lay.kv_heads, (lay.dim,), (lay.dc,)),
         _pad_rows(k, lay.kv_heads, (lay.dim,), (lay.dc,)),
-        _pad_rows(v, lay.heads, (lay.vdim,), (lay.vc,))]).float().contiguous()
+        _pad_rows(v, lay.heads, (lay.vdim,), (lay.vc,))]
+    ).float().t().contiguous()
 
 
 def pack_decay(lay: DeltaLayout, a_log, dt_bias):
@@ -148,7 +149,7 @@ def _recur_ref(y, y2, lay, conv_w, decay, state, batch, o, seqs):
         keep = float(int(batch.positions[t0]) != 0)
         S = S_all[slot] * keep
         raw = torch.cat([tails[slot].float() * keep, y[t0:t1, :n].float()])
-        x = sum(raw[j:j + T] * conv_w[:, j] for j in range(lay.taps))
+        x = sum(raw[j:j + T] * conv_w[j] for j in range(lay.taps))
         x = torch.nn.functional.silu(x)
 
         def unit(a):

@@ -40,6 +40,7 @@ import torch
 
 from .. import ops
 from ..models import Transformer, build_model
+from ..models.config import ModelConfig
 from ..models.ragged import Portion, StepPlan
 from ..parallel import comm
 from ..utils.trace import get_tracer
@@ -108,14 +109,14 @@ class Request:
 
 
 class Engine:
-    def __init__(self, model: Transformer | str, device=None,
+    def __init__(self, model: Transformer | ModelConfig | str, device=None,
                  dtype=torch.bfloat16, kv_blocks: int | None = None,
                  max_batch: int = 64, mem_fraction: float = 0.85, seed: int = 0,
                  load_in_8bit: bool = False, prefix_cache: bool | None = None,
                  kv_fp8: bool | None = None):
         self.device = device if device is not None else (
             f"cuda:{comm.local_rank()}" if torch.cuda.is_available() else "cpu")
-        if isinstance(model, str):
+        if isinstance(model, (str, ModelConfig)):
             model = build_model(model, dtype=dtype, seed=seed,
                                 device=self.device)
         self.model = model.to(self.device).eval()

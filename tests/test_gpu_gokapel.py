@@ -360,7 +360,8 @@ def test_routing(router, T):
         pairs, tiles = ops.ext().moe_plan(got.chosen, E, tile)
         pairs, tiles = pairs.cpu(), tiles.cpu()
         assert sorted(pairs.tolist()) == list(range(T * top))
-        seen = 0
+        used, seen = int(tiles[-1, 0]), 0
+        assert (tiles[:, 2] > 0).sum() == used < len(tiles)
         for e, first, n in tiles.tolist():
             if n:
                 assert first == seen and n <= tile
