@@ -71,7 +71,12 @@ template <typename T> RB_DEV float sigmoid(float x) {
     return 1.0f / (1.0f + expf(-x));
 }
 RB_DEV float gate(float x) { return 1.0f / (1.0f + expf(-x)); }
-RB_DEV float softplus(float x) {
+template <typename T> RB_DEV float softplus(float x) {
+  if constexpr (sizeof(T) == 2) {
+    const float e = __expf(-fabsf(x));
+    return fmaxf(x, 0.0f) +
+           (e < 1e-3f ? e - 0.5f * e * e : __logf(1.0f + e));
+  }
   return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x)));
 }
 
@@ -125,7 +130,7 @@ RB_DEV float log_decay(const Args &a, int64_t row, int h, int d) {
   const float x = rb::bf16_to_f32_or_id(
       ((const T *)a.y2)[row * a.ny2 + h * a.dc + d]);
   const float *w = a.decay + h * (a.dc + 1);
-  return LOG2E * w[a.dc] * softplus(x + w[d]);
+  return LOG2E * w[a.dc] * softplus<T>(x + w[d]);
 }
 
 // ---------------------------------------------------------------------------
@@ -567,11 +572,10 @@ union Frag { u32x4v u; bf16x8v v; };
 RB_DEV f32x4v mfma(const Frag &a, const Frag &b, f32x4v c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
 }
-// an fp32 product of two split factors
-RB_DEV f32x4v mfma3(const Frag *a, const Frag &bh, const Frag &bl, f32x4v c) {
-  c = mfma(a[0], bh, c);
-  c = mfma(a[0], bl, c);
-  return mfma(a[1], bh, c);
+// one of the three products that make an fp32 product of split factors
+RB_DEV f32x4v part(int i, const Frag *a, const Frag &bh, const Frag &bl,
+                   f32x4v c) {
+  return mfma(a[i == 2], i == 1 ? bl : bh, c);
 }
 
 template <int DCP, bool AHEAD>
@@ -649,34 +653,37 @@ __global__ __launch_bounds__(RB_WAVE, 1) void delta_scan_kernel(Args a) {
       split8(f, sh[ks].u, sl[ks].u);
     }
     f32x4v u[2] = {uf[0], uf[1]}, o[2] = {(f32x4v)(0.0f), (f32x4v)(0.0f)};
+    if constexpr (!AHEAD) get_q(e);
+    // four sums side by side
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
-      for (int m = 0; m < 2; ++m)
-        u[m] = mfma3(wf[m * KS + ks], sh[ks], sl[ks], u[m]);
+      for (int i = 0; i < 3; ++i)
+#pragma unroll
+        for (int m = 0; m < 2; ++m) {
+          u[m] = part(i, wf[m * KS + ks], sh[ks], sl[ks], u[m]);
+          o[m] = part(i, qf[m * KS + ks], sh[ks], sl[ks], o[m]);
+        }
     if constexpr (AHEAD) get_w(next);
-    else get_q(e);
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
-#pragma unroll
-      for (int m = 0; m < 2; ++m)
-        o[m] = mfma3(qf[m * KS + ks], sh[ks], sl[ks], o[m]);
     Frag uh, ul;
     {
       const float f[8] = {u[0][0], u[0][1], u[0][2], u[0][3],
                           u[1][0], u[1][1], u[1][2], u[1][3]};
       split8(f, uh.u, ul.u);
     }
+    if constexpr (!AHEAD) get_k(e);
 #pragma unroll
-    for (int m = 0; m < 2; ++m) o[m] = mfma3(pf[m], uh, ul, o[m]);
-    if constexpr (AHEAD) get_q(next);
-    else get_k(e);
-#pragma unroll
-    for (int d = 0; d < TD; ++d) {
+    for (int d = 0; d < TD; ++d)
 #pragma unroll
       for (int r = 0; r < 4; ++r) S[d][r] *= gf[d][r];
-      S[d] = mfma3(kf[d], uh, ul, S[d]);
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+#pragma unroll
+      for (int m = 0; m < 2; ++m) o[m] = part(i, pf[m], uh, ul, o[m]);
+#pragma unroll
+      for (int d = 0; d < TD; ++d) S[d] = part(i, kf[d], uh, ul, S[d]);
     }
+    if constexpr (AHEAD) get_q(next);
     if constexpr (AHEAD) get_k(next);
     const int t = (a.chunk0 + c) * C + grp * 4;
     if (col_ok)

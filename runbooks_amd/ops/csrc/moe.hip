@@ -360,8 +360,7 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       *reinterpret_cast<u32x4v *>(buf + dst[i]) = ok ? r.x[i] : zero;
-      *reinterpret_cast<u32x4v *>(buf + 128 * ROW + dst[i]) =
-          ok ? r.w[i] : zero;
+      *reinterpret_cast<u32x4v *>(buf + 128 * ROW + dst[i]) = r.w[i];
     }
   };
   f32x4v acc[4][4];
@@ -374,7 +373,7 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
                   const Step &next) __attribute__((always_inline)) {
     fetch(free, k0 + 2 * BK);
     const char *xs = buf, *ws = buf + 128 * ROW;
-#pragma unroll 1
+#pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
       bf16x8v xf[4], wf[4];
 #pragma unroll
@@ -400,9 +399,8 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
   fetch(r1, BK);
   stage(r0, 0, smem);
   __syncthreads();
-  for (int k0 = 0; k0 < a.K; k0 += 2 * BK) {
+  for (int k0 = 0; k0 < a.K; k0 += 2 * BK) {   // beyond K: zeros
     step(k0, smem, smem + BUF, r0, r1);
-    if (k0 + BK >= a.K) break;
     step(k0 + BK, smem + BUF, smem, r1, r0);
   }
 #pragma unroll

@@ -44,15 +44,28 @@ __global__ __launch_bounds__(BLOCK) void qkv_prep_kernel(
   const int64_t page_head = (int64_t)skv::PAGE * ec;
   const float *cr = cos + (int64_t)positions[t] * a.half;
   const float *sr = sin + (int64_t)positions[t] * a.half;
-  float cc[NV][4], ss[NV][4];
+  float cc[NV][4], ss[NV][4], wq[NV][8], wk[NV][8];
 #pragma unroll
-  for (int n = 0; n < NV; ++n)
+  for (int n = 0; n < NV; ++n) {
+    const int c0 = (n * L + lane) * 8;
+    const bool turns = c0 < 2 * a.half;
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-      const int p = (n * L + lane) * 4 + k;
-      cc[n][k] = p < a.half ? cr[p] : 1.0f;
-      ss[n][k] = p < a.half ? sr[p] : 0.0f;
+      const int p = c0 / 2 + k;
+      cc[n][k] = turns ? cr[min(p, a.half - 1)] : 1.0f;
+      ss[n][k] = turns ? sr[min(p, a.half - 1)] : 0.0f;
+      if (p >= a.half) {
+        cc[n][k] = 1.0f;
+        ss[n][k] = 0.0f;
+      }
     }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const int c = min(c0 + k, a.dim - 1);
+      wq[n][k] = c0 + k < a.dim ? norms[c] : 0.0f;
+      wk[n][k] = c0 + k < a.dim ? norms[a.dim + c] : 0.0f;
+    }
+  }
   const int n_heads = a.heads + a.kv;
   float ahead[NV][8];
   auto fetch = [&](int h) {
@@ -86,11 +99,10 @@ __global__ __launch_bounds__(BLOCK) void qkv_prep_kernel(
     for (int n = 0; n < NV; ++n) {
       const int c = (n * L + lane) * 8;
       if (c >= a.hc) continue;
-      const float *w = norms + (is_k ? a.dim : 0) + c;
       float r[8];
 #pragma unroll
       for (int k = 0; k < 8; ++k)
-        r[k] = c + k < a.dim ? v[n][k] * inv * w[k] : 0.0f;
+        r[k] = v[n][k] * inv * (is_k ? wk[n][k] : wq[n][k]);
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
         const float p = r[2 * k], q = r[2 * k + 1];

@@ -6,7 +6,7 @@ import torch
 import gokapel_oracle as oracle
 from gokapel_oracle import delta, dense, moe, twin
 from keralorn_helpers import portions  # noqa: F401
-from latent_helpers import (close, rel_err, run_cut, tokens_of,  # noqa: F401
+from latent_helpers import (rel_err, run_cut, tokens_of,  # noqa: F401
                             write_checkpoint)
 from runbooks_amd.models import build_model
 from runbooks_amd.models.load import (config_from_gokapel,
@@ -66,3 +66,16 @@ def make_engine(cfg, W, dtype=torch.float32, device="cpu", **kw):
     kw.setdefault("kv_blocks", 128)
     kw.setdefault("max_batch", 6)
     return Engine(load(cfg, W, dtype, device), device=device, **kw)
+
+
+def close(got, ref, dtype, slack=1.0):
+    """Engine logits against the oracle: 32-bit to rounding; bf16 to a mean
+    error. Rounding may decide a few tokens of such small models (experts of
+    nearly equal choice score, a unit vector or a head's result of a length
+    near zero), so single rows may differ."""
+    d = (got.double() - ref.double()).pow(2).mean(-1).sqrt() / \
+        ref.double().pow(2).mean().sqrt()
+    if dtype == torch.float32:
+        return float(d.max()) < 2e-5 * slack
+    return float(d.mean()) < 0.02 * slack and \
+        float((d > 0.15).double().mean()) < 0.03 * slack

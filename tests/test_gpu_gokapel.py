@@ -427,6 +427,7 @@ def test_unequal_requests_in_one_batch(name, dtype):
     refs = [oracle.forward(cfg, W, s) for s in seqs]
     eng = make_engine(cfg, W, dtype, DEV, kv_blocks=20, max_batch=2)
     live, waiting, turn = {}, list(range(len(seqs))), 0
+    got = [[] for _ in seqs]
     while waiting or live:
         while waiting and len(live) < 2:
             live[waiting.pop(0)] = [eng.open_request(), 0]
@@ -439,12 +440,13 @@ def test_unequal_requests_in_one_batch(name, dtype):
         turn += 1
         logits, row = eng.run_portions(entries).float().cpu(), 0
         for i, at, n in ids:
-            assert close(logits[row:row + n], refs[i][at:at + n], dtype,
-                         slack=3)
+            got[i].append(logits[row:row + n])
             row += n
             live[i][1] = at + n
             if at + n == len(seqs[i]):
                 eng.close_request(live.pop(i)[0])
+    assert close(torch.cat([x for g in got for x in g]), torch.cat(refs),
+                 dtype, slack=1.5)
     assert len(eng.allocator.free) == eng.allocator.num_blocks
 
 
