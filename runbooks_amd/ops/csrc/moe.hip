@@ -21,6 +21,8 @@ namespace {
 constexpr int BLOCK = 256;
 constexpr int MAX_EXPERTS = 1024;
 constexpr int MAX_TOP = 64;
+// a tile: expert, first pair, pairs, the expert's first tile, its tiles
+constexpr int TILE_INTS = 5;
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
 typedef __attribute__((ext_vector_type(4))) float f32x4v;
@@ -172,15 +174,17 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(
   const int first = at[src][i] - mine, first_t = tl[src][i] - mine_t;
   const int used = tl[src][MAX_EXPERTS - 1];
   for (int k = 0; k < mine_t; ++k) {
-    int *e = tiles + (first_t + k) * 3;
+    int *e = tiles + (first_t + k) * TILE_INTS;
     e[0] = i;
     e[1] = first + k * tile;
     e[2] = min(tile, mine - k * tile);
+    e[3] = first_t;
+    e[4] = mine_t;
   }
   for (int k = used + i; k < n_tiles; k += 1024) {
-    tiles[k * 3] = k == n_tiles - 1 ? used : 0;
-    tiles[k * 3 + 1] = 0;
-    tiles[k * 3 + 2] = 0;
+    int *e = tiles + k * TILE_INTS;
+    e[0] = k == n_tiles - 1 ? used : 0;
+    e[1] = e[2] = e[3] = e[4] = 0;
   }
   count[i] = first;
   __syncthreads();
@@ -259,7 +263,7 @@ __global__ __launch_bounds__(BLOCK) void moe_rows_kernel(Args a) {
   using V = typename S::V;
   constexpr int U = 4;
   __shared__ f32x4v red[BLOCK / RB_WAVE][2][64];
-  const int *tile = a.tiles + blockIdx.y * 3;
+  const int *tile = a.tiles + blockIdx.y * TILE_INTS;
   const int expert = tile[0], first = tile[1], count = tile[2];
   if (count <= 0) return;
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -317,16 +321,18 @@ template <bool DOWN>
 __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
                                                             int n_tiles) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  // neighbouring workgroups of one XCD share an expert
-  const int total = a.tiles[(n_tiles - 1) * 3] * nb;
+  // neighbouring workgroups are on one XCD and share an expert's columns,
+  // so that a weight is read once
+  const int total = a.tiles[(n_tiles - 1) * TILE_INTS] * nb;
   const int q8 = total / 8, r8 = total % 8;
   const int xcd = blockIdx.x % 8, pos = blockIdx.x / 8;
   if (pos >= q8 + (xcd < r8)) return;
   const int wg = xcd * q8 + min(xcd, r8) + pos;
-  const int *tile = a.tiles + wg / nb * 3;
+  const int *own = a.tiles + wg / nb * TILE_INTS;
+  const int local = wg - own[3] * nb;
+  const int *tile = a.tiles + (own[3] + local % own[4]) * TILE_INTS;
   const int expert = tile[0], first = tile[1], count = tile[2];
-  if (count <= 0) return;
-  const int n0 = wg % nb * 128;
+  const int n0 = local / own[4] * 128;
   const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
   const int l16 = lane & 15, grp = lane >> 4;
   const int wn = (wid & 1) * 64, wm = (wid >> 1) * 64;
@@ -475,7 +481,7 @@ std::vector<at::Tensor> moe_plan(at::Tensor chosen, int64_t experts,
   TORCH_CHECK(n < (1 << 30), "moe_plan: pairs");
   const int64_t n_tiles = (n + tile - 1) / tile + std::min(n, experts) + 1;
   auto pairs = at::empty({n}, chosen.options());
-  auto tiles = at::empty({n_tiles, 3}, chosen.options());
+  auto tiles = at::empty({n_tiles, TILE_INTS}, chosen.options());
   if (n == 0) return {pairs, tiles};
   hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0,
                      at::hip::getCurrentHIPStream(), chosen.data_ptr<int>(),
@@ -498,7 +504,7 @@ at::Tensor moe_gemm(at::Tensor x, at::Tensor w, at::Tensor pairs,
               weights.scalar_type() == at::kFloat && pairs.is_contiguous() &&
               pairs.scalar_type() == at::kInt &&
               pairs.numel() == weights.numel() && tiles.dim() == 2 &&
-              tiles.size(1) == 3 && tiles.is_contiguous() &&
+              tiles.size(1) == TILE_INTS && tiles.size(0) >= 1 && tiles.is_contiguous() &&
               tiles.scalar_type() == at::kInt, "moe_gemm: plan");
   const int64_t T = weights.size(0), top = weights.size(1), N = w.size(1),
                 K = w.size(2), n = pairs.numel();

@@ -31,7 +31,8 @@ class MoEPlan:
     chosen: torch.Tensor           # [T, top] int32
     weights: torch.Tensor          # [T, top] fp32
     pairs: torch.Tensor | None = None    # token * top + choice, by expert
-    # [n, 3] expert, first pair, pairs; the last row counts the used ones
+    # [n, 5] expert, first pair, pairs, the expert's first tile and its tiles;
+    # the last row counts the used ones
     tiles: torch.Tensor | None = None
     tile: int = 0                  # most pairs of a tile
 

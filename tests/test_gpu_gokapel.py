@@ -362,7 +362,7 @@ def test_routing(router, T):
         assert sorted(pairs.tolist()) == list(range(T * top))
         used, seen = int(tiles[-1, 0]), 0
         assert (tiles[:, 2] > 0).sum() == used < len(tiles)
-        for e, first, n in tiles.tolist():
+        for e, first, n, *_ in tiles.tolist():
             if n:
                 assert first == seen and n <= tile
                 assert (ref.chosen.view(-1)[pairs[first:first + n].long()]
