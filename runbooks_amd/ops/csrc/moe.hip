@@ -313,12 +313,12 @@ __global__ __launch_bounds__(BLOCK) void moe_rows_kernel(Args a) {
 }
 
 // 128 pairs x 128 columns per workgroup, 4 waves of 64 x 64, K in steps of 64
-// through two LDS buffers.
+// through LDS.
 constexpr int BK = 64, ROW = BK * 2 + 16;      // LDS bytes per row
 constexpr int BUF = 2 * 128 * ROW;
 
 template <bool DOWN>
-__global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
+__global__ __launch_bounds__(BLOCK, 3) void moe_tile_kernel(Args a, int nb,
                                                             int n_tiles) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   // neighbouring workgroups are on one XCD and share an expert's columns,
@@ -374,11 +374,15 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = (f32x4v)(0.0f);
-  // two steps ahead in registers, one in LDS
-  auto step = [&](int k0, char *buf, char *other, Step &free,
-                  const Step &next) __attribute__((always_inline)) {
-    fetch(free, k0 + 2 * BK);
-    const char *xs = buf, *ws = buf + 128 * ROW;
+  // one step in LDS, the next in registers; three workgroups per CU fill each
+  // other's waits
+  Step r;
+  fetch(r, 0);
+  for (int k0 = 0; k0 < a.K; k0 += BK) {
+    stage(r, k0, smem);
+    __syncthreads();
+    fetch(r, k0 + BK);
+    const char *xs = smem, *ws = smem + 128 * ROW;
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
       bf16x8v xf[4], wf[4];
@@ -397,17 +401,7 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_tile_kernel(Args a, int nb,
           acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
               wf[i], xf[j], acc[i][j], 0, 0, 0);
     }
-    stage(next, k0 + BK, other);
     __syncthreads();
-  };
-  Step r0, r1;
-  fetch(r0, 0);
-  fetch(r1, BK);
-  stage(r0, 0, smem);
-  __syncthreads();
-  for (int k0 = 0; k0 < a.K; k0 += 2 * BK) {   // beyond K: zeros
-    step(k0, smem, smem + BUF, r0, r1);
-    step(k0 + BK, smem + BUF, smem, r1, r0);
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
@@ -428,13 +422,13 @@ template <bool DOWN> void launch_tile(const Args &a, int n_tiles,
     return hipFuncSetAttribute(
                reinterpret_cast<const void *>(&moe_tile_kernel<DOWN>),
                hipFuncAttributeMaxDynamicSharedMemorySize,
-               2 * BUF) == hipSuccess;
+               BUF) == hipSuccess;
   }();
   TORCH_CHECK(once, "moe_gemm: LDS size");
   const int nb = (a.N + 127) / 128;
   const int total = (nb * n_tiles + 7) / 8 * 8;
   hipLaunchKernelGGL((moe_tile_kernel<DOWN>), dim3(total), dim3(BLOCK),
-                     2 * BUF, stream, a, nb, n_tiles);
+                     BUF, stream, a, nb, n_tiles);
 }
 
 }  // namespace
