@@ -313,14 +313,17 @@ __global__ __launch_bounds__(BLOCK) void moe_rows_kernel(Args a) {
 }
 
 // 128 pairs x 128 columns per workgroup, 4 waves of 64 x 64, K in steps of 64
-// through LDS.
-constexpr int BK = 64, ROW = BK * 2 + 16;      // LDS bytes per row
-constexpr int BUF = 2 * 128 * ROW;
+// straight to LDS; the workgroups of a CU fill each other's waits. A row's
+// eight 16-byte chunks are stored in an order that depends on the row, so that
+// 16 rows are read without bank conflicts.
+constexpr int BK = 64, ROW = BK * 2;           // LDS bytes per row
+
+RB_DEV int chunk_at(int row, int c) { return c ^ ((row >> 1) & 7); }
 
 template <bool DOWN>
-__global__ __launch_bounds__(BLOCK, 3) void moe_tile_kernel(Args a, int nb,
+__global__ __launch_bounds__(BLOCK, 4) void moe_tile_kernel(Args a, int nb,
                                                             int n_tiles) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
+  __shared__ __attribute__((aligned(16))) char smem[2 * 128 * ROW];
   // neighbouring workgroups are on one XCD and share an expert's columns,
   // so that a weight is read once
   const int total = a.tiles[(n_tiles - 1) * TILE_INTS] * nb;
@@ -333,62 +336,53 @@ __global__ __launch_bounds__(BLOCK, 3) void moe_tile_kernel(Args a, int nb,
   const int *tile = a.tiles + (own[3] + local % own[4]) * TILE_INTS;
   const int expert = tile[0], first = tile[1], count = tile[2];
   const int n0 = local / own[4] * 128;
-  const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63;
   const int l16 = lane & 15, grp = lane >> 4;
   const int wn = (wid & 1) * 64, wm = (wid >> 1) * 64;
 
+  // a lane's 16 bytes of eight rows at a time
   const uint16_t *xp[4], *wp[4];
-  int dst[4];
-  const int kc = tid & 7;                      // 16-byte chunk of a row
+  int kc[4];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const int row = (tid >> 3) + i * 32;
+    const int row = (wid * 4 + i) * 8 + (lane >> 3);
     const int pair = a.pairs[first + min(row, count - 1)];
     xp[i] = (const uint16_t *)a.x +
-            (int64_t)(DOWN ? pair : pair / a.top) * a.K + kc * 8;
+            (int64_t)(DOWN ? pair : pair / a.top) * a.K;
     wp[i] = (const uint16_t *)a.w +
-            ((int64_t)expert * a.N + min(n0 + row, a.N - 1)) * a.K + kc * 8;
-    dst[i] = row * ROW + kc * 16;
+            ((int64_t)expert * a.N + min(n0 + row, a.N - 1)) * a.K;
+    kc[i] = chunk_at(row, lane & 7) * 8;
   }
-  struct Step { u32x4v x[4], w[4]; };          // a thread's part of a step
-  auto fetch = [&](Step &r, int k0) {
-    const bool ok = k0 + kc * 8 < a.K;
-    const int k = ok ? k0 : 0;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      r.x[i] = *reinterpret_cast<const u32x4v *>(xp[i] + k);
-      r.w[i] = *reinterpret_cast<const u32x4v *>(wp[i] + k);
-    }
-  };
-  auto stage = [&](const Step &r, int k0, char *buf) {
-    const bool ok = k0 + kc * 8 < a.K;
-    const u32x4v zero = (u32x4v)(0u);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      *reinterpret_cast<u32x4v *>(buf + dst[i]) = ok ? r.x[i] : zero;
-      *reinterpret_cast<u32x4v *>(buf + 128 * ROW + dst[i]) = r.w[i];
-    }
+  auto to_lds = [](const uint16_t *p, char *dst) {
+    __builtin_amdgcn_global_load_lds(
+        (const __attribute__((address_space(1))) uint32_t *)(const void *)p,
+        (__attribute__((address_space(3))) uint32_t *)(void *)dst, 16, 0, 0);
   };
   f32x4v acc[4][4];
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = (f32x4v)(0.0f);
-  // one step in LDS, the next in registers; three workgroups per CU fill each
-  // other's waits
-  Step r;
-  fetch(r, 0);
   for (int k0 = 0; k0 < a.K; k0 += BK) {
-    stage(r, k0, smem);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      // beyond K any address of the row: those chunks are not read
+      const int k = k0 + kc[i] < a.K ? k0 + kc[i] : 0;
+      char *dst = smem + (wid * 4 + i) * 8 * ROW;
+      to_lds(xp[i] + k, dst);
+      to_lds(wp[i] + k, dst + 128 * ROW);
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    fetch(r, k0 + BK);
     const char *xs = smem, *ws = smem + 128 * ROW;
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
+      if (k0 + ks * 32 >= a.K) break;
       bf16x8v xf[4], wf[4];
+      const int at = chunk_at(l16, ks * 4 + grp) * 16;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int at = ks * 64 + grp * 16;
         xf[i] = *reinterpret_cast<const bf16x8v *>(
             xs + (wm + i * 16 + l16) * ROW + at);
         wf[i] = *reinterpret_cast<const bf16x8v *>(
@@ -418,17 +412,10 @@ __global__ __launch_bounds__(BLOCK, 3) void moe_tile_kernel(Args a, int nb,
 
 template <bool DOWN> void launch_tile(const Args &a, int n_tiles,
                                       hipStream_t stream) {
-  static bool once = [] {
-    return hipFuncSetAttribute(
-               reinterpret_cast<const void *>(&moe_tile_kernel<DOWN>),
-               hipFuncAttributeMaxDynamicSharedMemorySize,
-               BUF) == hipSuccess;
-  }();
-  TORCH_CHECK(once, "moe_gemm: LDS size");
   const int nb = (a.N + 127) / 128;
   const int total = (nb * n_tiles + 7) / 8 * 8;
   hipLaunchKernelGGL((moe_tile_kernel<DOWN>), dim3(total), dim3(BLOCK),
-                     BUF, stream, a, nb, n_tiles);
+                     0, stream, a, nb, n_tiles);
 }
 
 }  // namespace
