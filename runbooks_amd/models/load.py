@@ -412,7 +412,8 @@ def config_from_gokapel(d: dict, shapes: dict, name: str = "gokapel"
 
     def rows(i, tensor):
         seen = set()
-        while d["layers"][i].get("weights_of") is not None and i not in seen:
+        while i not in seen and i < len(d["layers"]) and \
+                d["layers"][i].get("weights_of") is not None:
             seen.add(i)
             i = d["layers"][i]["weights_of"]
         full = f"l{i}.mix.{tensor}"

@@ -35,7 +35,8 @@ def materialize_synthetic(name: str, out_dir: Path, seed: int = 0) -> None:
     cfg = get_config(name)
     model = build_model(cfg, dtype=torch.bfloat16, tp=1, seed=seed)
     save_file({k: v.contiguous() for k, v in model.state_dict().items()
-               if not k.startswith("rope_")},
+               if not k.startswith("rope_") and
+               not (cfg.tie_embeddings and k == "lm_head.weight")},
               str(out_dir / "model.safetensors"))
     (out_dir / "config.json").write_text(json.dumps({
         "runbooks_amd_config": cfg.name}))
