@@ -52,7 +52,7 @@ struct Args {
   int64_t ny, ny2;
   int heads, kv, dim, dc, vc, taps, off_k, off_v, off_b;
   const float *conv;                   // [taps, off_b]
-  const float *decay;                  // [heads, dc + 1]
+  const float *decay;                  // [heads, dc] biases, [heads] factors
   float *state;                        // [slots, heads, dc, vc]
   void *tails;                         // [slots, taps - 1, off_b]
   const int *positions, *cu_q, *slots;
@@ -80,6 +80,17 @@ template <typename T> RB_DEV float softplus(float x) {
   return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x)));
 }
 
+// N neighbouring values of T or fp32
+template <int N, typename E> RB_DEV void load_n(const E *p, float *f) {
+  if constexpr (N == 8) {
+    rb::VIO<E>::load(p, f);
+    if constexpr (rb::VIO<E>::W == 4) rb::VIO<E>::load(p + 4, f + 4);
+  } else {
+#pragma unroll
+    for (int k = 0; k < N; ++k) f[k] = rb::bf16_to_f32_or_id(p[k]);
+  }
+}
+
 // Convolution and silu of N neighbouring channels at token t of the portion
 // that starts at row q0.
 template <typename T, int N>
@@ -87,16 +98,6 @@ RB_DEV void conv(const Args &a, int q0, int t, bool fresh, int slot, int ch,
                  float *out) {
 #pragma unroll
   for (int k = 0; k < N; ++k) out[k] = 0.0f;
-  auto load = [](const auto *p, float *f) {
-    using E = std::remove_cv_t<std::remove_reference_t<decltype(*p)>>;
-    if constexpr (N == 8) {
-      rb::VIO<E>::load(p, f);
-      if constexpr (rb::VIO<E>::W == 4) rb::VIO<E>::load(p + 4, f + 4);
-    } else {
-#pragma unroll
-      for (int k = 0; k < N; ++k) f[k] = rb::bf16_to_f32_or_id(p[k]);
-    }
-  };
   const T *now = (const T *)a.y + (int64_t)(q0 + t) * a.ny + ch;
   for (int j0 = 0; j0 < a.taps; j0 += 4) {
     float f[4][N], w[4][N];
@@ -109,8 +110,8 @@ RB_DEV void conv(const Args &a, int q0, int t, bool fresh, int slot, int ch,
         p = (const T *)a.tails +
             ((int64_t)slot * (a.taps - 1) + a.taps - 1 + s) * a.off_b + ch;
       if (j >= a.taps || (s < 0 && fresh)) p = now;
-      load(p, f[i]);
-      load(a.conv + (int64_t)min(j, a.taps - 1) * a.off_b + ch, w[i]);
+      load_n<N>(p, f[i]);
+      load_n<N>(a.conv + (int64_t)min(j, a.taps - 1) * a.off_b + ch, w[i]);
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -124,13 +125,15 @@ RB_DEV void conv(const Args &a, int q0, int t, bool fresh, int slot, int ch,
   for (int k = 0; k < N; ++k) out[k] *= sigmoid<T>(out[k]);
 }
 
-// log2 g of one head and channel
-template <typename T>
-RB_DEV float log_decay(const Args &a, int64_t row, int h, int d) {
-  const float x = rb::bf16_to_f32_or_id(
-      ((const T *)a.y2)[row * a.ny2 + h * a.dc + d]);
-  const float *w = a.decay + h * (a.dc + 1);
-  return LOG2E * w[a.dc] * softplus<T>(x + w[d]);
+// log2 g of N neighbouring channels of one head
+template <typename T, int N>
+RB_DEV void log_decay(const Args &a, int64_t row, int h, int d, float *out) {
+  float x[N], b[N];
+  load_n<N>((const T *)a.y2 + row * a.ny2 + h * a.dc + d, x);
+  load_n<N>(a.decay + h * a.dc + d, b);
+  const float f = LOG2E * a.decay[a.heads * a.dc + h];
+#pragma unroll
+  for (int k = 0; k < N; ++k) out[k] = f * softplus<T>(x[k] + b[k]);
 }
 
 // ---------------------------------------------------------------------------
@@ -170,8 +173,9 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
         qk_s[buf][i] = f;
       } else if (i < 3 * DP) {
         const int d = i - 2 * DP;
-        g_s[buf][d] = d < a.dc
-            ? __builtin_amdgcn_exp2f(log_decay<T>(a, t, h, d)) : 0.0f;
+        float f = -INFINITY;
+        if (d < a.dc) log_decay<T, 1>(a, t, h, d, &f);
+        g_s[buf][d] = __builtin_amdgcn_exp2f(f);
       } else if (i < 3 * DP + STEP_COLS) {
         const int c = i - 3 * DP;
         float f = 0.0f;
@@ -314,6 +318,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
                              a.heads + h) * a.entry;
 
   auto stage_v = [&](int c0) {
+#pragma unroll 2
     for (int i = tid; i < C * (vb / 8); i += BLOCK) {
       const int t = i / (vb / 8), c = i % (vb / 8) * 8;
       float f[8] = {};
@@ -324,6 +329,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     }
   };
   // ---- q, k, log g, beta, v ----------------------------------------------
+#pragma unroll 2
   for (int i = tid; i < 2 * C * (DCP / 8); i += BLOCK) {
     const int which = i / (C * (DCP / 8)), r = i % (C * (DCP / 8));
     const int t = r / (DCP / 8), d = r % (DCP / 8) * 8;
@@ -335,10 +341,13 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
 #pragma unroll
     for (int k = 0; k < 8; ++k) dst[k] = f[k];
   }
-  for (int i = tid; i < C * DCP; i += BLOCK) {
-    const int t = i / DCP, d = i % DCP;
-    g_s[t * RS + d] =
-        t < len && d < a.dc ? log_decay<T>(a, q0 + t0 + t, h, d) : 0.0f;
+#pragma unroll 2
+  for (int i = tid; i < C * (DCP / 8); i += BLOCK) {
+    const int t = i / (DCP / 8), d = i % (DCP / 8) * 8;
+    float f[8] = {};
+    if (t < len && d < a.dc) log_decay<T, 8>(a, q0 + t0 + t, h, d, f);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) g_s[t * RS + d + k] = f[k];
   }
   if (tid < C)
     b_s[tid] = tid < len
@@ -368,12 +377,13 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     }
   }
   for (int d = tid; d < DCP; d += BLOCK) {
-    float s = 0.0f;
-#pragma unroll 8
-    for (int t = 0; t < C; ++t) {
-      s += g_s[t * RS + d];
-      g_s[t * RS + d] = s;
-    }
+    float s[C];
+#pragma unroll
+    for (int t = 0; t < C; ++t) s[t] = g_s[t * RS + d];
+#pragma unroll
+    for (int t = 1; t < C; ++t) s[t] += s[t - 1];
+#pragma unroll
+    for (int t = 1; t < C; ++t) g_s[t * RS + d] = s[t];
   }
   __syncthreads();
   // ---- A and P: tiles of 4 x 4 tokens, 4 lanes share a tile's channels.

@@ -126,11 +126,10 @@ def pack_conv(lay: DeltaLayout, q, k, v):
 
 
 def pack_decay(lay: DeltaLayout, a_log, dt_bias):
-    """[heads, dc + 1] fp32: the bias per channel, then -exp(a_log)."""
-    out = torch.zeros(lay.heads, lay.dc + 1, device=a_log.device)
-    out[:, :lay.dim] = dt_bias.float().view(lay.heads, lay.dim)
-    out[:, lay.dc] = -torch.exp(a_log.float())
-    return out
+    """fp32: [heads, dc] biases, then [heads] -exp(a_log)."""
+    bias = torch.zeros(lay.heads, lay.dc, device=a_log.device)
+    bias[:, :lay.dim] = dt_bias.float().view(lay.heads, lay.dim)
+    return torch.cat([bias.view(-1), -torch.exp(a_log.float())])
 
 
 def alloc_delta_state(slots: int, lay: DeltaLayout, device, dtype):
@@ -162,8 +161,8 @@ def _recur_ref(y, y2, lay, conv_w, decay, state, batch, o, seqs):
         v = x[:, lay.off_v:].reshape(T, H, lay.vc)
         beta = torch.sigmoid(y[t0:t1, n:n + H].float())
         a = y2[t0:t1, :lay.off_g].float().view(T, H, lay.dc)
-        g = torch.exp(decay[:, lay.dc:] * torch.nn.functional.softplus(
-            a + decay[:, :lay.dc]))
+        g = torch.exp(decay[H * lay.dc:, None] * torch.nn.functional.softplus(
+            a + decay[:H * lay.dc].view(H, lay.dc)))
         for t in range(T):
             S = g[t][:, :, None] * S
             u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S,
