@@ -39,11 +39,13 @@ namespace {
 constexpr int BLOCK = 256;
 constexpr int STEP_COLS = 32;          // state columns per workgroup, step
 constexpr int C = 32;                  // tokens per chunk
+constexpr int PREP = 512;              // threads of delta_prep
 constexpr int VB = 256;                // value columns staged at once
 constexpr float UNIT_EPS = 1e-6f;
 constexpr float LOG2E = 1.4426950408889634f;
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
+typedef __attribute__((ext_vector_type(2))) float f32x2v;
 typedef __attribute__((ext_vector_type(4))) float f32x4v;
 typedef __attribute__((ext_vector_type(4))) unsigned int u32x4v;
 
@@ -294,7 +296,7 @@ template <int DCP> constexpr int prep_lds(int vb) {
 }
 
 template <int DCP>
-__global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
+__global__ __launch_bounds__(PREP, 2) void delta_prep_kernel(Args a, int vb) {
   using E = Entry<DCP>;
   using T = uint16_t;
   constexpr int RS = DCP + 4, AS = C + 4;      // floats per LDS row
@@ -319,7 +321,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
 
   auto stage_v = [&](int c0) {
 #pragma unroll 2
-    for (int i = tid; i < C * (vb / 8); i += BLOCK) {
+    for (int i = tid; i < C * (vb / 8); i += PREP) {
       const int t = i / (vb / 8), c = i % (vb / 8) * 8;
       float f[8] = {};
       if (t < len && c0 + c < a.vc)
@@ -330,7 +332,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
   };
   // ---- q, k, log g, beta, v ----------------------------------------------
 #pragma unroll 2
-  for (int i = tid; i < 2 * C * (DCP / 8); i += BLOCK) {
+  for (int i = tid; i < 2 * C * (DCP / 8); i += PREP) {
     const int which = i / (C * (DCP / 8)), r = i % (C * (DCP / 8));
     const int t = r / (DCP / 8), d = r % (DCP / 8) * 8;
     float f[8] = {};
@@ -342,7 +344,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     for (int k = 0; k < 8; ++k) dst[k] = f[k];
   }
 #pragma unroll 2
-  for (int i = tid; i < C * (DCP / 8); i += BLOCK) {
+  for (int i = tid; i < C * (DCP / 8); i += PREP) {
     const int t = i / (DCP / 8), d = i % (DCP / 8) * 8;
     float f[8] = {};
     if (t < len && d < a.dc) log_decay<T, 8>(a, q0 + t0 + t, h, d, f);
@@ -358,25 +360,25 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
   __syncthreads();
   // ---- unit vectors (8 lanes per token); sums of log g --------------------
   {
-    const int t = tid >> 3, l = tid & 7;
+    const int t = tid >> 4, l = tid & 15;
     float sq = 0.0f, sk = 0.0f;
-    for (int d = l; d < DCP; d += 8) {
+    for (int d = l; d < DCP; d += 16) {
       sq += q_s[t * RS + d] * q_s[t * RS + d];
       sk += k_s[t * RS + d] * k_s[t * RS + d];
     }
 #pragma unroll
-    for (int o = 4; o > 0; o >>= 1) {
+    for (int o = 8; o > 0; o >>= 1) {
       sq += __shfl_xor(sq, o, 64);
       sk += __shfl_xor(sk, o, 64);
     }
     sq = a.qscale / sqrtf(sq + UNIT_EPS);
     sk = 1.0f / sqrtf(sk + UNIT_EPS);
-    for (int d = l; d < DCP; d += 8) {
+    for (int d = l; d < DCP; d += 16) {
       q_s[t * RS + d] *= sq;
       k_s[t * RS + d] *= sk;
     }
   }
-  for (int d = tid; d < DCP; d += BLOCK) {
+  for (int d = tid; d < DCP; d += PREP) {
     float s[C];
 #pragma unroll
     for (int t = 0; t < C; ++t) s[t] = g_s[t * RS + d];
@@ -386,37 +388,37 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     for (int t = 1; t < C; ++t) g_s[t * RS + d] = s[t];
   }
   __syncthreads();
-  // ---- A and P: tiles of 4 x 4 tokens, 4 lanes share a tile's channels.
+  // ---- A and P: tiles of 4 x 4 tokens, 8 lanes share a tile's channels.
   // Below the diagonal the exponents go through the tile's first token. -----
   {
-    const int part = tid & 3;
-    const bool off_diag = tid < 112, diag = tid >= 128 && tid < 160;
+    const int part = tid & 7;
+    const bool off_diag = tid < 224, diag = tid >= 256 && tid < 320;
     int ti = 0, tj = 0;
     if (off_diag) {
-      int i = tid >> 2;                        // 28 tiles
+      int i = tid >> 3;                        // 28 tiles
       ti = 1;
       while (i >= ti) i -= ti++;
       tj = i;
     } else if (diag) {
-      ti = tj = (tid - 128) >> 2;
+      ti = tj = (tid - 256) >> 3;
     }
     float A[4][4] = {}, P[4][4] = {};
     if (off_diag || diag) {
       const float *qp = q_s + ti * 4 * RS, *kp = k_s + ti * 4 * RS;
       const float *gp = g_s + ti * 4 * RS;
       const float *kj = k_s + tj * 4 * RS, *gj = g_s + tj * 4 * RS;
-      for (int d0 = part * 4; d0 < DCP; d0 += 16) {
-        f32x4v q[4], k[4], g[4], k2[4], g2[4];
+      for (int d0 = part * 2; d0 < DCP; d0 += 16) {
+        f32x2v q[4], k[4], g[4], k2[4], g2[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          q[r] = *reinterpret_cast<const f32x4v *>(qp + r * RS + d0);
-          k[r] = *reinterpret_cast<const f32x4v *>(kp + r * RS + d0);
-          g[r] = *reinterpret_cast<const f32x4v *>(gp + r * RS + d0);
-          k2[r] = *reinterpret_cast<const f32x4v *>(kj + r * RS + d0);
-          g2[r] = *reinterpret_cast<const f32x4v *>(gj + r * RS + d0);
+          q[r] = *reinterpret_cast<const f32x2v *>(qp + r * RS + d0);
+          k[r] = *reinterpret_cast<const f32x2v *>(kp + r * RS + d0);
+          g[r] = *reinterpret_cast<const f32x2v *>(gp + r * RS + d0);
+          k2[r] = *reinterpret_cast<const f32x2v *>(kj + r * RS + d0);
+          g2[r] = *reinterpret_cast<const f32x2v *>(gj + r * RS + d0);
         }
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
+        for (int e = 0; e < 2; ++e) {
           if (off_diag) {
             float x[4];
 #pragma unroll
@@ -452,10 +454,12 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
       for (int s = 0; s < 4; ++s) {
         A[r][s] += __shfl_xor(A[r][s], 1, 64);
         A[r][s] += __shfl_xor(A[r][s], 2, 64);
+        A[r][s] += __shfl_xor(A[r][s], 4, 64);
         P[r][s] += __shfl_xor(P[r][s], 1, 64);
         P[r][s] += __shfl_xor(P[r][s], 2, 64);
+        P[r][s] += __shfl_xor(P[r][s], 4, 64);
       }
-    for (int i = tid; i < C * C; i += BLOCK)   // above the diagonal
+    for (int i = tid; i < C * C; i += PREP)   // above the diagonal
       if (i % C / 4 > i / C / 4) p_s[(i / C) * AS + i % C] = 0.0f;
     if ((off_diag || diag) && part == 0) {
 #pragma unroll
@@ -478,7 +482,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     *reinterpret_cast<u32x4v *>(entry + at + 1024 + lane * 16) = small;
   };
   const int lane = tid & 63, wid = tid >> 6, l16 = lane & 15, grp = lane >> 4;
-  for (int i = wid; i < 2 * E::KS + 2 + E::TD; i += BLOCK / RB_WAVE) {
+  for (int i = wid; i < 2 * E::KS + 2 + E::TD; i += PREP / RB_WAVE) {
     float f[8];
     if (i < 2 * E::KS) {
       const int t = i / E::KS * 16 + l16, d = i % E::KS * 32 + grp * 4;
@@ -506,7 +510,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
       put(E::K + m * E::OP, lane, f);
     }
   }
-  for (int d = tid; d < DCP; d += BLOCK)
+  for (int d = tid; d < DCP; d += PREP)
     reinterpret_cast<float *>(entry + E::G)[d] =
         __builtin_amdgcn_exp2f(g_s[(C - 1) * RS + d]);
   __syncthreads();                             // q_s is free
@@ -541,7 +545,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
           (f32x4v){x[4 * i], x[4 * i + 1], x[4 * i + 2], x[4 * i + 3]};
   };
   const int vround = (a.vc + 15) / 16 * 16;
-  for (int i = tid; i < DCP + min(vb, vround); i += BLOCK) {
+  for (int i = tid; i < DCP + min(vb, vround); i += PREP) {
     if (i < DCP) {
 #pragma unroll
       for (int t = 0; t < C; ++t)
@@ -555,7 +559,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     }
   }
   __syncthreads();
-  for (int i = wid; i < 2 * E::KS; i += BLOCK / RB_WAVE) {
+  for (int i = wid; i < 2 * E::KS; i += PREP / RB_WAVE) {
     float f[8];
     const int t = i / E::KS * 16 + l16, d = i % E::KS * 32 + grp * 4;
 #pragma unroll
@@ -567,7 +571,7 @@ __global__ __launch_bounds__(BLOCK) void delta_prep_kernel(Args a, int vb) {
     __syncthreads();
     stage_v(c0);
     __syncthreads();
-    for (int c = tid; c < min(vb, vround - c0); c += BLOCK) solve_v(c, c0);
+    for (int c = tid; c < min(vb, vround - c0); c += PREP) solve_v(c, c0);
   }
 }
 
@@ -897,7 +901,7 @@ void launch_chunk(Args a, int64_t n_seqs, int64_t max_q,
   for (int64_t c = 0; c < all; c += a.chunks) {
     a.chunk0 = (int)c;
     hipLaunchKernelGGL((delta_prep_kernel<DCP>),
-                       dim3(a.heads, a.chunks, n_seqs), dim3(BLOCK), shmem,
+                       dim3(a.heads, a.chunks, n_seqs), dim3(PREP), shmem,
                        stream, a, vb);
     hipLaunchKernelGGL((delta_scan_kernel<DCP, DCP <= 128>), scan,
                        dim3(RB_WAVE), 0, stream, a);
