@@ -683,7 +683,7 @@ def _gokapel(name: str, pattern: str, width: int, vocab: int, ff: int,
     that layer."""
     made = {"d": GatedDeltaSpec(**delta),
             "p": TwinSpec(AttentionSpec(**attention), MinGRUSpec(gru),
-                          0.6, 0.5)}
+                          0.75, 0.5)}
     layers: list[LayerSpec] = []
     for c in pattern:
         if c.isdigit():
@@ -693,8 +693,8 @@ def _gokapel(name: str, pattern: str, width: int, vocab: int, ff: int,
             layers.append(LayerSpec(
                 made[c.lower()],
                 SquaredReluSpec(ff) if c.isupper() else MoESpec(**mixture)))
-    kw = {"streams": 4, "residual_mult": 0.7, "embed_scale": width ** 0.5,
-          "norm_eps": 1e-6, **kw}
+    kw = {"streams": 4, "residual_mult": 0.8, "embed_scale": width ** 0.5,
+          **kw}
     return register(layered_config(name, layers, width, vocab, norm="dyt",
                                    tie_embeddings=True, **kw))
 
