@@ -311,6 +311,27 @@ def test_delta_chunks_and_steps_agree(size):
             assert relative(a, ref.cpu()) < 2e-4
 
 
+def test_delta_chunks_of_long_portions():
+    """More chunks than the scratch memory holds at once, of two sequences,
+    against the steps."""
+    ps = portions((5000, 0, 0), (700, 300, 0), blocks=400)
+    T = 5700
+    lay, y, y2, conv, dec = delta_case((32, 4, 128, 128, 4, 16, 16), T, BF)
+    res = []
+    for expand in (True, False):
+        b = StepPlan(ps).build(16, [], DEV, expand=expand)
+        assert b.n_short == (0 if expand else 2)
+        st = DR.alloc_delta_state(2, lay, DEV, BF)
+        for x in st:
+            x.fill_(0.5)
+        o = torch.full((T, lay.n_o), float("nan"), device=DEV)
+        run = DR.delta_chunk if expand else DR.delta_step
+        run(y.to(DEV), y2.to(DEV), lay, conv.to(DEV), dec.to(DEV), st, b, o)
+        res.append((o, st[0]))
+    for a, ref in zip(*res):
+        assert relative(a, ref.cpu()) < 1e-3
+
+
 @pytest.mark.parametrize("batch", list(BATCHES) + ["long"])
 @pytest.mark.parametrize("dtype", [BF, F32])
 @pytest.mark.parametrize("R", [8, 40, 200, 1024])
