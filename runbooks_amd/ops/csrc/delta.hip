@@ -23,7 +23,7 @@
 //
 //    delta_prep, parallel over chunks, solves for both right sides and leaves
 //    what multiplies S or U as MFMA operands in lane order; delta_scan walks
-//    the chunks, 16 state columns per wave, all in registers. Exponents are
+//    the chunks, 16 state columns per two waves, in registers. Exponents are
 //    differences that are never positive. An fp32 factor enters a product as
 //    two bf16 parts, so the recurrence keeps fp32's quality.
 //  * delta_out: RMS norm per head, times weight and sigmoid gate; the
@@ -264,14 +264,19 @@ RB_DEV unsigned pack2(float lo, float hi) {
   c.b[1] = (__bf16)hi;
   return c.u;
 }
+// two floats as packed bf16 and the packed rest
+RB_DEV void split2(float x, float y, unsigned &big, unsigned &small) {
+  big = pack2(x, y);
+  small = pack2(x - __uint_as_float(big << 16),
+                y - __uint_as_float(big & 0xffff0000u));
+}
 RB_DEV void split8(const float *f, u32x4v &big, u32x4v &small) {
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const float x = f[2 * i], y = f[2 * i + 1];
-    const unsigned b = pack2(x, y);
+    unsigned b, s;
+    split2(f[2 * i], f[2 * i + 1], b, s);
     big[i] = b;
-    small[i] = pack2(x - __uint_as_float(b << 16),
-                     y - __uint_as_float(b & 0xffff0000u));
+    small[i] = s;
   }
 }
 
@@ -576,10 +581,12 @@ __global__ __launch_bounds__(PREP, 2) void delta_prep_kernel(Args a, int vb) {
 }
 
 // ---------------------------------------------------------------------------
-// chunks: the recurrence. One wave owns 16 state columns, as MFMA result
-// tiles: tile d, register r of a lane is S[16 d + 4 (lane / 16) + r]
-// [lane % 16]; two stacked tiles are, packed, an operand with the entries'
-// order of the summed index. So is U.
+// chunks: the recurrence. Two waves own 16 state columns, half of the rows
+// each, as MFMA result tiles: tile d, register r of a lane is
+// S[16 d + 4 (lane / 16) + r][lane % 16]; two stacked tiles are, packed, an
+// operand with the entries' order of the summed index. So is U. The waves give
+// each other their packed halves through LDS; the first one makes U, the
+// second one O.
 // ---------------------------------------------------------------------------
 union Frag { u32x4v u; bf16x8v v; };
 
@@ -592,11 +599,13 @@ RB_DEV f32x4v part(int i, const Frag *a, const Frag &bh, const Frag &bl,
   return mfma(a[i == 2], i == 1 ? bl : bh, c);
 }
 
-template <int DCP, bool AHEAD>
-__global__ __launch_bounds__(RB_WAVE, 1) void delta_scan_kernel(Args a) {
+template <int DCP>
+__global__ __launch_bounds__(2 * RB_WAVE, 1) void delta_scan_kernel(Args a) {
   using E = Entry<DCP>;
-  constexpr int KS = E::KS, TD = E::TD;
-  const int lane = threadIdx.x, l16 = lane & 15, grp = lane >> 4;
+  constexpr int KS = E::KS, HT = E::TD / 2;    // state tiles per wave
+  __shared__ u32x4v s_s[2][KS][64], u_s[2][64];
+  const int lane = threadIdx.x & 63, l16 = lane & 15, grp = lane >> 4;
+  const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int h = blockIdx.x % a.heads, cb = blockIdx.x / a.heads;
   const int seq = a.first_seq + blockIdx.z;
   const int q0 = a.cu_q[seq], n = a.cu_q[seq + 1] - q0;
@@ -606,115 +615,128 @@ __global__ __launch_bounds__(RB_WAVE, 1) void delta_scan_kernel(Args a) {
   const bool col_ok = col < a.vc;
   float *st = a.state + ((int64_t)a.slots[seq] * a.heads + h) * a.dc * a.vc;
   const bool zero = a.chunk0 == 0 && a.positions[q0] == 0;
-  f32x4v S[TD];
+  f32x4v S[HT];
 #pragma unroll
-  for (int d = 0; d < TD; ++d)
+  for (int d = 0; d < HT; ++d)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int dim = d * 16 + grp * 4 + r;
+      const int dim = (wid * HT + d) * 16 + grp * 4 + r;
       S[d][r] = !zero && col_ok && dim < a.dc
                     ? st[(int64_t)dim * a.vc + col] : 0.0f;
     }
   const int64_t stride = a.heads * a.entry;
   const char *base = a.scratch +
                      ((int64_t)blockIdx.z * a.chunks * a.heads + h) * a.entry;
-  const int lb = lane * 16;
+  const int64_t orow = (int64_t)a.heads * a.vc;
+  float *op = a.o + (int64_t)(q0 + a.chunk0 * C + grp * 4) * orow + h * a.vc +
+              col;
+  int left = n - a.chunk0 * C - grp * 4;       // tokens from this lane's on
 
-  Frag wf[2 * KS][2], qf[2 * KS][2], pf[2][2], kf[TD][2];
-  f32x4v gf[TD], uf[2];
-  auto get = [&](Frag *f, const char *e, int at) {
-    f[0].u = *reinterpret_cast<const u32x4v *>(e + at + lb);
-    f[1].u = *reinterpret_cast<const u32x4v *>(e + at + 1024 + lb);
+  // what multiplies S (-W and U, or Q), and what multiplies U
+  Frag ff[2 * KS][2], pf[2][2], kf[HT][2];
+  f32x4v gf[HT], uf[2];
+  auto get = [&](Frag *f, const char *e) __attribute__((always_inline)) {
+    f[0].u = *reinterpret_cast<const u32x4v *>(e + lane * 16);
+    f[1].u = *reinterpret_cast<const u32x4v *>(e + 1024 + lane * 16);
   };
-  auto get_w = [&](const char *e) {
+  auto get_f = [&](const char *e) __attribute__((always_inline)) {
+    const char *f = e + (wid == 0 ? E::W : E::Q);
+#pragma unroll
+    for (int i = 0; i < 2 * KS; ++i) get(ff[i], f + i * E::OP);
 #pragma unroll
     for (int i = 0; i < 2; ++i)
       uf[i] = *reinterpret_cast<const f32x4v *>(e + E::U + cb * 2048 +
-                                                i * 1024 + lb);
-#pragma unroll
-    for (int i = 0; i < 2 * KS; ++i) get(wf[i], e, E::W + i * E::OP);
+                                                i * 1024 + lane * 16);
   };
-  auto get_q = [&](const char *e) {
+  auto get_k = [&](const char *e) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < 2 * KS; ++i) get(qf[i], e, E::Q + i * E::OP);
+    for (int i = 0; i < 2; ++i) get(pf[i], e + E::P + i * E::OP);
 #pragma unroll
-    for (int i = 0; i < 2; ++i) get(pf[i], e, E::P + i * E::OP);
-  };
-  auto get_k = [&](const char *e) {
-#pragma unroll
-    for (int d = 0; d < TD; ++d) {
-      get(kf[d], e, E::K + d * E::OP);
+    for (int d = 0; d < HT; ++d) {
+      const int t = wid * HT + d;
+      get(kf[d], e + E::K + t * E::OP);
       gf[d] = *reinterpret_cast<const f32x4v *>(e + E::G +
-                                                (d * 16 + grp * 4) * 4);
+                                                (t * 16 + grp * 4) * 4);
     }
   };
-  if constexpr (AHEAD) {
-    get_w(base);
-    get_q(base);
-    get_k(base);
-  }
+  get_f(base);
+  get_k(base);
   for (int c = 0; c < nc; ++c) {
-    const char *e = base + c * stride;
     const char *next = base + min(c + 1, nc - 1) * stride;
-    if constexpr (!AHEAD) get_w(e);
+#pragma unroll
+    for (int d = 0; d < HT; ++d) {
+      const int t = wid * HT + d;
+      uint2 big, small;
+      split2(S[d][0], S[d][1], big.x, small.x);
+      split2(S[d][2], S[d][3], big.y, small.y);
+      reinterpret_cast<uint2 *>(&s_s[0][t >> 1][lane])[t & 1] = big;
+      reinterpret_cast<uint2 *>(&s_s[1][t >> 1][lane])[t & 1] = small;
+    }
+    __syncthreads();                           // S; U has been read
     Frag sh[KS], sl[KS];
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
-      const float f[8] = {S[2 * ks][0],     S[2 * ks][1],     S[2 * ks][2],
-                          S[2 * ks][3],     S[2 * ks + 1][0],
-                          S[2 * ks + 1][1], S[2 * ks + 1][2],
-                          S[2 * ks + 1][3]};
-      split8(f, sh[ks].u, sl[ks].u);
+      sh[ks].u = s_s[0][ks][lane];
+      sl[ks].u = s_s[1][ks][lane];
     }
-    f32x4v u[2] = {uf[0], uf[1]}, o[2] = {(f32x4v)(0.0f), (f32x4v)(0.0f)};
-    if constexpr (!AHEAD) get_q(e);
-    // four sums side by side
+    f32x4v x[2];                               // U, or what S gives to O
+#pragma unroll
+    for (int m = 0; m < 2; ++m) x[m] = wid == 0 ? uf[m] : (f32x4v)(0.0f);
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
       for (int i = 0; i < 3; ++i)
 #pragma unroll
-        for (int m = 0; m < 2; ++m) {
-          u[m] = part(i, wf[m * KS + ks], sh[ks], sl[ks], u[m]);
-          o[m] = part(i, qf[m * KS + ks], sh[ks], sl[ks], o[m]);
-        }
-    if constexpr (AHEAD) get_w(next);
-    Frag uh, ul;
-    {
-      const float f[8] = {u[0][0], u[0][1], u[0][2], u[0][3],
-                          u[1][0], u[1][1], u[1][2], u[1][3]};
-      split8(f, uh.u, ul.u);
+        for (int m = 0; m < 2; ++m)
+          x[m] = part(i, ff[m * KS + ks], sh[ks], sl[ks], x[m]);
+    __builtin_amdgcn_sched_barrier(0);
+    get_f(next);
+    __builtin_amdgcn_sched_barrier(0);
+    if (wid == 0) {
+      u32x4v big, small;
+      const float f[8] = {x[0][0], x[0][1], x[0][2], x[0][3],
+                          x[1][0], x[1][1], x[1][2], x[1][3]};
+      split8(f, big, small);
+      u_s[0][lane] = big;
+      u_s[1][lane] = small;
     }
-    if constexpr (!AHEAD) get_k(e);
 #pragma unroll
-    for (int d = 0; d < TD; ++d)
+    for (int d = 0; d < HT; ++d)
 #pragma unroll
       for (int r = 0; r < 4; ++r) S[d][r] *= gf[d][r];
+    __syncthreads();                           // U; S has been read
+    Frag uh, ul;
+    uh.u = u_s[0][lane];
+    ul.u = u_s[1][lane];
 #pragma unroll
-    for (int i = 0; i < 3; ++i) {
+    for (int i = 0; i < 3; ++i)
 #pragma unroll
-      for (int m = 0; m < 2; ++m) o[m] = part(i, pf[m], uh, ul, o[m]);
+      for (int d = 0; d < HT; ++d) S[d] = part(i, kf[d], uh, ul, S[d]);
+    if (wid == 1) {
 #pragma unroll
-      for (int d = 0; d < TD; ++d) S[d] = part(i, kf[d], uh, ul, S[d]);
+      for (int i = 0; i < 3; ++i)
+#pragma unroll
+        for (int m = 0; m < 2; ++m) x[m] = part(i, pf[m], uh, ul, x[m]);
     }
-    if constexpr (AHEAD) get_q(next);
-    if constexpr (AHEAD) get_k(next);
-    const int t = (a.chunk0 + c) * C + grp * 4;
-    if (col_ok)
+    __builtin_amdgcn_sched_barrier(0);
+    get_k(next);
+    __builtin_amdgcn_sched_barrier(0);
+    if (wid == 1 && col_ok) {
 #pragma unroll
       for (int m = 0; m < 2; ++m)
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (t + m * 16 + r < n)
-            a.o[(int64_t)(q0 + t + m * 16 + r) * a.heads * a.vc + h * a.vc +
-                col] = o[m][r];
+          if (m * 16 + r < left) op[(m * 16 + r) * orow] = x[m][r];
+    }
+    op += C * orow;
+    left -= C;
   }
   if (!col_ok) return;
 #pragma unroll
-  for (int d = 0; d < TD; ++d)
+  for (int d = 0; d < HT; ++d)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int dim = d * 16 + grp * 4 + r;
+      const int dim = (wid * HT + d) * 16 + grp * 4 + r;
       if (dim < a.dc) st[(int64_t)dim * a.vc + col] = S[d][r];
     }
 }
@@ -903,8 +925,8 @@ void launch_chunk(Args a, int64_t n_seqs, int64_t max_q,
     hipLaunchKernelGGL((delta_prep_kernel<DCP>),
                        dim3(a.heads, a.chunks, n_seqs), dim3(PREP), shmem,
                        stream, a, vb);
-    hipLaunchKernelGGL((delta_scan_kernel<DCP, DCP <= 128>), scan,
-                       dim3(RB_WAVE), 0, stream, a);
+    hipLaunchKernelGGL((delta_scan_kernel<DCP>), scan, dim3(2 * RB_WAVE), 0,
+                       stream, a);
   }
 }
 
