@@ -7,13 +7,16 @@ own runtime.
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 
 
 @dataclass(frozen=True)
 class LatentAttentionSpec:
     """Latent attention: keys and values are linear images of one cached
-    latent per token (plus one rotated key part all heads share)."""
+    latent per token (plus one rotated key part all heads share, unless
+    rot_dim is 0). A sigmoid gate on the result, one per value column or,
+    with head_gate, one per head."""
     heads: int
     dim: int                        # unrotated query/key size per head
     rot_dim: int                    # rotated query/key size per head
@@ -24,9 +27,13 @@ class LatentAttentionSpec:
     rope_dims: int | None = None    # rotated part of rot_dim (None: all)
     window: int | None = None       # keys a query sees, itself included
     kv_from: int | None = None      # layer whose latents this layer reads
+    q_rank: int | None = None       # latent of the queries (None: direct)
+    head_gate: bool = False
 
     @property
-    def rotation(self) -> tuple[float, int]:
+    def rotation(self) -> tuple[float, int] | None:
+        if self.rot_dim == 0:
+            return None
         return (self.rope_base, self.rope_dims or self.rot_dim)
 
 
@@ -144,6 +151,48 @@ class TwinSpec:
 
 
 @dataclass(frozen=True)
+class GeneralDeltaSpec:
+    """Generalized delta rule with a decay w and a removal rate a per head
+    and key channel: S <- diag(w) S - (a u)(u^T S) + k v^T with u = k / |k|,
+    o = S^T r; RMS norm per head, sigmoid gate. w = exp(decay_scale
+    sigmoid(..)) comes through a tanh bottleneck."""
+    heads: int
+    dim: int
+    decay_rank: int
+    decay_scale: float = -math.exp(-0.5)
+
+    rotation = None
+
+    @property
+    def vdim(self):
+        return self.dim
+
+
+@dataclass(frozen=True)
+class DiffAttentionSpec:
+    """Differential attention: two attention maps per head over the same
+    values, the second one subtracted times a learned factor, RMS norm per
+    head. Biased q, k, v pass a short causal convolution; no rotation."""
+    heads: int
+    kv_heads: int
+    dim: int                        # query/key size per head and map
+    vdim: int
+    scale: float                    # factor on the scores
+    diff: float                     # constant part of the factor
+    conv: int                       # taps of the convolution
+    window: int | None = None       # keys a query sees, itself included
+
+    rotation = None
+
+
+@dataclass(frozen=True)
+class PolyNormSpec:
+    """Feed-forward down(a N(z) + b N(z^2) + c N(z^3) + e), z = up, N an RMS
+    norm over all ff values."""
+    ff: int
+
+
+@dataclass(frozen=True)
 class SquaredReluSpec:
     """Feed-forward down(relu(up)^2)."""
     ff: int
@@ -171,18 +220,19 @@ class GLUSpec:
 
 @dataclass(frozen=True)
 class LayerSpec:
-    """One layer of a model whose layers differ, on a 32-bit residual. With
-    a latent mixer both sublayers read the same normed input and are summed;
-    with the others they follow each other, each behind a norm of its own."""
+    """One layer of a model whose layers differ, on a 32-bit residual.
+    ModelConfig.layout says how its sublayers follow each other."""
     mixer: (LatentAttentionSpec | SharedKVAttentionSpec | LightningSpec |
-            GatedDeltaSpec | TwinSpec)
-    mlp: GatedMLPSpec | GLUSpec | SquaredReluSpec | MoESpec | None
+            GatedDeltaSpec | TwinSpec | GeneralDeltaSpec | DiffAttentionSpec)
+    mlp: (GatedMLPSpec | GLUSpec | SquaredReluSpec | MoESpec | PolyNormSpec |
+          None)
     weights_of: int | None = None   # layer whose parameters this one uses
 
     @property
     def attends(self) -> bool:
         """The mixer reads cached keys."""
-        return not isinstance(self.mixer, (LightningSpec, GatedDeltaSpec))
+        return not isinstance(self.mixer, (LightningSpec, GatedDeltaSpec,
+                                           GeneralDeltaSpec))
 
     @property
     def reach(self) -> int | None:
@@ -205,10 +255,12 @@ class LayerSpec:
 class LoopSpec:
     """Layers start .. stop - 1 run `times` times in a row with the same
     weights, each pass on a cache of its own, behind a projection of
-    [residual; embedding output] that replaces the residual."""
+    [residual; embedding output] that replaces the residual; with `step`, a
+    learned vector of the pass is then added."""
     start: int
     stop: int
     times: int
+    step: bool = False
 
 
 @dataclass
@@ -246,6 +298,11 @@ class ModelConfig:
     # the factor on a sublayer's result that goes with them
     streams: int | None = None
     residual_mult: float = 1.0
+    # taps of a causal convolution that every sublayer's normed input passes
+    # (None: none); such sublayers run in parallel, each behind its own norm
+    canon: int | None = None
+    norm_offset: float = 0.0  # added to the weights of RMS norms
+    logit_softcap: float | None = None   # logits -> cap tanh(logits / cap)
 
     def __post_init__(self):
         if self.layers is not None:
@@ -255,16 +312,30 @@ class ModelConfig:
             self.head_dim = self.hidden_size // self.num_heads
 
     @property
-    def layer_runs(self) -> list[tuple[int, bool]]:
-        """(layer, starts a loop pass) in the order of execution."""
+    def layout(self) -> str:
+        """How a layer-by-layer model's sublayers meet: "streams" (several
+        residuals with learned mixing), "dual" (in parallel, each behind a
+        norm and input convolution of its own), "shared" (in parallel on one
+        normed input) or "sequence" (one after the other)."""
+        if self.streams is not None:
+            return "streams"
+        if self.canon is not None:
+            return "dual"
+        latent = isinstance(self.layers[0].mixer, LatentAttentionSpec)
+        return "shared" if latent else "sequence"
+
+    @property
+    def layer_runs(self) -> list[tuple[int, int | None]]:
+        """(layer, number of the loop pass it starts or None) in the order
+        of execution."""
         n, loop = len(self.layers), self.loop
         if loop is None:
-            return [(self.owner(i), False) for i in range(n)]
+            return [(self.owner(i), None) for i in range(n)]
         body = range(loop.start, loop.stop)
-        return ([(i, False) for i in range(loop.start)] +
-                [(i, i == loop.start) for _ in range(loop.times)
-                 for i in body] +
-                [(i, False) for i in range(loop.stop, n)])
+        return ([(i, None) for i in range(loop.start)] +
+                [(i, t if i == loop.start else None)
+                 for t in range(loop.times) for i in body] +
+                [(i, None) for i in range(loop.stop, n)])
 
     def owner(self, i: int) -> int:
         """The layer whose parameters layer i uses."""
@@ -288,33 +359,43 @@ class ModelConfig:
         """Kernel modules (ops/build.py) that serving this model needs."""
         if self.layers is None:
             return ("core", "main")
-        if self.streams is not None:
-            return ("core", "hybrid", "streams")
-        latent = any(isinstance(lay.mixer, LatentAttentionSpec)
-                     for lay in self.layers)
-        return ("core", "latent" if latent else "hybrid")
+        need = {LatentAttentionSpec: "latent",
+                SharedKVAttentionSpec: "shared_kv",
+                LightningSpec: "lightning", GatedDeltaSpec: "delta",
+                GeneralDeltaSpec: "delta", DiffAttentionSpec: "shared_kv",
+                TwinSpec: "shared_kv"}
+        groups = {need[type(lay.mixer)] for lay in self.layers}
+        groups |= {self.layout} & {"streams", "dual"}
+        return ("core", *sorted(groups))
 
     def _check_layers(self):
         checks = {LatentAttentionSpec: self._check_latent,
                   SharedKVAttentionSpec: self._check_shared_kv,
                   LightningSpec: self._check_lightning,
                   GatedDeltaSpec: self._check_delta,
-                  TwinSpec: self._check_twin}
+                  TwinSpec: self._check_twin,
+                  GeneralDeltaSpec: self._check_general_delta,
+                  DiffAttentionSpec: self._check_diff}
+        # what a layout's layers may consist of
+        mixers, mlps = {
+            "streams": ((GatedDeltaSpec, TwinSpec),
+                        (SquaredReluSpec, MoESpec)),
+            "dual": ((GeneralDeltaSpec, DiffAttentionSpec,
+                      LatentAttentionSpec), (PolyNormSpec,)),
+            "shared": ((LatentAttentionSpec,), (GatedMLPSpec,)),
+            "sequence": ((SharedKVAttentionSpec, LightningSpec), (GLUSpec,)),
+        }[self.layout]
         for i, lay in enumerate(self.layers):
+            if not isinstance(lay.mixer, mixers):
+                raise ValueError(f"layer {i}: no {lay.mixer} in the layout "
+                                 f"{self.layout!r}")
             if getattr(lay.mixer, "window", None) is not None and \
                     lay.mixer.window < 1:
                 raise ValueError(f"layer {i}: window {lay.mixer.window}")
             checks[type(lay.mixer)](i, lay.mixer)
-            kinds = ((SquaredReluSpec, MoESpec) if self.streams is not None
-                     else GatedMLPSpec
-                     if isinstance(lay.mixer, LatentAttentionSpec)
-                     else GLUSpec)
             if lay.mlp is not None and (
-                    lay.mlp.ff < 1 or not isinstance(lay.mlp, kinds)):
+                    lay.mlp.ff < 1 or not isinstance(lay.mlp, mlps)):
                 raise ValueError(f"layer {i}: mlp {lay.mlp}")
-            if isinstance(lay.mixer, (GatedDeltaSpec, TwinSpec)) != \
-                    (self.streams is not None):
-                raise ValueError(f"layer {i}: residual of {lay.mixer}")
             if isinstance(lay.mlp, MoESpec):
                 self._check_moe(i, lay.mlp)
             self._check_owner(i, lay)
@@ -332,6 +413,11 @@ class ModelConfig:
         if self.streams is not None and (self.streams < 1 or self.loop or
                                          self.norm != "dyt"):
             raise ValueError(f"bad streams {self.streams}")
+        if self.canon is not None and (self.canon < 1 or
+                                       self.norm != "rmsnorm"):
+            raise ValueError(f"bad input convolution {self.canon}")
+        if self.logit_softcap is not None and self.logit_softcap <= 0:
+            raise ValueError(f"bad logit_softcap {self.logit_softcap}")
 
     def _check_owner(self, i, lay):
         """Layer i's weights_of leads to a layer like it that has some."""
@@ -358,6 +444,16 @@ class ModelConfig:
                 (a.chunk is not None and a.chunk < 1):
             raise ValueError(f"layer {i}: bad mixer sizes {m}")
 
+    def _check_general_delta(self, i, m):
+        if min(m.heads, m.dim, m.decay_rank) < 1 or \
+                not -2.0 <= m.decay_scale <= 0.0:
+            raise ValueError(f"layer {i}: bad mixer sizes {m}")
+
+    def _check_diff(self, i, m):
+        if min(m.heads, m.kv_heads, m.dim, m.vdim, m.conv) < 1 or \
+                m.heads % m.kv_heads:
+            raise ValueError(f"layer {i}: bad mixer sizes {m}")
+
     def _check_moe(self, i, m):
         if m.experts < 1 or m.groups < 1 or m.experts % m.groups or \
                 not 1 <= m.keep <= m.groups or m.shared_ff < 0 or \
@@ -365,9 +461,17 @@ class ModelConfig:
             raise ValueError(f"layer {i}: bad mixture {m}")
 
     def _check_latent(self, i, m):
-        if min(m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank) < 1 or \
-                m.rotation[1] % 2 or m.rotation[1] > m.rot_dim:
+        rot = m.rotation[1] if m.rotation else 0
+        q_rank = 1 if m.q_rank is None else m.q_rank
+        if min(m.heads, m.dim, m.vdim, m.kv_rank, q_rank) < 1 or \
+                rot % 2 or not 0 <= rot <= m.rot_dim:
             raise ValueError(f"layer {i}: bad mixer sizes {m}")
+        # the "dual" layout has the one form, the "shared" one the other
+        dual = self.layout == "dual"
+        if (m.q_rank is not None, m.head_gate, m.rot_dim == 0) != (dual,) * 3 \
+                or (dual and m.kv_from is not None):
+            raise ValueError(f"layer {i}: latent attention {m} in the layout "
+                             f"{self.layout!r}")
         if m.kv_from is None:
             return
         if not 0 <= m.kv_from < i:
@@ -409,12 +513,22 @@ class ModelConfig:
                     a = m.left
                     n += h * (a.heads + a.kv_heads) * (a.dim + a.vdim) + \
                         4 * h * m.right.width
+                elif isinstance(m, GeneralDeltaSpec):
+                    n += m.heads * m.dim * (6 * h + m.decay_rank) + \
+                        h * m.decay_rank
+                elif isinstance(m, DiffAttentionSpec):
+                    n += h * (m.heads + m.kv_heads) * (2 * m.dim + m.vdim)
+                elif m.q_rank is not None:
+                    n += m.q_rank * (h + m.heads * m.dim) + \
+                        m.kv_rank * (h + m.heads * (m.dim + m.vdim)) + \
+                        h * m.heads * (1 + m.vdim)
                 else:
                     n += h * m.heads * (m.dim + m.rot_dim + 2 * m.vdim) + \
                         m.kv_rank * m.heads * (m.dim + m.vdim)
                     if m.kv_from is None:
                         n += h * (m.kv_rank + m.rot_dim)
-                if isinstance(lay.mlp, (MoESpec, SquaredReluSpec)):
+                if isinstance(lay.mlp, (MoESpec, SquaredReluSpec,
+                                        PolyNormSpec)):
                     n += 2 * h * (lay.mlp.ff * getattr(lay.mlp, "experts", 1)
                                   + getattr(lay.mlp, "shared_ff", 0))
                 elif lay.mlp is not None:
@@ -442,9 +556,8 @@ def layered_config(name: str, layers, width: int, vocab: int,
     outside every attention layer's window."""
     layers = tuple(layers)
     mixers = [lay.mixer for lay in layers]
-    latent = isinstance(mixers[0], LatentAttentionSpec)
-    if any(isinstance(m, LatentAttentionSpec) != latent for m in mixers):
-        raise ValueError("latent layers do not mix with others")
+    latent = isinstance(mixers[0], LatentAttentionSpec) and \
+        kw.get("canon") is None
     # sizes of the attention (a twin mixer's left side)
     heads = [getattr(m, "left", m) for m in mixers]
     windows = [lay.reach for lay in layers if lay.attends]
@@ -727,3 +840,51 @@ _gokapel("gokapel-1b", "DpPd" * 4, 2048, 32000, 8192,
          dict(heads=32, kv_heads=32, dim=64, vdim=64, scale=64 ** -0.5,
               rope_dims=32, rope_base=500000.0, chunk=2048), 2048,
          max_seq_len=32768)
+
+
+# --- Dopilorn family (generalized delta rule, differential and positionless
+# latent attention beside a PolyNorm unit, each behind a norm and an input
+# convolution; a looped stretch of layers) --------------------------------------
+def _dopilorn(name: str, pattern: str, width: int, vocab: int, ff: int,
+              delta: dict, attention: dict, latent: dict, loop=None,
+              **kw) -> ModelConfig:
+    """`pattern`: one letter a layer, D delta, A attention or L latent
+    attention (upper case with a feed-forward, lower case without)."""
+    made = {"d": GeneralDeltaSpec(**delta),
+            "a": DiffAttentionSpec(**attention),
+            "l": LatentAttentionSpec(rot_dim=0, head_gate=True, **latent)}
+    layers = [LayerSpec(made[c.lower()],
+                        PolyNormSpec(ff) if c.isupper() else None)
+              for c in pattern]
+    kw = {"canon": 4, "logit_softcap": 30.0, "norm_offset": 1.0, **kw}
+    return register(layered_config(
+        name, layers, width, vocab,
+        loop=loop and LoopSpec(*loop, step=True), **kw))
+
+
+_dopilorn("tiny-dopilorn", "AdLD", 64, 256, 96,
+          dict(heads=3, dim=16, decay_rank=8),
+          dict(heads=4, kv_heads=2, dim=12, vdim=24, scale=12 ** -0.5,
+               diff=0.5, conv=3, window=24),
+          dict(heads=3, dim=16, vdim=24, q_rank=40, kv_rank=24,
+               scale=0.25), loop=(1, 3, 2), max_seq_len=256)
+_dopilorn("smoke-dopilorn", "ALdA", 256, 512, 512,
+          dict(heads=4, dim=64, decay_rank=32),
+          dict(heads=4, kv_heads=2, dim=32, vdim=64, scale=32 ** -0.5,
+               diff=0.5, conv=3, window=80),
+          dict(heads=4, dim=64, vdim=64, q_rank=96, kv_rank=64, scale=0.125),
+          loop=(1, 3, 2), max_seq_len=1024)
+# layers of the width of llama2-7b and llama-1b and with about as many
+# parameters
+_dopilorn("dopilorn-7b", "ADLD" * 4, 4096, 32000, 16384,
+          dict(heads=32, dim=128, decay_rank=128),
+          dict(heads=16, kv_heads=16, dim=128, vdim=256, scale=128 ** -0.5,
+               diff=0.5, conv=4, window=4096),
+          dict(heads=32, dim=128, vdim=128, q_rank=1536, kv_rank=512,
+               scale=128 ** -0.5), max_seq_len=32768)
+_dopilorn("dopilorn-1b", "ADLD" * 4, 2048, 32000, 8192,
+          dict(heads=16, dim=128, decay_rank=64),
+          dict(heads=16, kv_heads=16, dim=64, vdim=128, scale=64 ** -0.5,
+               diff=0.5, conv=4, window=2048),
+          dict(heads=32, dim=64, vdim=64, q_rank=768, kv_rank=256,
+               scale=64 ** -0.5), max_seq_len=32768)

@@ -15,16 +15,14 @@ from pathlib import Path
 
 import torch
 
-from .config import LatentAttentionSpec, ModelConfig
+from .config import ModelConfig
 from .transformer import Transformer
 
 
 def detect_family(cfg: ModelConfig) -> str:
     if cfg.layers is not None:
-        if cfg.streams is not None:
-            return "gokapel"
-        latent = isinstance(cfg.layers[0].mixer, LatentAttentionSpec)
-        return "pimazen" if latent else "keralorn"
+        return {"streams": "gokapel", "dual": "dopilorn", "shared": "pimazen",
+                "sequence": "keralorn"}[cfg.layout]
     if cfg.pos == "learned":
         return "gpt2" if cfg.act == "gelu_tanh" else "opt"
     if cfg.parallel_residual:
@@ -183,6 +181,34 @@ def _map_gokapel(name: str, cfg: ModelConfig):
     return name
 
 
+_DOPILORN = {
+    **{f"mix.{n}": f"mixer.{n}_proj.weight" for n in
+       ("q", "k", "v", "o", "r", "a", "g", "w1", "w2", "dq", "uq", "dkv",
+        "uk", "uv")},
+    **{f"mix.{n}.b": f"mixer.{n}_proj.bias" for n in ("q", "k", "v", "a")},
+    **{f"mix.{n}.conv": f"mixer.{n}_conv" for n in ("q", "k", "v")},
+    **{f"mix.{n}": f"mixer.{n}" for n in
+       ("lq1", "lk1", "lq2", "lk2", "w0")},
+    "mix.norm": "mixer.norm.weight", "mix.dq.norm": "mixer.q_norm.weight",
+    "mix.dkv.norm": "mixer.kv_norm.weight",
+    "mlp.up": "mlp.up_proj.weight", "mlp.down": "mlp.down_proj.weight",
+    "mlp.act": "mlp.act",
+    **{f"norm{n}": f"norm{n}.weight" for n in "12"},
+    **{f"canon{n}": f"canon{n}" for n in "12"}}
+_DOPILORN_TOP = {"embed": "embed.weight", "final.norm": "norm_f.weight",
+                 "head": "lm_head.weight", "loop.in": "loop_in.weight",
+                 "loop.step": "loop_step"}
+
+
+def _map_dopilorn(name: str):
+    if name in _DOPILORN_TOP:
+        return _DOPILORN_TOP[name]
+    layer, _, rest = name.partition(".")
+    if layer[:1] == "l" and layer[1:].isdigit() and rest in _DOPILORN:
+        return f"blocks.{layer[1:]}.{_DOPILORN[rest]}"
+    return name
+
+
 def _split_falcon_qkv(w: torch.Tensor, cfg: ModelConfig):
     """Falcon fuses QKV as [n_kv_groups, (g_q + 2), head_dim, hidden] with
     the group's q heads followed by its k and v head."""
@@ -201,7 +227,7 @@ def convert_hf_state_dict(hf_state: dict, cfg: ModelConfig) -> dict:
     mapper = {"llama": _map_llama, "opt": _map_opt,
               "falcon": _map_falcon, "gpt2": _map_gpt2,
               "pimazen": _map_pimazen,
-              "keralorn": _map_keralorn,
+              "keralorn": _map_keralorn, "dopilorn": _map_dopilorn,
               "gokapel": lambda n: _map_gokapel(n, cfg)}[family]
     for name, w in hf_state.items():
         if name.endswith(".rotary_emb.inv_freq"):
@@ -518,6 +544,107 @@ def config_to_gokapel(cfg: ModelConfig) -> dict:
             "max_seq_len": cfg.max_seq_len}
 
 
+def config_from_dopilorn(d: dict, shapes: dict, name: str = "dopilorn"
+                         ) -> ModelConfig:
+    """ModelConfig from a Dopilorn config.json and the shapes of its tensors
+    (the inner size of the delta mixer's decay projection stands only there).
+    A type or kind this framework does not have is an error; an unknown key
+    is reported."""
+    from .config import (DiffAttentionSpec, GeneralDeltaSpec,
+                         LatentAttentionSpec, LayerSpec, LoopSpec,
+                         PolyNormSpec, layered_config)
+
+    def delta(m, where, i):
+        _only(m, ("heads", "dim"), where)
+        full = f"l{i}.mix.w1"
+        if full not in shapes:
+            raise ValueError(f"no tensor {full} to take a size from")
+        return GeneralDeltaSpec(m["heads"], m["dim"], shapes[full][0])
+
+    def attention(m, where, i):
+        _only(m, ("heads", "kv_heads", "dim", "vdim", "scale", "diff", "conv",
+                  "mask"), where)
+        mask = _only(m.get("mask") or {}, ("size",), where)
+        return DiffAttentionSpec(
+            m["heads"], m["kv_heads"], m["dim"], m["vdim"],
+            float(m["scale"]), float(m["diff"]), m["conv"], mask.get("size"))
+
+    def latent(m, where, i):
+        _only(m, ("heads", "dim", "vdim", "q_rank", "kv_rank", "scale"),
+              where)
+        return LatentAttentionSpec(
+            heads=m["heads"], dim=m["dim"], rot_dim=0, vdim=m["vdim"],
+            kv_rank=m["kv_rank"], scale=float(m["scale"]),
+            q_rank=m["q_rank"], head_gate=True)
+
+    mixers = {"general_delta": delta, "attention": attention,
+              "latent_attention": latent}
+    _only(d, ("architecture", "canon", "layers", "logit_softcap", "loop",
+              "norm", "vocab", "width", "max_seq_len"), "config")
+    layers = []
+    for i, lay in enumerate(d["layers"]):
+        where = f"layer {i}"
+        _only(lay, ("type", "mixer", "mlp"), where)
+        if lay["type"] not in mixers:
+            raise ValueError(f"{where}: type {lay['type']!r}")
+        mlp = lay.get("mlp")
+        if mlp is not None:
+            _only(mlp, ("kind", "ff"), where)
+            if mlp["kind"] != "dense":
+                raise ValueError(f"{where}: mlp kind {mlp['kind']!r}")
+            mlp = PolyNormSpec(mlp["ff"])
+        layers.append(LayerSpec(mixers[lay["type"]](lay["mixer"], where, i),
+                                mlp))
+    loop = d.get("loop")
+    if loop is not None:
+        keys = ("start", "stop", "times")
+        loop = LoopSpec(*(_only(loop, keys, "loop")[k] for k in keys),
+                        step=True)
+    kw = {"max_seq_len": d["max_seq_len"]} if "max_seq_len" in d else {}
+    cap = d.get("logit_softcap")
+    return layered_config(
+        name, layers, d["width"], d["vocab"],
+        norm_eps=float(_only(d["norm"], ("eps",), "norm")["eps"]),
+        norm_offset=1.0, loop=loop,
+        canon=_only(d["canon"], ("taps",), "canon")["taps"],
+        logit_softcap=None if cap is None else float(cap), **kw)
+
+
+def config_to_dopilorn(cfg: ModelConfig) -> dict:
+    """The config.json of a Dopilorn model (inverse of
+    config_from_dopilorn)."""
+    from .config import DiffAttentionSpec, GeneralDeltaSpec
+    layers = []
+    for lay in cfg.layers:
+        m = lay.mixer
+        if isinstance(m, GeneralDeltaSpec):
+            kind, mixer = "general_delta", {"heads": m.heads, "dim": m.dim}
+        elif isinstance(m, DiffAttentionSpec):
+            kind = "attention"
+            mixer = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim,
+                     "vdim": m.vdim, "scale": m.scale, "diff": m.diff,
+                     "conv": m.conv}
+            if m.window is not None:
+                mixer["mask"] = {"size": m.window}
+        else:
+            kind = "latent_attention"
+            mixer = {"heads": m.heads, "dim": m.dim, "vdim": m.vdim,
+                     "q_rank": m.q_rank, "kv_rank": m.kv_rank,
+                     "scale": m.scale}
+        layers.append({"type": kind, "mixer": mixer, "mlp": lay.mlp and
+                       {"kind": "dense", "ff": lay.mlp.ff}})
+    out = {"architecture": "Dopilorn", "canon": {"taps": cfg.canon},
+           "layers": layers, "norm": {"eps": cfg.norm_eps},
+           "vocab": cfg.vocab_size, "width": cfg.hidden_size,
+           "max_seq_len": cfg.max_seq_len}
+    if cfg.logit_softcap is not None:
+        out["logit_softcap"] = cfg.logit_softcap
+    if cfg.loop is not None:
+        out["loop"] = {k: getattr(cfg.loop, k)
+                       for k in ("start", "stop", "times")}
+    return out
+
+
 def config_from_pimazen(d: dict, name: str = "pimazen") -> ModelConfig:
     """ModelConfig from a Pimazen config.json. A layer type or kind this
     framework does not have is an error; an unknown key is reported."""
@@ -579,9 +706,9 @@ def config_to_pimazen(cfg: ModelConfig) -> dict:
 def config_from_dir(path: str | Path, default: str | None = None
                     ) -> ModelConfig:
     """The configuration of a checkpoint directory: a registered name or
-    explicit fields this framework wrote, a Pimazen, Keralorn or Gokapel
-    config, or an HF one; `default` names the registry entry of a directory
-    that says nothing."""
+    explicit fields this framework wrote, a Pimazen, Keralorn, Gokapel or
+    Dopilorn config, or an HF one; `default` names the registry entry of a
+    directory that says nothing."""
     from .config import get_config, list_configs, register
     marker = Path(path) / "config.json"
     meta = json.loads(marker.read_text()) if marker.exists() else {}
@@ -604,6 +731,8 @@ def config_from_hf_json(path: str | Path) -> ModelConfig:
         readers = {"Pimazen": config_from_pimazen,
                    "Keralorn": config_from_keralorn,
                    "Gokapel": lambda d: config_from_gokapel(
+                       d, tensor_shapes(Path(path).parent)),
+                   "Dopilorn": lambda d: config_from_dopilorn(
                        d, tensor_shapes(Path(path).parent))}
         if d["architecture"] not in readers:
             raise ValueError(f"unsupported architecture {d['architecture']}")

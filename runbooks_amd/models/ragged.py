@@ -40,6 +40,7 @@ class RaggedBatch:
     seq_lens: torch.Tensor     # [B] int32, retained tokens incl. new ones
     block_tables: torch.Tensor  # [B, n] int32
     state_slots: torch.Tensor  # [B] int32
+    seq_of: torch.Tensor       # [T] int32, sequence of each token
     rows: torch.Tensor | None  # token rows whose logits are wanted (None: all)
     n_seqs: int
     # sequences [0, n_short) are short portions
@@ -52,6 +53,11 @@ class RaggedBatch:
     # first query)
     long_plans: dict = field(default_factory=dict)
     max_q_long: int = 0
+
+    @property
+    def single(self) -> bool:
+        """Every portion is one token."""
+        return self.n_short == self.n_seqs and self.max_q <= 1
 
 
 class StepPlan:
@@ -114,7 +120,9 @@ class StepPlan:
         parts = {"tokens": tokens, "positions": np.concatenate(positions),
                  "slots": np.concatenate(slots), "cu_q": cu,
                  "seq_lens": seq_lens, "tables": tables.reshape(-1),
-                 "states": [P[i].slot for i in order], "rows": rows}
+                 "states": [P[i].slot for i in order],
+                 "seq_of": np.repeat(np.arange(len(P)), np.diff(cu)),
+                 "rows": rows}
         for w in windows if n_short < len(P) else ():
             ctx, meta, at = [], [], 0
             for k, i in enumerate(order[n_short:], n_short):
@@ -132,7 +140,8 @@ class StepPlan:
             tokens=dev["tokens"].long(), positions=dev["positions"],
             slots=dev["slots"], cu_q=dev["cu_q"], seq_lens=dev["seq_lens"],
             block_tables=dev["tables"].view(len(P), width),
-            state_slots=dev["states"], rows=dev["rows"].long(),
+            state_slots=dev["states"], seq_of=dev["seq_of"],
+            rows=dev["rows"].long(),
             n_seqs=len(P), n_short=n_short, t_short=cu[n_short],
             max_q=max((len(P[i].tokens) for i in short), default=0),
             max_keys=max(seq_lens[:n_short], default=0),

@@ -111,7 +111,7 @@ class GatedDelta(nn.Module):
         if batch.n_seqs > batch.n_short:
             DR.delta_chunk(*args)
         z, swz = _new_z(self, y, self.out_w, filled=True)
-        DR.delta_out(o, lay, self.norm_w, y2, z, self.eps, swz, y, cache,
+        DR.delta_out(o, lay, self.norm_w, y2, z, self.eps, swz, y, cache[1],
                      batch)
         return z
 

@@ -8,7 +8,7 @@ One implementation, three family knobs (ModelConfig):
   * parallel_residual: falcon's attn+mlp-in-parallel block
   * GQA/MQA via num_kv_heads (llama2-70b 8, falcon-40b 8, falcon-7b 1)
   * layers: models described layer by layer (models/latent.py,
-    models/hybrid.py, models/streams.py)
+    models/hybrid.py, models/streams.py, models/dual.py)
 
 Forward modes:
   * ``forward(tokens)``             — training, full causal attention
@@ -41,6 +41,7 @@ from ..parallel import (
     gather_from_tp,
 )
 from .config import LatentAttentionSpec, ModelConfig
+from .dual import DualBlock
 from .hybrid import SequentialBlock
 from .latent import ParallelBlock
 from .ragged import RaggedBatch
@@ -49,7 +50,8 @@ from .streams import StreamBlock
 
 def _norm_module(cfg: ModelConfig, dtype):
     if cfg.norm == "rmsnorm":
-        return ops.RMSNorm(cfg.hidden_size, eps=cfg.norm_eps, dtype=dtype)
+        return ops.RMSNorm(cfg.hidden_size, eps=cfg.norm_eps, dtype=dtype,
+                           offset=cfg.norm_offset)
     if cfg.norm == "dyt":
         return ops.DynamicTanh(cfg.hidden_size, dtype=dtype)
     return nn.LayerNorm(cfg.hidden_size, eps=cfg.norm_eps, dtype=dtype)
@@ -291,12 +293,12 @@ class Transformer(nn.Module):
         # beside decoded tokens) through forward_ragged
         self.ragged = cfg.layers is not None
         if self.ragged:
-            latent = isinstance(cfg.layers[0].mixer, LatentAttentionSpec)
-            kind = (StreamBlock if cfg.streams is not None else
-                    ParallelBlock if latent else SequentialBlock)
+            kind = {"streams": StreamBlock, "dual": DualBlock,
+                    "shared": ParallelBlock,
+                    "sequence": SequentialBlock}[cfg.layout]
             self.blocks = nn.ModuleList(
                 kind(cfg, cfg.layers[i], dtype, self.tp) for i in cfg.owners)
-            # (layer, starts a loop pass), in the order of execution: a
+            # (layer, loop pass it starts), in the order of execution: a
             # looped layer, or one whose weights another layer uses, runs,
             # and has a cache, every time
             self.runs = cfg.layer_runs
@@ -305,6 +307,9 @@ class Transformer(nn.Module):
                 self.loop_in = ops.Linear(2 * cfg.hidden_size,
                                           cfg.hidden_size, bias=False,
                                           dtype=dtype)
+                if cfg.loop.step:
+                    self.loop_step = nn.Parameter(torch.zeros(
+                        cfg.loop.times, cfg.hidden_size, dtype=dtype))
         else:
             self.blocks = nn.ModuleList(Block(cfg, dtype, self.tp)
                                         for _ in range(cfg.num_layers))
@@ -440,7 +445,8 @@ class Transformer(nn.Module):
             return self.forward_ragged(RaggedBatch(
                 tokens=tokens, positions=positions, slots=slot_mapping,
                 cu_q=self._decode_cu[B], seq_lens=seq_lens,
-                block_tables=block_tables, state_slots=state_slots, rows=None,
+                block_tables=block_tables, state_slots=state_slots,
+                seq_of=self._decode_cu[B][:B], rows=None,
                 n_seqs=B, n_short=B, t_short=B, max_q=1, max_keys=None),
                 caches)
         x = self._embed(tokens.view(B, 1), positions)
@@ -487,8 +493,8 @@ class Transformer(nn.Module):
             x = (x * self.cfg.embed_scale)[:, None].repeat(
                 1, self.cfg.streams, 1)
         for (i, enters), cache in zip(self.runs, caches):
-            if enters:
-                x, delta = self._enter_pass(x, delta, x0)
+            if enters is not None:
+                x, delta = self._enter_pass(x, delta, x0, enters)
             r = self._rope_of[i]
             rope = None if r is None else (getattr(self, f"rope_cos_{r}"),
                                            getattr(self, f"rope_sin_{r}"))
@@ -501,8 +507,13 @@ class Transformer(nn.Module):
         w, n = self.lm_head.weight, x.shape[0]
         ready = ops.decode_ready(w, n)
         y = ops.norm_res32(self.norm_f, x, delta, self.dtype, operand=ready)
-        logits = (ops.fast_linear(y, w).float() if ready
-                  else ops.linear_f32(y, w))
+        if self.cfg.logit_softcap is not None:
+            logits = ops.softcap(
+                ops.decode_linear_raw(y, w, f32=True)[0] if ready
+                else ops.linear_f32(y, w), self.cfg.logit_softcap)
+        else:
+            logits = (ops.fast_linear(y, w).float() if ready
+                      else ops.linear_f32(y, w))
         return gather_from_tp(logits) if self._lm_vocab_parallel else logits
 
     def _head_of_streams(self, x, pending, rows):
@@ -523,16 +534,21 @@ class Transformer(nn.Module):
         self._all_streams = torch.ones(self.cfg.streams,
                                        device=self._norm_f_v.device)
 
-    def _enter_pass(self, x, delta, x0):
-        """The residual a loop pass starts from: one product of the residual
-        and the embedding output. Returns (x, pending part of it)."""
+    def _enter_pass(self, x, delta, x0, t: int):
+        """The residual loop pass t starts from: one product of the residual
+        and the embedding output, plus the pass's vector where there is one.
+        Returns (x, pending part of it)."""
         w = self.loop_in.weight
         ready = ops.decode_ready(w, x.shape[0])
         h = ops.join_res32(x, delta, x0, operand=ready)
-        if not ready:
-            return ops.linear_f32(h, w), None
-        slab = ops.decode_linear_raw(h, w, f32=True)[0]
-        return slab[0], slab[1:] if len(slab) > 1 else None
+        if ready:
+            slab = ops.decode_linear_raw(h, w, f32=True)[0]
+            x, delta = slab[0], slab[1:] if len(slab) > 1 else None
+        else:
+            x, delta = ops.linear_f32(h, w), None
+        if self.cfg.loop.step:
+            x += self.loop_step[t]
+        return x, delta
 
     # -- cache helpers ----------------------------------------------------------
     def local_kv_heads(self) -> int:

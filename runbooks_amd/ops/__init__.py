@@ -5,7 +5,7 @@ plain-PyTorch fp32 references (the numerics oracles). A GPU tensor with no
 built extension raises — there is no silent eager fallback on the GPU.
 """
 from ._backend import ext, has_hip, use_hip  # noqa: F401
-from .activations import cross_entropy, geglu, swiglu  # noqa: F401
+from .activations import cross_entropy, geglu, softcap, swiglu  # noqa: F401
 from .adamw import FusedAdamW  # noqa: F401
 from .attention import (causal_attention, flash_prefill, paged_decode,  # noqa: F401
                         paged_decode_ref, paged_decode_with_operand)

@@ -13,10 +13,10 @@ import importlib
 
 import torch
 
-# The kernels are built as five modules (setup.py): ops shared by every
-# served model, latent attention, attention on shared keys and values with
-# lightning attention, layers around residual streams, and the rest.
-_MODULES = ("_hip_core", "_hip_latent", "_hip_hybrid", "_hip_streams", "_hip")
+# The kernels are built as several modules (setup.py): ops shared by every
+# served model, one per kind of mixer or layer, and the rest.
+_MODULES = ("_hip_core", "_hip_latent", "_hip_shared_kv", "_hip_lightning",
+            "_hip_delta", "_hip_streams", "_hip_dual", "_hip")
 _BUILD_HINT = ("Run `PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext "
                "--inplace` at the repo root.")
 

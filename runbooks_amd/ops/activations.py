@@ -74,3 +74,13 @@ def cross_entropy(logits: torch.Tensor, targets: torch.Tensor,
                                      ignore_index)
     return torch.nn.functional.cross_entropy(
         flat_l.float(), flat_t.long(), ignore_index=ignore_index)
+
+
+def softcap(logits, cap: float):
+    """cap tanh(logits / cap) in fp32; logits [n, V], or an uncombined
+    split-K slab [split, n, V] of them."""
+    if not _backend.use_hip(logits):
+        if logits.dim() == 3:
+            logits = logits.sum(0)
+        return cap * torch.tanh(logits.float() / cap)
+    return _backend.ext().softcap(logits, cap)

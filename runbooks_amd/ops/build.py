@@ -9,9 +9,8 @@ from pathlib import Path
 
 _OPS = Path(__file__).parent
 _ROOT = _OPS.parent.parent
-_MODULE = {"core": "_hip_core", "latent": "_hip_latent",
-           "hybrid": "_hip_hybrid", "streams": "_hip_streams",
-           "main": "_hip"}
+_MODULE = {"main": "_hip", **{g: f"_hip_{g}" for g in (
+    "core", "latent", "shared_kv", "lightning", "delta", "streams", "dual")}}
 
 
 def _missing(groups) -> list[str]:

@@ -7,7 +7,7 @@ std::vector<at::Tensor> rmsnorm_fwd(at::Tensor x, at::Tensor w, double eps);
 std::vector<at::Tensor> rmsnorm_fwd_dec(at::Tensor x, at::Tensor w, double eps);
 std::vector<at::Tensor> rmsnorm_res_fwd_dec(at::Tensor x, at::Tensor res, at::Tensor w, double eps);
 std::vector<at::Tensor> rmsnorm_res_slab_fwd_dec(at::Tensor x, at::Tensor slabs, at::Tensor w, double eps);
-std::vector<at::Tensor> rmsnorm_res32(at::Tensor x, c10::optional<at::Tensor> delta, at::Tensor w, double eps, bool want_swz);
+std::vector<at::Tensor> rmsnorm_res32(at::Tensor x, c10::optional<at::Tensor> delta, at::Tensor w, double eps, bool want_swz, double offset);
 std::vector<at::Tensor> rmsnorm_bwd(at::Tensor x, at::Tensor w, at::Tensor dy,
                                     at::Tensor inv_rms);
 std::vector<at::Tensor> layernorm_res32(at::Tensor x, c10::optional<at::Tensor> delta, at::Tensor w, at::Tensor b, double eps, bool want_swz);

@@ -13,7 +13,12 @@ void latent_prep(at::Tensor y, at::Tensor cos, at::Tensor sin,
 void head_gemm(at::Tensor x, int64_t x_off, int64_t xh, at::Tensor w,
                int64_t K, int64_t N, at::Tensor out, int64_t o_off, int64_t oh,
                c10::optional<at::Tensor> gate, int64_t g_off,
-               c10::optional<at::Tensor> swz, int64_t T, int64_t H);
+               c10::optional<at::Tensor> swz, int64_t T, int64_t H,
+               bool head_gate);
+void latent_norms(at::Tensor y, int64_t oq, int64_t nq, at::Tensor wq,
+                  at::Tensor out, c10::optional<at::Tensor> swz, int64_t oc,
+                  int64_t nc, at::Tensor wc, at::Tensor cache,
+                  at::Tensor slots, double eps);
 int64_t latent_attend_rows(int64_t rows, int64_t rc, int64_t rotc, bool bf16);
 at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
                          int64_t q_head, at::Tensor cache,
@@ -23,13 +28,16 @@ at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
                          int64_t rc);
 void latent_flash(at::Tensor y, at::Tensor kv, at::Tensor ctx, at::Tensor meta,
                   at::Tensor z, int64_t heads, int64_t dimc, int64_t rotc,
-                  int64_t vc, int64_t rc, int64_t off_g, int64_t max_q,
-                  double scale, int64_t window);
+                  int64_t vc, int64_t rc, at::Tensor gate, int64_t off_g,
+                  bool head_gate, int64_t max_q, double scale,
+                  int64_t window);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "runbooks_amd gfx950 HIP kernels: latent attention";
   m.def("latent_prep", &latent_prep,
         "rotations, latent norm, cache write and gated activation");
+  m.def("latent_norms", &latent_norms,
+        "norms of the queries' and the cached latent");
   m.def("head_gemm", &head_gemm,
         "per-head product with an optional sigmoid gate");
   m.def("latent_attend_rows", &latent_attend_rows,

@@ -1,5 +1,5 @@
-// Python bindings of the residual streams, gated delta rule, minGRU, mixture
-// of experts and the preparation of queries, keys and values.
+// Python bindings of the residual streams, minGRU, mixture of experts and the
+// preparation of queries, keys and values.
 
 #include <torch/extension.h>
 
@@ -13,19 +13,6 @@ void qkv_prep(at::Tensor y, at::Tensor cos, at::Tensor sin,
               at::Tensor positions, at::Tensor slots, at::Tensor cache,
               at::Tensor norms, int64_t heads, int64_t dim, int64_t hc,
               double eps);
-void delta_step(at::Tensor y, at::Tensor y2, at::Tensor conv, at::Tensor decay,
-                at::Tensor state, at::Tensor tails, at::Tensor positions,
-                at::Tensor cu_q, at::Tensor slots, at::Tensor o,
-                int64_t n_seqs, int64_t kv, int64_t dim);
-void delta_chunk(at::Tensor y, at::Tensor y2, at::Tensor conv,
-                 at::Tensor decay, at::Tensor state, at::Tensor tails,
-                 at::Tensor positions, at::Tensor cu_q, at::Tensor slots,
-                 at::Tensor o, int64_t first_seq, int64_t n_seqs,
-                 int64_t max_q, int64_t kv, int64_t dim);
-void delta_out(at::Tensor o, at::Tensor w, at::Tensor y2, int64_t off_g,
-               at::Tensor z, Opt swz, int64_t vdim, double eps, at::Tensor y,
-               at::Tensor tails, at::Tensor positions, at::Tensor cu_q,
-               at::Tensor slots, int64_t n_seqs);
 void min_gru_step(at::Tensor y, int64_t off, at::Tensor bias, at::Tensor state,
                   at::Tensor positions, at::Tensor cu_q, at::Tensor slots,
                   int64_t first_seq, int64_t n_seqs, at::Tensor z,
@@ -43,18 +30,13 @@ at::Tensor moe_gemm(at::Tensor x, at::Tensor w, at::Tensor pairs,
                     bool down);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
-  m.doc() = "runbooks_amd gfx950 HIP kernels: residual streams, gated delta "
-            "rule, minGRU, mixture of experts";
+  m.doc() = "runbooks_amd gfx950 HIP kernels: residual streams, minGRU, "
+            "mixture of experts";
   m.def("streams_norm", &streams_norm,
         "streams += pending result; next sublayer's normed input");
   m.def("squared_relu", &squared_relu, "relu(y[:, :n])^2");
   m.def("qkv_prep", &qkv_prep,
         "norms and rotations of queries and keys, cache write");
-  m.def("delta_step", &delta_step, "gated delta rule, token after token");
-  m.def("delta_chunk", &delta_chunk,
-        "gated delta rule of long portions in chunks");
-  m.def("delta_out", &delta_out,
-        "norm per head times sigmoid gate; the convolutions' last inputs");
   m.def("min_gru_step", &min_gru_step, "minGRU, token after token");
   m.def("min_gru_scan", &min_gru_scan, "minGRU of long portions in segments");
   m.def("moe_route", &moe_route, "chosen experts and their weights");

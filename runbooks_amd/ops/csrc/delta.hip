@@ -26,13 +26,14 @@
 //    the chunks, 16 state columns per two waves, in registers. Exponents are
 //    differences that are never positive. An fp32 factor enters a product as
 //    two bf16 parts, so the recurrence keeps fp32's quality.
-//  * delta_out: RMS norm per head, times weight and sigmoid gate; the
-//    convolutions' last inputs go to the sequences' slots.
+//
+// delta_out.hip norms and gates o and moves the convolutions' last inputs to
+// the sequences' slots.
 
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 
-#include "common.h"
+#include "split.h"
 
 namespace {
 
@@ -44,10 +45,9 @@ constexpr int VB = 256;                // value columns staged at once
 constexpr float UNIT_EPS = 1e-6f;
 constexpr float LOG2E = 1.4426950408889634f;
 
-typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8v;
+using namespace split;
+
 typedef __attribute__((ext_vector_type(2))) float f32x2v;
-typedef __attribute__((ext_vector_type(4))) float f32x4v;
-typedef __attribute__((ext_vector_type(4))) unsigned int u32x4v;
 
 struct Args {
   const void *y, *y2;
@@ -258,28 +258,6 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
 // ---------------------------------------------------------------------------
 // chunks: operands
 // ---------------------------------------------------------------------------
-RB_DEV unsigned pack2(float lo, float hi) {
-  union { __bf16 b[2]; unsigned u; } c;
-  c.b[0] = (__bf16)lo;
-  c.b[1] = (__bf16)hi;
-  return c.u;
-}
-// two floats as packed bf16 and the packed rest
-RB_DEV void split2(float x, float y, unsigned &big, unsigned &small) {
-  big = pack2(x, y);
-  small = pack2(x - __uint_as_float(big << 16),
-                y - __uint_as_float(big & 0xffff0000u));
-}
-RB_DEV void split8(const float *f, u32x4v &big, u32x4v &small) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    unsigned b, s;
-    split2(f[2 * i], f[2 * i + 1], b, s);
-    big[i] = b;
-    small[i] = s;
-  }
-}
-
 // One chunk and head in scratch. An operand is 64 lanes x 16 bytes, its big
 // and its small part behind each other. Its summed index runs, in lane l,
 // 4 (l / 16) + {0..3} and 16 + that.
@@ -588,17 +566,6 @@ __global__ __launch_bounds__(PREP, 2) void delta_prep_kernel(Args a, int vb) {
 // each other their packed halves through LDS; the first one makes U, the
 // second one O.
 // ---------------------------------------------------------------------------
-union Frag { u32x4v u; bf16x8v v; };
-
-RB_DEV f32x4v mfma(const Frag &a, const Frag &b, f32x4v c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
-}
-// one of the three products that make an fp32 product of split factors
-RB_DEV f32x4v part(int i, const Frag *a, const Frag &bh, const Frag &bl,
-                   f32x4v c) {
-  return mfma(a[i == 2], i == 1 ? bl : bh, c);
-}
-
 template <int DCP>
 __global__ __launch_bounds__(2 * RB_WAVE, 1) void delta_scan_kernel(Args a) {
   using E = Entry<DCP>;
@@ -739,98 +706,6 @@ __global__ __launch_bounds__(2 * RB_WAVE, 1) void delta_scan_kernel(Args a) {
       const int dim = (wid * HT + d) * 16 + grp * 4 + r;
       if (dim < a.dc) st[(int64_t)dim * a.vc + col] = S[d][r];
     }
-}
-
-// ---------------------------------------------------------------------------
-// z = rmsnorm per head(o) * w * sigmoid(gate), columns beyond o's zero; the
-// workgroups after the tokens' move the convolutions' last inputs
-// ---------------------------------------------------------------------------
-template <typename T> RB_DEV void load8(const T *p, float *f) {
-  rb::VIO<T>::load(p, f);
-  if constexpr (rb::VIO<T>::W == 4) rb::VIO<T>::load(p + 4, f + 4);
-}
-template <typename T> RB_DEV void store8(T *p, const float *f) {
-  rb::VIO<T>::store(p, f);
-  if constexpr (rb::VIO<T>::W == 4) rb::VIO<T>::store(p + 4, f + 4);
-}
-
-struct OutArgs {
-  const float *o, *w;
-  int64_t tokens, ny2, ny, nz;
-  int heads, vc, vdim, off_g;
-  float eps;
-  const void *y2, *y;
-  void *z, *swz, *tails;
-  const int *positions, *cu_q, *slots;
-  int taps, channels, tail_blocks;
-};
-
-// L lanes per head with NV times 8 columns each
-template <typename T, int L, int NV>
-__global__ __launch_bounds__(BLOCK) void delta_out_kernel(OutArgs a) {
-  if (blockIdx.x >= a.tokens) {
-    const int i = blockIdx.x - (int)a.tokens, seq = i / a.tail_blocks;
-    const int q0 = a.cu_q[seq], n = a.cu_q[seq + 1] - q0;
-    if (n <= 0) return;
-    const bool fresh = a.positions[q0] == 0;
-    const int keep = a.taps - 1;
-    T *tail = (T *)a.tails + (int64_t)a.slots[seq] * keep * a.channels;
-    const int c = (i % a.tail_blocks * BLOCK + threadIdx.x) * 8;
-    if (c >= a.channels) return;
-    for (int j = 0; j < keep; ++j) {
-      const int s = n - keep + j;              // token of the portion
-      float v[8] = {};
-      if (s >= 0)
-        load8((const T *)a.y + (int64_t)(q0 + s) * a.ny + c, v);
-      else if (!fresh)
-        load8(tail + (int64_t)(keep + s) * a.channels + c, v);
-      store8(tail + (int64_t)j * a.channels + c, v);
-    }
-    return;
-  }
-  constexpr int GROUPS = BLOCK / L;
-  const int64_t t = blockIdx.x;
-  const int lane = threadIdx.x % L, n = a.heads * a.vc;
-  const float *orow = a.o + t * n;
-  const T *g = (const T *)a.y2 + t * a.ny2 + a.off_g;
-  T *zr = (T *)a.z + t * a.nz;
-  auto put = [&](int col, const float *f) {
-    store8(zr + col, f);
-    if (a.swz != nullptr)
-      store8((T *)a.swz + (int64_t)(col >> 4) * 512 + ((col >> 3) & 1) * 256 +
-             t * 8, f);
-  };
-  for (int h0 = 0; h0 < a.heads; h0 += GROUPS) {
-    const int h = h0 + threadIdx.x / L;
-    float f[NV][8], sum = 0.0f;
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-      const int c = (v * L + lane) * 8;
-      if (h < a.heads && c < a.vc) {
-        load8(orow + h * a.vc + c, f[v]);
-#pragma unroll
-        for (int k = 0; k < 8; ++k) sum += f[v][k] * f[v][k];
-      }
-    }
-#pragma unroll
-    for (int o = L / 2; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
-    const float inv = 1.0f / sqrtf(sum / a.vdim + a.eps);
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-      const int c = (v * L + lane) * 8;
-      if (h < a.heads && c < a.vc) {
-        float gf[8], wf[8];
-        load8(g + h * a.vc + c, gf);
-        load8(a.w + c, wf);
-#pragma unroll
-        for (int k = 0; k < 8; ++k)
-          f[v][k] = f[v][k] * inv * wf[k] * sigmoid<T>(gf[k]);
-        put(h * a.vc + c, f[v]);
-      }
-    }
-  }
-  const float zero[8] = {};
-  for (int c = n + threadIdx.x * 8; c < a.nz; c += BLOCK * 8) put(c, zero);
 }
 
 Args check(const at::Tensor &y, const at::Tensor &y2, const at::Tensor &conv,
@@ -976,82 +851,4 @@ void delta_chunk(at::Tensor y, at::Tensor y2, at::Tensor conv,
   else if (a.dc <= 64) launch_chunk<64>(a, n_seqs, max_q, bytes, stream);
   else if (a.dc <= 128) launch_chunk<128>(a, n_seqs, max_q, bytes, stream);
   else launch_chunk<256>(a, n_seqs, max_q, bytes, stream);
-}
-
-// z [T, nz] (and its decode operand) from o [T, heads * vc], w [vc] f32; the
-// new `tails` of the n_seqs sequences
-void delta_out(at::Tensor o, at::Tensor w, at::Tensor y2, int64_t off_g,
-               at::Tensor z, c10::optional<at::Tensor> swz, int64_t vdim,
-               double eps, at::Tensor y, at::Tensor tails,
-               at::Tensor positions, at::Tensor cu_q, at::Tensor slots,
-               int64_t n_seqs) {
-  const auto dt = z.scalar_type();
-  TORCH_CHECK(o.is_cuda() && o.dim() == 2 && o.is_contiguous() &&
-              o.scalar_type() == at::kFloat && w.is_contiguous() &&
-              w.scalar_type() == at::kFloat && y2.dim() == 2 &&
-              y2.is_contiguous() && y2.scalar_type() == dt && z.dim() == 2 &&
-              z.is_contiguous() && y.dim() == 2 && y.is_contiguous() &&
-              y.scalar_type() == dt && tails.dim() == 3 &&
-              tails.is_contiguous() && tails.scalar_type() == dt,
-              "delta_out: tensors");
-  const int64_t T = o.size(0), n = o.size(1), vc = w.numel(), nz = z.size(1);
-  TORCH_CHECK(y2.size(0) == T && z.size(0) == T && y.size(0) == T &&
-              vc % 8 == 0 && vc >= 8 && vc <= 1024 && n % vc == 0 &&
-              nz % 8 == 0 && nz >= n && off_g % 8 == 0 && off_g >= 0 &&
-              y2.size(1) % 8 == 0 && off_g + n <= y2.size(1) && vdim >= 1 &&
-              vdim <= vc && tails.size(2) <= y.size(1) && tails.size(2) % 8 == 0 &&
-              y.size(1) % 8 == 0, "delta_out: layout");
-  TORCH_CHECK(positions.scalar_type() == at::kInt &&
-              positions.is_contiguous() && positions.numel() == T &&
-              cu_q.scalar_type() == at::kInt && cu_q.is_contiguous() &&
-              slots.scalar_type() == at::kInt && slots.is_contiguous() &&
-              n_seqs >= 0 && cu_q.numel() > n_seqs && slots.numel() >= n_seqs,
-              "delta_out: batch tensors");
-  const bool bf16 = dt == at::kBFloat16;
-  TORCH_CHECK(bf16 || dt == at::kFloat, "delta_out: dtype");
-  if (swz.has_value())
-    TORCH_CHECK(bf16 && T <= 32 && swz->is_contiguous() &&
-                swz->scalar_type() == dt && nz % 16 == 0 &&
-                swz->numel() == nz * 32, "delta_out: operand");
-  if (T == 0) return;
-  OutArgs a{};
-  a.o = o.data_ptr<float>();
-  a.w = w.data_ptr<float>();
-  a.tokens = T;
-  a.ny2 = y2.size(1);
-  a.ny = y.size(1);
-  a.nz = nz;
-  a.heads = (int)(n / vc);
-  a.vc = (int)vc;
-  a.vdim = (int)vdim;
-  a.off_g = (int)off_g;
-  a.eps = (float)eps;
-  a.y2 = y2.data_ptr();
-  a.y = y.data_ptr();
-  a.z = z.data_ptr();
-  a.swz = swz ? swz->data_ptr() : nullptr;
-  a.tails = tails.data_ptr();
-  a.positions = positions.data_ptr<int>();
-  a.cu_q = cu_q.data_ptr<int>();
-  a.slots = slots.data_ptr<int>();
-  a.taps = (int)tails.size(1) + 1;
-  a.channels = (int)tails.size(2);
-  a.tail_blocks = (a.channels + BLOCK * 8 - 1) / (BLOCK * 8);
-  auto stream = at::hip::getCurrentHIPStream();
-  auto launch = [&](auto tag, auto l, auto v) {
-    using E = decltype(tag);
-    hipLaunchKernelGGL(
-        (delta_out_kernel<E, decltype(l)::value, decltype(v)::value>),
-        dim3(T + n_seqs * a.tail_blocks), dim3(BLOCK), 0, stream, a);
-  };
-  constexpr std::integral_constant<int, 1> one{};
-  auto pick = [&](auto tag) {
-    if (vc <= 64) launch(tag, std::integral_constant<int, 8>{}, one);
-    else if (vc <= 128) launch(tag, std::integral_constant<int, 16>{}, one);
-    else if (vc <= 256) launch(tag, std::integral_constant<int, 32>{}, one);
-    else launch(tag, std::integral_constant<int, 64>{},
-                std::integral_constant<int, 2>{});
-  };
-  if (bf16) pick(uint16_t{});
-  else pick(float{});
 }

@@ -2,7 +2,7 @@
 //
 // All heads of a layer attend to the same cached row per token: the latent
 // (which is key and value at once, after q was moved into latent space) and
-// one rotated key part. Query rows are (token, head) pairs of one sequence,
+// one rotated key part (or none). Query rows are (token, head) pairs of one sequence,
 // heads fastest, so a workgroup reads each cache row once for 16-64 rows:
 // single decoded tokens and short prompt portions are the same kernel.
 //
@@ -35,7 +35,7 @@ namespace {
 constexpr int BLOCK = 512;             // MFMA kernel
 constexpr int ROWS_BLOCK = 256;        // scalar kernel
 constexpr int TK = 64;                 // keys per tile
-constexpr int ROTP = 64;               // padded rotated part
+constexpr int MAX_ROT = 64;            // padded rotated part
 constexpr int PAGE = 16;               // tokens per cache block
 constexpr int SSTRIDE = 68;            // floats per score row
 constexpr int PSTRIDE = 72;            // 16-bit weights per row
@@ -78,7 +78,7 @@ template <int N> RB_DEV float group_max(float v) {
   return v;
 }
 
-template <int RP, int MT>
+template <int RP, int MT, int ROTP>
 __global__ __launch_bounds__(BLOCK, 1) void latent_attend_kernel(AttendArgs a) {
   constexpr int M = MT * 16;
   constexpr int COLS = RP + ROTP;
@@ -529,12 +529,14 @@ __global__ __launch_bounds__(ROWS_BLOCK) void latent_attend_rows_kernel(
   }
 }
 
-bool mfma_sizes(int64_t rc, int64_t rotc) { return rc <= 512 && rotc <= ROTP; }
+bool mfma_sizes(int64_t rc, int64_t rotc) {
+  return rc <= 512 && rotc <= MAX_ROT;
+}
 int padded_rank(int64_t rc) {
   return rc <= 64 ? 64 : rc <= 128 ? 128 : rc <= 256 ? 256 : 512;
 }
 
-template <int RP, int MT>
+template <int RP, int MT, int ROTP>
 void launch_attend(const AttendArgs &a, dim3 grid, hipStream_t stream) {
   constexpr int planes = MT == 1 ? 2 : 1;
   constexpr size_t shmem =
@@ -543,12 +545,12 @@ void launch_attend(const AttendArgs &a, dim3 grid, hipStream_t stream) {
   static_assert(shmem <= 160 * 1024, "LDS");
   static bool once = [] {
     return hipFuncSetAttribute(
-               reinterpret_cast<const void *>(&latent_attend_kernel<RP, MT>),
+               reinterpret_cast<const void *>(&latent_attend_kernel<RP, MT, ROTP>),
                hipFuncAttributeMaxDynamicSharedMemorySize,
                (int)shmem) == hipSuccess;
   }();
   TORCH_CHECK(once, "latent_attend: LDS size");
-  hipLaunchKernelGGL((latent_attend_kernel<RP, MT>), grid, dim3(BLOCK), shmem,
+  hipLaunchKernelGGL((latent_attend_kernel<RP, MT, ROTP>), grid, dim3(BLOCK), shmem,
                      stream, a);
 }
 
@@ -576,7 +578,7 @@ at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
               cache.is_contiguous() && cache.scalar_type() == dt,
               "latent_attend: cache [blocks, 16, ec]");
   const int64_t ec = cache.size(2), rotc = ec - rc;
-  TORCH_CHECK(rc % 8 == 0 && rotc >= 8 && rotc % 8 == 0 && q_off % 8 == 0 &&
+  TORCH_CHECK(rc % 8 == 0 && rc >= 8 && rotc >= 0 && rotc % 8 == 0 && q_off % 8 == 0 &&
               q_head % 8 == 0 && y.size(1) % 8 == 0, "latent_attend: layout");
   TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && y.scalar_type() == dt &&
               y.size(0) >= T && q_off + (H - 1) * q_head + rotc <= y.size(1),
@@ -647,17 +649,20 @@ at::Tensor latent_attend(at::Tensor q_lat, at::Tensor y, int64_t q_off,
   }
   const dim3 grid(a.nsplit, (rows + M - 1) / M, n_seqs);
   const int rp = padded_rank(rc);
-#define RB_ATTEND(RP)                                     \
-  do {                                                    \
-    if (M == 16) launch_attend<RP, 1>(a, grid, stream);   \
-    else if (M == 32) launch_attend<RP, 2>(a, grid, stream); \
-    else if constexpr (RP < 512) launch_attend<RP, 4>(a, grid, stream); \
-  } while (0)
-  if (rp == 64) RB_ATTEND(64);
-  else if (rp == 128) RB_ATTEND(128);
-  else if (rp == 256) RB_ATTEND(256);
-  else RB_ATTEND(512);
-#undef RB_ATTEND
+  auto launch = [&](auto r, auto rot) {
+    constexpr int RP = decltype(r)::value, ROT = decltype(rot)::value;
+    if (M == 16) launch_attend<RP, 1, ROT>(a, grid, stream);
+    else if (M == 32) launch_attend<RP, 2, ROT>(a, grid, stream);
+    else if constexpr (RP < 512) launch_attend<RP, 4, ROT>(a, grid, stream);
+  };
+  auto pick = [&](auto rot) {
+    if (rp == 64) launch(std::integral_constant<int, 64>{}, rot);
+    else if (rp == 128) launch(std::integral_constant<int, 128>{}, rot);
+    else if (rp == 256) launch(std::integral_constant<int, 256>{}, rot);
+    else launch(std::integral_constant<int, 512>{}, rot);
+  };
+  if (rotc > 0) pick(std::integral_constant<int, MAX_ROT>{});
+  else pick(std::integral_constant<int, 0>{});
   if (a.nsplit > 1)
     hipLaunchKernelGGL(latent_combine_kernel, dim3(T * H), dim3(128), 0,
                        stream, a.part_o, a.part_ml, (uint16_t *)a.out,

@@ -4,7 +4,8 @@
 // kv[key][h] = [ unrotated key (dimc) | value (vc) ]; the rotated key part,
 // shared by all heads, is read from the context rows themselves
 // (ctx[key][rc..]). Queries lie in y ([dimc | rotc] per head). The sigmoid
-// output gate (also in y) is applied to the result, which goes to z.
+// output gate, per value column or per head, is applied to the result, which
+// goes to z.
 //
 // 4 waves, each 32 query rows of one head; 64-key tiles in LDS (next tile
 // prefetched to registers), scores transposed (key x query) so a query's
@@ -36,8 +37,9 @@ struct FlashArgs {
   const uint16_t *ctx;                 // [Tk, ec]
   const int *meta;                     // [n, 5]
   uint16_t *z;                         // [T, nz]
-  int64_t ny, nz;
-  int heads, dimc, rotc, vc, rc, ec, off_g, window;
+  const uint16_t *gate;                // [T, ng], from column off_g
+  int64_t ny, nz, ng;
+  int heads, dimc, rotc, vc, rc, ec, off_g, head_gate, window;
   float scale_log2e;
 };
 
@@ -225,7 +227,9 @@ __global__ __launch_bounds__(BLOCK, 2) void latent_flash_kernel(FlashArgs a) {
   const float l = l_run + __shfl_xor(l_run, 32, 64);
   const float inv = l > 0.0f ? 1.0f / l : 0.0f;
   const int64_t t = q_row0 + qi;
-  const uint16_t *gp = a.y + t * a.ny + a.off_g + h * a.vc;
+  const uint16_t *gp = a.gate + t * a.ng + a.off_g;
+  const uint32_t one = a.head_gate ? gp[h] * 0x10001u : 0;
+  gp += h * a.vc;
   uint16_t *zp = a.z + t * a.nz + h * a.vc;
 #pragma unroll
   for (int d = 0; d < DT; ++d)
@@ -233,7 +237,8 @@ __global__ __launch_bounds__(BLOCK, 2) void latent_flash_kernel(FlashArgs a) {
     for (int rq = 0; rq < 4; ++rq) {
       const int c = d * 32 + 8 * rq + 4 * hi;
       if (c >= a.vc) continue;
-      const uint2 gw = *reinterpret_cast<const uint2 *>(gp + c);
+      uint2 gw = make_uint2(one, one);
+      if (!a.head_gate) gw = *reinterpret_cast<const uint2 *>(gp + c);
       const uint32_t gu[2] = {gw.x, gw.y};
       float o[4];
 #pragma unroll
@@ -267,8 +272,9 @@ void launch_flash(const FlashArgs &a, dim3 grid, hipStream_t stream) {
 
 void latent_flash(at::Tensor y, at::Tensor kv, at::Tensor ctx, at::Tensor meta,
                   at::Tensor z, int64_t heads, int64_t dimc, int64_t rotc,
-                  int64_t vc, int64_t rc, int64_t off_g, int64_t max_q,
-                  double scale, int64_t window) {
+                  int64_t vc, int64_t rc, at::Tensor gate, int64_t off_g,
+                  bool head_gate, int64_t max_q, double scale,
+                  int64_t window) {
   TORCH_CHECK(y.is_cuda() && y.is_contiguous() && kv.is_contiguous() &&
               ctx.is_contiguous() && z.is_contiguous() &&
               meta.is_contiguous() && y.dim() == 2 && z.dim() == 2,
@@ -281,16 +287,22 @@ void latent_flash(at::Tensor y, at::Tensor kv, at::Tensor ctx, at::Tensor meta,
   TORCH_CHECK(dimc % 8 == 0 && rotc % 8 == 0 && vc % 8 == 0 && rc % 8 == 0 &&
               off_g % 8 == 0 && y.size(1) % 8 == 0 && z.size(1) % 8 == 0 &&
               heads * (dimc + rotc) <= y.size(1) &&
-              off_g + heads * vc <= y.size(1) && heads * vc <= z.size(1) &&
+              heads * vc <= z.size(1) &&
               kv.size(-1) == heads * (dimc + vc) && kv.size(0) == ctx.size(0) &&
               ctx.dim() == 2 && ctx.size(1) == rc + rotc &&
               y.size(0) == z.size(0) && meta.dim() == 2 && meta.size(1) == 5,
               "latent_flash: layout");
+  TORCH_CHECK(gate.dim() == 2 && gate.is_contiguous() &&
+              gate.scalar_type() == at::kBFloat16 &&
+              gate.size(0) == y.size(0) && gate.size(1) % 8 == 0 &&
+              off_g >= 0 && off_g + heads * (head_gate ? 1 : vc) <=
+              gate.size(1), "latent_flash: gate");
   FlashArgs a{(const uint16_t *)y.data_ptr(), (const uint16_t *)kv.data_ptr(),
               (const uint16_t *)ctx.data_ptr(), meta.data_ptr<int>(),
-              (uint16_t *)z.data_ptr(), y.size(1), z.size(1), (int)heads,
-              (int)dimc, (int)rotc, (int)vc, (int)rc, (int)ctx.size(1),
-              (int)off_g, (int)window,
+              (uint16_t *)z.data_ptr(), (const uint16_t *)gate.data_ptr(),
+              y.size(1), z.size(1), gate.size(1), (int)heads, (int)dimc,
+              (int)rotc, (int)vc, (int)rc, (int)ctx.size(1), (int)off_g,
+              (int)head_gate, (int)window,
               (float)(scale * 1.4426950408889634)};
   const dim3 grid(heads, (max_q + QB - 1) / QB, meta.size(0));
   auto stream = at::hip::getCurrentHIPStream();

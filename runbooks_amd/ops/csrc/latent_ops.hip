@@ -120,14 +120,57 @@ __global__ __launch_bounds__(BLOCK) void latent_prep_kernel(
 }
 
 // ---------------------------------------------------------------------------
+// RMS norms of two latents in y: blocks (token, 0) the queries' one, to `out`
+// (zeros up to its no columns), blocks (token, 1) the cached one
+// ---------------------------------------------------------------------------
+struct NormsArgs {
+  int64_t ny;
+  int oq, nq, no, oc, nc, ec;
+  float eps;
+};
+
+template <typename T>
+__global__ __launch_bounds__(BLOCK) void latent_norms_kernel(
+    const T *__restrict__ y, const float *__restrict__ wq,
+    const float *__restrict__ wc, T *__restrict__ out, T *__restrict__ swz,
+    T *__restrict__ cache, const int *__restrict__ slots, NormsArgs a) {
+  __shared__ float red[BLOCK / RB_WAVE];
+  const int64_t t = blockIdx.x;
+  const bool cached = blockIdx.y > 0;
+  const int n = cached ? a.nc : a.nq;
+  const T *row = y + t * a.ny + (cached ? a.oc : a.oq);
+  float ss = 0.0f;
+  for (int i = threadIdx.x; i < n; i += BLOCK) {
+    const float v = rb::bf16_to_f32_or_id(row[i]);
+    ss += v * v;
+  }
+  ss = rb::block_reduce_sum(ss, red);
+  const float ir = 1.0f / sqrtf(ss / (float)n + a.eps);
+  if (cached) {
+    T *dst = cache + (int64_t)slots[t] * a.ec;
+    for (int i = threadIdx.x; i < n; i += BLOCK)
+      rb::store_scalar(dst + i, rb::bf16_to_f32_or_id(row[i]) * ir * wc[i]);
+    return;
+  }
+  for (int i = threadIdx.x; i < a.no; i += BLOCK) {
+    const float v =
+        i < n ? rb::bf16_to_f32_or_id(row[i]) * ir * wq[i] : 0.0f;
+    rb::store_scalar(out + t * a.no + i, v);
+    if (swz != nullptr)
+      rb::store_scalar(swz + operand_at(i & ~7, (int)t) + (i & 7), v);
+  }
+}
+
+// ---------------------------------------------------------------------------
 // y_h = x_h @ w_h per head, optionally times sigmoid(gate).
 //   x element (m, h, k): x[x_off + m * xs + h * xh + k], k < K (K % 8 == 0)
 //   out element (m, h, n): out[o_off + m * os + h * oh + n], n < N
-//   gate element: g[g_off + m * gs + h * oh + n]
+//   gate element: g[g_off + m * gs + h * oh + n], or one per head:
+//                 g[g_off + m * gs + h]
 // ---------------------------------------------------------------------------
 struct HeadArgs {
   int64_t x_off, xs, o_off, os, g_off, gs;
-  int xh, oh, K, N, T;
+  int xh, oh, K, N, T, head_gate;
 };
 
 // Weights in fragment order [H][N/16][K/32][lane][8]: each step of a wave is
@@ -185,8 +228,10 @@ __global__ __launch_bounds__(BLOCK) void head_gemm_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = r4[r];
     if (gate != nullptr) {
-      const uint2 gw = *reinterpret_cast<const uint2 *>(
-          gate + a.g_off + m * a.gs + (int64_t)h * a.oh + n);
+      const uint16_t *gp = gate + a.g_off + m * a.gs;
+      uint2 gw;
+      if (a.head_gate) gw.x = gw.y = gp[h] * 0x10001u;
+      else gw = *reinterpret_cast<const uint2 *>(gp + (int64_t)h * a.oh + n);
       const uint32_t gu[2] = {gw.x, gw.y};
 #pragma unroll
       for (int r = 0; r < 4; ++r)
@@ -232,7 +277,8 @@ __global__ void head_gemm_f32_kernel(const float *__restrict__ x,
   float acc = 0.0f;
   for (int k = 0; k < a.K; ++k) acc = fmaf(xr[k], wr[(int64_t)k * a.N], acc);
   if (gate != nullptr)
-    acc *= sigmoidf<float>(gate[a.g_off + m * a.gs + (int64_t)h * a.oh + n]);
+    acc *= sigmoidf<float>(gate[a.g_off + m * a.gs +
+                                (a.head_gate ? h : (int64_t)h * a.oh + n)]);
   out[a.o_off + m * a.os + (int64_t)h * a.oh + n] = acc;
 }
 
@@ -296,10 +342,49 @@ void latent_prep(at::Tensor y, at::Tensor cos, at::Tensor sin,
   else TORCH_CHECK(false, "latent_prep: dtype");
 }
 
+void latent_norms(at::Tensor y, int64_t oq, int64_t nq, at::Tensor wq,
+                  at::Tensor out, c10::optional<at::Tensor> swz, int64_t oc,
+                  int64_t nc, at::Tensor wc, at::Tensor cache,
+                  at::Tensor slots, double eps) {
+  const auto dt = y.scalar_type();
+  const int64_t T = y.size(0), no = out.size(1), ec = cache.size(-1);
+  TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous() &&
+              (dt == at::kBFloat16 || dt == at::kFloat) && out.dim() == 2 &&
+              out.is_contiguous() && out.scalar_type() == dt &&
+              out.size(0) == T && cache.is_contiguous() &&
+              cache.scalar_type() == dt && slots.scalar_type() == at::kInt &&
+              slots.is_contiguous() && slots.numel() == T,
+              "latent_norms: tensors");
+  TORCH_CHECK(nq >= 1 && nq <= no && nc >= 1 && nc <= ec && oq >= 0 &&
+              oc >= 0 && oq + nq <= y.size(1) && oc + nc <= y.size(1) &&
+              wq.scalar_type() == at::kFloat && wq.is_contiguous() &&
+              wq.numel() == nq && wc.scalar_type() == at::kFloat &&
+              wc.is_contiguous() && wc.numel() == nc, "latent_norms: layout");
+  if (swz.has_value())
+    TORCH_CHECK(T <= 32 && no % 16 == 0 && swz->numel() == no * 32 &&
+                swz->is_contiguous() && swz->scalar_type() == dt &&
+                dt == at::kBFloat16, "latent_norms: operand");
+  if (T == 0) return;
+  const NormsArgs a{y.size(1), (int)oq, (int)nq, (int)no, (int)oc, (int)nc,
+                    (int)ec, (float)eps};
+  auto stream = at::hip::getCurrentHIPStream();
+  auto launch = [&](auto tag) {
+    using E = decltype(tag);
+    hipLaunchKernelGGL((latent_norms_kernel<E>), dim3(T, 2), dim3(BLOCK), 0,
+                       stream, (const E *)y.data_ptr(), wq.data_ptr<float>(),
+                       wc.data_ptr<float>(), (E *)out.data_ptr(),
+                       swz ? (E *)swz->data_ptr() : nullptr,
+                       (E *)cache.data_ptr(), slots.data_ptr<int>(), a);
+  };
+  if (dt == at::kBFloat16) launch(uint16_t{});
+  else launch(float{});
+}
+
 void head_gemm(at::Tensor x, int64_t x_off, int64_t xh, at::Tensor w,
                int64_t K, int64_t N, at::Tensor out, int64_t o_off, int64_t oh,
                c10::optional<at::Tensor> gate, int64_t g_off,
-               c10::optional<at::Tensor> swz, int64_t T, int64_t H) {
+               c10::optional<at::Tensor> swz, int64_t T, int64_t H,
+               bool head_gate) {
   TORCH_CHECK(x.is_cuda() && x.dim() == 2 && out.dim() == 2 &&
               x.stride(1) == 1 && out.stride(1) == 1 && w.is_contiguous() &&
               T <= x.size(0) && T <= out.size(0), "head_gemm: tensors");
@@ -315,7 +400,8 @@ void head_gemm(at::Tensor x, int64_t x_off, int64_t xh, at::Tensor w,
   if (gate.has_value())
     TORCH_CHECK(gate->dim() == 2 && gate->stride(1) == 1 &&
                 gate->stride(0) % 8 == 0 && T <= gate->size(0) &&
-                g_off + (H - 1) * oh + N <= gate->size(1) &&
+                g_off + (head_gate ? H : (H - 1) * oh + N) <=
+                    gate->size(1) &&
                 gate->scalar_type() == x.scalar_type(), "head_gemm: gate");
   if (swz.has_value())
     TORCH_CHECK(bf16 && T <= 32 && swz->is_contiguous() &&
@@ -323,7 +409,7 @@ void head_gemm(at::Tensor x, int64_t x_off, int64_t xh, at::Tensor w,
   if (T == 0) return;
   HeadArgs a{x_off, x.stride(0), o_off, out.stride(0), g_off,
              gate ? gate->stride(0) : 0, (int)xh, (int)oh, (int)K, (int)N,
-             (int)T};
+             (int)T, (int)head_gate};
   auto stream = at::hip::getCurrentHIPStream();
   if (!bf16) {
     TORCH_CHECK(w.numel() == H * K * N, "head_gemm: weight");

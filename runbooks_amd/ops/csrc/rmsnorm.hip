@@ -367,8 +367,8 @@ std::vector<at::Tensor> rmsnorm_res_slab_fwd_dec(at::Tensor x,
   return {sum, y, swz};
 }
 
-// Norm of a 32-bit residual: x += delta in place, y = rmsnorm(x) * w in w's
-// dtype. `nd` delta terms of type DT (0: none; > 1: the uncombined split-K
+// Norm of a 32-bit residual: x += delta in place, y = rmsnorm(x) * (offset + w)
+// in w's dtype. `nd` delta terms of type DT (0: none; > 1: the uncombined split-K
 // slab of decode_gemm_raw) lie n_rows * D apart. swz as above (bf16 only).
 namespace {
 template <typename T, typename DT, int V>
@@ -377,7 +377,8 @@ __global__ void rmsnorm_res32_kernel(float *__restrict__ x,
                                      const T *__restrict__ w,
                                      T *__restrict__ y,
                                      uint16_t *__restrict__ swz,
-                                     int64_t n_rows, int D, float eps) {
+                                     int64_t n_rows, int D, float eps,
+                                     float offset) {
   __shared__ float red[BLOCK / RB_WAVE];
   const int nvec = D / V;
   for (int64_t row = blockIdx.x; row < n_rows; row += gridDim.x) {
@@ -424,7 +425,7 @@ __global__ void rmsnorm_res32_kernel(float *__restrict__ x,
         rb::VIO<T>::load(w + i * 8, g);
         if constexpr (rb::VIO<T>::W == 4) rb::VIO<T>::load(w + i * 8 + 4, g + 4);
 #pragma unroll
-        for (int k = 0; k < 8; ++k) f[k] = f[k] * ir * g[k];
+        for (int k = 0; k < 8; ++k) f[k] = f[k] * ir * (offset + g[k]);
         rb::VIO<T>::store(y + row * D + i * 8, f);
         if constexpr (rb::VIO<T>::W == 4)
           rb::VIO<T>::store(y + row * D + i * 8 + 4, f + 4);
@@ -435,7 +436,7 @@ __global__ void rmsnorm_res32_kernel(float *__restrict__ x,
         }
       } else {
         rb::store_scalar(y + row * D + i,
-                         xr[i] * ir * rb::bf16_to_f32_or_id(w[i]));
+                         xr[i] * ir * (offset + rb::bf16_to_f32_or_id(w[i])));
       }
     }
     __syncthreads();
@@ -445,7 +446,8 @@ __global__ void rmsnorm_res32_kernel(float *__restrict__ x,
 
 std::vector<at::Tensor> rmsnorm_res32(at::Tensor x,
                                       c10::optional<at::Tensor> delta,
-                                      at::Tensor w, double eps, bool want_swz) {
+                                      at::Tensor w, double eps, bool want_swz,
+                                      double offset) {
   TORCH_CHECK(x.is_cuda() && x.is_contiguous() && w.is_contiguous() &&
               x.dim() == 2 && x.scalar_type() == at::kFloat &&
               w.numel() == x.size(1), "rmsnorm_res32: x [T, D] f32, w [D]");
@@ -479,7 +481,7 @@ std::vector<at::Tensor> rmsnorm_res32(at::Tensor x,
                      stream, x.data_ptr<float>(), (const DT *)dp, nd,        \
                      (const T *)w.data_ptr(), (T *)y.data_ptr(),             \
                      want_swz ? (uint16_t *)swz.data_ptr() : nullptr,        \
-                     n_rows, D, (float)eps)
+                     n_rows, D, (float)eps, (float)offset)
 #define RB_RES32_V(V)                                  \
   if (bf16 && d16) RB_RES32(uint16_t, uint16_t, V);    \
   else if (bf16) RB_RES32(uint16_t, float, V);         \

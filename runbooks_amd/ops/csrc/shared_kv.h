@@ -13,6 +13,9 @@
 // projection's weight has its columns in the value's order. Otherwise the
 // value follows the key. The cache is [blocks, kv heads, PAGE, ec]: a page of
 // one head is contiguous.
+//
+// With two maps a row is [ key 1 | key 2 | value ], and a head has a query for
+// each key; its result is rms_norm(o1 - lam o2) times out_scale.
 #pragma once
 
 #include "common.h"
@@ -42,8 +45,12 @@ struct Args {
   void *z;                             // [T, nz]; heads first
   int64_t nz;
   uint16_t *swz;                       // decode operand of z, or null
-  float *part_o;                       // [nsplit, T*H, vc]
+  float *part_o;                       // [nsplit, T*H, vc], or null
   float *part_ml;                      // [nsplit, T*H, 2]
+  const float *lam;                    // two maps
+  int count;                           // columns that their norm counts
+  float eps;
+  bool f32;                            // z's type
 };
 
 // First key that a query at retained position `pos` sees, possibly below 0;
@@ -107,23 +114,49 @@ RB_DEV void store4(const Args &a, int64_t t, int col, const float *v) {
                                (col & 7)) = w;
 }
 
-// Calls f with the padded head size (key's or value's, the larger) and the
-// chunks a lane copies per page.
-template <typename F> void pick_sizes(int hc, int ec, F f) {
-  const int ni = (ec + 31) / 32;
-  auto go = [&](auto hcp) {
-    constexpr int H = decltype(hcp)::value;
-    constexpr int few = H / 32 + (H < 128 ? 1 : H / 128);
-    constexpr int most = H / 16;
-    if (ni <= few) f(hcp, std::integral_constant<int, few>{});
-    else f(hcp, std::integral_constant<int, most>{});
-  };
+// Sizes that a kernel is made for: HCK columns of a key, HCP of a value (and a
+// key), NI chunks that a lane copies per page.
+template <int K, int P, int N, int M> struct Sizes {
+  static constexpr int HCK = K, HCP = P, NI = N, MAPS = M;
+};
+
+template <typename F> void pick_head(int hc, F go) {
   if (hc <= 32) go(std::integral_constant<int, 32>{});
   else if (hc <= 64) go(std::integral_constant<int, 64>{});
   else if (hc <= 96) go(std::integral_constant<int, 96>{});
   else if (hc <= 128) go(std::integral_constant<int, 128>{});
   else if (hc <= 192) go(std::integral_constant<int, 192>{});
   else go(std::integral_constant<int, 256>{});
+}
+
+// Calls f with the sizes for keys of hc columns, values (or keys) of up to
+// `hc`, rows of ec.
+template <typename F> void pick_sizes(int hc, int ec, F f) {
+  const int ni = (ec + 31) / 32;
+  auto go = [&](auto hcp) {
+    constexpr int H = decltype(hcp)::value;
+    constexpr int few = H / 32 + (H < 128 ? 1 : H / 128);
+    constexpr int most = H / 16;
+    if (ni <= few) f(Sizes<H, H, few, 1>{});
+    else f(Sizes<H, H, most, 1>{});
+  };
+  pick_head(hc, go);
+}
+// the same for two maps with keys of hc columns, values of vc
+template <typename F> void pick_sizes2(int hc, int vc, F f) {
+  const int ni = (2 * hc + vc + 31) / 32;
+  auto go = [&](auto hcp) {
+    constexpr int H = decltype(hcp)::value;
+    auto width = [&](auto k) {
+      constexpr int K = decltype(k)::value;
+      if constexpr (K < H) f(Sizes<K, H, (2 * K + H + 31) / 32, 2>{});
+      else if (ni <= H / 16) f(Sizes<K, H, H / 16, 2>{});
+      else f(Sizes<K, H, 3 * H / 32, 2>{});
+    };
+    if (hc <= H / 2) width(std::integral_constant<int, H / 2>{});
+    else width(hcp);
+  };
+  pick_head(hc > vc ? hc : vc, go);
 }
 
 }  // namespace skv

@@ -8,7 +8,9 @@
 // as they stand (the order of the summed keys is free, so the transposed
 // reads of V follow the order of the scores). The waves' partial results are
 // merged at the end; `nsplit` workgroups may share a sequence's keys, merged
-// by shared_kv_combine.
+// by shared_kv_combine. With two maps a row's query stands in its own key's
+// columns, zeros in the other's, so rows of both share a tile; their results
+// meet in shared_kv_diff_combine.
 //
 // The scalar kernel covers fp32 and head sizes beyond 256: one workgroup per
 // row, a wave per key, lanes across the columns.
@@ -27,6 +29,7 @@ constexpr int WAVES = 4;
 constexpr int TK = 2 * PAGE;           // keys per tile
 constexpr int M = 16;                  // query rows per workgroup
 constexpr int SLACK = 512;             // LDS bytes past a wave's tile
+constexpr size_t MAX_LDS = 158 * 1024;
 
 __host__ __device__ constexpr int wave_bytes(int ec) {
   return TK * row_stride(ec) + SLACK;
@@ -38,9 +41,10 @@ RB_DEV void wave_fence() {
   __builtin_amdgcn_wave_barrier();
 }
 
-template <int HCP, int NI>
+template <typename SZ>
 __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
-  constexpr int KS = HCP / 32;                 // QK steps
+  constexpr int HCP = SZ::HCP, NI = SZ::NI;
+  constexpr int KS = SZ::MAPS * SZ::HCK / 32;  // QK steps
   constexpr int DT = HCP / 16;                 // column tiles of the result
   constexpr int OSTRIDE = HCP + 4;             // floats
 
@@ -74,7 +78,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
     return (int64_t)(q0 + r / a.group) * a.heads + g * a.group + r % a.group;
   };
   if (t0 >= t1) {                              // nothing left for this split
-    if (a.nsplit > 1 && tid < min(M, rows - row0)) {
+    if (a.part_o != nullptr && tid < min(M, rows - row0)) {
       float *ml =
           a.part_ml + ((int64_t)split * a.total_rows + global_row(tid)) * 2;
       ml[0] = -INFINITY;
@@ -116,12 +120,13 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
     const int64_t gr = global_row(row_ok ? l16 : 0);
     const uint16_t *qp = (const uint16_t *)a.y + gr / a.heads * a.ny +
                          gr % a.heads * a.hc;
+    const int at = SZ::MAPS > 1 ? (int)(gr % SZ::MAPS) * a.hc : 0;
 #pragma unroll
     for (int s = 0; s < KS; ++s) {
-      const int c = s * 32 + grp * 8;
+      const int c = s * 32 + grp * 8 - at;
       union { u32x4v u; bf16x8v v; } q;
-      q.u = row_ok && c < a.hc ? *reinterpret_cast<const u32x4v *>(qp + c)
-                               : (u32x4v)(0u);
+      q.u = row_ok && c >= 0 && c < a.hc
+                ? *reinterpret_cast<const u32x4v *>(qp + c) : (u32x4v)(0u);
       qf[s] = q.v;
     }
   }
@@ -222,7 +227,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
   if (wid == 0 && grp == 0) {
     out_s[l16][0] = mx;
     out_s[l16][1] = l;
-    if (a.nsplit > 1 && row_ok) {
+    if (a.part_o != nullptr && row_ok) {
       float *ml =
           a.part_ml + ((int64_t)split * a.total_rows + global_row(l16)) * 2;
       ml[0] = mx;
@@ -239,7 +244,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_attend_kernel(Args a) {
     for (int w = 0; w < WAVES; ++w)
       o += *reinterpret_cast<const f32x4v *>(o_s + (w * M + m) * OSTRIDE + c);
     const int64_t gr = global_row(m);
-    if (a.nsplit > 1) {
+    if (a.part_o != nullptr) {
       *reinterpret_cast<f32x4v *>(
           a.part_o + ((int64_t)split * a.total_rows + gr) * a.vc + c) = o;
     } else {
@@ -282,6 +287,64 @@ __global__ __launch_bounds__(64) void shared_kv_combine_kernel(Args a) {
   }
 }
 
+// One block per token and head merges the splits of its two maps, subtracts the
+// second one's result and norms.
+__global__ __launch_bounds__(64) void shared_kv_diff_combine_kernel(Args a) {
+  constexpr int NV = 4;                        // vc <= 1024
+  const int64_t row = blockIdx.x * (int64_t)2;
+  const int lane = threadIdx.x;
+  __shared__ float w_s[2][64];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    float m = -INFINITY, l = 0.0f;
+    if (lane < a.nsplit) {
+      const float2 ml = *reinterpret_cast<const float2 *>(
+          a.part_ml + ((int64_t)lane * a.total_rows + row + i) * 2);
+      m = ml.x;
+      l = ml.y;
+    }
+    const float mx = rb::wave_reduce_max(m);
+    float w = l > 0.0f ? __builtin_amdgcn_exp2f(m - mx) : 0.0f;
+    w /= rb::wave_reduce_sum(l * w);
+    w_s[i][lane] = i == 0 ? w : -a.lam[0] * w;
+  }
+  __syncthreads();
+  float o[NV][4] = {}, sum = 0.0f;
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int c = (v * 64 + lane) * 4;
+    if (c >= a.vc) continue;
+    for (int s = 0; s < a.nsplit; ++s)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const float ws = w_s[i][s];
+        if (ws == 0.0f) continue;              // its part may be unwritten
+        const f32x4v p = *reinterpret_cast<const f32x4v *>(
+            a.part_o + ((int64_t)s * a.total_rows + row + i) * a.vc + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[v][e] += ws * p[e];
+      }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) sum += o[v][e] * o[v][e];
+  }
+  sum = rb::wave_reduce_sum(sum);
+  const float f = a.out_scale / sqrtf(sum / (float)a.count + a.eps);
+  const int64_t t = row / a.heads;
+  const int col = (int)(row % a.heads) / 2 * a.vc;
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int c = (v * 64 + lane) * 4;
+    if (c >= a.vc) continue;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[v][e] *= f;
+    if (a.f32)
+      *reinterpret_cast<f32x4v *>((float *)a.z + t * a.nz + col + c) =
+          (f32x4v){o[v][0], o[v][1], o[v][2], o[v][3]};
+    else
+      store4(a, t, col + c, o[v]);
+  }
+}
+
 // ---------------------------------------------------------------------------
 // scalar kernel: block = one (token, head) row, wave = every fourth key
 // ---------------------------------------------------------------------------
@@ -300,6 +363,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
   const int v0 = a.seq_lens[seq] - nq;
   const int lo = max(0, first_key(a, qpos, dropped_of(a, q0, v0)));
   const T *qp = (const T *)a.y + (q0 + tok) * a.ny + head * a.hc;
+  const int koff = a.lam != nullptr ? head % 2 * a.hc : 0;
   const int *table = a.tables + (int64_t)seq * a.table_width;
 
   float q[NE], o[NE];
@@ -322,7 +386,7 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
 #pragma unroll
     for (int i = 0; i < NE; ++i) {
       const int e = lane + i * 64;
-      if (e < a.hc) s = fmaf(q[i], rb::bf16_to_f32_or_id(c[e]), s);
+      if (e < a.hc) s = fmaf(q[i], rb::bf16_to_f32_or_id(c[koff + e]), s);
     }
     s = rb::wave_reduce_sum(s) * a.scale;
     const float mn = fmaxf(m, s);
@@ -352,10 +416,19 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
     w[k] = ml_s[k][1] > 0.0f ? expf(ml_s[k][0] - mx) : 0.0f;
     lt += w[k] * ml_s[k][1];
   }
+  const int64_t gr = (int64_t)(q0 + tok) * a.heads + head;
+  if (a.part_o != nullptr && threadIdx.x == 0) {
+    a.part_ml[gr * 2] = mx;
+    a.part_ml[gr * 2 + 1] = lt;
+  }
   for (int e = threadIdx.x; e < a.vc; e += BLOCK) {
     float v = 0.0f;
 #pragma unroll
     for (int k = 0; k < 4; ++k) v += w[k] * o_s[k * a.vc + e];
+    if (a.part_o != nullptr) {
+      a.part_o[gr * a.vc + e] = v;
+      continue;
+    }
     v *= a.out_scale / lt;
     const int col = head * a.vc + e;
     rb::store_scalar((T *)a.z + (q0 + tok) * a.nz + col, v);
@@ -366,24 +439,25 @@ __global__ __launch_bounds__(BLOCK) void shared_kv_rows_kernel(Args a) {
   }
 }
 
-template <int HCP, int NI>
+template <typename SZ>
 void launch_attend(const Args &a, dim3 grid, hipStream_t stream) {
+  constexpr int HCP = SZ::HCP;
   const size_t tiles = (size_t)WAVES * wave_bytes(a.ec);
   const size_t merge = (size_t)WAVES * M * (HCP + 4) * sizeof(float);
   const size_t shmem = std::max(tiles, merge);
-  constexpr size_t most =
-      std::max((size_t)WAVES * wave_bytes(2 * HCP),
-               (size_t)WAVES * M * (HCP + 4) * sizeof(float));
-  static_assert(most <= 159 * 1024, "LDS");
+  constexpr size_t most = std::min(
+      MAX_LDS, std::max((size_t)WAVES * wave_bytes(SZ::MAPS == 1 ? 2 * HCP
+                                                   : 2 * SZ::HCK + HCP),
+                        (size_t)WAVES * M * (HCP + 4) * sizeof(float)));
   static bool once = [] {
     return hipFuncSetAttribute(
                reinterpret_cast<const void *>(
-                   &shared_kv_attend_kernel<HCP, NI>),
+                   &shared_kv_attend_kernel<SZ>),
                hipFuncAttributeMaxDynamicSharedMemorySize,
                (int)most) == hipSuccess;
   }();
   TORCH_CHECK(once && shmem <= most, "shared_kv_attend: LDS size");
-  hipLaunchKernelGGL((shared_kv_attend_kernel<HCP, NI>), grid, dim3(BLOCK),
+  hipLaunchKernelGGL((shared_kv_attend_kernel<SZ>), grid, dim3(BLOCK),
                      shmem, stream, a);
 }
 
@@ -406,6 +480,16 @@ void check_mask(const at::Tensor &y, int64_t window, int64_t chunk,
                 "shared_kv: sink [heads] f32");
 }
 
+// Two maps: their norm's columns and the row's layout.
+void check_maps(const c10::optional<at::Tensor> &lam, int64_t count,
+                int64_t hc, int64_t voff, int64_t vc,
+                const c10::optional<at::Tensor> &sink) {
+  if (!lam.has_value()) return;
+  TORCH_CHECK(lam->is_cuda() && lam->scalar_type() == at::kFloat &&
+              lam->numel() == 1 && voff == 2 * hc && count >= 1 &&
+              count <= vc && !sink.has_value(), "shared_kv: two maps");
+}
+
 // Attention of the first n_seqs sequences, whose t_seqs tokens are the first
 // ones of y; the heads' results go to z's first columns, and to the decode
 // operand `swz` when given.
@@ -416,7 +500,9 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
                       int64_t hc, int64_t voff, at::Tensor z,
                       c10::optional<at::Tensor> swz, int64_t chunk,
                       c10::optional<at::Tensor> positions,
-                      c10::optional<at::Tensor> sink, double out_scale) {
+                      c10::optional<at::Tensor> sink, double out_scale,
+                      c10::optional<at::Tensor> lam, int64_t count,
+                      double eps) {
   const auto dt = y.scalar_type();
   const bool bf16 = dt == at::kBFloat16;
   TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous() &&
@@ -428,19 +514,21 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
               "shared_kv_attend: cache [blocks, kv heads, 16, ec]");
   const int64_t T = y.size(0), G = cache.size(1), ec = cache.size(3);
   const int64_t vc = ec - voff, wide = std::max(hc, vc);
+  const int64_t maps = lam.has_value() ? 2 : 1;
   TORCH_CHECK(heads % G == 0 && voff >= 0 && hc >= 8 && hc % 8 == 0 &&
-              voff % 8 == 0 && voff <= hc && hc <= ec && vc >= 8 &&
+              voff % 8 == 0 && voff <= maps * hc && hc <= ec && vc >= 8 &&
               ec % 8 == 0 && y.size(1) % 8 == 0 &&
-              z.size(1) % 8 == 0 && heads * hc <= y.size(1) &&
+              z.size(1) % 8 == 0 && heads * maps * hc <= y.size(1) &&
               heads * vc <= z.size(1), "shared_kv_attend: layout");
   check_mask(y, window, chunk, positions, sink, heads);
+  check_maps(lam, count, hc, voff, vc, sink);
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.is_contiguous() &&
               block_tables.scalar_type() == at::kInt &&
               cu_q.scalar_type() == at::kInt && cu_q.is_contiguous() &&
               seq_lens.scalar_type() == at::kInt && seq_lens.is_contiguous() &&
               block_tables.size(0) >= n_seqs && cu_q.numel() > n_seqs &&
               seq_lens.numel() >= n_seqs, "shared_kv_attend: batch tensors");
-  TORCH_CHECK(T * heads < (1 << 30) && n_seqs <= 65535 && t_seqs <= T,
+  TORCH_CHECK(T * heads * maps < (1 << 30) && n_seqs <= 65535 && t_seqs <= T,
               "shared_kv_attend: rows");
   if (swz.has_value())
     TORCH_CHECK(bf16 && T <= 32 && swz->is_contiguous() &&
@@ -455,9 +543,9 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   a.cu_q = cu_q.data_ptr<int>();
   a.seq_lens = seq_lens.data_ptr<int>();
   a.table_width = (int)block_tables.size(1);
-  a.heads = (int)heads;
+  a.heads = (int)(heads * maps);       // a map counts as a head
   a.kv = (int)G;
-  a.group = (int)(heads / G);
+  a.group = (int)(heads * maps / G);
   a.hc = (int)hc;
   a.vc = (int)vc;
   a.voff = (int)voff;
@@ -467,17 +555,41 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   a.positions = chunk > 0 ? positions->data_ptr<int>() : nullptr;
   a.sink = sink ? sink->data_ptr<float>() : nullptr;
   a.out_scale = (float)out_scale;
-  a.total_rows = (int)(t_seqs * heads);
+  a.total_rows = (int)(t_seqs * heads * maps);
+  a.lam = lam ? lam->data_ptr<float>() : nullptr;
+  a.count = (int)count;
+  a.eps = (float)eps;
+  a.f32 = !bf16;
   a.z = z.data_ptr();
   a.nz = z.size(1);
   a.swz = swz ? (uint16_t *)swz->data_ptr() : nullptr;
   a.nsplit = 1;
   auto stream = at::hip::getCurrentHIPStream();
 
-  if (!bf16 || wide > 256) {
+  const bool scalar = !bf16 || wide > 256 ||
+                      (size_t)WAVES * wave_bytes((int)ec) > MAX_LDS;
+  if (!scalar)
+    a.nsplit = (int)std::min<int64_t>(64, std::max<int64_t>(1, nsplit));
+  at::Tensor po, pml;
+  if (a.nsplit > 1 || maps > 1) {
+    const auto f32 = y.options().dtype(at::kFloat);
+    po = at::empty({a.nsplit, a.total_rows, vc}, f32);
+    pml = at::empty({a.nsplit, a.total_rows, 2}, f32);
+    a.part_o = po.data_ptr<float>();
+    a.part_ml = pml.data_ptr<float>();
+  }
+  auto combine = [&]() {
+    if (maps > 1)
+      hipLaunchKernelGGL(shared_kv_diff_combine_kernel, dim3(a.total_rows / 2),
+                         dim3(64), 0, stream, a);
+    else if (a.nsplit > 1)
+      hipLaunchKernelGGL(shared_kv_combine_kernel, dim3(a.total_rows),
+                         dim3(64), 0, stream, a);
+  };
+  if (scalar) {
     TORCH_CHECK(wide <= 1024, "shared_kv_attend: heads of ", wide);
     a.scale = (float)scale;
-    const dim3 grid(max_q * heads, n_seqs);
+    const dim3 grid(max_q * a.heads, n_seqs);
     const size_t shmem = 4 * vc * sizeof(float);
     auto pick = [&](auto tag) {
       using E = decltype(tag);
@@ -492,26 +604,18 @@ void shared_kv_attend(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
     };
     if (bf16) pick(uint16_t{});
     else pick(float{});
+    combine();
     return;
   }
 
   a.scale = (float)(scale * 1.4426950408889634);
-  a.nsplit = (int)std::min<int64_t>(64, std::max<int64_t>(1, nsplit));
-  at::Tensor po, pml;
-  if (a.nsplit > 1) {
-    const auto f32 = y.options().dtype(at::kFloat);
-    po = at::empty({a.nsplit, t_seqs * heads, vc}, f32);
-    pml = at::empty({a.nsplit, t_seqs * heads, 2}, f32);
-    a.part_o = po.data_ptr<float>();
-    a.part_ml = pml.data_ptr<float>();
-  }
   const int64_t tiles = (max_q * a.group + M - 1) / M;
   TORCH_CHECK(tiles * G <= 65535, "shared_kv_attend: portion of ", max_q);
   const dim3 grid(a.nsplit, tiles * G, n_seqs);
-  pick_sizes((int)wide, (int)ec, [&](auto h, auto n) {
-    launch_attend<decltype(h)::value, decltype(n)::value>(a, grid, stream);
-  });
-  if (a.nsplit > 1)
-    hipLaunchKernelGGL(shared_kv_combine_kernel, dim3(a.total_rows), dim3(64),
-                       0, stream, a);
+  auto go = [&](auto size) {
+    launch_attend<decltype(size)>(a, grid, stream);
+  };
+  if (maps > 1) pick_sizes2((int)hc, (int)vc, go);
+  else pick_sizes((int)wide, (int)ec, go);
+  combine();
 }

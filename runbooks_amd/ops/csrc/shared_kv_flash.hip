@@ -6,6 +6,10 @@
 // on a lane pair; the same LDS rows serve as keys, read by rows, and as
 // values, read by columns (ds_read_b64_tr_b16).
 //
+// With two maps 64 (token, head) pairs per workgroup: two waves take the first
+// key's scores, two the second's, over the same tiles; the latter hand their
+// result to the former through LDS, which subtract it and norm.
+//
 // Blocks of one kv head are `kv` apart in launch order, so with a head count
 // divisible by the XCDs a head's keys stay in one L2.
 
@@ -30,11 +34,13 @@ RB_DEV unsigned pack2(float lo, float hi) {
   return c.u;
 }
 
-template <int HCP, int NI>
-__global__ __launch_bounds__(BLOCK, HCP > 128 ? 1 : 2)
+template <typename SZ>
+__global__ __launch_bounds__(BLOCK, SZ::HCP > 128 ? 1 : 2)
 void shared_kv_flash_kernel(Args a, int first_seq) {
-  constexpr int QSTEPS = HCP / 16;
+  constexpr int HCP = SZ::HCP, NI = SZ::NI, MAPS = SZ::MAPS;
+  constexpr int QSTEPS = SZ::HCK / 16;
   constexpr int DT = HCP / 32;
+  constexpr int QR = QB / MAPS;                // (token, head) pairs
 
   extern __shared__ __attribute__((aligned(16))) char smem[];
 
@@ -42,13 +48,15 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
   const int q_tok0 = a.cu_q[seq], nq = a.cu_q[seq + 1] - q_tok0;
   const int rows = nq * a.group;
   // the blocks with the most keys first
-  const int q0 = (gridDim.y - 1 - blockIdx.y) * QB;
+  const int q0 = (gridDim.y - 1 - blockIdx.y) * QR;
   if (q0 >= rows) return;
   const int rel = a.seq_lens[seq] - nq;        // retained position of query 0
   const int g = blockIdx.x;
   const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
   const int hi = lane >> 5, col = lane & 31;
-  const int qi = q0 + wid * 32 + col;          // this lane's query row
+  const int map = MAPS == 2 ? wid / 2 : 0;
+  const int wrow = q0 + wid % (4 / MAPS) * 32;
+  const int qi = wrow + col;                   // this lane's query row
   const bool q_ok = qi < rows;
   const int tok = (q_ok ? qi : 0) / a.group;
   const int head = g * a.group + (q_ok ? qi : 0) % a.group;
@@ -58,9 +66,8 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
   const int stride = row_stride(a.ec);
 
   // key range of the workgroup, and of this wave's queries
-  const int wg_hi = rel + (min(rows, q0 + QB) - 1) / a.group + 1;
+  const int wg_hi = rel + (min(rows, q0 + QR) - 1) / a.group + 1;
   const int wg_lo = max(0, first_key(a, rel + q0 / a.group, dropped));
-  const int wrow = q0 + wid * 32;
   const int first = rel + wrow / a.group;
   const int last =
       wrow < rows ? rel + (min(rows, wrow + 32) - 1) / a.group : -1;
@@ -88,7 +95,7 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
   bf16x8v qf[QSTEPS];
   {
     const uint16_t *qp = (const uint16_t *)a.y + (q_tok0 + tok) * a.ny +
-                         head * a.hc;
+                         (head * MAPS + map) * a.hc;
 #pragma unroll
     for (int s = 0; s < QSTEPS; ++s) {
       const int d = s * 16 + hi * 8;
@@ -126,7 +133,8 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
       const int k0 = t * KB + it * 32;
       if (k0 > last || k0 + 31 < lo_first) continue;          // wave-uniform
       f32x16v s = (f32x16v)(0.0f);
-      const char *kp = smem + (it * 32 + col) * stride + hi * 16;
+      const char *kp = smem + (it * 32 + col) * stride + hi * 16 +
+                       map * a.hc * 2;
 #pragma unroll
       for (int ks = 0; ks < QSTEPS; ++ks) {
         const bf16x8v kf = *reinterpret_cast<const bf16x8v *>(kp + ks * 32);
@@ -188,9 +196,43 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
     }
   }
 
-  if (!q_ok) return;
   const float l = l_run + __shfl_xor(l_run, 32, 64);
-  const float inv = a.out_scale / l;
+  float inv = a.out_scale / l;
+  if constexpr (MAPS == 2) {
+    f32x4v *ex = reinterpret_cast<f32x4v *>(smem) + wid % 2 * DT * 4 * 64 +
+                 lane;
+    __syncthreads();                           // the tile has been read
+    if (map == 1) {
+      const float f = a.lam[0] / l;
+#pragma unroll
+      for (int d = 0; d < DT; ++d)
+#pragma unroll
+        for (int rq = 0; rq < 4; ++rq)
+          ex[(d * 4 + rq) * 64] =
+              (f32x4v){acc[d][rq * 4] * f, acc[d][rq * 4 + 1] * f,
+                       acc[d][rq * 4 + 2] * f, acc[d][rq * 4 + 3] * f};
+    }
+    __syncthreads();
+    if (map == 1) return;
+    inv = 1.0f / l;
+    float sum = 0.0f;
+#pragma unroll
+    for (int d = 0; d < DT; ++d)
+#pragma unroll
+      for (int rq = 0; rq < 4; ++rq) {
+        const f32x4v o2 = ex[(d * 4 + rq) * 64];
+        const bool real = d * 32 + 8 * rq + 4 * hi < a.vc;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float o = acc[d][rq * 4 + e] * inv - o2[e];
+          acc[d][rq * 4 + e] = o;
+          sum += real ? o * o : 0.0f;
+        }
+      }
+    sum += __shfl_xor(sum, 32, 64);
+    inv = a.out_scale / sqrtf(sum / (float)a.count + a.eps);
+  }
+  if (!q_ok) return;
   uint16_t *zp = (uint16_t *)a.z + (q_tok0 + tok) * a.nz + head * a.vc;
 #pragma unroll
   for (int d = 0; d < DT; ++d)
@@ -206,20 +248,25 @@ void shared_kv_flash_kernel(Args a, int first_seq) {
     }
 }
 
-template <int HCP, int NI>
+template <typename SZ>
 void launch_flash(const Args &a, int first_seq, dim3 grid,
                   hipStream_t stream) {
-  constexpr size_t most = (size_t)KB * row_stride(2 * HCP) + SLACK;
+  // a tile, or two waves' results
+  constexpr size_t merge = SZ::MAPS == 1 ? 0 : (size_t)2 * SZ::HCP * 128;
+  constexpr size_t most = std::max(
+      merge, (size_t)KB * row_stride(SZ::MAPS == 1 ? 2 * SZ::HCP
+                                     : 2 * SZ::HCK + SZ::HCP) + SLACK);
   static bool once = [] {
     return hipFuncSetAttribute(
                reinterpret_cast<const void *>(
-                   &shared_kv_flash_kernel<HCP, NI>),
+                   &shared_kv_flash_kernel<SZ>),
                hipFuncAttributeMaxDynamicSharedMemorySize,
                (int)most) == hipSuccess;
   }();
-  const size_t shmem = (size_t)KB * row_stride(a.ec) + SLACK;
+  const size_t shmem =
+      std::max(merge, (size_t)KB * row_stride(a.ec) + SLACK);
   TORCH_CHECK(once && shmem <= most, "shared_kv_flash: LDS size");
-  hipLaunchKernelGGL((shared_kv_flash_kernel<HCP, NI>), grid, dim3(BLOCK),
+  hipLaunchKernelGGL((shared_kv_flash_kernel<SZ>), grid, dim3(BLOCK),
                      shmem, stream, a, first_seq);
 }
 
@@ -228,6 +275,9 @@ void launch_flash(const Args &a, int first_seq, dim3 grid,
 void check_mask(const at::Tensor &y, int64_t window, int64_t chunk,
                 const c10::optional<at::Tensor> &positions,
                 const c10::optional<at::Tensor> &sink, int64_t heads);
+void check_maps(const c10::optional<at::Tensor> &lam, int64_t count,
+                int64_t hc, int64_t voff, int64_t vc,
+                const c10::optional<at::Tensor> &sink);
 
 // Attention of the sequences first_seq .. first_seq + n_seqs - 1.
 void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
@@ -236,7 +286,9 @@ void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
                      int64_t window, int64_t heads, int64_t hc, int64_t voff,
                      at::Tensor z, int64_t chunk,
                      c10::optional<at::Tensor> positions,
-                     c10::optional<at::Tensor> sink, double out_scale) {
+                     c10::optional<at::Tensor> sink, double out_scale,
+                     c10::optional<at::Tensor> lam, int64_t count,
+                     double eps) {
   TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous() &&
               y.scalar_type() == at::kBFloat16 && z.dim() == 2 &&
               z.is_contiguous() && z.size(0) == y.size(0) &&
@@ -245,13 +297,15 @@ void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
               cache.is_contiguous() && cache.scalar_type() == at::kBFloat16,
               "shared_kv_flash: cache [blocks, kv heads, 16, ec]");
   const int64_t G = cache.size(1), ec = cache.size(3), vc = ec - voff;
+  const int64_t maps = lam.has_value() ? 2 : 1;
   TORCH_CHECK(heads % G == 0 && voff >= 0 && hc >= 8 && hc <= 256 &&
-              hc % 8 == 0 && voff % 8 == 0 && voff <= hc && hc <= ec &&
+              hc % 8 == 0 && voff % 8 == 0 && voff <= maps * hc && hc <= ec &&
               vc >= 8 && vc <= 256 && ec % 8 == 0 &&
               y.size(1) % 8 == 0 && z.size(1) % 8 == 0 &&
-              heads * hc <= y.size(1) && heads * vc <= z.size(1),
+              heads * maps * hc <= y.size(1) && heads * vc <= z.size(1),
               "shared_kv_flash: layout");
   check_mask(y, window, chunk, positions, sink, heads);
+  check_maps(lam, count, hc, voff, vc, sink);
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.is_contiguous() &&
               block_tables.scalar_type() == at::kInt &&
               cu_q.scalar_type() == at::kInt && cu_q.is_contiguous() &&
@@ -282,15 +336,20 @@ void shared_kv_flash(at::Tensor y, at::Tensor cache, at::Tensor block_tables,
   a.positions = chunk > 0 ? positions->data_ptr<int>() : nullptr;
   a.sink = sink ? sink->data_ptr<float>() : nullptr;
   a.out_scale = (float)out_scale;
+  a.lam = lam ? lam->data_ptr<float>() : nullptr;
+  a.count = (int)count;
+  a.eps = (float)eps;
   a.scale = (float)(scale * 1.4426950408889634);
   a.z = z.data_ptr();
   a.nz = z.size(1);
-  const int64_t blocks = (max_q * a.group + QB - 1) / QB;
+  const int64_t rows = QB / maps;
+  const int64_t blocks = (max_q * a.group + rows - 1) / rows;
   TORCH_CHECK(blocks <= 65535, "shared_kv_flash: portion of ", max_q);
   const dim3 grid(G, blocks, n_seqs);
   auto stream = at::hip::getCurrentHIPStream();
-  pick_sizes((int)std::max(hc, vc), (int)ec, [&](auto h, auto n) {
-    launch_flash<decltype(h)::value, decltype(n)::value>(a, (int)first_seq,
-                                                         grid, stream);
-  });
+  auto go = [&](auto size) {
+    launch_flash<decltype(size)>(a, (int)first_seq, grid, stream);
+  };
+  if (maps > 1) pick_sizes2((int)hc, (int)vc, go);
+  else pick_sizes((int)std::max(hc, vc), (int)ec, go);
 }

@@ -199,17 +199,20 @@ def delta_chunk(y, y2, lay, conv_w, decay, state, batch, o):
         lay.kv_heads, lay.dim)
 
 
-def delta_out(o, lay, w, y2, z, eps, swz, y, state, batch):
-    """z = rmsnorm per head(o) * w * sigmoid(gate), padding zero. w [vc]
-    fp32. After it the slots hold the convolution's last inputs."""
+def delta_out(o, lay, w, gate, z, eps, swz, y, tails, batch, end=None):
+    """z = rmsnorm per head(o) * w * sigmoid(gate's columns from lay.off_g),
+    zeros behind it up to column `end` (None: all). w fp32, [vc] for every
+    head or [heads * vc]. After it the slots hold the last inputs, y's first
+    columns, of the convolution (tails None: there is none)."""
+    end = z.shape[1] if end is None else end
     if not _backend.use_hip(o):
         T = o.shape[0]
         r = o.view(T, lay.heads, lay.vc)
         r = r * torch.rsqrt(r.pow(2).sum(-1, keepdim=True) / lay.vdim + eps)
-        g = torch.sigmoid(y2[:, lay.off_g:lay.off_g + lay.n_o].float())
-        z[:, :lay.n_o] = ((r * w).view(T, -1) * g).to(z.dtype)
-        z[:, lay.n_o:] = 0
+        g = torch.sigmoid(gate[:, lay.off_g:lay.off_g + lay.n_o].float())
+        z[:, :lay.n_o] = ((r * w.view(-1, lay.vc)).view(T, -1) * g).to(z.dtype)
+        z[:, lay.n_o:end] = 0
         return
-    _backend.ext().delta_out(o, w, y2, lay.off_g, z, swz, lay.vdim, eps, y,
-                             state[1], batch.positions, batch.cu_q,
-                             batch.state_slots, batch.n_seqs)
+    _backend.ext().delta_out(o, w, gate, lay.off_g, z, swz, lay.heads,
+                             lay.vdim, eps, y, tails, batch.positions,
+                             batch.cu_q, batch.state_slots, batch.n_seqs, end)

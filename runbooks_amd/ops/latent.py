@@ -14,6 +14,14 @@ projection `y` and one output projection that reads `z`:
   * ``latent_flash``   the same attention for long portions, on keys and
                        values expanded from the context's latents
 
+Without a rotated part and with queries from a latent of their own,
+
+    y = [ query latent | latent | gates ],   q = product of the former
+
+``latent_norms`` takes the place of latent_prep: it norms both latents; the
+other ops then read q in a tensor of its own. The output gate is one number
+per value column, or (head_gate) one per head.
+
 Every per-head or per-section size is padded to a multiple of 8 elements
 inside y, z, the cache and the packed weights (zero rows), so the kernels
 read 16 bytes per lane for any model size.
@@ -256,7 +264,18 @@ def _attend_ref(q_lat, y, lay, cache, batch, scale, window):
     return out
 
 
-def _flash_ref(y, lay, kv, ctx, meta, scale, window, z):
+def gated_ref(o, lay, gate, off, head_gate):
+    """o [T, H, vc] times the sigmoid gates in `gate`'s columns from off."""
+    T = o.shape[0]
+    if head_gate:
+        g = gate[:, off:off + lay.heads].float()[..., None]
+    else:
+        g = gate[:, off:off + lay.heads * lay.vc].float().view(o.shape)
+    return (o * torch.sigmoid(g)).reshape(T, -1)
+
+
+def _flash_ref(y, lay, kv, ctx, meta, scale, window, z, gate, off_g,
+               head_gate):
     for q0, nq, k0, nk, rel in meta.tolist():
         q = y[q0:q0 + nq, :lay.off_kv].view(nq, lay.heads, lay.qc).float()
         e = kv[k0:k0 + nk].view(nk, lay.heads, lay.dimc + lay.vc).float()
@@ -267,9 +286,8 @@ def _flash_ref(y, lay, kv, ctx, meta, scale, window, z):
         p = _masked_softmax_ref(s, torch.arange(nq) + rel, torch.arange(nk),
                                 window)
         o = torch.einsum("hqk,khv->qhv", p, e[..., lay.dimc:])
-        g = y[q0:q0 + nq, lay.off_g:lay.off_gate].float()
-        z[q0:q0 + nq, :lay.off_act] = (
-            o.reshape(nq, -1) * torch.sigmoid(g)).to(z.dtype)
+        z[q0:q0 + nq, :lay.off_act] = gated_ref(
+            o, lay, gate[q0:q0 + nq], off_g, head_gate).to(z.dtype)
 
 
 # ---------------------------------------------------------------------------
@@ -294,6 +312,30 @@ def latent_prep(y, lay, cos, sin, positions, slots, cache, norm_w, eps, mlp,
         lay.fc, lay.off_act, eps, limit, alpha, shift)
 
 
+def latent_norms(y, parts, eps, slots, cache, swz=None):
+    """RMS norms of both latents in y. parts: (first columns, sizes, weights
+    fp32) of the query latent and of the cached one, as three pairs. Returns
+    the former, [T, its size padded to 32]; the latter goes to `cache` at
+    `slots`."""
+    (oq, oc), (nq, nc), (wq, wc) = parts
+    out = torch.empty(y.shape[0], pad_to(nq, 32), dtype=y.dtype,
+                      device=y.device)
+    if not _backend.use_hip(y):
+        def norm(at, n, w):
+            c = y[:, at:at + n].float()
+            return (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) *
+                    w).to(y.dtype)
+        out.zero_()
+        out[:, :nq] = norm(oq, nq, wq)
+        cache.view(-1, cache.shape[-1])[slots.long(), :nc] = norm(oc, nc, wc)
+        return out
+    _backend.ext().latent_norms(y, oq, nq, wq, out, swz, oc, nc, wc, cache,
+                                slots, eps)
+    if swz is not None:
+        out._rb_swz = swz
+    return out
+
+
 def latent_absorb(y, lay, w_absorb, T):
     """First T rows of q, unrotated part, into latent space:
     [T, heads, rc]."""
@@ -304,23 +346,24 @@ def latent_absorb(y, lay, w_absorb, T):
     out = torch.empty(T, lay.heads, lay.rc, dtype=y.dtype, device=y.device)
     _backend.ext().head_gemm(
         y, 0, lay.qc, w_absorb, lay.dimc, lay.rc, out.view(T, -1), 0, lay.rc,
-        None, 0, None, T, lay.heads)
+        None, 0, None, T, lay.heads, False)
     return out
 
 
-def latent_expand(o_lat, lay, w_expand, y, z, swz=None):
-    """z's head part of the first rows: value-space heads times the
-    sigmoid output gate (in y)."""
+def latent_expand(o_lat, lay, w_expand, gate, z, swz=None, off_g=None,
+                  head_gate=False):
+    """z's head part of the first rows: value-space heads times the sigmoid
+    output gates, in columns of `gate` from off_g (None: as y has them)."""
     T = o_lat.shape[0]
-    if not _backend.use_hip(y):
+    off_g = lay.off_g if off_g is None else off_g
+    if not _backend.use_hip(o_lat):
         o = torch.einsum("thr,hrv->thv", o_lat.float(), w_expand.float())
-        g = y[:T, lay.off_g:lay.off_gate].float()
-        z[:T, :lay.off_act] = (o.reshape(T, -1) *
-                               torch.sigmoid(g)).to(z.dtype)
+        z[:T, :lay.off_act] = gated_ref(o, lay, gate[:T], off_g,
+                                        head_gate).to(z.dtype)
         return
     _backend.ext().head_gemm(
         o_lat.view(T, -1), 0, lay.rc, w_expand, lay.rc, lay.vc, z, 0, lay.vc,
-        y, lay.off_g, swz, T, lay.heads)
+        gate, off_g, swz, T, lay.heads, head_gate)
 
 
 def attend_split(n_seqs: int, row_tiles: int, max_keys: int | None,
@@ -360,12 +403,16 @@ def latent_flash_supported(lay: LatentLayout, dtype) -> bool:
     return lay.dimc + lay.rotc <= 256 and lay.vc <= 256
 
 
-def latent_flash(y, lay, kv, ctx, meta, max_q, scale, window, z):
+def latent_flash(y, lay, kv, ctx, meta, max_q, scale, window, z, gate=None,
+                 off_g=None, head_gate=False):
     """z's head part of the long portions. kv [Tk, H, dimc + vc]: keys and
     values expanded from the context rows `ctx` [Tk, ec]; meta rows as in
-    RaggedBatch.long_plans."""
+    RaggedBatch.long_plans; gates as in latent_expand (None: in y)."""
+    gate = y if gate is None else gate
+    off_g = lay.off_g if off_g is None else off_g
     if not _backend.use_hip(y):
-        return _flash_ref(y, lay, kv, ctx, meta, scale, window, z)
+        return _flash_ref(y, lay, kv, ctx, meta, scale, window, z, gate,
+                          off_g, head_gate)
     _backend.ext().latent_flash(y, kv, ctx, meta, z, lay.heads, lay.dimc,
-                                lay.rotc, lay.vc, lay.rc, lay.off_g, max_q,
-                                scale, window or 0)
+                                lay.rotc, lay.vc, lay.rc, gate, off_g,
+                                head_gate, max_q, scale, window or 0)

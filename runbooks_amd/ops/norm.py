@@ -47,18 +47,19 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float = 1e-5) -> torch.T
 
 def rmsnorm_res32(x: torch.Tensor, delta: torch.Tensor | None,
                   weight: torch.Tensor, eps: float, dtype: torch.dtype,
-                  operand: bool = False) -> torch.Tensor:
+                  operand: bool = False, offset: float = 0.0
+                  ) -> torch.Tensor:
     """Norm of a 32-bit residual: x [T, D] fp32 += delta in place, returns
-    rmsnorm(x) * weight in `dtype`. delta: fp32 or `dtype` [T, D], an
+    rmsnorm(x) * (offset + weight) in `dtype`. delta: fp32 or `dtype` [T, D], an
     uncombined fp32 split-K slab [split, T, D], or None. operand=True also
     attaches the decode GEMM's pre-swizzled operand (T <= 32)."""
     if not _backend.use_hip(x):
         if delta is not None:
             x += delta.float() if delta.dim() == 2 else delta.sum(0)
-        return rmsnorm_ref(x, weight, eps).to(dtype)
+        return rmsnorm_ref(x, offset + weight.float(), eps).to(dtype)
     y, swz = _backend.ext().rmsnorm_res32(
         x, None if delta is None else delta.contiguous(), weight, eps,
-        operand)
+        operand, offset)
     if operand:
         y._rb_swz = swz
     return y
@@ -95,7 +96,8 @@ def norm_res32(norm: torch.nn.Module, x: torch.Tensor,
     """x += delta, then `norm` (an RMSNorm, or a LayerNorm with bias)."""
     bias = getattr(norm, "bias", None)
     if bias is None:
-        return rmsnorm_res32(x, delta, norm.weight, norm.eps, dtype, operand)
+        return rmsnorm_res32(x, delta, norm.weight, norm.eps, dtype, operand,
+                             norm.offset)
     return layernorm_res32(x, delta, norm.weight, bias, norm.eps, dtype,
                            operand)
 
@@ -117,12 +119,19 @@ def join_res32(x: torch.Tensor, delta: torch.Tensor | None,
 
 
 class RMSNorm(torch.nn.Module):
-    def __init__(self, dim: int, eps: float = 1e-5, dtype=None):
+    """`offset` is added to the stored weight (served residual norms
+    only)."""
+
+    def __init__(self, dim: int, eps: float = 1e-5, dtype=None,
+                 offset: float = 0.0):
         super().__init__()
-        self.weight = torch.nn.Parameter(torch.ones(dim, dtype=dtype))
-        self.eps = eps
+        self.weight = torch.nn.Parameter(
+            torch.full((dim,), 1.0 - offset, dtype=dtype))
+        self.eps, self.offset = eps, offset
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
+        if self.offset:
+            raise NotImplementedError("RMSNorm.forward with an offset")
         return rmsnorm(x, self.weight, self.eps)
 
     def extra_repr(self) -> str:

@@ -1,17 +1,22 @@
 """Attention on keys and values of their own, over the paged rows of
-ops/shared_kv.py: normed, rotated queries and keys.
+ops/shared_kv.py: queries and keys that are normed and rotated, or that pass,
+with the values, a short causal convolution.
 
 Around one projection `y` and one output projection that reads `z`:
 
     y = [ q heads | k heads | v heads | .. ],   z = [ heads of the result | .. ]
 
   * ``qkv_prep``  RMS norms and rotations of q (in y) and k, cache write
+  * ``qkv_conv``  biases and convolutions of q (to a tensor of its own), k
+    and v, cache write, the convolutions' last inputs to the slots
 
-then shared_kv_attend and shared_kv_flash. A cached row is [ key | value ];
-sizes per head are padded to a multiple of 8 with zero rows of the packed
-weight.
+then shared_kv_attend and shared_kv_flash. With several maps a head has a
+query, and a kv head a key, for each, all with the kv head's value. A cached
+row is [ keys | value ]; sizes per head are padded to a multiple of 8 with
+zero rows of the packed weight.
 
-GPU tensors run csrc/qkv_prep.hip; CPU tensors the plain reference here.
+GPU tensors run csrc/qkv_prep.hip and csrc/qkv_conv.hip; CPU tensors the plain
+references here.
 """
 from __future__ import annotations
 
@@ -20,6 +25,7 @@ from dataclasses import dataclass
 import torch
 
 from . import _backend
+from .canon import history_ref
 from .kvcache import BLOCK_SIZE
 from .latent import _pad_rows, pad_to, rope_interleaved_ref
 
@@ -32,7 +38,8 @@ class QKVLayout:
     kv_heads: int
     dim: int
     vdim: int
-    rot: int                   # rotated dimensions
+    rot: int = 0               # rotated dimensions
+    maps: int = 1              # attention maps per head
 
     @property
     def group(self):
@@ -48,19 +55,19 @@ class QKVLayout:
 
     @property
     def ec(self):              # one cached row
-        return self.hc + self.vc
+        return self.voff + self.vc
 
     @property
     def voff(self):            # first column of the value in a row
-        return self.hc
+        return self.maps * self.hc
 
     @property
     def off_k(self):
-        return self.heads * self.hc
+        return self.heads * self.maps * self.hc
 
     @property
     def off_v(self):
-        return self.off_k + self.kv_heads * self.hc
+        return self.off_k + self.kv_heads * self.maps * self.hc
 
     @property
     def n_y(self):
@@ -73,8 +80,9 @@ class QKVLayout:
 
 def pack_qkv(lay: QKVLayout, q, k, v):
     """Rows of the joint projection, in y's layout."""
-    return torch.cat([_pad_rows(q, lay.heads, (lay.dim,), (lay.hc,)),
-                      _pad_rows(k, lay.kv_heads, (lay.dim,), (lay.hc,)),
+    m = lay.maps
+    return torch.cat([_pad_rows(q, lay.heads * m, (lay.dim,), (lay.hc,)),
+                      _pad_rows(k, lay.kv_heads * m, (lay.dim,), (lay.hc,)),
                       _pad_rows(v, lay.kv_heads, (lay.vdim,), (lay.vc,))])
 
 
@@ -116,3 +124,43 @@ def qkv_prep(y, lay: QKVLayout, cos, sin, positions, slots, cache, norms,
                          eps)
     _backend.ext().qkv_prep(y, cos, sin, positions, slots, cache, norms,
                             lay.heads, lay.dim, lay.hc, eps)
+
+
+def _conv_ref(y, lay, bias, conv_w, tails, batch, cache, q):
+    T, n = y.shape[0], lay.n_y
+    out = torch.empty(T, n)
+    for b in range(batch.n_seqs):
+        t0, t1 = int(batch.cu_q[b]), int(batch.cu_q[b + 1])
+        slot, p0 = int(batch.state_slots[b]), int(batch.positions[t0])
+        rows = history_ref(y[t0:t1, :n].float(), tails[slot], p0)
+        pos = torch.arange(p0 - rows.shape[0] + t1 - t0, p0 + t1 - t0)
+        u = rows + bias * (pos >= 0)[:, None]     # none before the start
+        out[t0:t1] = sum(u[j:j + t1 - t0] * w for j, w in enumerate(conv_w))
+        tails[slot] = rows[t1 - t0:].to(tails.dtype)
+    q.copy_(out[:, :lay.off_k])
+    s = batch.slots.long()
+    cache[s // BLOCK_SIZE, :, s % BLOCK_SIZE] = torch.cat(
+        [out[:, lay.off_k:lay.off_v].view(T, lay.kv_heads, lay.voff),
+         out[:, lay.off_v:].view(T, lay.kv_heads, lay.vc)],
+        dim=-1).to(cache.dtype)
+
+
+def alloc_conv_tails(slots: int, taps: int, lay: QKVLayout, device, dtype):
+    """The last projections of every slot, the oldest first."""
+    return torch.zeros(slots, taps - 1, lay.n_y, device=device, dtype=dtype)
+
+
+def qkv_conv(y, lay: QKVLayout, bias, conv_w, tails, batch, cache):
+    """Adds the biases [n_y] to y's first columns and convolves them over
+    time with conv_w [taps, n_y] (both fp32). Returns q [T, off_k]; keys and
+    values go to `cache`. Afterwards `tails` holds the sequences' last
+    projections (without biases)."""
+    q = torch.empty(y.shape[0], lay.off_k, dtype=y.dtype, device=y.device)
+    if not _backend.use_hip(y):
+        _conv_ref(y, lay, bias, conv_w, tails, batch, cache, q)
+        return q
+    _backend.ext().qkv_conv(
+        y, bias, conv_w, tails, batch.positions, batch.cu_q,
+        batch.state_slots, batch.seq_of, batch.slots, batch.single,
+        batch.n_seqs, cache, lay.voff, q)
+    return q

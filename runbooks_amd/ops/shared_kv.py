@@ -155,17 +155,29 @@ def visible_ref(qpos, kpos, window, chunk=None, dropped=0):
     return seen
 
 
+@dataclass(frozen=True)
+class DiffMaps:
+    """Two attention maps per head, the second one's result subtracted:
+    rms_norm(o1 - factor o2) per head."""
+    factor: torch.Tensor       # [1] fp32
+    vdim: int                  # columns the norm counts
+    eps: float
+
+
 def _attend_ref(y, lay, cache, batch, seqs, scale, window, z, chunk=None,
-                sink=None, out_scale=1.0):
+                sink=None, out_scale=1.0, diff=None):
+    maps = 1 if diff is None else 2
     for b in seqs:
         t0, t1 = int(batch.cu_q[b]), int(batch.cu_q[b + 1])
         n = int(batch.seq_lens[b])
         pos = torch.arange(n)
         blk = batch.block_tables[b].long()[pos // BLOCK_SIZE]
         rows = cache[blk, :, pos % BLOCK_SIZE].float()     # [n, G, ec]
+        # group members are heads, or (head, map) pairs
         q = y[t0:t1, :lay.off_k].float().view(
-            t1 - t0, lay.kv_heads, lay.group, lay.hc)
-        s = torch.einsum("qgrd,kgd->grqk", q, rows[..., :lay.hc]) * scale
+            t1 - t0, lay.kv_heads, lay.group, maps, lay.hc)
+        k = rows[..., :maps * lay.hc].view(n, lay.kv_heads, maps, lay.hc)
+        s = torch.einsum("qgrmd,kgmd->grmqk", q, k).flatten(1, 2) * scale
         dropped = int(batch.positions[t0]) - (n - (t1 - t0))
         hidden = ~visible_ref(pos[n - (t1 - t0):], pos, window, chunk,
                               dropped)
@@ -176,6 +188,10 @@ def _attend_ref(y, lay, cache, batch, seqs, scale, window, z, chunk=None,
             s = torch.cat([s, extra], dim=-1)
         p = torch.softmax(s, dim=-1)[..., :n]
         o = torch.einsum("grqk,kgd->qgrd", p, rows[..., lay.voff:])
+        if diff is not None:
+            o = o[:, :, 0::2] - diff.factor * o[:, :, 1::2]
+            o = o * torch.rsqrt(o.pow(2).sum(-1, keepdim=True) / diff.vdim +
+                                diff.eps)
         o = (o * out_scale).reshape(t1 - t0, -1)
         z[t0:t1, :o.shape[1]] = o.to(z.dtype)
 
@@ -207,22 +223,30 @@ def attend_split(n_seqs: int, workgroups: int, max_keys: int | None,
 
 
 def shared_kv_attend(y, lay, cache, batch, scale, window, z, swz=None,
-                     chunk=None, sink=None, out_scale=1.0):
+                     chunk=None, sink=None, out_scale=1.0, diff=None):
     """z's first t_short rows: attention of the batch's short portions. A
     query at retained position i sees keys j with 0 <= i - j < window, or
     those up to its own of its chunk. `sink` [heads] fp32: one more entry of
-    the softmax's denominator. The result is multiplied by out_scale."""
+    the softmax's denominator. The result is multiplied by out_scale. With
+    `diff` (DiffMaps) every head has two queries, the kv heads' rows two keys,
+    [ key | key | value ]."""
     if not _backend.use_hip(y):
         return _attend_ref(y, lay, cache, batch, range(batch.n_short), scale,
-                           window, z, chunk, sink, out_scale)
-    tiles = -(-batch.max_q * lay.group // 16) * lay.kv_heads
+                           window, z, chunk, sink, out_scale, diff)
+    maps = 1 if diff is None else 2
+    tiles = -(-batch.max_q * lay.group * maps // 16) * lay.kv_heads
     nsplit = attend_split(batch.n_short, tiles, batch.max_keys,
                           window or chunk, batch.max_q)
     _backend.ext().shared_kv_attend(
         y, cache, batch.block_tables, batch.cu_q, batch.seq_lens,
         batch.n_short, batch.t_short, batch.max_q, nsplit, scale, window or 0,
         lay.heads, lay.hc, lay.voff, z, swz, chunk or 0, batch.positions,
-        sink, out_scale)
+        sink, out_scale, *_diff_args(diff))
+
+
+def _diff_args(diff):
+    return (None, 0, 0.0) if diff is None else (diff.factor, diff.vdim,
+                                                diff.eps)
 
 
 def shared_kv_flash_supported(lay: SharedKVLayout, dtype) -> bool:
@@ -230,14 +254,15 @@ def shared_kv_flash_supported(lay: SharedKVLayout, dtype) -> bool:
 
 
 def shared_kv_flash(y, lay, cache, batch, scale, window, z, chunk=None,
-                    sink=None, out_scale=1.0):
+                    sink=None, out_scale=1.0, diff=None):
     """z's other rows: the same attention for the long portions."""
     n = batch.n_seqs - batch.n_short
     if not _backend.use_hip(y):
         return _attend_ref(y, lay, cache, batch,
                            range(batch.n_short, batch.n_seqs), scale, window,
-                           z, chunk, sink, out_scale)
+                           z, chunk, sink, out_scale, diff)
     _backend.ext().shared_kv_flash(
         y, cache, batch.block_tables, batch.cu_q, batch.seq_lens,
         batch.n_short, n, batch.max_q_long, scale, window or 0, lay.heads,
-        lay.hc, lay.voff, z, chunk or 0, batch.positions, sink, out_scale)
+        lay.hc, lay.voff, z, chunk or 0, batch.positions, sink, out_scale,
+        *_diff_args(diff))

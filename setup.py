@@ -19,28 +19,31 @@ CSRC = ROOT / "runbooks_amd" / "ops" / "csrc"
 
 # One extension module per group, so that a caller can build just what a
 # model needs (RB_EXT_GROUPS=core,latent): `core` holds the ops every
-# served model runs, `latent` the latent-attention kernels, `hybrid` the
-# attention on shared keys and values and the lightning attention, `streams`
-# the layers around several residual streams, `main` the rest.
-CORE = ("rmsnorm", "layernorm", "glu", "decode_gemm", "sampling")
-STREAMS = ("streams", "qkv_prep", "delta", "min_gru", "moe")
+# served model runs, `latent` the latent-attention kernels, `shared_kv` the
+# attention over rows of keys and values, `lightning` the lightning attention,
+# `delta` the delta rules, `streams` the layers around several residual
+# streams, `dual` those with norms and input convolutions side by side, `main`
+# the rest.
+GROUPS = {"core": ("rmsnorm", "layernorm", "glu", "decode_gemm", "sampling"),
+          "streams": ("streams", "qkv_prep", "min_gru", "moe"),
+          "delta": ("delta", "delta_out", "general_delta"),
+          "dual": ("canon", "qkv_conv", "poly_norm")}
+PREFIXES = {"shared_kv": "shared_kv", "lightning": "lightning",
+            "latent_": "latent"}
 
 
 def _group_of(stem: str) -> str:
-    if stem in CORE:
-        return "core"
-    if stem in STREAMS:
-        return "streams"
-    if stem.startswith(("shared_kv", "lightning")):
-        return "hybrid"
-    return "latent" if stem.startswith("latent_") else "main"
+    for group, stems in GROUPS.items():
+        if stem in stems:
+            return group
+    return next((g for p, g in PREFIXES.items() if stem.startswith(p)),
+                "main")
 
 
-MODULES = {"core": ("_hip_core", "bindings_core.cpp"),
-           "latent": ("_hip_latent", "bindings_latent.cpp"),
-           "hybrid": ("_hip_hybrid", "bindings_hybrid.cpp"),
-           "streams": ("_hip_streams", "bindings_streams.cpp"),
-           "main": ("_hip", "bindings.cpp")}
+MODULES = {"main": ("_hip", "bindings.cpp"),
+           **{g: (f"_hip_{g}", f"bindings_{g}.cpp")
+              for g in ("core", "latent", "shared_kv", "lightning", "delta",
+                        "streams", "dual")}}
 
 # *_hip.hip are build-time copies torch's extension builder leaves behind
 kernels = [p for p in sorted(CSRC.glob("*.hip"))

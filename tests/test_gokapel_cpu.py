@@ -564,7 +564,8 @@ def test_checkpoint_directory_round_trip(tmp_path):
     assert mc.layers[0].mixer.decay_rank == 6      # from the tensors
     assert mc.layers[0].mixer.gate_rank == 10
     assert mc.sliding_window == 35 and mc.norm_eps == 2e-5
-    assert mc.kernel_groups == ("core", "hybrid", "streams")
+    assert mc.kernel_groups == ("core", "delta", "shared_kv",
+                                "streams")
     m = build_model(mc, dtype=torch.float32)
     load_pretrained(m, d)
     ref = load(cfg, W, torch.float32)
@@ -639,7 +640,7 @@ def test_parts_serve_another_design():
     toks = [3, 1, 4, 1, 5, 9, 2, 6]
     whole = run_cut(eng, toks, [8])
     assert torch.allclose(whole, run_cut(eng, toks, [1]), atol=1e-5)
-    with pytest.raises(ValueError, match="residual"):
+    with pytest.raises(ValueError, match="layout"):
         layered_config("q", [LayerSpec(TwinSpec(left, MinGRUSpec(5)), None)],
                        16, 20)
     with pytest.raises(ValueError, match="mlp"):

@@ -443,8 +443,8 @@ def test_every_pass_has_a_cache_of_its_own():
     cfg, W = make("mixed")
     eng = make_engine(cfg, W)
     assert [i for i, _ in eng.model.runs] == [0, 1, 2, 3, 1, 2, 3, 4]
-    assert [e for _, e in eng.model.runs] == [False, True, False, False, True,
-                                              False, False, False]
+    assert [e for _, e in eng.model.runs] == [None, 0, None, None, 1, None,
+                                              None, None]
     assert len({c.data_ptr() for c in eng.caches}) == 8
     # state slots for the running requests and one for padded rows
     assert eng.caches[1].shape == (7, 3, 24, 16)
@@ -578,7 +578,7 @@ def test_checkpoint_directory_round_trip(tmp_path):
     back = config_from_keralorn(config_to_keralorn(mc))
     assert back.layers == mc.layers and back.loop == mc.loop
     assert mc.sliding_window == 64 and mc.norm_eps == 2e-5
-    assert mc.kernel_groups == ("core", "hybrid")
+    assert mc.kernel_groups == ("core", "lightning", "shared_kv")
     assert config_from_keralorn(make("full")[0]).sliding_window is None
     m = build_model(mc, dtype=torch.float32)
     load_pretrained(m, d)
@@ -679,7 +679,7 @@ def test_parts_serve_another_design():
     ref = oracle.rms_norm(x, g["norm_f.weight"], mc.norm_eps) @ \
         g["lm_head.weight"].T
     assert rel_err(whole, ref) < TOL
-    with pytest.raises(ValueError, match="do not mix"):
+    with pytest.raises(ValueError, match="layout"):
         layered_config("q", [LayerSpec(spec, None),
                              get_config("tiny-pimazen").layers[0]], 16, 20)
     with pytest.raises(ValueError, match="share latents"):
