@@ -10,8 +10,9 @@ bench ESTABLISHES the baseline. --mode train / serve select a single
 metric; --mode latent (latent attention) and --mode hybrid (attention on
 shared keys and values, lightning attention) measure prefill and decode of
 those models beside llama models of equal layer sizes, --mode streams (gated
-delta rule, minGRU, mixtures on residual streams) beside hybrid models of as
-many layers.
+delta rule, minGRU, mixtures on residual streams) and --mode dual (generalized
+delta rule, differential and positionless latent attention, PolyNorm) beside
+hybrid models of as many layers.
 
 Launch (driver):
   python bench.py --gpus 1 --steps K --warmup W
@@ -201,7 +202,10 @@ PAIRS = {"latent": (("pimazen-7b", "llama2-7b"), ("pimazen-1b", "llama-1b"),
                     ("tiny-keralorn", "tiny-llama")),
          "streams": (("gokapel-7b", "keralorn-7b"),
                      ("gokapel-1b", "keralorn-1b"),
-                     ("tiny-gokapel", "tiny-keralorn"))}
+                     ("tiny-gokapel", "tiny-keralorn")),
+         "dual": (("dopilorn-7b", "keralorn-7b"),
+                  ("dopilorn-1b", "keralorn-1b"),
+                  ("tiny-dopilorn", "tiny-keralorn"))}
 
 
 def _cut(name: str, layers: int):
@@ -248,7 +252,7 @@ def bench_pairs(args) -> list[dict]:
     cfgs = []
     for pair in pairs:
         cfgs += [get_config(m) for m in pair]
-        if args.mode == "streams":     # as many layers as the first
+        if args.mode in ("streams", "dual"):   # as many layers as the first
             cfgs[-1] = _cut(pair[1], cfgs[-2].num_layers)
     for cfg in cfgs:
         name = cfg.name
@@ -300,7 +304,7 @@ def main():
     p.add_argument("--steps", type=int, default=20)
     p.add_argument("--warmup", type=int, default=5)
     p.add_argument("--mode", choices=["both", "train", "serve", "latent",
-                                      "hybrid", "streams"],
+                                      "hybrid", "streams", "dual"],
                    default="both")
     p.add_argument("--model", default=None)
     p.add_argument("--seq-len", type=int, default=512)

@@ -29,8 +29,10 @@ def _project(z, w, tp: int):
     """The sublayer's pending output: fp32, or a split-K slab."""
     if tp == 1 and ops.decode_ready(w, z.shape[0]):
         return ops.decode_linear_raw(z, w, f32=True)[0]
-    out = ops.linear_f32(z, w)
-    return reduce_from_tp(out) if tp > 1 else out
+    out = ops.linear_f32_parts(z, w)
+    if tp == 1:
+        return out
+    return reduce_from_tp(out if out.dim() == 2 else out.sum(0))
 
 
 def _new_z(lay, y, w, filled: bool):

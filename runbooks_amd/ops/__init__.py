@@ -13,7 +13,8 @@ from .kvcache import BLOCK_SIZE, alloc_kv_cache, kv_append, kv_append_ref  # noq
 from .latent import alloc_latent_cache, pad_to  # noqa: F401
 from .lightning import alloc_lightning_state  # noqa: F401
 from .linear import (Linear, decode_linear_raw, decode_operand,  # noqa: F401
-                     decode_ready, fast_linear, linear_f32)
+                     decode_ready, fast_linear, linear_f32,
+                     linear_f32_parts)
 from .norm import (RMSNorm, join_res32, layernorm_res32, norm_res32,  # noqa: F401
                    rmsnorm, rmsnorm_ref, rmsnorm_res32)
 from .rope import rope, rope_frequencies, rope_ref, rope_tables  # noqa: F401

@@ -6,10 +6,12 @@
 // (norm weight, convolution and the direct path in one). A sequence's slot
 // keeps its last taps - 1 rows of n.
 //
-//  * canon_token: batches of single tokens, a workgroup per token
+//  * canon_token: batches of single tokens, a workgroup per token (with up to
+//    MAX_TAPS taps and one column group per thread everything is on its way
+//    before the reduction)
 //  * canon_rows, canon_conv, canon_tails: portions; the rows' factors first,
-//    then every token and column on its own (a tap's row comes from a cache),
-//    then the slots, which canon_conv has read
+//    then the convolution (with up to MAX_TAPS taps a thread inside a portion
+//    reads every row once), then the slots, which canon_conv has read
 
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
@@ -22,8 +24,9 @@ using rb::Ragged;
 
 constexpr int BLOCK = 256;
 constexpr int MAX_SUBS = 2;
+constexpr int MAX_TAPS = 4;            // taps that kernels are made for
 constexpr int TPT = 4;                 // tokens per thread
-constexpr int VECS = 32;               // column groups per workgroup
+constexpr int VECS = 64;               // column groups per workgroup
 constexpr int TILE = BLOCK / VECS * TPT;   // tokens per workgroup
 
 struct Args {
@@ -117,6 +120,52 @@ __global__ __launch_bounds__(BLOCK) void canon_token_kernel(Args a) {
   clear_padding<T>(a, t);
 }
 
+// the same with one column group per thread
+template <typename T, typename DT, int TAPS, int BLK>
+__global__ __launch_bounds__(BLK) void canon_token_wide_kernel(Args a) {
+  __shared__ float red[BLK / RB_WAVE];
+  const int64_t t = blockIdx.x;
+  const int c = threadIdx.x * 8, pos = a.b.positions[t];
+  const bool ok = c < a.D;
+  const int cc = ok ? c : 0;
+  float *tail = a.tails + (int64_t)a.b.slots[t] * (TAPS - 1) * a.D + cc;
+  float n[TAPS][8], f[MAX_SUBS][TAPS][8], ss = 0.0f;
+#pragma unroll
+  for (int j = 0; j < TAPS - 1; ++j)
+    rb::load_v<8>(tail + (int64_t)j * a.D, n[j]);
+#pragma unroll
+  for (int s = 0; s < MAX_SUBS; ++s)
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+      rb::load_v<8>(a.coef + ((int64_t)min(s, a.subs - 1) * TAPS + j) * a.D +
+                        cc, f[s][j]);
+  if (ok) {
+    add_pending<DT, 8>(a, t, c, n[TAPS - 1]);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) ss += n[TAPS - 1][k] * n[TAPS - 1][k];
+  }
+  ss = rb::block_reduce_sum(ss, red);
+  const float inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+  if (ok) {
+    float out[MAX_SUBS][8] = {};
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const bool real = pos >= TAPS - 1 - j;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        n[j][k] = j == TAPS - 1 ? n[j][k] * inv : real ? n[j][k] : 0.0f;
+#pragma unroll
+        for (int s = 0; s < MAX_SUBS; ++s) out[s][k] += f[s][j][k] * n[j][k];
+      }
+      if (j > 0) rb::store_v<8>(tail + (int64_t)(j - 1) * a.D, n[j]);
+    }
+#pragma unroll
+    for (int s = 0; s < MAX_SUBS; ++s)
+      if (s < a.subs) put<T, 8>(a, s, t, c, out[s]);
+  }
+  clear_padding<T>(a, t);
+}
+
 template <typename T, typename DT, int V>
 __global__ __launch_bounds__(BLOCK) void canon_rows_kernel(Args a) {
   __shared__ float red[BLOCK / RB_WAVE];
@@ -134,47 +183,70 @@ __global__ __launch_bounds__(BLOCK) void canon_rows_kernel(Args a) {
   clear_padding<T>(a, t);
 }
 
-template <typename T, int V>
+template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(BLOCK) void canon_conv_kernel(Args a) {
   const int c = (blockIdx.x * VECS + threadIdx.x % VECS) * V;
   const int t0 = blockIdx.y * TILE + threadIdx.x / VECS * TPT;
   if (c >= a.D || t0 >= a.T) return;
-  const int taps = a.b.taps;
-  rb::Source src[TPT];
+  if constexpr (TAPS > 1) {
+    const int end = t0 + TPT - 1;
+    if (end < a.T && a.b.seq_of[end] == a.b.seq_of[t0] &&
+        t0 - (TAPS - 1) >= a.b.cu_q[a.b.seq_of[t0]]) {
+      // the rows of this thread and those before them are one portion's
+      float n[TPT + TAPS - 1][V], f[MAX_SUBS][TAPS][V];
 #pragma unroll
-  for (int i = 0; i < TPT; ++i)
-    src[i] = rb::source_of(a.b, min(t0 + i, (int)a.T - 1));
-  float out[MAX_SUBS][TPT][V] = {};
-  for (int j = 0; j < taps; ++j) {
-    float f[MAX_SUBS][V] = {};
-#pragma unroll
-    for (int s = 0; s < MAX_SUBS; ++s)
-      if (s < a.subs)
-        rb::load_v<V>(a.coef + ((int64_t)s * taps + j) * a.D + c, f[s]);
-#pragma unroll
-    for (int i = 0; i < TPT; ++i) {
-      const int t = min(t0 + i, (int)a.T - 1), at = src[i].at(t, j, taps);
-      const float *row =
-          at >= 0 ? a.x + (int64_t)at * a.D
-                  : a.tails + ((int64_t)src[i].slot * (taps - 1) + ~at) * a.D;
-      const float m = at >= 0 ? a.inv[at] : 1.0f;
-      if (at == (int)0x80000000) continue;
-      float v[V];
-      rb::load_v<V>(row + c, v);
-#pragma unroll
-      for (int k = 0; k < V; ++k) v[k] *= m;
+      for (int i = 0; i < TPT + TAPS - 1; ++i)
+        rb::load_v<V>(a.x + (int64_t)(t0 - (TAPS - 1) + i) * a.D + c, n[i]);
 #pragma unroll
       for (int s = 0; s < MAX_SUBS; ++s)
 #pragma unroll
-        for (int k = 0; k < V; ++k) out[s][i][k] += f[s][k] * v[k];
+        for (int j = 0; j < TAPS; ++j)
+          rb::load_v<V>(a.coef + ((int64_t)min(s, a.subs - 1) * TAPS + j) *
+                            a.D + c, f[s][j]);
+#pragma unroll
+      for (int i = 0; i < TPT + TAPS - 1; ++i) {
+        const float m = a.inv[t0 - (TAPS - 1) + i];
+#pragma unroll
+        for (int k = 0; k < V; ++k) n[i][k] *= m;
+      }
+#pragma unroll
+      for (int i = 0; i < TPT; ++i)
+#pragma unroll
+        for (int s = 0; s < MAX_SUBS; ++s) {
+          float out[V] = {};
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+            for (int k = 0; k < V; ++k) out[k] += f[s][j][k] * n[i + j][k];
+          if (s < a.subs) put<T, V>(a, s, t0 + i, c, out);
+        }
+      return;
     }
   }
+  const int taps = a.b.taps;
+  for (int t = t0; t < min(t0 + TPT, (int)a.T); ++t) {
+    const rb::Source src = rb::source_of(a.b, t);
+    float out[MAX_SUBS][V] = {};
+    for (int j = 0; j < taps; ++j) {
+      const int at = src.at(t, j, taps);
+      if (at == (int)0x80000000) continue;
+      const float m = at >= 0 ? a.inv[at] : 1.0f;
+      float v[V];
+      rb::load_v<V>((at >= 0 ? a.x + (int64_t)at * a.D
+                             : a.tails + ((int64_t)src.slot * (taps - 1) +
+                                          ~at) * a.D) + c, v);
 #pragma unroll
-  for (int s = 0; s < MAX_SUBS; ++s) {
-    if (s >= a.subs) break;
+      for (int s = 0; s < MAX_SUBS; ++s) {
+        if (s >= a.subs) break;
+        float f[V];
+        rb::load_v<V>(a.coef + ((int64_t)s * taps + j) * a.D + c, f);
 #pragma unroll
-    for (int i = 0; i < TPT; ++i)
-      if (t0 + i < a.T) put<T, V>(a, s, t0 + i, c, out[s][i]);
+        for (int k = 0; k < V; ++k) out[s][k] += f[k] * (v[k] * m);
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < MAX_SUBS; ++s)
+      if (s < a.subs) put<T, V>(a, s, t, c, out[s]);
   }
 }
 
@@ -280,10 +352,31 @@ void canon_norm(at::Tensor x, c10::optional<at::Tensor> delta, at::Tensor coef,
     a.inv = inv.data_ptr<float>();
   }
   auto stream = at::hip::getCurrentHIPStream();
+  auto with_taps = [&](auto f) {
+    if (a.b.taps == 2) f(std::integral_constant<int, 2>{});
+    else if (a.b.taps == 3) f(std::integral_constant<int, 3>{});
+    else f(std::integral_constant<int, MAX_TAPS>{});
+  };
+  const bool made = D % 8 == 0 && a.b.taps >= 2 && a.b.taps <= MAX_TAPS;
   auto go = [&](auto tag, auto dtag, auto v) {
     using E = decltype(tag);
     using DT = decltype(dtag);
     constexpr int V = decltype(v)::value;
+    if (single && made && D <= 8192) {
+      with_taps([&](auto n) {
+        constexpr int N = decltype(n)::value;
+        if (D <= 2048)
+          hipLaunchKernelGGL((canon_token_wide_kernel<E, DT, N, 256>), dim3(T),
+                             dim3(256), 0, stream, a);
+        else if (D <= 4096)
+          hipLaunchKernelGGL((canon_token_wide_kernel<E, DT, N, 512>), dim3(T),
+                             dim3(512), 0, stream, a);
+        else
+          hipLaunchKernelGGL((canon_token_wide_kernel<E, DT, N, 1024>),
+                             dim3(T), dim3(1024), 0, stream, a);
+      });
+      return;
+    }
     if (single) {
       hipLaunchKernelGGL((canon_token_kernel<E, DT, V>), dim3(T), dim3(BLOCK),
                          0, stream, a);
@@ -293,9 +386,17 @@ void canon_norm(at::Tensor x, c10::optional<at::Tensor> delta, at::Tensor coef,
                        stream, a);
     const int64_t tiles = (T + TILE - 1) / TILE;
     TORCH_CHECK(tiles <= 65535, "canon_norm: ", T, " tokens");
-    hipLaunchKernelGGL((canon_conv_kernel<E, V>),
-                       dim3((D / V + VECS - 1) / VECS, tiles), dim3(BLOCK), 0,
-                       stream, a);
+    const dim3 grid((D / V + VECS - 1) / VECS, tiles);
+    if constexpr (V == 8) {
+      if (made)
+        with_taps([&](auto n) {
+          hipLaunchKernelGGL((canon_conv_kernel<E, 8, decltype(n)::value>),
+                             grid, dim3(BLOCK), 0, stream, a);
+        });
+    }
+    if (!made)
+      hipLaunchKernelGGL((canon_conv_kernel<E, V, 0>), grid, dim3(BLOCK), 0,
+                         stream, a);
     if (a.b.taps > 1)
       hipLaunchKernelGGL((canon_tails_kernel<V>),
                          dim3((D / V + BLOCK - 1) / BLOCK, n_seqs),

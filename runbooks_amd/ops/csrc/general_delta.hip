@@ -29,13 +29,23 @@
 //      S <- exp(G_C) S + (exp(G_C - G) k)^T V - (exp(G_C - G) alpha)^T P
 //
 //    A step's decay is bounded (|scale| <= 2), so the exponentials split into
-//    two factors around the chunk's middle, and all four matrices are plain
-//    products. general_delta_prep, parallel over chunks, inverts I + A (two
-//    triangular blocks, then the one below them) and leaves everything that
-//    multiplies S, V or P as MFMA operands in lane order; general_delta_scan
-//    walks the chunks, 16 state columns per four waves, in registers. An fp32
-//    factor enters a product as two bf16 parts (split.h), so the recurrence
-//    keeps fp32's quality; k, r and v are bf16 as they come.
+//    two factors around the chunk's middle, G_m. With
+//
+//      R_t = exp(G_t - G_m) r_t,   U_t = exp(G_(t-1) - G_m) u_t,
+//      K_s = exp(G_m - G_s) k_s,   N_s = exp(G_m - G_s) alpha_s
+//
+//    all four matrices are plain products of these rows, and so is the rest,
+//    on the state Z = exp(G_m) S:
+//
+//      P = (I + A)^-1 (U Z + B V),   O = R Z + Pk V - Pa P
+//      Z <- Z + K^T V - N^T P,       S <- exp(G_C - G_m) Z
+//
+//    general_delta_prep, parallel over chunks, inverts I + A (two triangular
+//    blocks, then the one below them) and leaves everything that multiplies Z,
+//    V or P as MFMA operands in lane order; general_delta_scan walks the
+//    chunks, 16 state columns per four waves, in registers. An fp32 factor
+//    enters a product as two bf16 parts (split.h), so the recurrence keeps
+//    fp32's quality; k, r and v are bf16 as they come.
 
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
@@ -189,15 +199,15 @@ __global__ __launch_bounds__(BLOCK) void general_delta_step_kernel(Args a) {
 // behind each other; V, exact in bf16, only the one.
 template <int DCP> struct Entry {
   static constexpr int KS = DCP / 32, TD = DCP / 16, OP = 2048;
-  static constexpr int W = 0;                  // [2 token tiles][KS], negative
-  static constexpr int Q = W + 2 * KS * OP;    // [2 token tiles][KS]
-  static constexpr int TB = Q + 2 * KS * OP;   // [2 token tiles], negative
+  static constexpr int W = 0;                  // -(I + A)^-1 U, [2 tiles][KS]
+  static constexpr int R = W + 2 * KS * OP;    // [2 token tiles][KS]
+  static constexpr int TB = R + 2 * KS * OP;   // -(I + A)^-1 B, [2 tiles]
   static constexpr int PK = TB + 2 * OP;       // [2 token tiles]
   static constexpr int PA = PK + 2 * OP;       // [2 token tiles]
   static constexpr int K = PA + 2 * OP;        // [TD]
-  static constexpr int A = K + TD * OP;        // [TD]
-  static constexpr int G = A + TD * OP;        // exp(G_C), [DCP] fp32
-  static constexpr int V = G + DCP * 4;        // [vc / 16][64 lanes]
+  static constexpr int N = K + TD * OP;        // [TD]
+  static constexpr int F = N + TD * OP;        // exp(G_m), exp(G_C - G_m) fp32
+  static constexpr int V = F + DCP * 8;        // [vc / 16][64 lanes]
   static __host__ __device__ int64_t bytes(int vc) {
     return V + (int64_t)((vc + 15) / 16) * 1024;
   }
@@ -207,10 +217,11 @@ constexpr int AS = C + 4;              // floats per row of a token matrix
 template <int DCP> struct Lds {
   static constexpr int RB = DCP + 8;   // 16-bit elements per row
   static constexpr int RS = DCP + 4;   // floats per row
-  static constexpr int bytes(int vcp) {
-    return C * RB * 4 + C * RS * 8 + C * (vcp + 8) * 2 + 3 * C * AS * 4 +
-           C * 4;
-  }
+  // four kinds of rows in two parts; before them, in their place, G and V
+  static constexpr int rows = 8 * C * RB * 2;
+  static constexpr int g = C * RS * 4;
+  static constexpr int bytes = rows + 2 * C * AS * 4;
+  static_assert(g + C * RB * 2 <= rows, "G and V");
 };
 
 // element k of a lane of group grp: the summed index within 32
@@ -222,7 +233,7 @@ RB_DEV void wave_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   __builtin_amdgcn_wave_barrier();
 }
-// the eight elements of a lane in a row of floats, of 16-bit values
+// a lane's elements of 32 columns of a row
 RB_DEV void row8(const float *row, int grp, float *f) {
   const f32x4v lo = *reinterpret_cast<const f32x4v *>(row + grp * 4);
   const f32x4v hi = *reinterpret_cast<const f32x4v *>(row + grp * 4 + 16);
@@ -232,15 +243,16 @@ RB_DEV void row8(const float *row, int grp, float *f) {
     f[k + 4] = hi[k];
   }
 }
-RB_DEV void row8(const uint16_t *row, int grp, float *f) {
+RB_DEV void row8(const uint16_t *row, int grp, Frag &f) {
   const uint2 lo = *reinterpret_cast<const uint2 *>(row + grp * 4);
   const uint2 hi = *reinterpret_cast<const uint2 *>(row + grp * 4 + 16);
-  const uint32_t w[4] = {lo.x, lo.y, hi.x, hi.y};
-#pragma unroll
-  for (int k = 0; k < 4; ++k) {
-    f[2 * k] = __uint_as_float(w[k] << 16);
-    f[2 * k + 1] = __uint_as_float(w[k] & 0xffff0000u);
-  }
+  f.u = (u32x4v){lo.x, lo.y, hi.x, hi.y};
+}
+// its elements of a column (l16) of 32 rows
+template <int RB> RB_DEV void column8(const uint16_t *rows, int lane, Frag &f) {
+  const int l16 = lane & 15, grp = lane >> 4;
+  const uint16_t *p = rows + (grp * 4 + (l16 >> 2)) * RB + (l16 & 3) * 4;
+  f.v = rb::lds_column8((const char *)p, (const char *)(p + 16 * RB));
 }
 RB_DEV void split_frag(const float *f, Frag *out) {
   split8(f, out[0].u, out[1].u);
@@ -253,19 +265,21 @@ RB_DEV f32x4v product(const Frag *a, const Frag *b, f32x4v c) {
 }
 
 template <int DCP>
-__global__ __launch_bounds__(PREP, 2) void general_delta_prep_kernel(Args a,
-                                                                     int vcp) {
+__global__ __launch_bounds__(PREP, DCP > 128 ? 2 : 4)
+void general_delta_prep_kernel(Args a, int vcp) {
   using E = Entry<DCP>;
   using T = uint16_t;
   constexpr int RB = Lds<DCP>::RB, RS = Lds<DCP>::RS, KS = E::KS;
+  constexpr int L = DCP / 8;                   // threads per token
+  constexpr int NV = (C * L + PREP - 1) / PREP;
+  constexpr int PART = C * RB;                 // elements of a part
+  enum { R = 0, U = 2, K = 4, N = 6 };         // first part of a kind of rows
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  float *al_s = reinterpret_cast<float *>(lds);          // alpha [C][RS]
-  float *g_s = al_s + C * RS;                            // G [C][RS]
-  float *a_s = g_s + C * RS, *b_s = a_s + C * AS, *t_s = b_s + C * AS;
-  float *nk_s = t_s + C * AS;                            // 1 / |k|
-  uint16_t *r_s = reinterpret_cast<uint16_t *>(nk_s + C);  // [C][RB]
-  uint16_t *k_s = r_s + C * RB, *v_s = k_s + C * RB;     // v [C][VB]
-  const int VB = vcp + 8;
+  uint16_t *rows = reinterpret_cast<uint16_t *>(lds);     // [8][C][RB]
+  float *g_s = reinterpret_cast<float *>(lds);            // [C][RS]
+  uint16_t *v_s = reinterpret_cast<uint16_t *>(lds + Lds<DCP>::g);  // [C][RB]
+  float *a_s = reinterpret_cast<float *>(lds + Lds<DCP>::rows);
+  float *b_s = a_s + C * AS;                   // A (then its inverse), B
 
   const int tid = threadIdx.x;
   const int lane = tid & 63, l16 = lane & 15, grp = lane >> 4;
@@ -278,72 +292,134 @@ __global__ __launch_bounds__(PREP, 2) void general_delta_prep_kernel(Args a,
   const int len = min(C, n - t0);
   char *entry = a.scratch + (((int64_t)blockIdx.z * a.chunks + blockIdx.y) *
                              a.heads + h) * a.entry;
-  auto put = [&](int at, const float *f) {
-    Frag x[2];
-    split_frag(f, x);
+  auto put = [&](int at, const Frag *x) {
     *reinterpret_cast<u32x4v *>(entry + at + lane * 16) = x[0].u;
     *reinterpret_cast<u32x4v *>(entry + at + 1024 + lane * 16) = x[1].u;
   };
 
-  // ---- r, k, v as they are; a and log2 w ----------------------------------
-  const T *rows = (const T *)a.y + (int64_t)(q0 + t0) * a.ny;
-  const T *rows2 = (const T *)a.y2 + (int64_t)(q0 + t0) * a.ny2;
-  const u32x4v zero4 = (u32x4v)(0u);
-#pragma unroll 2
-  for (int i = tid; i < C * (DCP / 8); i += PREP) {
-    const int t = i / (DCP / 8), d = i % (DCP / 8) * 8;
-    const bool ok = t < len && d < a.dc;
-    const T *p = rows + (int64_t)(ok ? t : 0) * a.ny + h * a.dc + (ok ? d : 0);
-    const T *p2 =
-        rows2 + (int64_t)(ok ? t : 0) * a.ny2 + h * a.dc + (ok ? d : 0);
-    const u32x4v r = *reinterpret_cast<const u32x4v *>(p);
-    const u32x4v k = *reinterpret_cast<const u32x4v *>(p + a.off_k);
-    float x[8], z[8];
-    rb::VIO<T>::load(p + a.off_a, x);
-    rb::VIO<T>::load(p2, z);
-    const float *b = a.bias + h * a.dc + (ok ? d : 0);
-    *reinterpret_cast<u32x4v *>(r_s + t * RB + d) = ok ? r : zero4;
-    *reinterpret_cast<u32x4v *>(k_s + t * RB + d) = ok ? k : zero4;
+  // ---- this thread's columns of r, k, a; log2 w and v to LDS ---------------
+  const T *y = (const T *)a.y + (int64_t)(q0 + t0) * a.ny;
+  const T *y2 = (const T *)a.y2 + (int64_t)(q0 + t0) * a.ny2;
+  float r[NV][8], k[NV][8], al[NV][8], nk[NV];
+  // the first round covers every thread when there are fewer vectors
+  auto vec = [&](int i, int &t, int &d) {
+    const int v = tid + i * PREP;
+    t = v / L;
+    d = v % L * 8;
+    return v < C * L;
+  };
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    int t, d;
+    const bool mine = vec(i, t, d), ok = mine && t < len && d < a.dc;
+    const int64_t tt = ok ? t : 0;
+    const int c = h * a.dc + (ok ? d : 0);
+    float z[8], b[2][8];
+    rb::VIO<T>::load(y + tt * a.ny + c, r[i]);
+    rb::VIO<T>::load(y + tt * a.ny + a.off_k + c, k[i]);
+    rb::VIO<T>::load(y + tt * a.ny + a.off_a + c, al[i]);
+    rb::VIO<T>::load(y2 + tt * a.ny2 + c, z);
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      al_s[t * RS + d + e] = ok ? sigmoid(x[e] + b[a.heads * a.dc + e]) : 0.0f;
-      g_s[t * RS + d + e] = ok ? a.scale * sigmoid(z[e] + b[e]) : 0.0f;
+      b[0][e] = a.bias[c + e];
+      b[1][e] = a.bias[a.heads * a.dc + c + e];
     }
+    float s = 0.0f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      if (!ok) r[i][e] = k[i][e] = 0.0f;
+      al[i][e] = sigmoid(al[i][e] + b[1][e]);
+      z[e] = ok ? a.scale * sigmoid(z[e] + b[0][e]) : 0.0f;
+      s += k[i][e] * k[i][e];
+    }
+#pragma unroll
+    for (int o = L / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+    nk[i] = 1.0f / sqrtf(s + UNIT_EPS);
+    if (mine) rb::VIO<float>::store(g_s + t * RS + d, z);
+    if (mine) rb::VIO<float>::store(g_s + t * RS + d + 4, z + 4);
   }
   for (int i = tid; i < C * (vcp / 8); i += PREP) {
     const int t = i / (vcp / 8), c = i % (vcp / 8) * 8;
-    u32x4v v = zero4;
+    u32x4v v = (u32x4v)(0u);
     if (t < len && c < a.vc)
-      v = *reinterpret_cast<const u32x4v *>(rows + (int64_t)t * a.ny +
-                                            a.off_v + h * a.vc + c);
-    *reinterpret_cast<u32x4v *>(v_s + t * VB + c) = v;
+      v = *reinterpret_cast<const u32x4v *>(y + (int64_t)t * a.ny + a.off_v +
+                                            h * a.vc + c);
+    *reinterpret_cast<u32x4v *>(v_s + t * RB + c) = v;
   }
   __syncthreads();
-  // ---- unit keys (16 lanes per token), alpha; sums of log2 w --------------
-  {
-    const int t = tid >> 4, l = tid & 15;
-    float s = 0.0f;
-    for (int d = l * 2; d < DCP; d += 32) {
-      const uint32_t w = *reinterpret_cast<const uint32_t *>(k_s + t * RB + d);
-      const float x = __uint_as_float(w << 16);
-      const float z = __uint_as_float(w & 0xffff0000u);
-      s += x * x + z * z;
+  // ---- G: sums of log2 w over tokens; the other waves write V -------------
+  constexpr int SUMS = (DCP + RB_WAVE - 1) / RB_WAVE;      // waves
+  if (wid < SUMS) {
+    const int d = tid;
+    if (d < DCP) {
+      float s[C];
+#pragma unroll
+      for (int t = 0; t < C; ++t) s[t] = g_s[t * RS + d];
+#pragma unroll
+      for (int t = 1; t < C; ++t) s[t] += s[t - 1];
+#pragma unroll
+      for (int t = 1; t < C; ++t) g_s[t * RS + d] = s[t];
+      float *f = reinterpret_cast<float *>(entry + E::F);
+      f[d] = __builtin_amdgcn_exp2f(s[C / 2 - 1]);
+      f[DCP + d] = __builtin_amdgcn_exp2f(s[C - 1] - s[C / 2 - 1]);
+    }
+  } else {
+    for (int i = wid - SUMS; i < vcp / 16; i += PREP / RB_WAVE - SUMS) {
+      Frag x;
+      column8<RB>(v_s + i * 16, lane, x);
+      *reinterpret_cast<u32x4v *>(entry + E::V + i * 1024 + lane * 16) = x.u;
+    }
+  }
+  __syncthreads();
+  // ---- the four kinds of rows, in two parts each ----------------------------
+  u32x4v part_r[NV][2], part_u[NV][2], part_k[NV][2], part_n[NV][2];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    int t, d;
+    if (!vec(i, t, d)) t = d = 0;
+    float g[8], before[8], mid[8], u[8], x[8];
+    const float *gp = g_s + t * RS + d;
+    const float *bp = gp - (t > 0 ? RS : 0), *mp = g_s + (C / 2 - 1) * RS + d;
+#pragma unroll
+    for (int e = 0; e < 8; e += 4) {
+      rb::VIO<float>::load(gp + e, g + e);
+      rb::VIO<float>::load(bp + e, before + e);
+      rb::VIO<float>::load(mp + e, mid + e);
     }
 #pragma unroll
-    for (int o = 8; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
-    const float nk = 1.0f / sqrtf(s + UNIT_EPS);
-    if (l == 0) nk_s[t] = nk;
-    for (int d = l; d < DCP; d += 16)
-      al_s[t * RS + d] *= rb::bf16_to_f32(k_s[t * RB + d]) * nk;
+    for (int e = 0; e < 8; ++e) {
+      u[e] = k[i][e] * nk[i];
+      x[e] = r[i][e] * __builtin_amdgcn_exp2f(g[e] - mid[e]);
+    }
+    split8(x, part_r[i][0], part_r[i][1]);
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+      x[e] = u[e] *
+             __builtin_amdgcn_exp2f((t > 0 ? before[e] : 0.0f) - mid[e]);
+    split8(x, part_u[i][0], part_u[i][1]);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      g[e] = __builtin_amdgcn_exp2f(mid[e] - g[e]);
+      x[e] = k[i][e] * g[e];
+    }
+    split8(x, part_k[i][0], part_k[i][1]);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = al[i][e] * u[e] * g[e];
+    split8(x, part_n[i][0], part_n[i][1]);
   }
-  for (int d = tid; d < DCP; d += PREP) {
-    float s[C];
+  __syncthreads();                             // G and V have been read
 #pragma unroll
-    for (int t = 0; t < C; ++t) s[t] = g_s[t * RS + d];
+  for (int i = 0; i < NV; ++i) {
+    int t, d;
+    if (!vec(i, t, d)) continue;
 #pragma unroll
-    for (int t = 1; t < C; ++t) s[t] += s[t - 1];
-#pragma unroll
-    for (int t = 1; t < C; ++t) g_s[t * RS + d] = s[t];
+    for (int p = 0; p < 2; ++p) {
+      uint16_t *at = rows + p * PART + t * RB + d;
+      *reinterpret_cast<u32x4v *>(at + R * PART) = part_r[i][p];
+      *reinterpret_cast<u32x4v *>(at + U * PART) = part_u[i][p];
+      *reinterpret_cast<u32x4v *>(at + K * PART) = part_k[i][p];
+      *reinterpret_cast<u32x4v *>(at + N * PART) = part_n[i][p];
+    }
   }
   __syncthreads();
   // ---- the four token matrices: a wave has 16 rows (tokens t) of one. The
@@ -352,47 +428,35 @@ __global__ __launch_bounds__(PREP, 2) void general_delta_prep_kernel(Args a,
   {
     const int with_r = wid >> 2, m = (wid >> 1) & 1, with_k = wid & 1;
     const int t = m * 16 + l16;
+    const uint16_t *tp = rows + (with_r ? R : U) * PART + t * RB;
+    const uint16_t *sp = rows + (with_k ? K : N) * PART + l16 * RB;
     f32x4v acc[2] = {(f32x4v)(0.0f), (f32x4v)(0.0f)};
-    const float nk = nk_s[t];
+#pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
-      float mid[8], f[8], e[8];
-      row8(g_s + (C / 2 - 1) * RS + ks * 32, grp, mid);
-      if (with_r) {
-        row8(r_s + t * RB + ks * 32, grp, f);
-        row8(g_s + t * RS + ks * 32, grp, e);
-      } else {
-        row8(k_s + t * RB + ks * 32, grp, f);
-        row8(g_s + max(t - 1, 0) * RS + ks * 32, grp, e);
-      }
       Frag row[2], col[2];
 #pragma unroll
-      for (int k = 0; k < 8; ++k) {
-        const float g = with_r || t > 0 ? e[k] : 0.0f;
-        f[k] *= __builtin_amdgcn_exp2f(g - mid[k]) * (with_r ? 1.0f : nk);
-      }
-      split_frag(f, row);
+      for (int p = 0; p < 2; ++p) row8(tp + p * PART + ks * 32, grp, row[p]);
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         if (j > m) break;                      // above the diagonal
-        const int s = j * 16 + l16;
-        if (with_k) row8(k_s + s * RB + ks * 32, grp, f);
-        else row8(al_s + s * RS + ks * 32, grp, f);
-        row8(g_s + s * RS + ks * 32, grp, e);
 #pragma unroll
-        for (int k = 0; k < 8; ++k)
-          f[k] *= __builtin_amdgcn_exp2f(mid[k] - e[k]);
-        split_frag(f, col);
+        for (int p = 0; p < 2; ++p)
+          row8(sp + p * PART + j * 16 * RB + ks * 32, grp, col[p]);
         acc[j] = product(col, row, acc[j]);
       }
+      if (with_r && with_k)                    // these rows multiply Z, too
+        put(E::R + (m * KS + ks) * E::OP, row);
     }
     float f[8];
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
-      const int s = index_of(grp, k);
-      f[k] = s < t || (with_r && s == t) ? acc[k >> 2][k & 3] : 0.0f;
+    for (int e = 0; e < 8; ++e) {
+      const int s = index_of(grp, e);
+      f[e] = s < t || (with_r && s == t) ? acc[e >> 2][e & 3] : 0.0f;
     }
     if (with_r) {
-      put((with_k ? E::PK : E::PA) + m * E::OP, f);
+      Frag x[2];
+      split_frag(f, x);
+      put((with_k ? E::PK : E::PA) + m * E::OP, x);
     } else {
       float *dst = (with_k ? b_s : a_s) + t * AS + grp * 4;
       *reinterpret_cast<f32x4v *>(dst) = (f32x4v){f[0], f[1], f[2], f[3]};
@@ -401,10 +465,10 @@ __global__ __launch_bounds__(PREP, 2) void general_delta_prep_kernel(Args a,
   }
   __syncthreads();
   if (wid == 0) {
-    // ---- (I + A)^-1: column l16 of a 16 x 16 block per lane, then the block
-    // below the diagonal, -T22 (A21 T11) -------------------------------------
+    // ---- (I + A)^-1 in A's place: column l16 of a 16 x 16 block per lane,
+    // then the block below the diagonal, -T22 (A21 T11) ---------------------
     const int b0 = (lane >> 4 & 1) * 16;
-    float x[16];
+    float x[16], f[8] = {}, z[8] = {};
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       x[i] = i == l16 ? 1.0f : 0.0f;
@@ -412,112 +476,80 @@ __global__ __launch_bounds__(PREP, 2) void general_delta_prep_kernel(Args a,
       for (int j = 0; j < i; ++j)
         x[i] -= a_s[(b0 + i) * AS + b0 + j] * x[j];
     }
+    wave_fence();
     if (lane < 32) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        t_s[(b0 + i) * AS + b0 + l16] = x[i];
-        if (b0 == 0) t_s[i * AS + 16 + l16] = 0.0f;
-      }
+      for (int i = 0; i < 16; ++i)
+        a_s[(b0 + i) * AS + b0 + l16] = x[i];
     }
     wave_fence();
-    float f[8] = {}, z[8] = {};
     Frag fa[2], fb[2];
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      f[k] = a_s[(16 + l16) * AS + grp * 4 + k];
-      z[k] = t_s[(grp * 4 + k) * AS + l16];
+    for (int e = 0; e < 4; ++e) {
+      f[e] = a_s[(16 + l16) * AS + grp * 4 + e];
+      z[e] = a_s[(grp * 4 + e) * AS + l16];
     }
     split_frag(f, fa);
     split_frag(z, fb);
     f32x4v c = product(fa, fb, (f32x4v)(0.0f));
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      f[k] = t_s[(16 + l16) * AS + 16 + grp * 4 + k];
-      z[k] = c[k];
+    for (int e = 0; e < 4; ++e) {
+      f[e] = a_s[(16 + l16) * AS + 16 + grp * 4 + e];
+      z[e] = c[e];
     }
     split_frag(f, fa);
     split_frag(z, fb);
     c = product(fa, fb, (f32x4v)(0.0f));
+    wave_fence();
 #pragma unroll
-    for (int k = 0; k < 4; ++k)
-      t_s[(16 + grp * 4 + k) * AS + l16] = -c[k];
+    for (int e = 0; e < 4; ++e)
+      a_s[(16 + grp * 4 + e) * AS + l16] = -c[e];
   } else {
-    // ---- operands that need no inverse ------------------------------------
-    const int nv = vcp / 16;
-    for (int i = wid - 1; i < 2 * KS + E::TD + nv; i += PREP / RB_WAVE - 1) {
-      float f[8], e[8];
-      if (i < 2 * KS) {
-        const int t = i / KS * 16 + l16, d = i % KS * 32;
-        row8(r_s + t * RB + d, grp, f);
-        row8(g_s + t * RS + d, grp, e);
-#pragma unroll
-        for (int k = 0; k < 8; ++k) f[k] *= __builtin_amdgcn_exp2f(e[k]);
-        put(E::Q + i * E::OP, f);
-      } else if (i < 2 * KS + E::TD) {
-        const int tile = i - 2 * KS, d = tile * 16 + l16;
-        const float last = g_s[(C - 1) * RS + d];
-#pragma unroll
-        for (int k = 0; k < 8; ++k) {
-          const int s = index_of(grp, k);
-          const float x = __builtin_amdgcn_exp2f(last - g_s[s * RS + d]);
-          f[k] = rb::bf16_to_f32(k_s[s * RB + d]) * x;
-          e[k] = al_s[s * RS + d] * x;
-        }
-        put(E::K + tile * E::OP, f);
-        put(E::A + tile * E::OP, e);
-      } else {
-        const int tile = i - 2 * KS - E::TD;
-        const uint16_t *p =
-            v_s + (grp * 4 + (l16 >> 2)) * VB + tile * 16 + (l16 & 3) * 4;
-        Frag x;
-        x.v = rb::lds_column8((const char *)p, (const char *)(p + 16 * VB));
-        *reinterpret_cast<u32x4v *>(entry + E::V + tile * 1024 + lane * 16) =
-            x.u;
-      }
+    // ---- the keys and alphas of a state row ---------------------------------
+    for (int i = wid - 1; i < 2 * E::TD; i += PREP / RB_WAVE - 1) {
+      const int tile = i >> 1;
+      const uint16_t *p = rows + (i & 1 ? N : K) * PART + tile * 16;
+      Frag x[2];
+      column8<RB>(p, lane, x[0]);
+      column8<RB>(p + PART, lane, x[1]);
+      put((i & 1 ? E::N : E::K) + tile * E::OP, x);
     }
-    for (int d = tid - RB_WAVE; d < DCP; d += PREP - RB_WAVE)
-      reinterpret_cast<float *>(entry + E::G)[d] =
-          __builtin_amdgcn_exp2f(g_s[(C - 1) * RS + d]);
   }
   __syncthreads();
-  // ---- what the inverse multiplies: exp(G_(t-1)) u, and B. A result's rows
-  // are the other factor's columns, so that it is an operand, too. -------------
+  // ---- what the inverse multiplies: U, and B. A result's rows are the other
+  // factor's columns, so that it is an operand, too. ---------------------------
   for (int i = wid; i < 2 * KS + 2; i += PREP / RB_WAVE) {
     const int m = i < 2 * KS ? i / KS : i - 2 * KS;
     float f[8], out[8];
     Frag inv[2], x[2];
-    row8(t_s + (m * 16 + l16) * AS, grp, f);
+    row8(a_s + (m * 16 + l16) * AS, grp, f);
     split_frag(f, inv);
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
       if (i < 2 * KS) {
-        const int d = i % KS * 32 + j * 16 + l16;
-#pragma unroll
-        for (int k = 0; k < 8; ++k) {
-          const int s = index_of(grp, k);
-          const float g = s > 0 ? g_s[(s - 1) * RS + d] : 0.0f;
-          f[k] = rb::bf16_to_f32(k_s[s * RB + d]) * nk_s[s] *
-                 __builtin_amdgcn_exp2f(g);
-        }
+        const uint16_t *p = rows + U * PART + i % KS * 32 + j * 16;
+        column8<RB>(p, lane, x[0]);
+        column8<RB>(p + PART, lane, x[1]);
       } else {
 #pragma unroll
-        for (int k = 0; k < 8; ++k)
-          f[k] = b_s[index_of(grp, k) * AS + j * 16 + l16];
+        for (int e = 0; e < 8; ++e)
+          f[e] = b_s[index_of(grp, e) * AS + j * 16 + l16];
+        split_frag(f, x);
       }
-      split_frag(f, x);
       const f32x4v c = product(x, inv, (f32x4v)(0.0f));
 #pragma unroll
-      for (int k = 0; k < 4; ++k) out[j * 4 + k] = -c[k];
+      for (int e = 0; e < 4; ++e) out[j * 4 + e] = -c[e];
     }
-    put(i < 2 * KS ? E::W + i * E::OP : E::TB + m * E::OP, out);
+    split_frag(out, x);
+    put(i < 2 * KS ? E::W + i * E::OP : E::TB + m * E::OP, x);
   }
 }
 
 // ---------------------------------------------------------------------------
 // chunks: the recurrence. Four waves own 16 state columns, a quarter of the
 // rows each, as MFMA result tiles; packed, two stacked ones are an operand.
-// They exchange their packed tiles through LDS. Two waves (one per tile of 16
-// tokens) make -P, the two others O; all four bring their rows up to date.
+// They exchange Z, packed, through LDS. Two waves (one per tile of 16 tokens)
+// make -P, the two others O; all four bring their rows up to date.
 // ---------------------------------------------------------------------------
 template <int DCP>
 __global__ __launch_bounds__(4 * RB_WAVE, 1)
@@ -557,34 +589,39 @@ void general_delta_scan_kernel(Args a) {
   float *op = a.o + (int64_t)(q0 + tok) * orow + h * a.vc + col;
   int left = n - tok;                          // tokens from this lane's on
 
-  // what multiplies S, V (TB or Pk; the keys) and P (Pa; alpha)
-  Frag ff[KS][2], tf[2], pf[2], kf[HT][2], af[HT][2], vf;
-  f32x4v gf[HT];
+  // what multiplies Z, V (TB or Pk; the keys) and P (Pa; the alphas)
+  struct Operands {
+    Frag ff[KS][2], tf[2], pf[2], kf[HT][2], af[HT][2], vf;
+    f32x4v f0[HT], f1[HT];                     // S to Z and back
+  };
   auto get = [&](Frag *f, const char *e) __attribute__((always_inline)) {
     f[0].u = *reinterpret_cast<const u32x4v *>(e + lane * 16);
     f[1].u = *reinterpret_cast<const u32x4v *>(e + 1024 + lane * 16);
   };
-  auto get_first = [&](const char *e) __attribute__((always_inline)) {
-    const char *f = e + (out ? E::Q : E::W) + m * KS * E::OP;
-#pragma unroll
-    for (int i = 0; i < KS; ++i) get(ff[i], f + i * E::OP);
-    get(tf, e + (out ? E::PK : E::TB) + m * E::OP);
-  };
-  auto get_second = [&](const char *e) __attribute__((always_inline)) {
-    get(pf, e + E::PA + m * E::OP);
+  auto load = [&](Operands &o, int c) __attribute__((always_inline)) {
+    const char *e = base + min(c, nc - 1) * stride;
+    o.vf.u = *reinterpret_cast<const u32x4v *>(e + E::V + cb * 1024 +
+                                               lane * 16);
 #pragma unroll
     for (int d = 0; d < HT; ++d) {
-      get(kf[d], e + E::K + (first + d) * E::OP);
-      get(af[d], e + E::A + (first + d) * E::OP);
-      gf[d] = *reinterpret_cast<const f32x4v *>(
-          e + E::G + ((first + d) * 16 + grp * 4) * 4);
+      const char *f = e + E::F + ((first + d) * 16 + grp * 4) * 4;
+      o.f0[d] = *reinterpret_cast<const f32x4v *>(f);
+      o.f1[d] = *reinterpret_cast<const f32x4v *>(f + DCP * 4);
+      get(o.kf[d], e + E::K + (first + d) * E::OP);
     }
-    vf.u = *reinterpret_cast<const u32x4v *>(e + E::V + cb * 1024 + lane * 16);
+    get(o.tf, e + (out ? E::PK : E::TB) + m * E::OP);
+    const char *f = e + (out ? E::R : E::W) + m * KS * E::OP;
+#pragma unroll
+    for (int i = 0; i < KS; ++i) get(o.ff[i], f + i * E::OP);
+#pragma unroll
+    for (int d = 0; d < HT; ++d) get(o.af[d], e + E::N + (first + d) * E::OP);
+    if (out) get(o.pf, e + E::PA + m * E::OP);
   };
-  get_first(base);
-  get_second(base);
-  for (int c = 0; c < nc; ++c) {
-    const char *next = base + min(c + 1, nc - 1) * stride;
+  auto step = [&](const Operands &o) __attribute__((always_inline)) {
+#pragma unroll
+    for (int d = 0; d < HT; ++d)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[d][r] *= o.f0[d][r];
     if (owns) {
 #pragma unroll
       for (int d = 0; d < HT; ++d) {
@@ -598,17 +635,13 @@ void general_delta_scan_kernel(Args a) {
     }
     // meanwhile: what V gives to the state and to the tokens
     f32x4v x[2];
-    x[0] = mfma(tf[0], vf, (f32x4v)(0.0f));
-    x[1] = mfma(tf[1], vf, (f32x4v)(0.0f));
-#pragma unroll
-    for (int d = 0; d < HT; ++d)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) S[d][r] *= gf[d][r];
+    x[0] = mfma(o.tf[0], o.vf, (f32x4v)(0.0f));
+    x[1] = mfma(o.tf[1], o.vf, (f32x4v)(0.0f));
 #pragma unroll
     for (int i = 0; i < 2; ++i)
 #pragma unroll
-      for (int d = 0; d < HT; ++d) S[d] = mfma(kf[d][i], vf, S[d]);
-    __syncthreads();                           // S; P has been read
+      for (int d = 0; d < HT; ++d) S[d] = mfma(o.kf[d][i], o.vf, S[d]);
+    __syncthreads();                           // Z; P has been read
     Frag sf[KS][2];
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -619,7 +652,7 @@ void general_delta_scan_kernel(Args a) {
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
       for (int i = 0; i < 3; ++i)
-        x[(ks * 3 + i) & 1] = part(i, ff[ks], sf[ks][0], sf[ks][1],
+        x[(ks * 3 + i) & 1] = part(i, o.ff[ks], sf[ks][0], sf[ks][1],
                                    x[(ks * 3 + i) & 1]);
     f32x4v y = x[0] + x[1];
     if (!out) {
@@ -629,30 +662,40 @@ void general_delta_scan_kernel(Args a) {
       reinterpret_cast<uint2 *>(&u_s[0][lane])[m] = big;
       reinterpret_cast<uint2 *>(&u_s[1][lane])[m] = small;
     }
-    __builtin_amdgcn_sched_barrier(0);
-    get_first(next);
-    __builtin_amdgcn_sched_barrier(0);
-    __syncthreads();                           // P; S has been read
+    __syncthreads();                           // P; Z has been read
     Frag u[2];
     u[0].u = u_s[0][lane];
     u[1].u = u_s[1][lane];
 #pragma unroll
     for (int i = 0; i < 3; ++i)
 #pragma unroll
-      for (int d = 0; d < HT; ++d) S[d] = part(i, af[d], u[0], u[1], S[d]);
+      for (int d = 0; d < HT; ++d) S[d] = part(i, o.af[d], u[0], u[1], S[d]);
+#pragma unroll
+    for (int d = 0; d < HT; ++d)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[d][r] *= o.f1[d][r];
     if (out) {
-      y = product(pf, u, y);
+      y = product(o.pf, u, y);
       if (col_ok) {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
           if (r < left) op[r * orow] = y[r];
       }
     }
-    __builtin_amdgcn_sched_barrier(0);
-    get_second(next);
-    __builtin_amdgcn_sched_barrier(0);
     op += C * orow;
     left -= C;
+  };
+  // a chunk's operands are on their way while the one before it is walked
+  Operands even, odd;
+  load(even, 0);
+  for (int c = 0; c < nc; c += 2) {
+    load(odd, c + 1);
+    __builtin_amdgcn_sched_barrier(0);
+    step(even);
+    if (c + 1 >= nc) break;
+    load(even, c + 2);
+    __builtin_amdgcn_sched_barrier(0);
+    step(odd);
   }
   if (!col_ok || !owns) return;
 #pragma unroll
@@ -721,20 +764,19 @@ template <int DCP>
 void launch_chunk(Args a, int64_t n_seqs, int64_t max_q,
                   const at::TensorOptions &options, hipStream_t stream) {
   const int vcp = (a.vc + 15) / 16 * 16;
-  constexpr int most = Lds<DCP>::bytes(256);
-  static_assert(most <= 159 * 1024, "LDS");
+  constexpr int shmem = Lds<DCP>::bytes;
+  static_assert(shmem <= 159 * 1024, "LDS");
   static bool once = [] {
     return hipFuncSetAttribute(
                reinterpret_cast<const void *>(&general_delta_prep_kernel<DCP>),
                hipFuncAttributeMaxDynamicSharedMemorySize,
-               most) == hipSuccess;
+               shmem) == hipSuccess;
   }();
-  const int shmem = Lds<DCP>::bytes(vcp);
-  TORCH_CHECK(once && shmem <= most, "general_delta_chunk: LDS size");
+  TORCH_CHECK(once && vcp <= DCP, "general_delta_chunk: LDS size");
   a.entry = Entry<DCP>::bytes(a.vc);
   // as many chunks at once as keep the entries in the last-level cache
   const int64_t all = (max_q + C - 1) / C;
-  const int64_t fit = ((int64_t)160 << 20) / (n_seqs * a.heads * a.entry);
+  const int64_t fit = ((int64_t)192 << 20) / (n_seqs * a.heads * a.entry);
   a.chunks = (int)std::min<int64_t>(all, std::max<int64_t>(fit, 16));
   TORCH_CHECK(a.chunks <= 65535, "general_delta_chunk: portion of ", max_q);
   auto scratch = at::empty({n_seqs * a.chunks * a.heads * a.entry}, options);
@@ -790,8 +832,9 @@ void general_delta_chunk(at::Tensor y, at::Tensor y2, at::Tensor bias,
   if (n_seqs == 0 || max_q == 0) return;
   const auto bytes = y.options().dtype(at::kByte);
   auto stream = at::hip::getCurrentHIPStream();
-  if (a.dc <= 32) launch_chunk<32>(a, n_seqs, max_q, bytes, stream);
-  else if (a.dc <= 64) launch_chunk<64>(a, n_seqs, max_q, bytes, stream);
-  else if (a.dc <= 128) launch_chunk<128>(a, n_seqs, max_q, bytes, stream);
+  const int wide = std::max(a.dc, a.vc);
+  if (wide <= 32) launch_chunk<32>(a, n_seqs, max_q, bytes, stream);
+  else if (wide <= 64) launch_chunk<64>(a, n_seqs, max_q, bytes, stream);
+  else if (wide <= 128) launch_chunk<128>(a, n_seqs, max_q, bytes, stream);
   else launch_chunk<256>(a, n_seqs, max_q, bytes, stream);
 }

@@ -24,17 +24,28 @@ RB_DEV void add_powers(Sums &a, float z) {
   a.s[2] += r * q;
 }
 
-// the first ff of ny columns of a row, V at a time
-template <typename T, int V>
-RB_DEV Sums row_sums(const T *row, int ff, float (*red)[BLOCK / RB_WAVE]) {
+// The first ff columns of a row, 8 at a time; the first NV groups of a thread
+// stay in `keep`.
+template <typename T, int BLK, int NV>
+RB_DEV Sums row_sums(const T *row, int ff, float (*red)[BLK / RB_WAVE],
+                     float (*keep)[8]) {
   Sums a{};
-#pragma unroll 2
-  for (int c = threadIdx.x * V; c < ff; c += BLOCK * V) {
-    float f[V];
-    rb::load_v<V>(row + c, f);
 #pragma unroll
-    for (int k = 0; k < V; ++k)
+  for (int n = 0; n < NV; ++n) {
+    const int c = (n * BLK + threadIdx.x) * 8;
+    if (c < ff) rb::load_v<8>(row + c, keep[n]);
+  }
+  auto add = [&](const float *f, int c) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k)
       if (c + k < ff) add_powers(a, f[k]);
+  };
+#pragma unroll
+  for (int n = 0; n < NV; ++n) add(keep[n], (n * BLK + threadIdx.x) * 8);
+  for (int c = (NV * BLK + threadIdx.x) * 8; c < ff; c += BLK * 8) {
+    float f[8];
+    rb::load_v<8>(row + c, f);
+    add(f, c);
   }
 #pragma unroll
   for (int i = 0; i < 3; ++i) {
@@ -46,7 +57,7 @@ RB_DEV Sums row_sums(const T *row, int ff, float (*red)[BLOCK / RB_WAVE]) {
   for (int i = 0; i < 3; ++i) {
     a.s[i] = 0.0f;
 #pragma unroll
-    for (int w = 0; w < BLOCK / RB_WAVE; ++w) a.s[i] += red[i][w];
+    for (int w = 0; w < BLK / RB_WAVE; ++w) a.s[i] += red[i][w];
   }
   return a;
 }
@@ -56,7 +67,8 @@ __global__ __launch_bounds__(BLOCK) void power_sums_kernel(
     const T *__restrict__ u, int64_t nu, int ff, float *__restrict__ out) {
   __shared__ float red[3][BLOCK / RB_WAVE];
   const int64_t t = blockIdx.x;
-  const Sums s = row_sums<T, 8>(u + t * nu, ff, red);
+  float keep[1][8];
+  const Sums s = row_sums<T, BLOCK, 1>(u + t * nu, ff, red, keep);
   if (threadIdx.x < 3) out[t * 3 + threadIdx.x] = s.s[threadIdx.x];
 }
 
@@ -66,20 +78,19 @@ struct PolyArgs {
   float total, eps;
 };
 
-template <typename T>
-__global__ __launch_bounds__(BLOCK) void poly_norm_kernel(
+template <typename T, int BLK, int NV>
+__global__ __launch_bounds__(BLK) void poly_norm_kernel(
     const T *__restrict__ u, const float *__restrict__ act,
     const float *__restrict__ sums, T *__restrict__ z, T *__restrict__ swz,
     PolyArgs a) {
-  __shared__ float red[3][BLOCK / RB_WAVE];
+  __shared__ float red[3][BLK / RB_WAVE];
   const int64_t t = blockIdx.x;
   const T *row = u + t * a.nu;
-  Sums s;
-  if (sums != nullptr) {
+  float keep[NV][8];
+  Sums s = row_sums<T, BLK, NV>(row, a.ff, red, keep);
+  if (sums != nullptr) {                       // of all ranks
 #pragma unroll
     for (int i = 0; i < 3; ++i) s.s[i] = sums[t * 3 + i];
-  } else {
-    s = row_sums<T, 8>(row, a.ff, red);
   }
   float f[3];
 #pragma unroll
@@ -88,10 +99,7 @@ __global__ __launch_bounds__(BLOCK) void poly_norm_kernel(
   const float e = act[3];
   const int n = (int)(a.nz - a.off);
   T *zr = z + t * a.nz + a.off;
-#pragma unroll 2
-  for (int c = threadIdx.x * 8; c < n; c += BLOCK * 8) {
-    float v[8] = {};
-    if (c < a.ff) rb::load_v<8>(row + c, v);
+  auto finish = [&](float *v, int c) {
 #pragma unroll
     for (int k = 0; k < 8; ++k)
       v[k] = c + k < a.ff
@@ -99,6 +107,16 @@ __global__ __launch_bounds__(BLOCK) void poly_norm_kernel(
     rb::store_v<8>(zr + c, v);
     if (swz != nullptr)
       rb::store_v<8>(swz + rb::operand_slot(a.off + c, (int)t), v);
+  };
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * BLK + threadIdx.x) * 8;
+    if (c < n) finish(keep[i], c);
+  }
+  for (int c = (NV * BLK + threadIdx.x) * 8; c < n; c += BLK * 8) {
+    float v[8] = {};
+    if (c < a.ff) rb::load_v<8>(row + c, v);
+    finish(v, c);
   }
 }
 
@@ -186,11 +204,21 @@ void poly_norm(at::Tensor u, int64_t ff, int64_t total, at::Tensor act,
   auto stream = at::hip::getCurrentHIPStream();
   auto go = [&](auto tag) {
     using E = decltype(tag);
-    hipLaunchKernelGGL((poly_norm_kernel<E>), dim3(T), dim3(BLOCK), 0, stream,
-                       (const E *)u.data_ptr(), act.data_ptr<float>(),
-                       sums ? sums->data_ptr<float>() : nullptr,
-                       (E *)z.data_ptr(), swz ? (E *)swz->data_ptr() : nullptr,
-                       a);
+    auto launch = [&](auto blk, auto nv) {
+      constexpr int B = decltype(blk)::value, N = decltype(nv)::value;
+      hipLaunchKernelGGL((poly_norm_kernel<E, B, N>), dim3(T), dim3(B), 0,
+                         stream, (const E *)u.data_ptr(),
+                         act.data_ptr<float>(),
+                         sums ? sums->data_ptr<float>() : nullptr,
+                         (E *)z.data_ptr(),
+                         swz ? (E *)swz->data_ptr() : nullptr, a);
+    };
+    constexpr std::integral_constant<int, 256> few{};
+    constexpr std::integral_constant<int, 1024> many{};
+    if (ff <= 256 * 8 * 2) launch(few, std::integral_constant<int, 2>{});
+    else if (T > 256 && ff <= 256 * 8 * 8)
+      launch(few, std::integral_constant<int, 8>{});
+    else launch(many, std::integral_constant<int, 2>{});
   };
   if (dt == at::kBFloat16) go(uint16_t{});
   else go(float{});

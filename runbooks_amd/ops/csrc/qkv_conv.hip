@@ -5,7 +5,8 @@
 // there is neither.
 //
 // With single tokens a thread also moves its columns of the slot; after
-// portions qkv_tails does.
+// portions qkv_tails does. With 2 to 4 taps a thread inside a portion reads
+// every row once.
 
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
@@ -20,6 +21,7 @@ using rb::Ragged;
 constexpr int BLOCK = 256;
 constexpr int VECS = 32;               // column groups per workgroup
 constexpr int MAX_TPT = 4;             // tokens per thread
+constexpr int MAX_TAPS = 4;            // taps that kernels are made for
 
 struct Args {
   const void *y;
@@ -48,40 +50,62 @@ RB_DEV void put(const Args &a, int64_t t, int c, const float *f) {
   rb::store_v<8>(row + col, f);
 }
 
-template <typename T, int TPT, bool SINGLE>
+template <typename T, int TPT, int TAPS, bool SINGLE>
 __global__ __launch_bounds__(BLOCK) void qkv_conv_kernel(Args a) {
   const int c = (blockIdx.x * VECS + threadIdx.x % VECS) * 8;
   const int t0 = (blockIdx.y * (BLOCK / VECS) + threadIdx.x / VECS) * TPT;
   if (c >= a.n || t0 >= a.T) return;
-  const int taps = a.b.taps;
-  rb::Source src[TPT];
-#pragma unroll
-  for (int i = 0; i < TPT; ++i)
-    src[i] = rb::source_of(a.b, min(t0 + i, (int)a.T - 1));
-  float bias[8], out[TPT][8] = {};
+  float bias[8];
   rb::load_v<8>(a.bias + c, bias);
-  for (int j = 0; j < taps; ++j) {
-    float w[8];
-    rb::load_v<8>(a.conv + (int64_t)j * a.n + c, w);
+  if constexpr (TAPS > 1 && !SINGLE) {
+    const int end = t0 + TPT - 1;
+    if (end < a.T && a.b.seq_of[end] == a.b.seq_of[t0] &&
+        t0 - (TAPS - 1) >= a.b.cu_q[a.b.seq_of[t0]]) {
+      // the rows of this thread and those before them are one portion's
+      float u[TPT + TAPS - 1][8], w[TAPS][8];
 #pragma unroll
-    for (int i = 0; i < TPT; ++i) {
-      const int t = min(t0 + i, (int)a.T - 1), at = src[i].at(t, j, taps);
-      T *tail = (T *)a.tails + (int64_t)src[i].slot * (taps - 1) * a.n + c;
+      for (int i = 0; i < TPT + TAPS - 1; ++i)
+        rb::load_v<8>((const T *)a.y + (t0 - (TAPS - 1) + i) * a.ny + c, u[i]);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+        rb::load_v<8>(a.conv + (int64_t)j * a.n + c, w[j]);
+#pragma unroll
+      for (int i = 0; i < TPT + TAPS - 1; ++i)
+#pragma unroll
+        for (int k = 0; k < 8; ++k) u[i][k] += bias[k];
+#pragma unroll
+      for (int i = 0; i < TPT; ++i) {
+        float out[8] = {};
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+          for (int k = 0; k < 8; ++k) out[k] += w[j][k] * u[i + j][k];
+        put<T>(a, t0 + i, c, out);
+      }
+      return;
+    }
+  }
+  const int taps = a.b.taps;
+  for (int t = t0; t < min(t0 + TPT, (int)a.T); ++t) {
+    const rb::Source src = rb::source_of(a.b, t);
+    T *tail = (T *)a.tails + (int64_t)src.slot * (taps - 1) * a.n + c;
+    float out[8] = {};
+    for (int j = 0; j < taps; ++j) {
+      const int at = src.at(t, j, taps);
       float v[8] = {};
       const bool some = at != (int)0x80000000;
       if (some)
         rb::load_v<8>(at >= 0 ? (const T *)a.y + at * a.ny + c
                               : tail + (int64_t)~at * a.n, v);
       if (SINGLE && j > 0) rb::store_v<8>(tail + (int64_t)(j - 1) * a.n, v);
-      if (some) {
+      if (!some) continue;
+      float w[8];
+      rb::load_v<8>(a.conv + (int64_t)j * a.n + c, w);
 #pragma unroll
-        for (int k = 0; k < 8; ++k) out[i][k] += w[k] * (v[k] + bias[k]);
-      }
+      for (int k = 0; k < 8; ++k) out[k] += w[k] * (v[k] + bias[k]);
     }
+    put<T>(a, t, c, out);
   }
-#pragma unroll
-  for (int i = 0; i < TPT; ++i)
-    if (t0 + i < a.T) put<T>(a, t0 + i, c, out[i]);
 }
 
 template <typename T>
@@ -169,12 +193,19 @@ void qkv_conv(at::Tensor y, at::Tensor bias, at::Tensor conv, at::Tensor tails,
       return dim3(groups, m);
     };
     if (single) {
-      hipLaunchKernelGGL((qkv_conv_kernel<E, 1, true>), tiles(1), dim3(BLOCK),
-                         0, stream, a);
+      hipLaunchKernelGGL((qkv_conv_kernel<E, 1, 0, true>), tiles(1),
+                         dim3(BLOCK), 0, stream, a);
       return;
     }
-    hipLaunchKernelGGL((qkv_conv_kernel<E, MAX_TPT, false>), tiles(MAX_TPT),
-                       dim3(BLOCK), 0, stream, a);
+    auto go = [&](auto n) {
+      hipLaunchKernelGGL(
+          (qkv_conv_kernel<E, MAX_TPT, decltype(n)::value, false>),
+          tiles(MAX_TPT), dim3(BLOCK), 0, stream, a);
+    };
+    if (a.b.taps == 2) go(std::integral_constant<int, 2>{});
+    else if (a.b.taps == 3) go(std::integral_constant<int, 3>{});
+    else if (a.b.taps == 4) go(std::integral_constant<int, MAX_TAPS>{});
+    else go(std::integral_constant<int, 0>{});
     if (a.b.taps > 1)
       hipLaunchKernelGGL((qkv_tails_kernel<E>),
                          dim3((n / 8 + BLOCK - 1) / BLOCK, n_seqs),

@@ -155,6 +155,26 @@ def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
     return F.linear(x, weight).float()
 
 
+# Row length beyond which hipBLASLt's choice is often poor: 300 to 570 us by
+# the number of rows around 2048, where two products of half the length
+# together take about 310 us at each.
+_LONG_ROW = 16384
+
+
+def linear_f32_parts(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """linear_f32 for a consumer that takes several parts: [T, N], or, of
+    long rows, [2, T, N] to be summed."""
+    K = x.shape[1]
+    if not (x.is_cuda and x.dtype == torch.bfloat16 and K > _LONG_ROW):
+        return linear_f32(x, weight)
+    out = torch.empty(2, x.shape[0], weight.shape[0], dtype=torch.float32,
+                      device=x.device)
+    half = K // 128 * 64
+    for o, at in zip(out, (slice(0, half), slice(half, K))):
+        torch.mm(x[:, at], weight[:, at].t(), out_dtype=torch.float32, out=o)
+    return out
+
+
 class Linear(torch.nn.Linear):
     """nn.Linear with the decode-GEMM fast path."""
 

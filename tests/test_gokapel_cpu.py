@@ -181,7 +181,7 @@ def test_delta_rule(taps, H, G, d, e):
             step = DR.delta_step if b.n_short else DR.delta_chunk
             step(a, a2, lay, conv, decay, state, b, o)
             z = torch.ones(n, lay.n_o + 8)
-            DR.delta_out(o, lay, w, a2, z, 1e-4, None, a, state, b)
+            DR.delta_out(o, lay, w, a2, z, 1e-4, None, a, state[1], b)
             assert not z[:, lay.n_o:].any()
             out.append(z[:, :lay.n_o].view(n, H, lay.vc)[..., :e])
             at, i = at + n, i + 1

@@ -249,7 +249,7 @@ def delta_run(lay, y, y2, conv, dec, state, ps, dev, dtype):
         swz = ops.decode_operand(len(y), n_z, z)
     w = torch.zeros(lay.vc, device=dev)
     w[:lay.vdim] = torch.linspace(0.5, 1.5, lay.vdim, device=dev)
-    DR.delta_out(o, lay, w, y2, z, 1e-5, swz, y, state, b)
+    DR.delta_out(o, lay, w, y2, z, 1e-5, swz, y, state[1], b)
     if swz is not None:
         assert torch.equal(operand_rows(swz, len(y)), z)
     return o, z
