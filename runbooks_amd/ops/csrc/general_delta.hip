@@ -301,7 +301,7 @@ void general_delta_prep_kernel(Args a, int vcp) {
   const T *y = (const T *)a.y + (int64_t)(q0 + t0) * a.ny;
   const T *y2 = (const T *)a.y2 + (int64_t)(q0 + t0) * a.ny2;
   float r[NV][8], k[NV][8], al[NV][8], nk[NV];
-  // the first round covers every thread when there are fewer vectors
+  // vector i of this thread: token and first column; false where there is none
   auto vec = [&](int i, int &t, int &d) {
     const int v = tid + i * PREP;
     t = v / L;

@@ -120,8 +120,8 @@ __global__ __launch_bounds__(BLOCK) void latent_prep_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// RMS norms of two latents in y: blocks (token, 0) the queries' one, to `out`
-// (zeros up to its no columns), blocks (token, 1) the cached one
+// RMS norms of two latents in y: blocks (token, 0) the queries' one, to `out`,
+// blocks (token, 1) the cached one, both with zeros up to the row's end
 // ---------------------------------------------------------------------------
 struct NormsArgs {
   int64_t ny;
@@ -135,29 +135,48 @@ __global__ __launch_bounds__(BLOCK) void latent_norms_kernel(
     const float *__restrict__ wc, T *__restrict__ out, T *__restrict__ swz,
     T *__restrict__ cache, const int *__restrict__ slots, NormsArgs a) {
   __shared__ float red[BLOCK / RB_WAVE];
+  constexpr int NV = 2;                        // 8-wide vectors kept
   const int64_t t = blockIdx.x;
   const bool cached = blockIdx.y > 0;
-  const int n = cached ? a.nc : a.nq;
+  const int n = cached ? a.nc : a.nq, width = cached ? a.ec : a.no;
   const T *row = y + t * a.ny + (cached ? a.oc : a.oq);
-  float ss = 0.0f;
-  for (int i = threadIdx.x; i < n; i += BLOCK) {
-    const float v = rb::bf16_to_f32_or_id(row[i]);
-    ss += v * v;
+  const float *w = cached ? wc : wq;
+  float v[NV][8], ss = 0.0f;
+  auto add = [&](const float *f, int c) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k) ss += c + k < n ? f[k] * f[k] : 0.0f;
+  };
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * BLOCK + threadIdx.x) * 8;
+    if (c < n) load8(row + c, v[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < NV; ++i) add(v[i], (i * BLOCK + threadIdx.x) * 8);
+  for (int c = (NV * BLOCK + threadIdx.x) * 8; c < n; c += BLOCK * 8) {
+    float f[8];
+    load8(row + c, f);
+    add(f, c);
   }
   ss = rb::block_reduce_sum(ss, red);
   const float ir = 1.0f / sqrtf(ss / (float)n + a.eps);
-  if (cached) {
-    T *dst = cache + (int64_t)slots[t] * a.ec;
-    for (int i = threadIdx.x; i < n; i += BLOCK)
-      rb::store_scalar(dst + i, rb::bf16_to_f32_or_id(row[i]) * ir * wc[i]);
-    return;
+  T *dst = cached ? cache + (int64_t)slots[t] * a.ec : out + t * a.no;
+  auto finish = [&](float *f, int c) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k)
+      f[k] = c + k < n ? f[k] * ir * w[c + k] : 0.0f;
+    store8(dst + c, f);
+    if (!cached && swz != nullptr) store8(swz + operand_at(c, (int)t), f);
+  };
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * BLOCK + threadIdx.x) * 8;
+    if (c < width) finish(v[i], c);
   }
-  for (int i = threadIdx.x; i < a.no; i += BLOCK) {
-    const float v =
-        i < n ? rb::bf16_to_f32_or_id(row[i]) * ir * wq[i] : 0.0f;
-    rb::store_scalar(out + t * a.no + i, v);
-    if (swz != nullptr)
-      rb::store_scalar(swz + operand_at(i & ~7, (int)t) + (i & 7), v);
+  for (int c = (NV * BLOCK + threadIdx.x) * 8; c < width; c += BLOCK * 8) {
+    float f[8] = {};
+    if (c < n) load8(row + c, f);
+    finish(f, c);
   }
 }
 
@@ -355,8 +374,12 @@ void latent_norms(at::Tensor y, int64_t oq, int64_t nq, at::Tensor wq,
               cache.scalar_type() == dt && slots.scalar_type() == at::kInt &&
               slots.is_contiguous() && slots.numel() == T,
               "latent_norms: tensors");
+  // rows of both latents are padded to 8 columns in y
   TORCH_CHECK(nq >= 1 && nq <= no && nc >= 1 && nc <= ec && oq >= 0 &&
-              oc >= 0 && oq + nq <= y.size(1) && oc + nc <= y.size(1) &&
+              oc >= 0 && oq % 8 == 0 && oc % 8 == 0 && no % 8 == 0 &&
+              ec % 8 == 0 && y.size(1) % 8 == 0 &&
+              oq + (nq + 7) / 8 * 8 <= y.size(1) &&
+              oc + (nc + 7) / 8 * 8 <= y.size(1) &&
               wq.scalar_type() == at::kFloat && wq.is_contiguous() &&
               wq.numel() == nq && wc.scalar_type() == at::kFloat &&
               wc.is_contiguous() && wc.numel() == nc, "latent_norms: layout");

@@ -286,11 +286,11 @@ def test_latent_attention_matches_plain_form(size, dtype, batch):
 
 @pytest.mark.parametrize("T", [1, 32, 300])
 @pytest.mark.parametrize("dtype", [BF, F32])
-@pytest.mark.parametrize("rq,rank", [(64, 512), (1, 3), (1500, 24)])
+@pytest.mark.parametrize("rq,rank", [(64, 512), (1, 3), (1500, 24),
+                                     (5000, 9000)])
 def test_norms_of_both_latents(rq, rank, dtype, T):
-    r = randn(T)
-    y = torch.nn.functional.pad(r(T, 8 + rq + rank), (0, -(rq + rank) % 8)
-                                ).to(dtype)
+    r, off = randn(T), 8 + -(-rq // 8) * 8
+    y = r(T, off + -(-rank // 8) * 8).to(dtype)
     slots = torch.randperm(320, generator=torch.Generator().manual_seed(1))
     slots = slots[:T].int()
     wq, wc = r(rq), r(rank)
@@ -302,7 +302,7 @@ def test_norms_of_both_latents(rq, rank, dtype, T):
         swz = None
         if operand and dev == DEV:
             swz = ops.decode_operand(T, -(-rq // 32) * 32, cache)
-        out = L.latent_norms(y.to(dev), ((8, 8 + rq), (rq, rank),
+        out = L.latent_norms(y.to(dev), ((8, off), (rq, rank),
                                          (wq.to(dev), wc.to(dev))), 1e-5,
                              slots.to(dev), cache, swz)
         res[dev] = (out, cache)
